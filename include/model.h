@@ -20,7 +20,8 @@ extern "C" {
  * reference, and the forward pass runs on the fp32 operators -- exact weights,
  * slower.  Prints the reference's report of the header and the detected format.
  * Fills p (incl. head_dim, rope_theta) and w.  Fatal errors print to stderr and
- * exit(1) like the reference.  Reference: src/model.c:110-285. */
+ * exit(1) like the reference.  Reference: src/model.c:110-285.
+ * A folder instead of a file: see "model folders" in nvllm.h. */
 void load_model(Weights* w, Config* p, const char* checkpoint_path);
 
 /* Allocate the activation workspace for up to p->max_seq_len tokens.

@@ -61,6 +61,54 @@ int nvllm_argmax_rows(int* out, const float* logits, int num_rows, int vocab_siz
 void nvllm_set_kv_elem_bytes(int bytes);
 int  nvllm_get_kv_elem_bytes(void);
 
+/* ------------------------------------------------------------- model folders */
+/* No counterpart in the reference, whose models are single files of one design.  load_model() also takes
+ * a FOLDER with config.json and model.safetensors: config.json's "architecture" picks the design from the
+ * library's registry (today: "Suselorn" -- latent attention with sinks, hyper-connected residual streams,
+ * Dynamic Tanh norms, a repeated span of layers).  Everything else -- transformer_batch, the block pool,
+ * the driver, sample() -- is used as with a model file; Config carries the sizes that make sense for both
+ * (n_layers counts layer RUNS), max_seq_len is the caller's to set before malloc_run_state (2048 on return).
+ *
+ * How such a model computes; to be set before load_model:
+ *   NVLLM_COMPUTE_BF16  (default) bf16 weights, activations and cache, fp32 accumulation; residual streams,
+ *                       norms, positions, attention scores and weights in fp32
+ *   NVLLM_COMPUTE_F32   everything in fp32 (weights expanded, an fp32 cache), on plain fp32 operators */
+enum { NVLLM_COMPUTE_BF16 = 0, NVLLM_COMPUTE_F32 = 1 };
+void nvllm_set_compute_dtype(int dtype);
+int  nvllm_get_compute_dtype(void);
+/* Is there a design of this name in the registry? */
+int nvllm_has_architecture(const char* name);
+
+/* The block pool of a loaded model, file or folder: what init_kv_cache_manager() is to a model file. */
+void nvllm_init_model_kv(KVCacheManager* mgr, int block_size, int num_blocks, const Config* p, const Weights* w);
+
+/* ---- operators of these designs (HBM pointers, fp32; enqueued on the library stream) */
+
+/* One hyper-connection step on x [num_tokens][streams][dim]:
+ *   y given (else x stays):  y' = (y + bias) * scale (bias may be null),
+ *                            x_to <- sum_from mix[from][to] x_from + out[to] y', all from the old x;
+ *   u = sum_s in[s] x_s;  out = tanh(alpha u) * norm_w + norm_b  (norm_w null: out = u; out null: not wanted).
+ * record: mix [streams][streams], out [streams], in [streams], alpha -- streams*streams + 2*streams + 1 floats. */
+void nvllm_hyper_step(float* x, const float* y, const float* bias, const float* scale, const float* record,
+                      const float* norm_w, const float* norm_b, float* out, int streams, int dim, int num_tokens);
+
+/* silu(g + bg) * (u + bu), biases per feature;  x <- cap * tanh(x / cap) */
+void nvllm_swiglu_bias(float* out, const float* g, const float* u, const float* bg, const float* bu, int hidden_dim, int num_tokens);
+void nvllm_softcap(float* x, float cap, long n);
+
+/* Attention over cached latents (one layer).  A pool of rows [latent (rank) | rotated key part (rot)] per position,
+ * fp32 rows (elem_bytes 4) or bf16 pages of 16 positions (elem_bytes 2). */
+void nvllm_latent_pool_init(KVCacheManager* mgr, int block_size, int num_blocks, int rank, int rot, int elem_bytes);
+/* kv [num_tokens][rank + rot]: RMS norm of the latent (gain, eps inside the root), rotation of the rest (pairs
+ * (2i, 2i+1) by pos * base^(-2i/rot)), write into the pool. */
+void nvllm_latent_cache_write(KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr, const float* kv, const float* gain,
+                              float eps, double base, int rank, int rot, int elem_bytes, int num_tokens);
+/* out [num_tokens][n_heads][rank]: softmax over the sequence's positions <= the token's, with exp(sink) in the
+ * denominator, of scale * (q . row), times the rows' latents.  q [num_tokens][n_heads][rank + rot] (rounded to bf16
+ * for a bf16 pool). */
+void nvllm_latent_attention(float* out, const float* q, KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr,
+                            const float* sink, float scale, int n_heads, int rank, int rot, int elem_bytes, int num_tokens);
+
 /* -------------------------------------------------- one launch per decode step */
 /* No counterpart in the reference, whose layer loop (src/model.c:358-394) calls one operator
  * after the other.  With the switch on (off by default; environment NVLLM_DECODE_CHAIN=1 turns it
@@ -264,6 +312,17 @@ int nvllm_engine_seq_state(const NvllmEngine* e, int seq, int* status, int* curr
                            int* n_prompt, int* seq_len);
 int nvllm_engine_history(const NvllmEngine* e, int seq, int* out, int cap);
 int nvllm_engine_block_table(const NvllmEngine* e, int seq, int* out, int cap);
+
+/* ---- the same driver, fed from outside (a server or a replay decides what each pass carries; nothing is
+ * sampled).  A slot that is idle (no request set, or ended) takes tokens portion by portion: */
+/* Append the next n tokens of slot `seq` to the coming pass, and ask for the logits at `want` (n_want indices into
+ * these tokens, ascending).  Blocks are allocated as by the scheduler.  Returns 0; -1 bad argument; -2 the pass or the
+ * sequence would exceed max_seq_len tokens; -3 the pool has no free block left (nothing of this call is kept). */
+int nvllm_engine_feed(NvllmEngine* e, int seq, const int* tokens, int n, const int* want, int n_want);
+/* Run the pass fed so far.  Returns its number of logits rows (nvllm_engine_logits(), in the order fed), -1 if nothing was fed. */
+int nvllm_engine_feed_run(NvllmEngine* e);
+/* The slot's sequence is over: its blocks go back to the pool and the slot is idle again. */
+int nvllm_engine_feed_end(NvllmEngine* e, int seq);
 
 /* The ragged batch of the most recent forward pass. */
 int nvllm_engine_last_batch(const NvllmEngine* e, int* tokens, int* pos, int* seq_ids, int cap,

@@ -138,6 +138,9 @@ _COMMON = {
     "nvllm_engine_last_batch": (_I, [_P, c_int_p, c_int_p, c_int_p, _I, c_int_p, c_int_p, _I, c_int_p]),
     "nvllm_engine_logits": (c_float_p, [_P]),
     "nvllm_engine_alloc_trace": (_I, [_P, c_int_p, _I]),
+    "nvllm_engine_feed": (_I, [_P, _I, c_int_p, _I, c_int_p, _I]),
+    "nvllm_engine_feed_run": (_I, [_P]),
+    "nvllm_engine_feed_end": (_I, [_P, _I]),
 }
 
 # only in the HIP library (include/backend.h, include/nvllm.h)
@@ -159,6 +162,18 @@ _HIP_ONLY = {
     "nvllm_forward_collect": (_I, [_L, c_int_p, _I]),
     "nvllm_set_kv_elem_bytes": (_V, [_I]),
     "nvllm_get_kv_elem_bytes": (_I, []),
+    "nvllm_set_compute_dtype": (_V, [_I]),
+    "nvllm_get_compute_dtype": (_I, []),
+    "nvllm_has_architecture": (_I, [C.c_char_p]),
+    "nvllm_init_model_kv": (_V, [C.POINTER(KVCacheManager), _I, _I, C.POINTER(Config), C.POINTER(Weights)]),
+    "nvllm_hyper_step": (_V, [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I]),
+    "nvllm_swiglu_bias": (_V, [_P, _P, _P, _P, _P, _I, _I]),
+    "nvllm_softcap": (_V, [_P, _F, _L]),
+    "nvllm_latent_pool_init": (_V, [C.POINTER(KVCacheManager), _I, _I, _I, _I, _I]),
+    "nvllm_latent_cache_write": (_V, [C.POINTER(KVCacheManager), C.POINTER(C.POINTER(BlockTable)), c_int_p, c_int_p, _P, _P,
+                                      _F, C.c_double, _I, _I, _I, _I]),
+    "nvllm_latent_attention": (_V, [_P, _P, C.POINTER(KVCacheManager), C.POINTER(C.POINTER(BlockTable)), c_int_p, c_int_p,
+                                    _P, _F, _I, _I, _I, _I, _I]),
     "nvllm_prof_enable": (_V, [_I]),
     "nvllm_prof_reset": (_V, []),
     "nvllm_prof_num_classes": (_I, []),
@@ -184,6 +199,7 @@ _HIP_ONLY = {
 }
 
 DEVICE_TO_HOST, DEVICE_TO_DEVICE, HOST_TO_DEVICE = 0, 1, 2
+COMPUTE_BF16, COMPUTE_F32 = 0, 1   # nvllm_set_compute_dtype
 
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 REPO_DIR = os.path.dirname(PKG_DIR)
@@ -346,6 +362,25 @@ class Engine:
         buf = (C.c_int * (3 * max(n, 1)))()
         self.lib.nvllm_engine_alloc_trace(self.h, buf, n)
         return np.array(buf[:3 * n], dtype=np.int32).reshape(n, 3)
+
+    # ---- passes put together by the caller
+    def feed(self, seq, tokens, want=()):
+        """The next tokens of slot `seq` join the coming pass; logits are wanted at the places `want` among them."""
+        t, w = ints(tokens), ints(sorted(want))
+        rc = self.lib.nvllm_engine_feed(self.h, seq, t, len(t), w, len(w))
+        if rc != 0:
+            raise ValueError({-2: "max_seq_len exceeded", -3: "out of cache blocks"}.get(rc, "bad portion") + f" (slot {seq})")
+
+    def feed_run(self) -> np.ndarray:
+        """Run the pass; logits rows in the order fed."""
+        n = self.lib.nvllm_engine_feed_run(self.h)
+        if n < 0:
+            raise ValueError("nothing was fed")
+        return self.logits(n) if n else np.zeros((0, self.config.vocab_size), np.float32)
+
+    def feed_end(self, seq):
+        if self.lib.nvllm_engine_feed_end(self.h, seq) != 0:
+            raise ValueError(f"slot {seq} is not a fed sequence")
 
     def close(self):
         if self.h:

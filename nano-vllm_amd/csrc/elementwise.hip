@@ -184,10 +184,18 @@ __global__ __launch_bounds__(256) void k_gather_rows_f32(float* __restrict__ dst
     for (int i = threadIdx.x; i < D / 4; i += blockDim.x) d[i] = s[i];
 }
 
+__global__ __launch_bounds__(256) void k_gather_rows_f32_any(float* __restrict__ dst, const float* __restrict__ src,
+                                                             const int* __restrict__ idx, int D) {
+    for (int i = threadIdx.x; i < D; i += blockDim.x) dst[(size_t)blockIdx.x * D + i] = src[(size_t)idx[blockIdx.x] * D + i];
+}
+
 void launch_gather_rows_f32(float* dst, const float* src, const int* idx, int B, int D) {
     if (B <= 0) return;
-    if (D % 4) NVLLM_FATAL("row width %d is not a multiple of 4", D);
     ProfScope ps(PC_EMBED, (double)B * D * 8.0, 0);
+    if (D % 4) {
+        NVLLM_LAUNCH(k_gather_rows_f32_any, dim3(B), dim3(256), 0, dst, src, idx, D);
+        return;
+    }
     NVLLM_LAUNCH(k_gather_rows_f32, dim3(B), dim3(256), 0, dst, src, idx, D);
 }
 

@@ -10,6 +10,26 @@ typedef _Float16 h8_t __attribute__((ext_vector_type(8)));
 typedef float f4_t __attribute__((ext_vector_type(4)));
 typedef unsigned int u4_t __attribute__((ext_vector_type(4)));
 
+typedef __bf16 b8_t __attribute__((ext_vector_type(8)));
+typedef __bf16 b4_t __attribute__((ext_vector_type(4)));
+
+// How activations enter a projection, and the multiply that goes with it.  Fragments travel as eight 16-bit
+// values per lane either way (h8_t); OpBf16 reinterprets their bits.
+struct OpF16x2 {   // fp16 weights; fp32 activations as fp16 hi + lo planes
+    static constexpr int PLANES = 2;
+    static __device__ __forceinline__ f4_t mfma(h8_t w, h8_t a, f4_t c) { return __builtin_amdgcn_mfma_f32_16x16x32_f16(w, a, c, 0, 0, 0); }
+};
+struct OpBf16 {    // bf16 weights, bf16 activations
+    static constexpr int PLANES = 1;
+    static __device__ __forceinline__ f4_t mfma(h8_t w, h8_t a, f4_t c) {
+        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, w), __builtin_bit_cast(b8_t, a), c, 0, 0, 0);
+    }
+};
+// epilogues that act on four consecutive features of one token at a time (epi_point below)
+constexpr bool epi_is_point(int kind) { return kind >= GemmEpilogue::TILE_B16; }
+// epilogues that also leave sums of squares per 32 features
+constexpr bool epi_has_ss(int kind) { return kind == GemmEpilogue::RESID_A16 || kind == GemmEpilogue::LATENT_IN; }
+
 struct GemmArgs {
     const __half* W;
     long nb_stride;   // halves between 16-row blocks
@@ -18,6 +38,9 @@ struct GemmArgs {
     const __half* A;  // activation tiles [Tb][Kb][2][512]
     int Tb;
     int N, T;
+    int act_Kb;       // k tiles per token block of A (Kb, or Kb * groups of a block-diagonal product)
+    int group_nb;     // block-diagonal product: 16-row blocks per group, 0 = one group ...
+    int group_tiles;  // ... and feature tiles per group (streaming kernel: grid columns)
     int kb_per_split;
     int ksplit;
     float* slab;      // [tile][slice][round][item] float4
@@ -99,6 +122,103 @@ template <>
 __device__ __forceinline__ void kv_put4_strided<__half>(__half* dst, const float* y) {
 #pragma unroll
     for (int e = 0; e < 4; e++) dst[4 * e] = kv_sat_half(y[e]);
+}
+
+__device__ __forceinline__ b4_t to_b4(const float* y) {
+    const f4_t v = {y[0], y[1], y[2], y[3]};
+    return __builtin_convertvector(v, b4_t);
+}
+// 4 consecutive k of token t into bf16 activation tiles (n % 4 == 0)
+__device__ __forceinline__ void store_b16_4(__half* act, int Kb_out, int t, int n, const float* y) {
+    const size_t tile = (size_t)(t >> 4) * Kb_out + (n >> 5);
+    const size_t off = (size_t)((t & 15) + 16 * ((n >> 3) & 3)) * 8 + (n & 7);
+    *reinterpret_cast<b4_t*>(act + tile * TILE_HALVES + off) = to_b4(y);
+}
+
+// Hyper-connection update of one token's features n .. n+3 and the next sublayer's input from it:
+//   x_to <- sum_from mix[from][to] x_from + out[to] * (y + bias) * scale;   u = sum_s in[s] x_s;
+//   act = tanh(alpha u) w + b
+template <int SMAX>
+__device__ __forceinline__ void hyper_update_4(const GemmEpilogue& ep, int N, int t, int n, const float* y_in) {
+    const int S = ep.streams;
+    float y[4];
+    const f4_t ls = *reinterpret_cast<const f4_t*>(ep.hyper_scale + n);
+    const f4_t bias = ep.bias ? *reinterpret_cast<const f4_t*>(ep.bias + n) : f4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int r = 0; r < 4; r++) y[r] = (y_in[r] + bias[r]) * ls[r];
+    f4_t xs[SMAX];
+    float* xr = ep.x + (size_t)t * S * N + n;
+#pragma unroll
+    for (int s = 0; s < SMAX; s++)
+        if (s < S) xs[s] = *reinterpret_cast<const f4_t*>(xr + (size_t)s * N);
+    const float* mix = ep.hyper;
+    const float* out = mix + S * S;
+    const float* in = out + S;
+    const float alpha = in[S];
+    f4_t u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int to = 0; to < SMAX; to++)
+        if (to < S) {
+            const float o = out[to], ii = in[to];
+            f4_t v;
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] = o * y[r];
+#pragma unroll
+            for (int s = 0; s < SMAX; s++)
+                if (s < S) {
+                    const float m = mix[s * S + to];
+#pragma unroll
+                    for (int r = 0; r < 4; r++) v[r] = fmaf(m, xs[s][r], v[r]);
+                }
+            *reinterpret_cast<f4_t*>(xr + (size_t)to * N) = v;
+#pragma unroll
+            for (int r = 0; r < 4; r++) u[r] = fmaf(ii, v[r], u[r]);
+        }
+    const f4_t w = *reinterpret_cast<const f4_t*>(ep.norm_w + n), b = *reinterpret_cast<const f4_t*>(ep.norm_b + n);
+    float z[4];
+#pragma unroll
+    for (int r = 0; r < 4; r++) z[r] = fmaf(tanhf(alpha * u[r]), w[r], b[r]);
+    store_b16_4(ep.a16_out, ep.Kb_out, t, n, z);
+}
+
+// One token's features n .. n+3 through a point epilogue; returns their share of the sum of squares.
+template <int EPI>
+__device__ __forceinline__ float epi_point(const GemmEpilogue& ep, int N, int t, int n, const float* y) {
+    if constexpr (EPI == GemmEpilogue::TILE_B16) {
+        store_b16_4(ep.a16_out, ep.Kb_out, t, n, y);
+    } else if constexpr (EPI == GemmEpilogue::ROWS_B16) {
+        const int h = n / ep.head_ld, d = n - h * ep.head_ld;
+        *reinterpret_cast<b4_t*>(ep.q_rows + ((size_t)t * ep.q_heads + h) * ep.q_row + d) = to_b4(y);
+    } else if constexpr (EPI == GemmEpilogue::LATENT_IN) {
+        if (n < ep.latent_q) {
+            const f4_t g = *reinterpret_cast<const f4_t*>(ep.gain_next + n);
+            const float z[4] = {y[0] * g[0], y[1] * g[1], y[2] * g[2], y[3] * g[3]};
+            store_b16_4(ep.a16_out, ep.Kb_out, t, n, z);
+            return y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3];
+        }
+        *reinterpret_cast<f4_t*>(ep.out + (size_t)t * ep.ldo + (n - ep.latent_q)) = f4_t{y[0], y[1], y[2], y[3]};
+    } else if constexpr (EPI == GemmEpilogue::LATENT_Q) {
+        if (n < ep.q_plain) {
+            store_b16_4(ep.a16_out, ep.Kb_out, t, n, y);
+        } else {
+            const int m = n - ep.q_plain, h = m / ep.rot_ld, d = m - h * ep.rot_ld;
+            float z[4] = {0.f, 0.f, 0.f, 0.f};
+            const float2* tab = ep.rope + (size_t)ep.pos[t] * (ep.rot_dim >> 1);
+#pragma unroll
+            for (int e = 0; e < 4; e += 2)
+                if (d + e < ep.rot_dim) {   // (features past rot_dim are padding)
+                    const float2 cs = tab[(d + e) >> 1];
+                    z[e] = y[e] * cs.x - y[e + 1] * cs.y;
+                    z[e + 1] = y[e + 1] * cs.x + y[e] * cs.y;
+                }
+            *reinterpret_cast<b4_t*>(ep.q_rows + ((size_t)t * ep.q_heads + h) * ep.q_row + ep.head_ld + d) = to_b4(z);
+        }
+    } else if constexpr (EPI == GemmEpilogue::HYPER_2) {
+        hyper_update_4<2>(ep, N, t, n, y);
+    } else {
+        hyper_update_4<4>(ep, N, t, n, y);
+    }
+    return 0.f;
 }
 
 // gemm_prefill.hip: 128 x 128 output tiles through LDS, for batches of hundreds of tokens

@@ -136,7 +136,8 @@ __device__ __forceinline__ void gemm_tile_prefetch(const GemmArgs& p, const Tile
 // spread over its last RW steps: the place to start loads for later work, a few at a time.
 // PRE: 0 = the tile requests its first RW K-steps of weights itself; 1 = the caller has (gemm_tile_prefetch);
 // 2 = the caller says at run time (`prefetched`, uniform over the workgroup).
-template <int NBW, int TB, int NW, int RW, int RA, int EPI, typename KVT, bool COH, int PRE, typename Hook>
+// OP: operand format (gemm_common.h); GRP: a block-diagonal product, whose tiles never cross a group.
+template <int NBW, int TB, int NW, int RW, int RA, int EPI, typename KVT, bool COH, int PRE, typename OP = OpF16x2, bool GRP = false, typename Hook>
 __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, unsigned char* lds_dyn, h8_t (&w)[RW][NBW],
                                           Hook&& slot_free, const int tid, const bool prefetched = true) {
     static_assert(NBW % 2 == 0, "row blocks are reduced in pairs");
@@ -157,8 +158,10 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
 
     const int lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int nb0 = ix.x * NBW;
-    if (nb0 >= p.NB) {   // grid padded for XCD alignment
+    const int grp = GRP ? ix.x / p.group_tiles : 0;
+    const int nb0 = GRP ? grp * p.group_nb + (ix.x - grp * p.group_tiles) * NBW : ix.x * NBW;
+    const int nb_lim = GRP ? min(p.NB, (grp + 1) * p.group_nb) : p.NB;   // row blocks this tile may touch
+    if (nb0 >= nb_lim) {   // grid padded for XCD alignment
 #pragma unroll
         for (int r = 0; r < RW; r++) slot_free(r);
         return false;
@@ -175,18 +178,21 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
     const h8_t* wp[NBW];
 #pragma unroll
     for (int i = 0; i < NBW; i++)
-        wp[i] = reinterpret_cast<const h8_t*>(p.W + (size_t)min(nb0 + i, p.NB - 1) * p.nb_stride) + lane;
+        wp[i] = reinterpret_cast<const h8_t*>(p.W + (size_t)min(nb0 + i, nb_lim - 1) * p.nb_stride) + lane;
     // activations: pointers (plain loads), or byte offsets into a buffer descriptor (sc1 loads)
     const h8_t* ap[TB];
     int aoff[TB];
     __amdgpu_buffer_rsrc_t rs_a = gemm_rsrc(p.A, (unsigned)p.Tb * (unsigned)p.Kb * 2048u);
 #pragma unroll
     for (int j = 0; j < TB; j++) {
-        ap[j] = reinterpret_cast<const h8_t*>(p.A + (size_t)min(tb0 + j, p.Tb - 1) * p.Kb * 2 * TILE_HALVES) + lane;
+        ap[j] = reinterpret_cast<const h8_t*>(p.A + ((size_t)min(tb0 + j, p.Tb - 1) * (GRP ? p.act_Kb : p.Kb) + (GRP ? grp * p.Kb : 0)) * OP::PLANES * TILE_HALVES) + lane;
         aoff[j] = min(tb0 + j, p.Tb - 1) * p.Kb * 2048 + lane * 16;
     }
+    static_assert(!COH || (OP::PLANES == 2 && !GRP), "the one-launch step runs fp16 models");
     auto load_act = [&](int j, int kb, h8_t& hi, h8_t& lo) {
-        if constexpr (COH) {
+        if constexpr (OP::PLANES == 1) {
+            hi = ap[j][(size_t)kb * 64];
+        } else if constexpr (COH) {
             hi = __builtin_bit_cast(h8_t, __builtin_amdgcn_raw_buffer_load_b128(rs_a, aoff[j], kb * 2048, AUX_SC1));
             lo = __builtin_bit_cast(h8_t, __builtin_amdgcn_raw_buffer_load_b128(rs_a, aoff[j] + 1024, kb * 2048, AUX_SC1));
         } else {
@@ -255,9 +261,9 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
                 for (int i = 0; i < NBW; i++)
 #pragma unroll
                     for (int j = 0; j < TB; j++) {
-                        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(w[r][i], ah[r % RA][j], acc[i][j], 0, 0, 0);
+                        acc[i][j] = OP::mfma(w[r][i], ah[r % RA][j], acc[i][j]);
 #ifndef NVLLM_ABLATE_LO
-                        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(w[r][i], al[r % RA][j], acc[i][j], 0, 0, 0);
+                        if constexpr (OP::PLANES == 2) acc[i][j] = OP::mfma(w[r][i], al[r % RA][j], acc[i][j]);
 #endif
                     }
                 if (s == 0) NVLLM_TSTAMP(2, acc[NBW - 1][TB - 1][0]);
@@ -429,10 +435,17 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
             const int t = tb0 * 16 + tl;
             const int nb = nb0 + 2 * h + i;
             const int n = nb * 16 + 4 * (l >> 4);
-            const bool live = t < p.T && tb0 + j < p.Tb && nb < p.NB;
+            const bool live = t < p.T && tb0 + j < p.Tb && nb < nb_lim;
             const float rinv = ep.ss_in ? s_rinv[tl] : 1.0f;
             float y[4] = {v[s][0] * rinv, v[s][1] * rinv, v[s][2] * rinv, v[s][3] * rinv};
-            if (EPI == GemmEpilogue::F32) {
+            if constexpr (epi_is_point(EPI)) {
+                if (live) ssq[s] += epi_point<EPI>(ep, p.N, t, n, y);
+            } else if (EPI == GemmEpilogue::F32) {
+                if constexpr (OP::PLANES == 1) {
+                    if (ep.softcap > 0.f)
+#pragma unroll
+                        for (int r = 0; r < 4; r++) y[r] = ep.softcap * tanhf(y[r] / ep.softcap);
+                }
                 if (live) {
                     float* o = ep.out + (size_t)t * ep.ldo + n;
                     if (n + 3 < p.N && (ep.ldo & 3) == 0) {
@@ -469,9 +482,19 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
                     const f4_t u = red[0][2 * h + 1][j][l];
                     float z[4];
 #pragma unroll
-                    for (int r = 0; r < 4; r++) z[r] = silu_mul(y[r], u[r] * rinv);
+                    for (int r = 0; r < 4; r++) {
+                        float gate = y[r], up = u[r] * rinv;
+                        if constexpr (OP::PLANES == 1) {   // (the up row of a hidden unit is 16 rows further on)
+                            if (ep.bias) {
+                                gate += ep.bias[n + r];
+                                up += ep.bias[n + 16 + r];
+                            }
+                        }
+                        z[r] = silu_mul(gate, up);
+                    }
                     const int hid = (nb >> 1) * 16 + 4 * (l >> 4);
-                    if constexpr (COH) store_a16_4_sc1(rs_o, ep.Kb_out, t, hid, z, l);
+                    if constexpr (OP::PLANES == 1) store_b16_4(ep.a16_out, ep.Kb_out, t, hid, z);
+                    else if constexpr (COH) store_a16_4_sc1(rs_o, ep.Kb_out, t, hid, z, l);
                     else store_a16_4(ep.a16_out, ep.Kb_out, t, hid, z);
                 }
             } else if (EPI == GemmEpilogue::RESID_A16) {
@@ -548,10 +571,10 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
             if (t < p.T) ep.amax_pairs[(size_t)ix.x * ep.amax_ld + t] = best;
         }
     }
-    if (EPI == GemmEpilogue::RESID_A16) {
+    if (epi_has_ss(EPI)) {
         // per-token sum of x^2 over each 32-feature group (= one round: two row blocks):
         // over the 4 lane groups (l>>4), then over the round's two row blocks (i)
-        const int ss_cols = (p.N + 31) >> 5;
+        const int ss_cols = EPI == GemmEpilogue::LATENT_IN ? ep.latent_q >> 5 : (p.N + 31) >> 5;
         // all rounds' halves meet in the array of the partial tiles (consumed: a barrier back), [round][half][token]:
         // one barrier for all rounds
         float (*ss_lds)[2][TB * 16] = reinterpret_cast<float (*)[2][TB * 16]>(lds_dyn);

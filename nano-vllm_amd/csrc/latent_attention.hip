@@ -1,0 +1,637 @@
+// latent_attention.hip -- attention over cached latents (latent_attention.h).
+//
+// k_latent_attn (bf16 pages).  A work item is up to CT consecutive tokens of one sequence x up to 16*C (token,
+// head) columns x a slice of the pages; all heads of a token share every cached row, so a row is read once per item.
+// The four waves of a workgroup walk the item's positions in blocks of 64 (four pages):
+//   copy    wave w brings page w global -> LDS with direct-to-LDS loads (pages are stored in operand order, so the
+//           image is lane-linear), one block ahead of the multiplication, two buffers;
+//   scores  wave w: S^T[key, col] = K_w Q^T over the whole row, C column groups per key fragment;
+//   softmax block maxima meet in LDS; every wave turns its 16 keys into weights, bf16, in the operand order of the
+//           next product (a score tile's registers ARE the k order that product uses, no shuffle);
+//   values  O^T[d, col] += V^T P: the latents again, as the transposed operand, through the LDS transpose read; the
+//           waves split the latent's dims, and `col` stays on the lane, so rescaling needs no exchange.
+// Scores, maxima and sums are fp32; queries, latents and weights enter the matrix cores as bf16.
+// The sink joins the denominator once, after the last slice (here, or in k_latent_combine when pages are sliced
+// across workgroups).
+//
+// k_latent_attn_any (fp32 rows, and bf16 rows wider than the kernel above has registers for): one workgroup per
+// (token, head), fp32 arithmetic on the vector units.
+#include "latent_attention.h"
+
+#include "attn_tile.h"
+#include "gemm_common.h"
+
+namespace nvllm {
+
+LatentPool latent_pool(void* base, int elem_bytes, int block_size, int rank, int rot) {
+    LatentPool p{base, elem_bytes, block_size, rank, rot, rank, rot};
+    if (elem_bytes == 2) {
+        if (block_size % LATENT_PAGE) NVLLM_FATAL("bf16 latent pages hold 16 positions: block size %d is not a multiple of 16", block_size);
+        p.rank_ld = (rank + 31) & ~31;
+        p.rot_ld = (rot + 31) & ~31;
+    }
+    return p;
+}
+
+// half index of element d of the row at pool row r (block * block_size + slot)
+__device__ __forceinline__ size_t latent_off(long r, int d, int row) {
+    return (size_t)(r >> 4) * 16 * row + (size_t)(d >> 5) * 512 + (size_t)(((int)r & 15) + 16 * ((d >> 3) & 3)) * 8 + (d & 7);
+}
+__device__ __forceinline__ float bf16_to_f32(unsigned short v) { return __builtin_bit_cast(float, (unsigned)v << 16); }
+
+// ------------------------------------------------------------------ cache write
+template <bool B16>
+__global__ __launch_bounds__(256) void k_latent_kv(void* base, const float* __restrict__ raw, int raw_ld, int rot_at, const float* __restrict__ gain,
+                                                   float eps, const float2* __restrict__ rope, const int* __restrict__ pos,
+                                                   const int* __restrict__ kv_row, int T, int rank, int rot, int rank_ld, int rot_ld) {
+    const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t >= T) return;
+    const long row = kv_row[t];
+    if (row < 0) return;
+    const float* src = raw + (size_t)t * raw_ld;
+    const int width = rank_ld + rot_ld;
+    float ss = 0.f;
+    for (int d = lane; d < rank; d += 64) ss = fmaf(src[d], src[d], ss);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float rms = sqrtf(ss / (float)rank + eps);
+    const float2* tab = rope + (size_t)pos[t] * (rot >> 1);
+    for (int d = 2 * lane; d < width; d += 128) {   // a pair of elements per lane (rank_ld is even in the padded layout)
+        float v[2] = {0.f, 0.f};
+        if (d >= rank_ld) {
+            const int r = d - rank_ld;
+            if (r < rot) {
+                const float2 cs = tab[r >> 1];
+                const float u = src[rot_at + r], w = src[rot_at + r + 1];
+                v[0] = u * cs.x - w * cs.y;
+                v[1] = w * cs.x + u * cs.y;
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 2; e++)
+                if (d + e < rank) v[e] = src[d + e] / rms * gain[d + e];
+        }
+        if (B16) {
+            typedef __bf16 b2_t __attribute__((ext_vector_type(2)));
+            typedef float f2_t __attribute__((ext_vector_type(2)));
+            const f2_t f = {v[0], v[1]};
+            *reinterpret_cast<b2_t*>(reinterpret_cast<__half*>(base) + latent_off(row, d, width)) = __builtin_convertvector(f, b2_t);
+        } else {
+            float* dst = reinterpret_cast<float*>(base) + (size_t)row * width + d;
+            dst[0] = v[0];
+            dst[1] = v[1];
+        }
+    }
+}
+// fp32 rows whose latent size is odd: pairs would straddle the two parts, so one element per lane
+__global__ __launch_bounds__(256) void k_latent_kv_odd(float* base, const float* __restrict__ raw, int raw_ld, int rot_at, const float* __restrict__ gain,
+                                                       float eps, const float2* __restrict__ rope, const int* __restrict__ pos,
+                                                       const int* __restrict__ kv_row, int T, int rank, int rot) {
+    const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t >= T) return;
+    const long row = kv_row[t];
+    if (row < 0) return;
+    const float* src = raw + (size_t)t * raw_ld;
+    float ss = 0.f;
+    for (int d = lane; d < rank; d += 64) ss = fmaf(src[d], src[d], ss);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float rms = sqrtf(ss / (float)rank + eps);
+    float* dst = base + (size_t)row * (rank + rot);
+    for (int d = lane; d < rank; d += 64) dst[d] = src[d] / rms * gain[d];
+    for (int i = lane; i < rot / 2; i += 64) {
+        const float2 cs = rope[(size_t)pos[t] * (rot >> 1) + i];
+        const float u = src[rot_at + 2 * i], w = src[rot_at + 2 * i + 1];
+        dst[rank + 2 * i] = u * cs.x - w * cs.y;
+        dst[rank + 2 * i + 1] = w * cs.x + u * cs.y;
+    }
+}
+
+void launch_latent_kv(const LatentPool& pool, const float* raw, int raw_ld, int rot_at, const float* gain, float eps, const float2* rope,
+                      const StepArrays& st) {
+    if (st.T <= 0) return;
+    ProfScope ps(PC_LATENT_KV, (double)st.T * ((double)raw_ld * 4.0 + (double)pool.row() * pool.elem_bytes), 0);
+    const dim3 grid(cdiv(st.T, 4));
+    if (pool.elem_bytes == 2)
+        NVLLM_LAUNCH((k_latent_kv<true>), grid, dim3(256), 0, pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
+                     pool.rot, pool.rank_ld, pool.rot_ld);
+    else if (pool.rank % 2)
+        NVLLM_LAUNCH(k_latent_kv_odd, grid, dim3(256), 0, (float*)pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
+                     pool.rot);
+    else
+        NVLLM_LAUNCH((k_latent_kv<false>), grid, dim3(256), 0, pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
+                     pool.rot, pool.rank_ld, pool.rot_ld);
+}
+
+// ------------------------------------------------------------------ attention, any size
+template <bool B16>
+__device__ __forceinline__ float latent_elem(const void* base, long r, int d, int row) {
+    if (B16) return bf16_to_f32(reinterpret_cast<const unsigned short*>(base)[latent_off(r, d, row)]);
+    return reinterpret_cast<const float*>(base)[(size_t)r * row + d];
+}
+
+template <bool B16>
+__global__ __launch_bounds__(256) void k_latent_attn_any(const void* base, const void* q, const float* __restrict__ sink, float scale,
+                                                         const int* __restrict__ pos, const int* __restrict__ seq,
+                                                         const int* __restrict__ tbl_off, const int* __restrict__ tables, int block_size, int H,
+                                                         int rank, int rank_ld, int row, float* out_f32, __half* out_b16, int Kb_out) {
+    extern __shared__ float lds_any[];   // q row [row], accumulators [rank_ld], weights [256], reductions [8]
+    float* sq = lds_any;
+    float* acc = sq + row;
+    float* sp = acc + rank_ld;
+    float* red = sp + 256;
+    const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    for (int d = tid; d < row; d += 256) {
+        const size_t i = ((size_t)t * H + h) * row + d;
+        sq[d] = B16 ? bf16_to_f32(reinterpret_cast<const unsigned short*>(q)[i]) : reinterpret_cast<const float*>(q)[i];
+    }
+    for (int d = tid; d < rank_ld; d += 256) acc[d] = 0.f;
+    const int p = pos[t];
+    const int* table = tables + tbl_off[seq[t]];
+    float m = -INFINITY, l = 0.f;   // the same in every thread
+    __syncthreads();
+    for (int k0 = 0; k0 <= p; k0 += 256) {
+        const int key = k0 + tid;
+        float s = -INFINITY;
+        if (key <= p) {
+            const long r = (long)table[key / block_size] * block_size + key % block_size;
+            float dot = 0.f;
+            for (int d = 0; d < row; d++) dot = fmaf(sq[d], latent_elem<B16>(base, r, d, row), dot);
+            s = dot * scale;
+        }
+        float mx = s;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
+        if (lane == 0) red[wave] = mx;
+        __syncthreads();
+        const float mn = fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+        const float e = key <= p ? expf(s - mn) : 0.f;
+        sp[tid] = e;
+        float sum = e;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
+        if (lane == 0) red[4 + wave] = sum;
+        __syncthreads();
+        const float alpha = m == -INFINITY ? 0.f : expf(m - mn);
+        l = l * alpha + ((red[4] + red[5]) + (red[6] + red[7]));
+        m = mn;
+        const int n = min(256, p - k0 + 1);
+        for (int d = tid; d < rank; d += 256) {
+            float a = acc[d] * alpha;
+            for (int k = 0; k < n; k++) {
+                const int kk = k0 + k;
+                const long r = (long)table[kk / block_size] * block_size + kk % block_size;
+                a = fmaf(sp[k], latent_elem<B16>(base, r, d, row), a);
+            }
+            acc[d] = a;
+        }
+        __syncthreads();   // weights and reductions are free again
+    }
+    const float top = fmaxf(m, sink[h]);
+    const float f = expf(m - top), den = l * f + expf(sink[h] - top);
+    for (int d = tid; d < rank_ld; d += 256) {
+        const float o = d < rank ? acc[d] * f / den : 0.f;
+        if (B16) {
+            const int k = h * rank_ld + d;
+            const __bf16 b = (__bf16)o;
+            reinterpret_cast<__bf16*>(out_b16)[((size_t)(t >> 4) * Kb_out + (k >> 5)) * TILE_HALVES + (size_t)((t & 15) + 16 * ((k >> 3) & 3)) * 8 + (k & 7)] = b;
+        } else {
+            out_f32[((size_t)t * H + h) * rank + d] = o;
+        }
+    }
+}
+
+// ------------------------------------------------------------------ attention, bf16 pages
+typedef short s4_t __attribute__((ext_vector_type(4)));
+typedef short s8_t __attribute__((ext_vector_type(8)));
+typedef __attribute__((address_space(3))) s4_t lds_s4;
+typedef __attribute__((address_space(3))) void lds_void_t;
+
+struct LatentKArgs {
+    const __half* base;
+    const __half* q;
+    const float* sink;
+    float scale;
+    const int* tables;
+    const int4* runs;     // (first token, count, last position, table offset)
+    int n_sub;            // items of CT tokens per run
+    int CT, HG, NG;       // tokens and heads per item; head groups
+    int H, nsplit;
+    int chunks;           // row / 32
+    int n_tiles;          // rank_ld / 16
+    int rank_ld;
+    int page_shift;       // log2(pages per block)
+    __half* out;
+    int Kb_out;
+    float* part_acc;      // [token][head][slice][rank_ld]
+    float* part_ml;       // [token][head][slice][2], log2 domain
+};
+
+constexpr int LATENT_BLOCK_PAGES = 4;
+static size_t latent_attn_lds(int chunks, int C) { return (size_t)2 * LATENT_BLOCK_PAGES * chunks * 1024 + (size_t)C * 2048 + (size_t)C * 2 * 4 * 16 * 4; }
+
+__device__ __forceinline__ void latent_copy_tile(const __half* lane_src, unsigned lds_byte_address) {
+    unsigned keep;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+                 : "=&s"(keep)
+                 : "v"(lane_src), "s"(lds_byte_address)
+                 : "memory");
+}
+// LDS stores of this wave are done, then everybody meets (copies to LDS in flight stay in flight)
+__device__ __forceinline__ void latent_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+
+// RC: row chunks of 32 held as query fragments; NT: 16-dim value tiles per wave; C: column groups of 16.
+// EXACT: the row has exactly RC chunks and 4 * NT value tiles.
+template <int RC, int NT, int C, bool EXACT>
+__global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds_latent[];
+    const int nc = EXACT ? RC : a.chunks;
+    const int n_tiles = EXACT ? 4 * NT : a.n_tiles;
+    __half* pages = reinterpret_cast<__half*>(lds_latent);                          // [2][4][nc][512]
+    __half* s_p = pages + (size_t)2 * LATENT_BLOCK_PAGES * nc * TILE_HALVES;        // [C][2][64][8]
+    float* s_max = reinterpret_cast<float*>(s_p + C * 2 * 64 * 8);                  // [C][4][16]
+    float* s_sum = s_max + C * 4 * 16;                                              // [C][4][16]
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int x = lane & 15, g = lane >> 4;
+
+    unsigned idx = blockIdx.x;
+    const int split = (int)(idx % (unsigned)a.nsplit);
+    idx /= (unsigned)a.nsplit;
+    const int hg = (int)(idx % (unsigned)a.NG);
+    idx /= (unsigned)a.NG;
+    const int sub = (int)(idx % (unsigned)a.n_sub);
+    const int4 run = a.runs[idx / (unsigned)a.n_sub];
+    const int first = sub * a.CT;
+    if (first >= run.y) return;
+    const int ntok = min(a.CT, run.y - first), t0 = run.x + first;
+    const int plast = run.z - (run.y - first - ntok);
+    const int h0 = hg * a.HG;
+    const int* table = a.tables + run.w;
+    const int npages = (plast >> 4) + 1, nblocks = (npages + LATENT_BLOCK_PAGES - 1) / LATENT_BLOCK_PAGES;
+    const int per = (nblocks + a.nsplit - 1) / a.nsplit;
+    const int b0 = split * per, b1 = min(nblocks, b0 + per);
+    const int row = nc * 32;
+
+    // this lane's columns: (token, head), the last position they see
+    int colt[C], colh[C], plim[C];
+    bool valid[C];
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        const int j = 16 * c + x, tok = j / a.HG, h = h0 + j - tok * a.HG;
+        valid[c] = tok < ntok && h < a.H;
+        colt[c] = t0 + (valid[c] ? tok : 0);
+        colh[c] = valid[c] ? h : 0;
+        plim[c] = valid[c] ? plast - (ntok - 1 - tok) : -1;
+    }
+
+    const unsigned lds0 = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(wave * nc) * 1024u;
+    auto issue = [&](int b, int buf) {   // page `wave` of block b (past the end: the last page again, its keys are masked)
+        const int pg = min(b * LATENT_BLOCK_PAGES + wave, npages - 1);
+        const long page = ((long)table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1));
+        const __half* src = a.base + (size_t)page * LATENT_PAGE * row + lane * 8;
+        const unsigned dst = lds0 + (unsigned)(buf * LATENT_BLOCK_PAGES * nc) * 1024u;
+#pragma unroll
+        for (int c = 0; c < RC; c++)
+            if (EXACT || c < nc) latent_copy_tile(src + (size_t)c * TILE_HALVES, __builtin_amdgcn_readfirstlane(dst + (unsigned)c * 1024u));
+    };
+
+    float m[C], lsum[C];
+    f4_t acc[NT][C];
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        m[c] = -INFINITY;
+        lsum[c] = 0.f;
+#pragma unroll
+        for (int n = 0; n < NT; n++) acc[n][c] = f4_t{0.f, 0.f, 0.f, 0.f};
+    }
+    if (b0 < b1) issue(b0, 0);
+    // queries as the B operand: column x, dims 32k + 8g .. +7
+    b8_t qf[C][RC];
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        const __half* qr = a.q + ((size_t)colt[c] * a.H + colh[c]) * row + 8 * g;
+#pragma unroll
+        for (int k = 0; k < RC; k++) {
+            qf[c][k] = b8_t{};
+            if ((EXACT || k < nc) && valid[c]) qf[c][k] = *reinterpret_cast<const b8_t*>(qr + 32 * k);
+        }
+    }
+    const float sl2 = a.scale * 1.44269504088896340736f;   // scores in the log2 domain
+    // transpose read: 16 lanes bring 4 keys x 16 dims, lane i gets dim i of the 4 keys
+    const int tr_key = 4 * g + (x >> 2), tr_sub = (x & 3) >> 1, tr_off = 4 * (x & 1);
+
+    for (int b = b0; b < b1; b++) {
+        const int buf = (b - b0) & 1;
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // this wave's page of block b is in LDS
+        latent_barrier();                                   // ... and everybody's; block b - 1 has been consumed
+        if (b + 1 < b1) issue(b + 1, buf ^ 1);
+        const __half* blk = pages + (size_t)buf * LATENT_BLOCK_PAGES * nc * TILE_HALVES;
+        // ---- scores of this wave's page
+        f4_t s[C];
+#pragma unroll
+        for (int c = 0; c < C; c++) s[c] = f4_t{0.f, 0.f, 0.f, 0.f};
+        const b8_t* kp = reinterpret_cast<const b8_t*>(blk + (size_t)wave * nc * TILE_HALVES) + lane;
+#pragma unroll
+        for (int k = 0; k < RC; k++)
+            if (EXACT || k < nc) {
+                const b8_t kf = kp[k * 64];
+#pragma unroll
+                for (int c = 0; c < C; c++) s[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[c][k], s[c], 0, 0, 0);
+            }
+        const int kfirst = (b * LATENT_BLOCK_PAGES + wave) * LATENT_PAGE + 4 * g;
+#pragma unroll
+        for (int c = 0; c < C; c++) {
+            float mx = -INFINITY;
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                s[c][r] = kfirst + r <= plim[c] ? s[c][r] * sl2 : -INFINITY;
+                mx = fmaxf(mx, s[c][r]);
+            }
+            mx = rows_max(mx);
+            if (g == 0) s_max[(c * 4 + wave) * 16 + x] = mx;
+        }
+        latent_barrier();
+        // ---- weights
+        float alpha[C];
+        bool rises = false;
+#pragma unroll
+        for (int c = 0; c < C; c++) {
+            const float* bm = s_max + c * 64 + x;
+            const float mn = fmaxf(m[c], fmaxf(fmaxf(bm[0], bm[16]), fmaxf(bm[32], bm[48])));
+            alpha[c] = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[c] - mn);
+            rises |= mn > m[c];
+            m[c] = mn;
+            const float msafe = fmaxf(mn, -1.0e30f);   // nothing visible yet: exp2(-inf - finite) = 0, no NaN
+            lsum[c] *= alpha[c];
+            float p[4];
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                p[r] = __builtin_amdgcn_exp2f(s[c][r] - msafe);
+                lsum[c] += p[r];
+            }
+            *reinterpret_cast<b4_t*>(s_p + ((size_t)(c * 2 + (wave >> 1)) * 64 + lane) * 8 + (wave & 1) * 4) = to_b4(p);
+        }
+        if (__any(rises)) {
+#pragma unroll
+            for (int n = 0; n < NT; n++)
+#pragma unroll
+                for (int c = 0; c < C; c++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) acc[n][c][r] *= alpha[c];
+        }
+        latent_barrier();
+        // ---- values: keys of pages (0, 1), then (2, 3)
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            b8_t pf[C];
+#pragma unroll
+            for (int c = 0; c < C; c++) pf[c] = *reinterpret_cast<const b8_t*>(s_p + ((size_t)(c * 2 + h) * 64 + lane) * 8);
+            const __half* v0 = blk + (size_t)(2 * h) * nc * TILE_HALVES + tr_off;
+            const __half* v1 = v0 + (size_t)nc * TILE_HALVES;
+#pragma unroll
+            for (int i = 0; i < NT; i++) {
+                const int n = wave + 4 * i;
+                if (EXACT || n < n_tiles) {
+                    const int off = (n >> 1) * TILE_HALVES + (tr_key + 16 * (2 * (n & 1) + tr_sub)) * 8;
+                    const s4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(v0 + off));
+                    const s4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(v1 + off));
+                    const s8_t both = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+                    const b8_t vf = __builtin_bit_cast(b8_t, both);
+#pragma unroll
+                    for (int c = 0; c < C; c++) acc[i][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[c], acc[i][c], 0, 0, 0);
+                }
+            }
+        }
+    }
+    // ---- the waves' partial sums meet; the sink; the result
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        lsum[c] += __shfl_xor(lsum[c], 16, 64);
+        lsum[c] += __shfl_xor(lsum[c], 32, 64);
+        if (g == 0) s_sum[(c * 4 + wave) * 16 + x] = lsum[c];
+    }
+    latent_barrier();
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        const float* bs = s_sum + c * 64 + x;
+        const float L = (bs[0] + bs[16]) + (bs[32] + bs[48]);
+        if (!valid[c]) continue;
+        float f = 1.f;
+        const size_t th = (size_t)colt[c] * a.H + colh[c];
+        if (a.nsplit == 1) {
+            const float sk = a.sink[colh[c]] * 1.44269504088896340736f, top = fmaxf(m[c], sk);
+            const float w = __builtin_amdgcn_exp2f(m[c] - top);
+            f = w / fmaf(L, w, __builtin_amdgcn_exp2f(sk - top));
+        } else if (wave == 0 && g == 0) {
+            a.part_ml[(th * a.nsplit + split) * 2] = m[c];
+            a.part_ml[(th * a.nsplit + split) * 2 + 1] = L;
+        }
+#pragma unroll
+        for (int i = 0; i < NT; i++) {
+            const int n = wave + 4 * i;
+            if (!(EXACT || n < n_tiles)) continue;
+            const int d = 16 * n + 4 * g;
+            if (a.nsplit == 1) {
+                const float o[4] = {acc[i][c][0] * f, acc[i][c][1] * f, acc[i][c][2] * f, acc[i][c][3] * f};
+                store_b16_4(a.out, a.Kb_out, colt[c], colh[c] * a.rank_ld + d, o);
+            } else {
+                *reinterpret_cast<f4_t*>(a.part_acc + (th * a.nsplit + split) * a.rank_ld + d) = acc[i][c];
+            }
+        }
+    }
+}
+
+// slices of one (token, head) -> the attended latent, the sink in the denominator
+__global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
+                                                        const float* __restrict__ sink, int H, int nsplit, int rank_ld, __half* out, int Kb_out) {
+    const int t = blockIdx.x / H, h = blockIdx.x % H;
+    const size_t th = blockIdx.x;
+    const float* ml = part_ml + th * nsplit * 2;
+    const float sk = sink[h] * 1.44269504088896340736f;
+    float top = sk;
+    for (int s = 0; s < nsplit; s++) top = fmaxf(top, ml[2 * s]);
+    float den = __builtin_amdgcn_exp2f(sk - top);
+    for (int s = 0; s < nsplit; s++) den = fmaf(ml[2 * s + 1], __builtin_amdgcn_exp2f(ml[2 * s] - top), den);
+    const float inv = 1.0f / den;
+    for (int d = 4 * (int)threadIdx.x; d < rank_ld; d += 512) {
+        f4_t o = {0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < nsplit; s++) {
+            const float f = __builtin_amdgcn_exp2f(ml[2 * s] - top) * inv;   // a slice without pages: exp2(-inf) = 0, its sums are zeros
+            const f4_t v = *reinterpret_cast<const f4_t*>(part_acc + (th * nsplit + s) * rank_ld + d);
+#pragma unroll
+            for (int r = 0; r < 4; r++) o[r] = fmaf(v[r], f, o[r]);
+        }
+        const float z[4] = {o[0], o[1], o[2], o[3]};
+        store_b16_4(out, Kb_out, t, h * rank_ld + d, z);
+    }
+}
+
+template <int RC, int NT, int C>
+static void launch_latent_c(const LatentKArgs& k, long units) {
+    const size_t lds = latent_attn_lds(k.chunks, C);
+    const bool exact = k.chunks == RC && k.n_tiles == 4 * NT;
+    static bool ready = false;
+    if (!ready) {
+        const int most = (int)latent_attn_lds(RC, C);
+        if (most > 64 * 1024) {
+            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, true>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
+            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, false>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
+        }
+        ready = true;
+    }
+    if (exact) NVLLM_LAUNCH((k_latent_attn<RC, NT, C, true>), dim3((unsigned)units), dim3(256), lds, k);
+    else NVLLM_LAUNCH((k_latent_attn<RC, NT, C, false>), dim3((unsigned)units), dim3(256), lds, k);
+}
+template <int RC, int NT>
+static void launch_latent_rc(const LatentKArgs& k, long units, int C) {
+    if (C == 1) launch_latent_c<RC, NT, 1>(k, units);
+    else launch_latent_c<RC, NT, 2>(k, units);
+}
+
+void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
+    if (st.T <= 0) return;
+    const LatentPool& P = a.pool;
+    const int row = P.row(), chunks = row / 32, vt = cdiv(P.rank_ld, 64);   // value tiles per wave
+    // algorithmic work: every run's rows read once; per (token, key, head) the two products
+    const double bytes = (double)st.kv_positions * row * P.elem_bytes + (double)st.T * a.H * (row + P.rank_ld) * P.elem_bytes;
+    const double flops = 2.0 * (double)st.qk_pairs * a.H * (row + P.rank_ld);
+    const bool tiled = P.elem_bytes == 2 && ((chunks <= 4 && vt <= 1) || (chunks <= 6 && vt <= 2) || (chunks <= 10 && vt <= 4) || (chunks <= 18 && vt <= 8));
+    int pages_per_block = P.block_size / LATENT_PAGE, page_shift = 0;
+    while ((1 << page_shift) < pages_per_block) page_shift++;
+    if (!tiled || (1 << page_shift) != pages_per_block) {
+        const size_t lds = ((size_t)row + P.rank_ld + 256 + 8) * sizeof(float);
+        if (lds > 64 * 1024) NVLLM_FATAL("latent attention: a cached row of %d values is not supported", row);
+        ProfScope ps(PC_LATENT_ATTN, bytes, flops);
+        const dim3 grid(st.T, a.H);
+        if (P.elem_bytes == 2)
+            NVLLM_LAUNCH((k_latent_attn_any<true>), grid, dim3(256), lds, P.base, a.q, a.sink, a.scale, st.d_pos, st.d_seq, st.d_tbl_off, st.d_tables,
+                         P.block_size, a.H, P.rank, P.rank_ld, row, a.out_f32, a.out_b16, a.H * P.rank_ld / 32);
+        else
+            NVLLM_LAUNCH((k_latent_attn_any<false>), grid, dim3(256), lds, P.base, a.q, a.sink, a.scale, st.d_pos, st.d_seq, st.d_tbl_off, st.d_tables,
+                         P.block_size, a.H, P.rank, P.rank_ld, row, a.out_f32, a.out_b16, 0);
+        return;
+    }
+    // columns per item: 32, or 16 when no item would fill more
+    const int C = (a.H <= 16 && a.H * st.max_run <= 16) ? 1 : 2, W = 16 * C;
+    LatentKArgs k{};
+    k.base = (const __half*)P.base;
+    k.q = (const __half*)a.q;
+    k.sink = a.sink;
+    k.scale = a.scale;
+    k.tables = st.d_tables;
+    k.runs = (const int4*)st.d_runs;
+    k.HG = a.H < W ? a.H : W;
+    k.NG = cdiv(a.H, k.HG);
+    k.CT = W / k.HG;
+    k.n_sub = cdiv(st.max_run < LATENT_RUN ? st.max_run : LATENT_RUN, k.CT);
+    k.H = a.H;
+    k.chunks = chunks;
+    k.n_tiles = P.rank_ld / 16;
+    k.rank_ld = P.rank_ld;
+    k.page_shift = page_shift;
+    k.out = a.out_b16;
+    k.Kb_out = a.H * P.rank_ld / 32;
+    // slices of pages until the chip is full: as many workgroups as fit by LDS (at most two per CU), two blocks per slice at least
+    const long items = (long)st.n_runs * k.n_sub * k.NG;
+    const int per_cu = latent_attn_lds(chunks, C) * 2 <= 160 * 1024 ? 2 : 1;
+    const int nblocks = cdiv(st.max_pos / LATENT_PAGE + 1, LATENT_BLOCK_PAGES);
+    int nsplit = (int)(((long)per_cu * rt().num_cus + items / 2) / items);
+    if (nsplit > cdiv(nblocks, 2)) nsplit = cdiv(nblocks, 2);
+    if (nsplit > 64) nsplit = 64;
+    if (nsplit < 1) nsplit = 1;
+    k.nsplit = nsplit;
+    if (nsplit > 1) {
+        const size_t rows = (size_t)st.T * a.H * nsplit;
+        float* part = (float*)ws_get(WS_ATT_PART, rows * (P.rank_ld + 2) * sizeof(float));
+        k.part_acc = part;
+        k.part_ml = part + rows * P.rank_ld;
+    }
+    {
+        ProfScope ps(PC_LATENT_ATTN, bytes, flops);
+        const long units = items * nsplit;
+        if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, C);
+        else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, C);
+        else if (chunks <= 10 && vt <= 4) launch_latent_rc<10, 4>(k, units, C);
+        else launch_latent_rc<18, 8>(k, units, C);
+    }
+    if (nsplit > 1) {
+        ProfScope ps(PC_LATENT_COMBINE, (double)st.T * a.H * ((double)nsplit * (P.rank_ld + 2) * 4.0 + P.rank_ld * 2.0), 0);
+        NVLLM_LAUNCH(k_latent_combine, dim3((unsigned)st.T * a.H), dim3(128), 0, k.part_acc, k.part_ml, a.sink, a.H, nsplit, P.rank_ld, a.out_b16, k.Kb_out);
+    }
+}
+
+// ------------------------------------------------------------------ fp32 head products
+__global__ __launch_bounds__(256) void k_latent_q_f32(float* __restrict__ rows, const float* __restrict__ q, const float* __restrict__ uk,
+                                                      const float2* __restrict__ rope, const int* __restrict__ pos, int H, int dim, int rot, int rank) {
+    const int t = blockIdx.x, h = blockIdx.y;
+    const float* qh = q + ((size_t)t * H + h) * (dim + rot);
+    float* dst = rows + ((size_t)t * H + h) * (rank + rot);
+    for (int j = threadIdx.x; j < rank; j += 256) {
+        float s = 0.f;
+        for (int d = 0; d < dim; d++) s = fmaf(qh[d], uk[((size_t)h * dim + d) * rank + j], s);
+        dst[j] = s;
+    }
+    for (int i = threadIdx.x; i < rot / 2; i += 256) {
+        const float2 cs = rope[(size_t)pos[t] * (rot / 2) + i];
+        const float u = qh[dim + 2 * i], v = qh[dim + 2 * i + 1];
+        dst[rank + 2 * i] = u * cs.x - v * cs.y;
+        dst[rank + 2 * i + 1] = v * cs.x + u * cs.y;
+    }
+}
+void launch_latent_q_f32(float* rows, const float* q, const float* uk, const float2* rope, const int* pos, int T, int H, int dim, int rot, int rank) {
+    if (T <= 0) return;
+    ProfScope ps(PC_GEMM_ABSORB, (double)H * dim * rank * 4.0 + (double)T * H * (dim + rank + 2 * rot) * 4.0, 2.0 * T * (double)H * dim * rank);
+    NVLLM_LAUNCH(k_latent_q_f32, dim3(T, H), dim3(256), 0, rows, q, uk, rope, pos, H, dim, rot, rank);
+}
+
+__global__ __launch_bounds__(256) void k_latent_v_f32(float* __restrict__ out, const float* __restrict__ lat, const float* __restrict__ uv, int H, int vdim,
+                                                      int rank) {
+    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
+    const float* lh = lat + ((size_t)t * H + h) * rank;
+    for (int v = threadIdx.x >> 6; v < vdim; v += 4) {   // a wave per output
+        const float* w = uv + ((size_t)h * vdim + v) * rank;
+        float s = 0.f;
+        for (int c = lane; c < rank; c += 64) s = fmaf(lh[c], w[c], s);
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+        if (lane == 0) out[((size_t)t * H + h) * vdim + v] = s;
+    }
+}
+void launch_latent_v_f32(float* out, const float* lat, const float* uv, int T, int H, int vdim, int rank) {
+    if (T <= 0) return;
+    ProfScope ps(PC_GEMM_VALUE, (double)H * vdim * rank * 4.0 + (double)T * H * (vdim + rank) * 4.0, 2.0 * T * (double)H * vdim * rank);
+    NVLLM_LAUNCH(k_latent_v_f32, dim3(T, H), dim3(256), 0, out, lat, uv, H, vdim, rank);
+}
+
+// ------------------------------------------------------------------ converters
+__global__ __launch_bounds__(256) void k_latent_rows_b16(__bf16* __restrict__ dst, const float* __restrict__ src, int rank, int rot, int rank_ld, int rot_ld) {
+    const size_t r = blockIdx.x;
+    for (int d = threadIdx.x; d < rank_ld + rot_ld; d += 256) {
+        const int part = d >= rank_ld, i = part ? d - rank_ld : d;
+        const float v = i < (part ? rot : rank) ? src[r * (rank + rot) + (part ? rank : 0) + i] : 0.f;
+        dst[r * (rank_ld + rot_ld) + d] = (__bf16)v;
+    }
+}
+void launch_latent_rows_b16(__half* dst, const float* src, int rows, const LatentPool& pool) {
+    if (rows <= 0) return;
+    NVLLM_LAUNCH(k_latent_rows_b16, dim3(rows), dim3(256), 0, (__bf16*)dst, src, pool.rank, pool.rot, pool.rank_ld, pool.rot_ld);
+}
+
+__global__ __launch_bounds__(256) void k_untile_b16(float* __restrict__ dst, const unsigned short* __restrict__ tiles, int H, int width, int width_ld, int Kb) {
+    const int t = blockIdx.x, h = blockIdx.y;
+    for (int d = threadIdx.x; d < width; d += 256) {
+        const int k = h * width_ld + d;
+        dst[((size_t)t * H + h) * width + d] =
+            bf16_to_f32(tiles[((size_t)(t >> 4) * Kb + (k >> 5)) * TILE_HALVES + (size_t)((t & 15) + 16 * ((k >> 3) & 3)) * 8 + (k & 7)]);
+    }
+}
+void launch_untile_b16(float* dst, const __half* tiles, int T, int H, int width, int width_ld) {
+    if (T <= 0) return;
+    NVLLM_LAUNCH(k_untile_b16, dim3(T, H), dim3(256), 0, dst, (const unsigned short*)tiles, H, width, width_ld, cdiv(H * width_ld, 32));
+}
+
+}  // namespace nvllm

@@ -3,8 +3,11 @@
 // enqueues the fused per-layer kernel sequence and hands back logits / arg-max.
 #include <algorithm>
 #include <cstring>
+#include <memory>
+#include <sys/stat.h>
 #include <vector>
 
+#include "model_dir.h"
 #include "nvllm_internal.h"
 #include "step_arrays.h"
 
@@ -42,6 +45,7 @@ struct ModelPriv {
     // forward pass runs the fp32 operators one by one.
     bool f32 = false;
     std::vector<void*> f32_bufs;
+    std::unique_ptr<DirModel> dir;        // a model folder: everything about its design lives there, nothing above is used
     ChainLayer* chain_layers = nullptr;   // per-layer weight pointers in HBM, for the one-launch decode step (chain.hip)
 };
 
@@ -119,13 +123,50 @@ static PassSlot g_pass[PASS_RING];
 // overwritten by the next pass's classifier, which therefore waits for `g_rows_copied` first.
 static hipEvent_t g_kernels_done = nullptr;
 static hipEvent_t g_rows_copied = nullptr;   // the event of the latest such copy that nobody has waited for yet
-static void wait_for_row_copies() {
+void wait_for_row_copies() {
     if (!g_rows_copied) return;
     HIP_CHECK(hipStreamWaitEvent(rt().stream, g_rows_copied, 0));
     g_rows_copied = nullptr;
 }
 static long g_next_ticket = 0;
 static PassView g_seen;                // the most recently collected pass
+
+// ---- designs that come as folders: config.json's "architecture" -> loader
+static const struct {
+    const char* name;
+    DirModelLoader load;
+} kArchitectures[] = {
+    {"Suselorn", load_latent_hyper_model},
+};
+static DirModelLoader find_architecture(const char* name) {
+    for (const auto& a : kArchitectures)
+        if (strcmp(a.name, name) == 0) return a.load;
+    return nullptr;
+}
+
+static void load_model_dir(Weights* w, Config* p, const char* path) {
+    if (tp().active) {
+        fprintf(stderr, "model folders are not split over tensor-parallel ranks\n");
+        exit(1);
+    }
+    const ModelDir dir(path);
+    const std::string arch = json_get(dir.config, "architecture", Json::STRING, "config").text;
+    const DirModelLoader load = find_architecture(arch.c_str());
+    if (!load) {
+        fprintf(stderr, "nvllm: unknown architecture '%s'; known:", arch.c_str());
+        for (const auto& a : kArchitectures) fprintf(stderr, " %s", a.name);
+        fprintf(stderr, "\n");
+        exit(1);
+    }
+    memset(w, 0, sizeof *w);
+    memset(p, 0, sizeof *p);
+    std::unique_ptr<ModelPriv> m(new ModelPriv());
+    m->dir.reset(load(dir, p));
+    m->cfg = *p;
+    w->_data_buffer = m.release();
+    printf("Model loaded: %s, width %d, %d layer runs, vocabulary %d, %s\n", arch.c_str(), p->dim, p->n_layers, p->vocab_size,
+           rt().compute_dtype == NVLLM_COMPUTE_F32 ? "fp32" : "bf16");
+}
 
 static void read_exact(FILE* f, void* dst, size_t bytes, const char* what) {
     if (fread(dst, 1, bytes, f) != bytes) {
@@ -176,10 +217,10 @@ static long finish_pass(RunState* s, float* d_logits, int* d_argmax, int B, int 
     }
     // (with the status word of a one-launch step, which sits right behind the indices)
     // (a copy operation between two passes costs the stream ~10 us: the copy kernel and the switch around it)
-    if (!host_written)
+    if (!host_written && (B > 0 || chained))
         HIP_CHECK(hipMemcpyAsync(slot.host, d_argmax, (size_t)(B + (chained ? 1 : 0)) * sizeof(int), hipMemcpyDeviceToHost, stream));
     slot.chained = chained;
-    if (rt().logits_mode == NVLLM_LOGITS_HOST)
+    if (rt().logits_mode == NVLLM_LOGITS_HOST && B > 0)
         HIP_CHECK(hipMemcpyAsync(s->logits, d_logits, (size_t)B * V * sizeof(float), hipMemcpyDeviceToHost, stream));
     HIP_CHECK(hipEventRecord(slot.ev, stream));
     if (rt().logits_mode == NVLLM_LOGITS_HOST) g_rows_copied = slot.ev;
@@ -325,6 +366,11 @@ extern "C" {
 // File format and tensor order: reference src/model.c:118-279.
 void load_model(Weights* w, Config* p, const char* checkpoint_path) {
     ensure_init();
+    struct stat info;
+    if (stat(checkpoint_path, &info) == 0 && S_ISDIR(info.st_mode)) {
+        load_model_dir(w, p, checkpoint_path);
+        return;
+    }
     FILE* f = fopen(checkpoint_path, "rb");
     if (!f) {
         fprintf(stderr, "Failed to open model file: %s\n", checkpoint_path);
@@ -569,6 +615,15 @@ void load_model(Weights* w, Config* p, const char* checkpoint_path) {
     }
 }
 
+int nvllm_has_architecture(const char* name) { return name && find_architecture(name) != nullptr; }
+
+void nvllm_init_model_kv(KVCacheManager* mgr, int block_size, int num_blocks, const Config* p, const Weights* w) {
+    ensure_init();
+    ModelPriv* m = (ModelPriv*)w->_data_buffer;
+    if (m && m->dir) m->dir->init_kv(mgr, block_size, num_blocks);
+    else init_kv_cache_manager(mgr, block_size, num_blocks, p->n_layers, p->n_kv_heads, p->head_dim);
+}
+
 void nvllm_free_model(Weights* w) {
     if (!w || !w->_data_buffer) return;
     ModelPriv* m = (ModelPriv*)w->_data_buffer;
@@ -643,6 +698,15 @@ static long enqueue_pass(int* tokens, int num_tokens, int* pos_arr, int* seq_ids
     const int T = num_tokens, B = num_outputs;
     if (T <= 0) return -1;
     if (T > p->max_seq_len || B > p->max_seq_len) NVLLM_FATAL("batch of %d tokens exceeds the workspace (%d)", T, p->max_seq_len);
+    if (m->dir) {
+        if (tp().active) NVLLM_FATAL("model folders are not split over tensor-parallel ranks");
+        const bool to_host = rt().logits_mode == NVLLM_LOGITS_ARGMAX && B > 0;
+        PassArgs a{tokens, pos_arr, seq_ids, output_indices, token_src, T, B, p->max_seq_len, block_tables, &g_kv_manager,
+                   (float*)ws_get(WS_LOGITS, (size_t)B * p->vocab_size * sizeof(float)),
+                   (int*)ws_get(WS_ARGMAX, (size_t)(p->max_seq_len + 64) * sizeof(int)), to_host ? next_slot(B).host : nullptr};
+        m->dir->forward(a);
+        return finish_pass(s, a.d_logits, a.d_argmax, B, p->vocab_size, PassView{}, false, to_host);
+    }
     // H, KVH, F, QD, KD: what THIS process computes (its tensor-parallel slice; the whole model when world == 1)
     const int D = p->dim, F = m->sh.hidden, hd = p->head_dim, H = m->sh.n_heads, KVH = m->sh.n_kv_heads;
     const int QD = H * hd, KD = KVH * hd, V = p->vocab_size;
@@ -784,6 +848,7 @@ static long enqueue_pass(int* tokens, int num_tokens, int* pos_arr, int* seq_ids
             }
         }
     }
+    if (B <= 0) return finish_pass(s, d_logits, d_argmax, 0, V, PassView{}, chained);   // nobody wants a row of this pass
     // logits only for the rows named by output_indices                            (model.c:396,411-418)
     wait_for_row_copies();   // the previous pass's rows have left the workspaces the classifier writes
     bool identity = B == T;

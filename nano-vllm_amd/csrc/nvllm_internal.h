@@ -81,6 +81,7 @@ struct Runtime {
     hipStream_t copy_stream = nullptr;   // result copies of a pass when logits rows travel to the host (created on first use)
     int logits_mode = NVLLM_LOGITS_HOST;
     int kv_elem_bytes = 4;
+    int compute_dtype = NVLLM_COMPUTE_BF16;   // of models loaded from a folder
     bool kv_elem_set = false;   // nvllm_set_kv_elem_bytes was called: the environment default does not apply
     int num_cus = 256;
 };
@@ -130,6 +131,13 @@ enum WsSlot {
     WS_TP_GATHER,   // ... and what the ranks gathered
     WS_CHAIN_SYNC,  // arrival counters of the one-launch decode step
     WS_AMAX_PAIRS,  // the classifier tiles' (maximum, index) pairs
+    WS_STREAMS,     // hyper-connections: the residual streams [T][streams][width]
+    WS_KV_RAW,      // latent attention: a batch's latents and rotated key parts before norm and rotation
+    WS_Q_ROWS,      // ... its absorbed queries
+    WS_LATENT,      // ... its attended latents
+    WS_F32_A,       // fp32 models: activations between operators
+    WS_F32_B,
+    WS_F32_C,
     WS_COUNT
 };
 void* ws_get(WsSlot slot, size_t bytes);
@@ -141,6 +149,9 @@ int* pinned_ints(size_t n);   // ring allocation, for callers that fill it thems
 // float2 {cos, sin} per (position, pair), computed on the host with the same libm
 // calls as the reference (src/kernels/layers.c:119-122) and cached in HBM.
 const float2* rope_table(float theta, int head_dim, int min_positions);
+// The same layout for pair i of `dims` rotated dimensions turning by base^(-2i/dims) per position, with the angle
+// and its sine and cosine formed in double and rounded once.
+const float2* rotation_table(double base, int dims, int min_positions);
 
 // ---------------------------------------------------------------- profiling
 enum ProfClass {
@@ -159,6 +170,14 @@ enum ProfClass {
     PC_ARGMAX,
     PC_PACK,
     PC_CHAIN,      // all layers of a decode step in one launch (chain.hip)
+    PC_GEMM_LATENT_IN,   // latent attention: the two down-projections ...
+    PC_GEMM_LATENT_Q,    // ... queries from their latent
+    PC_GEMM_ABSORB,      // ... queries times the key up-projection, head by head
+    PC_GEMM_VALUE,       // ... attended latents times the value up-projection, head by head
+    PC_LATENT_KV,        // ... norm, rotation and cache write of a token's latent row
+    PC_LATENT_ATTN,
+    PC_LATENT_COMBINE,
+    PC_HYPER,            // hyper-connection update and norm as a launch of its own
     PC_COUNT
 };
 hipEvent_t prof_start_event();   // events of the enclosing ProfScope, or null when timing is off
@@ -188,7 +207,16 @@ struct ProfScope {  // names the class of, and attaches timing events to, the ON
 // ----------------------------------------------------- kernel launchers (device ptrs)
 // What a projection does with its complete sums (see gemm.hip).
 struct GemmEpilogue {
-    enum Kind { F32 = 0, SWIGLU_A16 = 1, RESID_A16 = 2, ROPE_KV = 3 } kind = F32;
+    enum Kind {
+        F32 = 0, SWIGLU_A16 = 1, RESID_A16 = 2, ROPE_KV = 3,
+        // bf16 models (gemm_b16.hip): everything below is element-wise on four consecutive features of a token
+        TILE_B16 = 4,    // activation tiles for the next projection
+        ROWS_B16 = 5,    // bf16 rows of the latent attention's queries
+        LATENT_IN = 6,   // query latent * gain -> tiles + sums of squares; key/value latent and rotated key part -> fp32 rows
+        LATENT_Q = 7,    // unrotated query parts -> tiles; rotated parts -> query rows
+        HYPER_2 = 8,     // hyper-connection update of up to 2 (4) residual streams, and the next sublayer's
+        HYPER_4 = 9      //   input (their weighted sum through the Dynamic Tanh norm) -> tiles
+    } kind = F32;
     // Input normalisation.  When ss_in is set the activations fed to the projection are
     // x * gain (not yet divided by the RMS) and the result is scaled per token by
     // 1/sqrt(sum_j ss_in[t, j] / d_in + eps); ss_gather (optional) maps the projection's
@@ -226,7 +254,26 @@ struct GemmEpilogue {
     int kv_elem_bytes = 4;
     int bs = 16;
     long layer_off = 0;
+    // ---- bf16 models
+    const float* bias = nullptr;   // SWIGLU_A16, HYPER_*: one fp32 per output feature, added before anything else
+    float softcap = 0.f;           // F32: out = softcap * tanh(out / softcap) when positive
+    // LATENT_IN: features [0, latent_q) are the query latent (gain_next, a16_out, ss_out), the rest goes to out[t, ldo]
+    int latent_q = 0;
+    // LATENT_Q: features [0, q_plain) are the unrotated parts (a16_out); then per head rot_ld features, rotated by
+    // `rope` (rot_dim / 2 pairs per position) into q_rows;  ROWS_B16: head_ld features per head into q_rows
+    int q_plain = 0, rot_ld = 0, rot_dim = 0, head_ld = 0;
+    __bf16* q_rows = nullptr;      // [T][q_heads][q_row]: head_ld latent features, then rot_ld rotated ones
+    int q_heads = 0, q_row = 0;
+    // HYPER_*: x = [T][streams][hyper_ld] fp32
+    const float* hyper = nullptr;  // hyper_record() of the sublayer and the one after it
+    const float* hyper_scale = nullptr;   // layer scale [N]
+    const float* norm_w = nullptr;        // the next sublayer's norm [N]
+    const float* norm_b = nullptr;
+    int streams = 0;
 };
+// Where a sublayer's hyper-connection numbers sit in its record: mix[from][to], out[to], then the next
+// sublayer's in[s] and the alpha of its norm.
+constexpr int hyper_record_floats(int streams) { return streams * streams + 2 * streams + 1; }
 // Memory a projection launch needs beyond its operands, when the caller brings it instead of the
 // library's grow-only buffers: a slab for split-K partial tiles and zeroed arrival counters (every
 // launch leaves them zero again).  A slab too small for the chosen K split means no K split.
@@ -293,6 +340,17 @@ int chain_enabled();
 size_t chain_sync_words(int n_layers);
 bool launch_decode_chain(const ChainStep& s);
 
+// ---- gemm_b16.hip: the same projection kernels on bf16 weights and one bf16 activation plane
+// A weight matrix in tile order.  groups > 1: a block-diagonal product -- rows [g * N/groups, ...) meet only the
+// K-wide slice g of the activations (one head each); N / groups is a multiple of 16.
+struct B16Weight {
+    const __half* tiles = nullptr;   // bf16 bit patterns, 16 rows x 32 k per 1-KiB tile
+    int N = 0, K = 0;                // K: per group, a multiple of 32
+    int groups = 1;
+};
+static inline size_t b16_halves(int tokens, int K) { return (size_t)cdiv(tokens, 16) * cdiv(K, 32) * TILE_HALVES; }
+void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls);
+
 void launch_pack_a16(__half* a16, const float* in, int T, int K);
 void launch_matmul_f32w(float* out, const float* in, const float* w, int T, int K, int N);
 
@@ -350,6 +408,31 @@ struct AttnArgs {
 };
 void launch_paged_attention(const AttnArgs& a);
 int attn_tokens_per_item(int H, int KVH);
+
+// ---- hyper.hip: hyper-connections with the Dynamic Tanh norm, as launches of their own
+// One hyper-connection step on x [T][streams][ld] (all pointers device; width <= ld, the rest is padding):
+//   y given:  y <- (y + bias) * scale (bias optional), then x_to <- sum_from mix[from][to] x_from + out[to] y
+//   then      u = sum_s in[s] x_s, and z = tanh(alpha u) * norm_w + norm_b (norm_w null: z = u)
+//   z goes to out_f32 rows [T][ld] and / or out_b16 activation tiles, whichever is given.
+// record: hyper_record_floats(streams) floats (mix, out, in, alpha); any number of streams up to 64.
+struct HyperStep {
+    float* x;
+    const float* y = nullptr;     // [T][ld]
+    const float* bias = nullptr;
+    const float* scale = nullptr;
+    const float* record;
+    const float* norm_w = nullptr;
+    const float* norm_b = nullptr;
+    float* out_f32 = nullptr;
+    __half* out_b16 = nullptr;
+    int streams, ld;
+};
+void launch_hyper_step(const HyperStep& h, int T);
+// every stream of token t = its embedding row (fp32 or bf16 table rows of ld values); tok_src / prev as in launch_embed_prescale
+void launch_embed_streams(float* x, const void* table, bool bf16, const int* tokens, int T, int streams, int ld, const int* tok_src, const int* prev);
+void launch_gather_b16(__half* dst, const __half* src, const int* idx, int B, int K);   // rows of activation tiles
+void launch_swiglu_bias(float* out, const float* g, const float* u, const float* bg, const float* bu, int T, int F);
+void launch_softcap(float* x, float cap, long n);
 
 // x[t,:] = table[tokens[t],:]; a16 = x * gain in hi/lo tiles; ss[t, j] = sum of x^2 over features 32j..32j+31
 // tok_src / prev (optional): where tok_src[t] >= 0 the token id is prev[tok_src[t]] instead of tokens[t]

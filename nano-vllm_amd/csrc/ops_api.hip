@@ -5,6 +5,8 @@
 #include <unordered_map>
 #include <vector>
 
+#include "latent_attention.h"
+#include "model_dir.h"
 #include "nvllm_internal.h"
 #include "step_arrays.h"
 
@@ -90,6 +92,8 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
             runs.push_back(pos_of(t + n - 1));
             runs.push_back(tbl_off[seq_of(t)]);
             s.kv_positions += pos_of(t + n - 1) + 1;
+            for (int i = 0; i < n; i++) s.qk_pairs += pos_of(t + i) + 1;
+            if (n > s.max_run) s.max_run = n;
             for (int tb = t >> 4; tb <= (t + n - 1) >> 4; tb++)
                 if (tb < 4) s.runs_in_tb[tb]++;
             t += n;
@@ -227,6 +231,14 @@ void accum(float* a, float* b, int size) {
 
 // ------------------------------------------------------- KV block pool
 // Host bookkeeping exactly as reference memory.c:8-82; the two pools are HBM.
+static void init_free_stack(KVCacheManager* mgr, int block_size, int num_blocks) {
+    mgr->block_size = block_size;
+    mgr->num_blocks = num_blocks;
+    mgr->free_blocks_count = num_blocks;
+    mgr->free_block_indices = (int*)malloc((size_t)num_blocks * sizeof(int));
+    for (int slot = 0; slot < num_blocks; slot++) mgr->free_block_indices[slot] = num_blocks - 1 - slot;
+}
+
 void init_kv_cache_manager(KVCacheManager* mgr, int block_size, int num_blocks, int n_layers,
                            int n_kv_heads, int head_dim) {
     ensure_init();
@@ -236,11 +248,7 @@ void init_kv_cache_manager(KVCacheManager* mgr, int block_size, int num_blocks, 
         if (n_kv_heads % tp().world) NVLLM_FATAL("%d kv heads do not divide over %d tensor-parallel ranks", n_kv_heads, tp().world);
         n_kv_heads /= tp().world;
     }
-    mgr->block_size = block_size;
-    mgr->num_blocks = num_blocks;
-    mgr->free_blocks_count = num_blocks;
-    mgr->free_block_indices = (int*)malloc((size_t)num_blocks * sizeof(int));
-    for (int slot = 0; slot < num_blocks; slot++) mgr->free_block_indices[slot] = num_blocks - 1 - slot;
+    init_free_stack(mgr, block_size, num_blocks);
     const size_t elems = (size_t)n_layers * num_blocks * block_size * n_kv_heads * head_dim;
     const int eb = rt().kv_elem_bytes;
     if (eb == 2 && (block_size != KV16_PAGE_KEYS || head_dim % 16 != 0))
@@ -256,6 +264,18 @@ void init_kv_cache_manager(KVCacheManager* mgr, int block_size, int num_blocks, 
     mgr->pool_v = (float*)pv;
     pools()[pk] = PoolInfo{eb, n_layers, n_kv_heads, head_dim};
 }
+
+}  // extern "C"
+void nvllm::init_block_pool(KVCacheManager* mgr, int block_size, int num_blocks, size_t bytes) {
+    ensure_init();
+    init_free_stack(mgr, block_size, num_blocks);
+    void* pool = nullptr;
+    if (device_malloc(&pool, bytes) != 0) NVLLM_FATAL("cannot allocate the block pool (%zu bytes)", bytes);
+    HIP_CHECK(hipMemsetAsync(pool, 0, bytes, rt().stream));   // rows nobody has written are finite
+    mgr->pool_k = (float*)pool;
+    mgr->pool_v = nullptr;
+}
+extern "C" {
 
 void free_kv_cache_manager(KVCacheManager* mgr) {
     if (mgr->free_block_indices) free(mgr->free_block_indices);
@@ -409,6 +429,69 @@ void paged_attention_batch(float* out, float* q, KVCacheManager* mgr, BlockTable
     a.n_runs = s.n_runs;
     a.kv_positions = s.kv_positions;
     launch_paged_attention(a);
+}
+
+}  // extern "C"
+
+// -------------------------------------------------- operators of folder models (include/nvllm.h)
+extern "C" {
+
+void nvllm_hyper_step(float* x, const float* y, const float* bias, const float* scale, const float* record, const float* norm_w,
+                      const float* norm_b, float* out, int streams, int dim, int num_tokens) {
+    ensure_init();
+    HyperStep h{};
+    h.x = x; h.y = y; h.bias = bias; h.scale = scale; h.record = record; h.norm_w = norm_w; h.norm_b = norm_b; h.out_f32 = out;
+    h.streams = streams; h.ld = dim;
+    launch_hyper_step(h, num_tokens);
+}
+
+void nvllm_swiglu_bias(float* out, const float* g, const float* u, const float* bg, const float* bu, int hidden_dim, int num_tokens) {
+    ensure_init();
+    launch_swiglu_bias(out, g, u, bg, bu, num_tokens, hidden_dim);
+}
+
+void nvllm_softcap(float* x, float cap, long n) {
+    ensure_init();
+    launch_softcap(x, cap, n);
+}
+
+void nvllm_latent_pool_init(KVCacheManager* mgr, int block_size, int num_blocks, int rank, int rot, int elem_bytes) {
+    init_block_pool(mgr, block_size, num_blocks, latent_pool_bytes(latent_pool(nullptr, elem_bytes, block_size, rank, rot), num_blocks));
+}
+
+void nvllm_latent_cache_write(KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr, const float* kv, const float* gain,
+                              float eps, double base, int rank, int rot, int elem_bytes, int num_tokens) {
+    ensure_init();
+    if (num_tokens <= 0) return;
+    StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size);
+    if (s.table_short) NVLLM_FATAL("latent cache write: a position lies beyond its sequence's block table");
+    launch_latent_kv(latent_pool(mgr->pool_k, elem_bytes, mgr->block_size, rank, rot), kv, rank + rot, rank, gain, eps,
+                     rotation_table(base, rot, s.max_pos + 1), s);
+}
+
+void nvllm_latent_attention(float* out, const float* q, KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr,
+                            const float* sink, float scale, int n_heads, int rank, int rot, int elem_bytes, int num_tokens) {
+    ensure_init();
+    if (num_tokens <= 0) return;
+    StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size, LATENT_RUN);
+    if (s.table_short) NVLLM_FATAL("latent attention: a position lies beyond its sequence's block table");
+    LatentAttn a{};
+    a.pool = latent_pool(mgr->pool_k, elem_bytes, mgr->block_size, rank, rot);
+    a.sink = sink;
+    a.scale = scale;
+    a.H = n_heads;
+    if (elem_bytes == 4) {
+        a.q = q;
+        a.out_f32 = out;
+        launch_latent_attention(a, s);
+        return;
+    }
+    __half* rows = (__half*)ws_get(WS_Q_ROWS, (size_t)num_tokens * n_heads * a.pool.row() * sizeof(__half));
+    launch_latent_rows_b16(rows, q, num_tokens * n_heads, a.pool);
+    a.q = rows;
+    a.out_b16 = (__half*)ws_get(WS_LATENT, b16_halves(num_tokens, n_heads * a.pool.rank_ld) * sizeof(__half));
+    launch_latent_attention(a, s);
+    launch_untile_b16(out, a.out_b16, num_tokens, n_heads, rank, a.pool.rank_ld);
 }
 
 }  // extern "C"

@@ -8,6 +8,7 @@
 #include "nvllm_internal.h"
 
 extern "C" void nvllm_host_rope_table(float* table, float theta, int head_dim, int first_pos, int n_pos);
+extern "C" void nvllm_host_rotation_table(float* table, double base, int dims, int n_pos);
 
 namespace nvllm {
 
@@ -87,24 +88,26 @@ void unregister_weight(const void* handle) { registry().erase(handle); }
 
 // -------------------------------------------------------------- RoPE tables
 struct RopeTab {
-    float theta;
+    double theta;
     int head_dim;
+    bool exact;   // angles formed in double (rotation_table)
     int n_pos;
     float2* dev;
 };
 static std::vector<RopeTab> g_rope;
 
-const float2* rope_table(float theta, int head_dim, int min_positions) {
+static const float2* angle_table(double theta, int head_dim, int min_positions, bool exact) {
     ensure_init();
     RopeTab* hit = nullptr;
     for (auto& t : g_rope)
-        if (t.theta == theta && t.head_dim == head_dim) hit = &t;
+        if (t.theta == theta && t.head_dim == head_dim && t.exact == exact) hit = &t;
     if (hit && hit->n_pos >= min_positions) return hit->dev;
     int n = 1024;
     while (n < min_positions) n *= 2;
     const size_t floats = (size_t)n * (head_dim / 2) * 2;
     std::vector<float> host(floats);
-    nvllm_host_rope_table(host.data(), theta, head_dim, 0, n);
+    if (exact) nvllm_host_rotation_table(host.data(), theta, head_dim, n);
+    else nvllm_host_rope_table(host.data(), (float)theta, head_dim, 0, n);
     float2* dev = nullptr;
     HIP_CHECK(hipMalloc(&dev, floats * sizeof(float)));
     HIP_CHECK(hipMemcpyAsync(dev, host.data(), floats * sizeof(float), hipMemcpyHostToDevice, g_rt.stream));
@@ -114,10 +117,12 @@ const float2* rope_table(float theta, int head_dim, int min_positions) {
         hit->dev = dev;
         hit->n_pos = n;
     } else {
-        g_rope.push_back({theta, head_dim, n, dev});
+        g_rope.push_back({theta, head_dim, exact, n, dev});
     }
     return dev;
 }
+const float2* rope_table(float theta, int head_dim, int min_positions) { return angle_table(theta, head_dim, min_positions, false); }
+const float2* rotation_table(double base, int dims, int min_positions) { return angle_table(base, dims, min_positions, true); }
 
 // ---------------------------------------------------------------- profiling
 struct ProfRec {
@@ -185,7 +190,7 @@ static void prof_drain() {
 static const char* kProfNames[PC_COUNT] = {
     "embed",      "rmsnorm",  "gemm_qkv", "gemm_wo",      "gemm_gateup", "gemm_down", "gemm_head",
     "gemm_other", "rope_kv",  "attn",     "attn_combine", "elementwise", "argmax",    "pack",
-    "decode_chain"};
+    "decode_chain", "gemm_latent_in", "gemm_latent_q", "gemm_absorb", "gemm_value", "latent_kv", "latent_attn", "latent_combine", "hyper"};
 
 // --------------------------------------------------------------------- init
 void ensure_init() {
@@ -244,6 +249,11 @@ void nvllm_set_kv_elem_bytes(int bytes) {
     g_rt.kv_elem_set = true;
 }
 int nvllm_get_kv_elem_bytes(void) { return g_rt.kv_elem_bytes; }
+void nvllm_set_compute_dtype(int dtype) {
+    if (dtype != NVLLM_COMPUTE_BF16 && dtype != NVLLM_COMPUTE_F32) NVLLM_FATAL("unknown compute type %d", dtype);
+    g_rt.compute_dtype = dtype;
+}
+int nvllm_get_compute_dtype(void) { return g_rt.compute_dtype; }
 
 void nvllm_prof_enable(int on) {
     ensure_init();

@@ -46,6 +46,9 @@ extern long nvllm_forward_enqueue(int* tokens, int num_tokens, int* pos_arr, int
                                   BlockTable** block_tables) __attribute__((weak));
 extern int nvllm_forward_collect(long ticket, int* argmax_out, int cap) __attribute__((weak));
 extern int nvllm_get_logits_mode(void) __attribute__((weak));
+/* Optional: a backend whose models bring block pools of their own layout. */
+extern void nvllm_init_model_kv(KVCacheManager* mgr, int block_size, int num_blocks, const Config* p, const Weights* w)
+    __attribute__((weak));
 
 struct NvllmEngine {
     NvllmEngineOptions opt;
@@ -69,6 +72,7 @@ struct NvllmEngine {
     int* batch_output_indices;
     int* batch_sampled;
     BlockTable** batch_block_tables;
+    int fed_tokens, fed_outputs;   /* the pass a caller is putting together (nvllm_engine_feed) */
     int last_batch_count;
     int last_output_count;
     /* the pass in flight (two-halves mode): which sequence each output row belongs to and where
@@ -130,8 +134,8 @@ NvllmEngine* nvllm_engine_create(const char* model_path, int n_seqs, const Nvllm
     e->max_blocks_per_seq = (e->config.max_seq_len + bs - 1) / bs;
     int pool_blocks = e->opt.num_blocks;
     if (pool_blocks <= 0) pool_blocks = n_seqs * e->max_blocks_per_seq; /* main.c:189-193 */
-    init_kv_cache_manager(&g_kv_manager, bs, pool_blocks, e->config.n_layers, e->config.n_kv_heads,
-                          e->config.head_dim);
+    if (nvllm_init_model_kv) nvllm_init_model_kv(&g_kv_manager, bs, pool_blocks, &e->config, &e->weights);
+    else init_kv_cache_manager(&g_kv_manager, bs, pool_blocks, e->config.n_layers, e->config.n_kv_heads, e->config.head_dim);
     for (int i = 0; i < n_seqs; i++) {
         Sequence* s = &e->seqs[i];
         s->id = i;
@@ -144,7 +148,8 @@ NvllmEngine* nvllm_engine_create(const char* model_path, int n_seqs, const Nvllm
     e->batch_tokens = (int*)malloc((size_t)e->capacity * sizeof(int));
     e->batch_pos = (int*)malloc((size_t)e->capacity * sizeof(int));
     e->batch_seq_ids = (int*)malloc((size_t)e->capacity * sizeof(int));
-    e->batch_output_indices = (int*)malloc((size_t)n_seqs * sizeof(int));
+    /* (the scheduler asks for one row per sequence, a feeding caller for any tokens of the pass) */
+    e->batch_output_indices = (int*)malloc((size_t)(n_seqs > e->capacity ? n_seqs : e->capacity) * sizeof(int));
     e->batch_sampled = (int*)malloc((size_t)n_seqs * sizeof(int));
     e->batch_block_tables = (BlockTable**)malloc((size_t)n_seqs * sizeof(BlockTable*));
     for (int i = 0; i < n_seqs; i++) e->batch_block_tables[i] = &e->seqs[i].table;
@@ -250,14 +255,13 @@ int nvllm_engine_set_request(NvllmEngine* e, int seq, const int* prompt, int n_p
     return 0;
 }
 
-int nvllm_engine_skip_prefill(NvllmEngine* e, int seq, int upto) {
-    if (!e || seq < 0 || seq >= e->n_seqs) return -1;
+/* A block for every position in [start, start + n) that begins one (main.c:322-335); 0, or -1 when the pool ran out
+ * (blocks allocated so far stay in the table). */
+static int cover_positions(NvllmEngine* e, int seq, int start, int n) {
     Sequence* s = &e->seqs[seq];
-    if (s->status != SEQ_WAITING || s->pos != 0 || !s->prompt_tokens || upto < 0) return -1;
-    if (upto > s->num_prompt_tokens - 1) upto = s->num_prompt_tokens - 1;
     const int bs = g_kv_manager.block_size;
-    for (int p = 0; p < upto; p++) {
-        if (p % bs == 0) {                                  /* main.c:322-335 */
+    for (int p = start; p < start + n; p++) {
+        if (p % bs == 0) {
             const int blk = alloc_block(&g_kv_manager);
             if (blk == -1) return -1;
             s->table.block_indices[p / bs] = blk;
@@ -265,6 +269,15 @@ int nvllm_engine_skip_prefill(NvllmEngine* e, int seq, int upto) {
             trace_push(e, seq, p / bs, blk);
         }
     }
+    return 0;
+}
+
+int nvllm_engine_skip_prefill(NvllmEngine* e, int seq, int upto) {
+    if (!e || seq < 0 || seq >= e->n_seqs) return -1;
+    Sequence* s = &e->seqs[seq];
+    if (s->status != SEQ_WAITING || s->pos != 0 || !s->prompt_tokens || upto < 0) return -1;
+    if (upto > s->num_prompt_tokens - 1) upto = s->num_prompt_tokens - 1;
+    if (cover_positions(e, seq, 0, upto) != 0) return -1;
     s->pos = upto;
     s->current_token = s->prompt_tokens[upto];
     return upto;
@@ -317,19 +330,9 @@ int nvllm_engine_step(NvllmEngine* e) {
         }
         if (batch_count + n_tokens > e->capacity) continue; /* main.c:315-318 */
 
-        const int bs = g_kv_manager.block_size;             /* main.c:322-335 */
-        for (int t = 0; t < n_tokens; t++) {
-            const int p = start_pos + t;
-            if (p % bs == 0) {
-                const int blk = alloc_block(&g_kv_manager);
-                if (blk == -1) {
-                    printf("Error: Out of KV Cache blocks!\n");
-                    exit(1);
-                }
-                s->table.block_indices[p / bs] = blk;
-                s->table.num_blocks++;
-                trace_push(e, i, p / bs, blk);
-            }
+        if (cover_positions(e, i, start_pos, n_tokens) != 0) {  /* main.c:322-335 */
+            printf("Error: Out of KV Cache blocks!\n");
+            exit(1);
         }
         for (int t = 0; t < n_tokens; t++) {                /* main.c:338-342 */
             e->batch_tokens[batch_count + t] = token_ptr[t];
@@ -478,6 +481,60 @@ int nvllm_engine_step(NvllmEngine* e) {
         return 0;
     }
     return 1;
+}
+
+/* ---- passes put together by the caller (include/nvllm.h) */
+int nvllm_engine_feed(NvllmEngine* e, int seq, const int* tokens, int n, const int* want, int n_want) {
+    if (!e || seq < 0 || seq >= e->n_seqs || n <= 0 || !tokens || n_want < 0 || n_want > n || (n_want && !want)) return -1;
+    Sequence* s = &e->seqs[seq];
+    if (s->status != SEQ_FINISHED || s->prompt_tokens) return -1;   /* the scheduler's slot */
+    for (int k = 0; k < n_want; k++)
+        if (want[k] < 0 || want[k] >= n || (k && want[k] <= want[k - 1])) return -1;
+    for (int t = 0; t < n; t++)
+        if (tokens[t] < 0 || tokens[t] >= e->config.vocab_size) return -1;
+    for (int t = 0; t < e->fed_tokens; t++)
+        if (e->batch_seq_ids[t] == seq) return -1;                  /* one portion per sequence and pass */
+    if (e->fed_tokens + n > e->capacity || s->pos + n > e->config.max_seq_len) return -2;
+    const int had = s->table.num_blocks;
+    if (cover_positions(e, seq, s->pos, n) != 0) {
+        while (s->table.num_blocks > had) free_block(&g_kv_manager, s->table.block_indices[--s->table.num_blocks]);
+        return -3;
+    }
+    engine_flush(e);
+    for (int t = 0; t < n; t++) {
+        e->batch_tokens[e->fed_tokens + t] = tokens[t];
+        e->batch_pos[e->fed_tokens + t] = s->pos + t;
+        e->batch_seq_ids[e->fed_tokens + t] = seq;
+    }
+    for (int k = 0; k < n_want; k++) e->batch_output_indices[e->fed_outputs++] = e->fed_tokens + want[k];
+    e->fed_tokens += n;
+    s->pos += n;
+    return 0;
+}
+
+int nvllm_engine_feed_run(NvllmEngine* e) {
+    if (!e || e->fed_tokens == 0) return -1;
+    const int n = e->fed_tokens, rows = e->fed_outputs;
+    e->fed_tokens = e->fed_outputs = 0;
+    e->seen_state = 0;
+    const double t0 = now_seconds();
+    transformer_batch(e->batch_tokens, n, e->batch_pos, e->batch_seq_ids, e->batch_output_indices, rows, &e->config, &e->state,
+                      &e->weights, e->batch_block_tables);
+    e->stats.forward_seconds += now_seconds() - t0;
+    e->stats.steps += 1;
+    e->stats.tokens_forwarded += n;
+    e->last_batch_count = n;
+    e->last_output_count = 0;   /* nothing was sampled */
+    return rows;
+}
+
+int nvllm_engine_feed_end(NvllmEngine* e, int seq) {
+    if (!e || seq < 0 || seq >= e->n_seqs) return -1;
+    Sequence* s = &e->seqs[seq];
+    if (s->status != SEQ_FINISHED || s->prompt_tokens) return -1;
+    release_blocks(e, s);
+    s->pos = 0;
+    return 0;
 }
 
 int nvllm_engine_run(NvllmEngine* e, int n) {

@@ -23,5 +23,18 @@ void nvllm_host_rope_table(float* table, float theta, int head_dim, int first_po
     }
 }
 
+/* Angles p * base^(-2i/dims), i < dims/2, formed in double; {cos, sin} rounded once.  Same layout. */
+void nvllm_host_rotation_table(float* table, double base, int dims, int n_pos) {
+    const int half = dims / 2;
+    for (int i = 0; i < half; i++) {
+        const double freq = pow(base, -2.0 * i / dims);
+        for (int p = 0; p < n_pos; p++) {
+            float* dst = table + ((size_t)p * half + i) * 2;
+            dst[0] = (float)cos(p * freq);
+            dst[1] = (float)sin(p * freq);
+        }
+    }
+}
+
 /* 1/sqrtf(head_dim), the attention scale (reference src/kernels/attention.c:259). */
 float nvllm_host_attn_scale(int head_dim) { return 1.0f / sqrtf(head_dim); }
