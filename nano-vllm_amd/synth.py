@@ -170,3 +170,118 @@ def make_requests(n: int, prompt_lo: int, prompt_hi: int, vocab_size: int, seed:
         p[0] = bos
         out.append(p)
     return out
+
+
+# ------------------------------------------------------------------ model folders
+# config.json + model.safetensors (random bf16 weights) of the "Suselorn" design.  Test-sized models come with
+# weights that make every mechanism matter (attention scores of several units, sinks of their size, streams that
+# mix); `plain=True` writes the same tensors from one repeated random block, for benchmark-sized files.
+
+def latent_mixer(heads, dim, rot_dim, vdim, kv_rank, q_rank, scale=None, base=10000.0) -> dict:
+    return dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank,
+                scale=float(scale if scale is not None else (dim + rot_dim) ** -0.5), rot=dict(base=float(base), dims=rot_dim))
+
+
+def latent_config(width, vocab, layers, streams=2, loop=None, softcap=20.0, eps=1e-5) -> dict:
+    """layers: (mixer dict, ff width or None) per layer; loop: (start, stop, times) or None."""
+    return dict(architecture="Suselorn", width=width, vocab=vocab, streams=streams, logit_softcap=softcap, norm=dict(eps=eps),
+                loop=None if loop is None else dict(start=loop[0], stop=loop[1], times=loop[2]),
+                layers=[dict(type="latent_attention", mixer=m, mlp=None if ff is None else dict(kind="dense", ff=ff)) for m, ff in layers])
+
+
+def latent_tensors(cfg: dict) -> dict:
+    """name -> (shape, kind) of every tensor of the design, in file order."""
+    D, S = cfg["width"], cfg["streams"]
+    out = {"embed": ((cfg["vocab"], D), "embed")}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        H, parts = m["heads"], (1, 2) if layer["mlp"] else (1,)
+        for q in parts:
+            out[f"{p}norm{q}"] = ((D,), "gain")
+            out[f"{p}norm{q}.b"] = ((D,), "bias")
+            out[f"{p}norm{q}.alpha"] = ((), "alpha")
+        x = p + "mix."
+        out[x + "dq"] = ((m["q_rank"], D), "matrix")
+        out[x + "dq.norm"] = ((m["q_rank"],), "gain")
+        out[x + "uq"] = ((H * (m["dim"] + m["rot_dim"]), m["q_rank"]), "sharp")
+        out[x + "dkv"] = ((m["kv_rank"] + m["rot_dim"], D), "matrix")
+        out[x + "dkv.norm"] = ((m["kv_rank"],), "gain")
+        out[x + "uk"] = ((H * m["dim"], m["kv_rank"]), "sharp")
+        out[x + "uv"] = ((H * m["vdim"], m["kv_rank"]), "matrix")
+        out[x + "sink"] = ((H,), "sink")
+        out[x + "o"] = ((D, H * m["vdim"]), "matrix")
+        if layer["mlp"]:
+            ff, x = layer["mlp"]["ff"], p + "mlp."
+            for n, shape in (("gate", (ff, D)), ("up", (ff, D)), ("down", (D, ff))):
+                out[x + n] = (shape, "matrix")
+                out[x + n + ".b"] = ((shape[0],), "bias")
+        for q in parts:
+            out[f"{p}ls{q}"] = ((D,), "gain")
+            out[f"{p}hc{q}.in"] = ((S,), "weight")
+            out[f"{p}hc{q}.out"] = ((S,), "weight")
+            out[f"{p}hc{q}.mix"] = ((S, S), "mix")
+    out["final.norm"] = ((D,), "gain")
+    out["final.norm.b"] = ((D,), "bias")
+    out["final.norm.alpha"] = ((), "alpha")
+    return out
+
+
+def to_bf16(a: np.ndarray) -> np.ndarray:
+    """fp32 -> bf16 bit patterns, to nearest even."""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def from_bf16(u: np.ndarray) -> np.ndarray:
+    return (u.astype(np.uint32) << 16).view(np.float32)
+
+
+def _latent_values(shape, kind, rng) -> np.ndarray:
+    n = rng.standard_normal(shape)
+    fan = shape[-1] if shape else 1
+    return {"embed": lambda: n, "matrix": lambda: n * fan ** -0.5, "sharp": lambda: n * 1.7 * fan ** -0.5,
+            "gain": lambda: 1.0 + 0.2 * n, "bias": lambda: 0.2 * n, "alpha": lambda: 0.6 + 0.2 * rng.random(shape),
+            "sink": lambda: 1.5 + 2.0 * n, "weight": lambda: 0.4 + 0.8 * rng.random(shape),
+            "mix": lambda: 0.9 * np.eye(fan) + 0.2 * n}[kind]()
+
+
+def write_model_dir(path: str, cfg: dict, seed: int = 0, plain: bool = False, edit=None) -> dict:
+    """Write config.json and model.safetensors into folder `path`; returns the tensors (as fp32, exactly what the file
+    holds; none with `plain`).  `edit(name, array)` may return a replacement for a tensor's values before rounding."""
+    import json
+    os.makedirs(path, exist_ok=True)
+    rng = np.random.Generator(np.random.PCG64(seed))
+    tensors = latent_tensors(cfg)
+    header, at = {}, 0
+    for name, (shape, _) in tensors.items():
+        size = 2 * int(np.prod(shape, dtype=np.int64))
+        header[name] = dict(dtype="BF16", shape=list(shape), data_offsets=[at, at + size])
+        at += size
+    text = json.dumps(header).encode()
+    text += b" " * (-len(text) % 8)
+    out = {}
+    block = rng.standard_normal(1 << 22).astype(np.float32) if plain else None
+    tmp = os.path.join(path, "model.safetensors.tmp")
+    with open(tmp, "wb") as f:
+        f.write(struct.pack("<Q", len(text)))
+        f.write(text)
+        for name, (shape, kind) in tensors.items():
+            if plain and kind in ("embed", "matrix", "sharp"):
+                scale = {"embed": 1.0, "matrix": shape[-1] ** -0.5, "sharp": shape[-1] ** -0.5}[kind]
+                chunk, left = to_bf16(block * np.float32(scale)), int(np.prod(shape, dtype=np.int64))
+                while left > 0:
+                    chunk[:min(left, len(chunk))].tofile(f)
+                    left -= len(chunk)
+                continue
+            v = np.asarray(_latent_values(shape, kind, rng), np.float32)
+            if edit is not None:
+                new = edit(name, v)
+                v = v if new is None else np.asarray(new, np.float32)
+            bits = to_bf16(v.reshape(shape))
+            bits.tofile(f)
+            if not plain:
+                out[name] = from_bf16(bits)
+    os.replace(tmp, os.path.join(path, "model.safetensors"))
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f, indent=1)
+    return out
