@@ -293,6 +293,119 @@ def run_gpu(args, env, shape, model_path, kv_bytes=None, logits_host=None, steps
                 prof=prof, ctx=int(np.mean(ctx_mid)), tail=hist, forward_ms=forward_ms)
 
 
+# ------------------------------------------------------- designs side by side (--design)
+# Sizes that resemble real models' layers.  `llama` is the closest model the framework had: the same width, feed-forward,
+# layer count, heads and vocabulary with grouped-query attention.
+DESIGN_SIZES = {
+    "0.4b": dict(width=1024, ff=2816, layers=16, vocab=32000, heads=16, kv_heads=4, dim=64, rot=32, vdim=64, kv_rank=256, q_rank=512, batch=64),
+    "1.2b": dict(width=2048, ff=5632, layers=22, vocab=32000, heads=32, kv_heads=4, dim=64, rot=64, vdim=64, kv_rank=512, q_rank=1024, batch=64),
+    "7b-8l": dict(width=4096, ff=11008, layers=8, vocab=32000, heads=32, kv_heads=32, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=1536, batch=64),
+}
+
+
+def write_design_model(which, z, args):
+    """A random-weight model of size `z` (cached in --model-dir); returns its path."""
+    from nvllm_amd import synth
+    tag = "_".join(f"{k}{v}" for k, v in sorted(z.items()))
+    if which == "llama":
+        shape = synth.ModelShape(z["width"], z["ff"], z["layers"], z["heads"], z["kv_heads"], z["vocab"], args.max_seq_len)
+        path = os.path.join(args.model_dir, f"nvllm_llama_{tag}_s{args.max_seq_len}.bin")
+        if not (os.path.exists(path) and os.path.getsize(path) == 28 + 2 * shape.n_params()):
+            synth.write_model(path, shape, seed=0)
+        return path
+    path = os.path.join(args.model_dir, f"nvllm_suselorn_{tag}")
+    if not os.path.exists(os.path.join(path, "config.json")):
+        m = synth.latent_mixer(z["heads"], z["dim"], z["rot"], z["vdim"], z["kv_rank"], z["q_rank"])
+        synth.write_model_dir(path, synth.latent_config(z["width"], z["vocab"], [(m, z["ff"])] * z["layers"], streams=2), plain=True)
+    return path
+
+
+def kernel_table(lib):
+    """Timing class -> launches, average us, and the share of the roofline: the larger of bytes / HBM peak and flops /
+    matrix peak, over the measured time."""
+    out = {}
+    for c in range(lib.nvllm_prof_num_classes()):
+        n, ms, by, fl = C.c_longlong(), C.c_double(), C.c_double(), C.c_double()
+        lib.nvllm_prof_get(c, C.byref(n), C.byref(ms), C.byref(by), C.byref(fl))
+        if n.value:
+            hbm, mfma = by.value / (HBM_PEAK_GBS * 1e9), fl.value / (MFMA_PEAK_TFLOPS * 1e12)
+            out[lib.nvllm_prof_name(c).decode()] = dict(launches=n.value, avg_us=round(ms.value / n.value * 1e3, 2), total_ms=round(ms.value, 3),
+                                                        bound="hbm" if hbm >= mfma else "mfma", roofline=round(max(hbm, mfma) / (ms.value * 1e-3), 4))
+    return out
+
+
+def run_design(lib, path, z, args, profile):
+    """Prefill `batch` prompts in chunks, then decode; returns throughputs, or with `profile` the kernels' tables."""
+    from nvllm_amd import capi, synth
+    B = z["batch"]
+    chunks = -(-args.prompt_len // args.chunk)
+    per_step = max(1, args.max_seq_len // min(args.chunk, args.prompt_len))
+    n_new = -(-B * chunks // per_step) + 2 + args.warmup + args.steps + 8
+    eng = capi.Engine(lib, path, B, chunk_size=args.chunk, temperature=0.0, max_seq_len=args.max_seq_len, max_steps=1 << 30)
+    for i, p in enumerate(synth.make_requests(B, args.prompt_len, args.prompt_len, z["vocab"], seed=11)):
+        eng.set_request(i, p, n_new, 0)
+    eng.step()                                     # the first pass allocates workspaces and loads code
+    lib.device_sync()
+    eng.reset_stats()
+    if profile:
+        lib.nvllm_prof_reset()
+        lib.nvllm_prof_enable(1)
+    t0 = time.perf_counter()
+    while not all(s["pos"] >= s["n_prompt"] for s in (eng.seq_state(i) for i in range(B))):
+        eng.step()
+    lib.device_sync()
+    prefill_s = time.perf_counter() - t0
+    tokens = eng.stats().tokens_forwarded
+    out = {}
+    if profile:
+        out["prefill"] = kernel_table(lib)
+        lib.nvllm_prof_enable(0)
+    for _ in range(args.warmup):
+        eng.step()
+    lib.device_sync()
+    if profile:
+        lib.nvllm_prof_reset()
+        lib.nvllm_prof_enable(1)
+    t0 = time.perf_counter()
+    for _ in range(args.steps):
+        eng.step()
+    lib.device_sync()
+    decode_s = time.perf_counter() - t0
+    if profile:
+        out["decode"] = kernel_table(lib)
+        lib.nvllm_prof_enable(0)
+    else:
+        out = dict(prefill_tokens_per_s=round(tokens / prefill_s, 1), decode_tokens_per_s=round(B * args.steps / decode_s, 1),
+                   decode_ms_per_step=round(decode_s / args.steps * 1e3, 4))
+    eng.close()
+    return out
+
+
+def bench_designs(args):
+    """--design suselorn: the design beside the closest model at equal sizes, one JSON line per size."""
+    from nvllm_amd import capi
+    lib = capi.load_hip()
+    lib.nvllm_set_kv_elem_bytes(2)
+    lib.nvllm_set_logits_mode(1)
+    lib.nvllm_set_compute_dtype(capi.COMPUTE_BF16)
+    sys.stdout.flush()
+    real_stdout = os.dup(1)
+    os.dup2(2, 1)
+    for size in args.sizes.split(","):
+        z = dict(DESIGN_SIZES[size])
+        line = dict(metric="prefill and decode tokens/s, designs at equal size", size=size, shape=z, prompt_len=args.prompt_len, chunk=args.chunk,
+                    steps=args.steps, data="synthetic", dtype={"suselorn": "bf16", "llama": "f32 (fp16 hi/lo)"}, models={})
+        for which in args.design.split(",") + ([] if args.alone else ["llama"]):
+            t0 = time.time()
+            path = write_design_model(which, z, args)
+            print(f"bench: {path} ready after {time.time() - t0:.1f} s", file=sys.stderr, flush=True)
+            line["models"][which] = run_design(lib, path, z, args, False)
+            print(f"bench: {which} {size} {line['models'][which]}", file=sys.stderr, flush=True)
+            if args.profile_steps > 0:
+                line["models"][which]["kernels"] = run_design(lib, path, z, args, True)
+        os.write(real_stdout, (json.dumps(line) + "\n").encode())
+
+
 def cpu_baseline(args, shape, model_path, context):
     """The reference CPU path (oracle/_ref, the reference's own kernels compiled here)
     or, where that build is absent, this repository's restatement of it, timed on a
@@ -365,7 +478,14 @@ def main():
                     help="skip the `variants` block (N = 1 only: the same workload with the fp32 row pool and with logits rows to the host)")
     ap.add_argument("--cpu-steps", type=int, default=8, help="decode steps of the CPU baseline leg (about 1.7 s each on 16 cores); 0 disables it")
     ap.add_argument("--model-dir", default=os.environ.get("NVLLM_MODEL_DIR", "/tmp"))
+    ap.add_argument("--design", default=None, choices=("suselorn",),
+                    help="another benchmark: prefill and decode throughput of this design beside the closest model at equal sizes (bf16, random weights)")
+    ap.add_argument("--sizes", default=",".join(DESIGN_SIZES), help="with --design: which of " + ", ".join(DESIGN_SIZES))
+    ap.add_argument("--alone", action="store_true", help="with --design: without the closest model")
     args = ap.parse_args()
+    if args.design:
+        args.prompt_len, args.max_seq_len = args.prompt_len or 1024, args.max_seq_len or 2048
+        return bench_designs(args)
     if args.tp_slice:
         if not args.tp or int(os.environ.get("WORLD_SIZE", "1")) != 1:
             raise SystemExit("bench: --tp-slice goes with --tp in a single process")

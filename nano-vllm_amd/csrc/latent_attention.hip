@@ -1,15 +1,16 @@
 // latent_attention.hip -- attention over cached latents (latent_attention.h).
 //
-// k_latent_attn (bf16 pages).  A work item is up to CT consecutive tokens of one sequence x up to 16*C (token,
-// head) columns x a slice of the pages; all heads of a token share every cached row, so a row is read once per item.
-// The four waves of a workgroup walk the item's positions in blocks of 64 (four pages):
-//   copy    wave w brings page w global -> LDS with direct-to-LDS loads (pages are stored in operand order, so the
+// k_latent_attn (bf16 pages).  A work item is up to CT consecutive tokens of one sequence x up to 16, 32 or 64
+// (token, head) columns x a slice of the pages; all heads of a token share every cached row, so a row is read once per
+// item.  The workgroup walks the item's positions in blocks of 64 (four pages); wave = page + 4 * column part:
+//   copy    the waves bring the block global -> LDS with direct-to-LDS loads (pages are stored in operand order, so the
 //           image is lane-linear), one block ahead of the multiplication, two buffers;
-//   scores  wave w: S^T[key, col] = K_w Q^T over the whole row, C column groups per key fragment;
+//   scores  S^T[key, col] = K Q^T over the whole row of the wave's page, for the columns of its part;
 //   softmax block maxima meet in LDS; every wave turns its 16 keys into weights, bf16, in the operand order of the
 //           next product (a score tile's registers ARE the k order that product uses, no shuffle);
 //   values  O^T[d, col] += V^T P: the latents again, as the transposed operand, through the LDS transpose read; the
-//           waves split the latent's dims, and `col` stays on the lane, so rescaling needs no exchange.
+//           waves of a part split the latent's dims, and `col` stays on the lane, so rescaling needs no exchange.
+// Two waves per SIMD (32 and 64 columns) alternate between LDS reads and multiplies.
 // Scores, maxima and sums are fp32; queries, latents and weights enter the matrix cores as bf16.
 // The sink joins the denominator once, after the last slice (here, or in k_latent_combine when pages are sliced
 // across workgroups).
@@ -244,19 +245,23 @@ __device__ __forceinline__ void latent_barrier() {
     asm volatile("" ::: "memory");
 }
 
-// RC: row chunks of 32 held as query fragments; NT: 16-dim value tiles per wave; C: column groups of 16.
+typedef const __attribute__((address_space(4))) int* const_int_p;   // read-only for the whole launch: scalar loads
+
+// RC: row chunks of 32 held as query fragments; NT: 16-dim value tiles per wave; C: column groups of 16 per wave; WC: waves
+// side by side over the columns (4 * WC waves: wave = page of the block + 4 * column part).
 // EXACT: the row has exactly RC chunks and 4 * NT value tiles.
-template <int RC, int NT, int C, bool EXACT>
-__global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
+template <int RC, int NT, int C, int WC, bool EXACT>
+__global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds_latent[];
     const int nc = EXACT ? RC : a.chunks;
     const int n_tiles = EXACT ? 4 * NT : a.n_tiles;
     __half* pages = reinterpret_cast<__half*>(lds_latent);                          // [2][4][nc][512]
-    __half* s_p = pages + (size_t)2 * LATENT_BLOCK_PAGES * nc * TILE_HALVES;        // [C][2][64][8]
-    float* s_max = reinterpret_cast<float*>(s_p + C * 2 * 64 * 8);                  // [C][4][16]
-    float* s_sum = s_max + C * 4 * 16;                                              // [C][4][16]
+    __half* s_p = pages + (size_t)2 * LATENT_BLOCK_PAGES * nc * TILE_HALVES;        // [C * WC][2][64][8]
+    float* s_max = reinterpret_cast<float*>(s_p + C * WC * 2 * 64 * 8);             // [C * WC][4][16]
+    float* s_sum = s_max + C * WC * 4 * 16;                                         // [C * WC][4][16]
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int x = lane & 15, g = lane >> 4;
+    const int page = wave & 3, part = wave >> 2;   // this wave's page of a block, its part of the columns
 
     unsigned idx = blockIdx.x;
     const int split = (int)(idx % (unsigned)a.nsplit);
@@ -270,33 +275,43 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
     const int ntok = min(a.CT, run.y - first), t0 = run.x + first;
     const int plast = run.z - (run.y - first - ntok);
     const int h0 = hg * a.HG;
-    const int* table = a.tables + run.w;
-    const int npages = (plast >> 4) + 1, nblocks = (npages + LATENT_BLOCK_PAGES - 1) / LATENT_BLOCK_PAGES;
+    const const_int_p table = (const_int_p)(uintptr_t)(a.tables + __builtin_amdgcn_readfirstlane(run.w));
+    const int npages = __builtin_amdgcn_readfirstlane((plast >> 4) + 1), nblocks = (npages + LATENT_BLOCK_PAGES - 1) / LATENT_BLOCK_PAGES;
     const int per = (nblocks + a.nsplit - 1) / a.nsplit;
     const int b0 = split * per, b1 = min(nblocks, b0 + per);
     const int row = nc * 32;
 
-    // this lane's columns: (token, head), the last position they see
-    int colt[C], colh[C], plim[C];
-    bool valid[C];
+    // this lane's columns: (token of the item, head); -1 where the item has none.  (Formed again where needed: the page loop
+    // keeps only the last position each column sees.)
+    auto column = [&](int c, int& tok, int& h) {
+        const int j = 16 * (part * C + c) + (int)(threadIdx.x & 15);
+        tok = j / a.HG;
+        h = h0 + j - tok * a.HG;
+        const bool valid = tok < ntok && h < a.H;
+        tok = valid ? tok : 0;
+        h = valid ? h : -1;
+    };
+    int plim[C];
 #pragma unroll
     for (int c = 0; c < C; c++) {
-        const int j = 16 * c + x, tok = j / a.HG, h = h0 + j - tok * a.HG;
-        valid[c] = tok < ntok && h < a.H;
-        colt[c] = t0 + (valid[c] ? tok : 0);
-        colh[c] = valid[c] ? h : 0;
-        plim[c] = valid[c] ? plast - (ntok - 1 - tok) : -1;
+        int tok, h;
+        column(c, tok, h);
+        plim[c] = h >= 0 ? plast - (ntok - 1 - tok) : -1;
     }
 
-    const unsigned lds0 = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(wave * nc) * 1024u;
-    auto issue = [&](int b, int buf) {   // page `wave` of block b (past the end: the last page again, its keys are masked)
-        const int pg = min(b * LATENT_BLOCK_PAGES + wave, npages - 1);
-        const long page = ((long)table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1));
-        const __half* src = a.base + (size_t)page * LATENT_PAGE * row + lane * 8;
+    // the page id of a block's page `page` (past the end: the last page again, its keys are masked)
+    auto page_of = [&](int b) {
+        const int pg = min(b * LATENT_BLOCK_PAGES + page, npages - 1);
+        return (table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1));
+    };
+    const unsigned lds0 = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(page * nc + part) * 1024u;
+    auto issue = [&](int page_id, int buf) {   // tiles part, part + WC, ... of the page
+        const __half* src = a.base + (size_t)page_id * (LATENT_PAGE * row) + (size_t)part * TILE_HALVES + lane * 8;
         const unsigned dst = lds0 + (unsigned)(buf * LATENT_BLOCK_PAGES * nc) * 1024u;
 #pragma unroll
-        for (int c = 0; c < RC; c++)
-            if (EXACT || c < nc) latent_copy_tile(src + (size_t)c * TILE_HALVES, __builtin_amdgcn_readfirstlane(dst + (unsigned)c * 1024u));
+        for (int c = 0; c < RC; c += WC)
+            if (EXACT ? c + WC <= RC || c + part < RC : c + part < nc)
+                latent_copy_tile(src + (size_t)c * TILE_HALVES, __builtin_amdgcn_readfirstlane(dst + (unsigned)c * 1024u));
     };
 
     float m[C], lsum[C];
@@ -308,41 +323,58 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int n = 0; n < NT; n++) acc[n][c] = f4_t{0.f, 0.f, 0.f, 0.f};
     }
-    if (b0 < b1) issue(b0, 0);
-    // queries as the B operand: column x, dims 32k + 8g .. +7
+    int next_page = page_of(min(b0, nblocks - 1));
+    if (b0 < b1) issue(next_page, 0);
+    next_page = page_of(min(b0 + 1, nblocks - 1));
+    // queries as the B operand: column x, dims 32k + 8g .. +7 (columns nobody owns read a real row; their scores are masked)
     b8_t qf[C][RC];
 #pragma unroll
     for (int c = 0; c < C; c++) {
-        const __half* qr = a.q + ((size_t)colt[c] * a.H + colh[c]) * row + 8 * g;
+        int tok, h;
+        column(c, tok, h);
+        const __half* qr = a.q + ((size_t)(t0 + tok) * a.H + max(h, 0)) * row + 8 * g;
 #pragma unroll
-        for (int k = 0; k < RC; k++) {
-            qf[c][k] = b8_t{};
-            if ((EXACT || k < nc) && valid[c]) qf[c][k] = *reinterpret_cast<const b8_t*>(qr + 32 * k);
-        }
+        for (int k = 0; k < RC; k++) qf[c][k] = *reinterpret_cast<const b8_t*>(qr + 32 * (EXACT ? k : min(k, nc - 1)));
     }
+    // the queries have arrived before the loop: inside it the compiler then has no load of its own to wait for, and
+    // the only waits on memory are the ones below
+#pragma unroll
+    for (int c = 0; c < C; c++)
+#pragma unroll
+        for (int k = 0; k < RC; k++) asm volatile("" : "+v"(qf[c][k]));
     const float sl2 = a.scale * 1.44269504088896340736f;   // scores in the log2 domain
     // transpose read: 16 lanes bring 4 keys x 16 dims, lane i gets dim i of the 4 keys
     const int tr_key = 4 * g + (x >> 2), tr_sub = (x & 3) >> 1, tr_off = 4 * (x & 1);
 
     for (int b = b0; b < b1; b++) {
         const int buf = (b - b0) & 1;
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // this wave's page of block b is in LDS
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // this wave's tiles of block b are in LDS
         latent_barrier();                                   // ... and everybody's; block b - 1 has been consumed
-        if (b + 1 < b1) issue(b + 1, buf ^ 1);
+        if (b + 1 < b1) {
+            issue(next_page, buf ^ 1);
+            next_page = page_of(min(b + 2, nblocks - 1));
+        }
         const __half* blk = pages + (size_t)buf * LATENT_BLOCK_PAGES * nc * TILE_HALVES;
-        // ---- scores of this wave's page
+        // ---- scores of this wave's page; key fragments a few chunks ahead of the multiplies
         f4_t s[C];
 #pragma unroll
         for (int c = 0; c < C; c++) s[c] = f4_t{0.f, 0.f, 0.f, 0.f};
-        const b8_t* kp = reinterpret_cast<const b8_t*>(blk + (size_t)wave * nc * TILE_HALVES) + lane;
+        const b8_t* kp = reinterpret_cast<const b8_t*>(blk + (size_t)page * nc * TILE_HALVES) + lane;
+        constexpr int KA = C == 2 ? 3 : RC < 6 ? RC : 6;
+        b8_t kf[KA];
 #pragma unroll
-        for (int k = 0; k < RC; k++)
+        for (int k = 0; k < KA; k++) kf[k] = kp[(EXACT ? k : min(k, nc - 1)) * 64];
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int k = 0; k < RC; k++) {
             if (EXACT || k < nc) {
-                const b8_t kf = kp[k * 64];
 #pragma unroll
-                for (int c = 0; c < C; c++) s[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[c][k], s[c], 0, 0, 0);
+                for (int c = 0; c < C; c++) s[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k % KA], qf[c][k], s[c], 0, 0, 0);
+                if (k + KA < RC && (EXACT || k + KA < nc)) kf[k % KA] = kp[(k + KA) * 64];
             }
-        const int kfirst = (b * LATENT_BLOCK_PAGES + wave) * LATENT_PAGE + 4 * g;
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        const int kfirst = (b * LATENT_BLOCK_PAGES + page) * LATENT_PAGE + 4 * g;
 #pragma unroll
         for (int c = 0; c < C; c++) {
             float mx = -INFINITY;
@@ -352,16 +384,20 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
                 mx = fmaxf(mx, s[c][r]);
             }
             mx = rows_max(mx);
-            if (g == 0) s_max[(c * 4 + wave) * 16 + x] = mx;
+            if (g == 0) s_max[((part * C + c) * 4 + page) * 16 + x] = mx;
         }
         latent_barrier();
         // ---- weights
+        float bm[C][4];
+#pragma unroll
+        for (int c = 0; c < C; c++)
+#pragma unroll
+            for (int w = 0; w < 4; w++) bm[c][w] = s_max[((part * C + c) * 4 + w) * 16 + x];
         float alpha[C];
         bool rises = false;
 #pragma unroll
         for (int c = 0; c < C; c++) {
-            const float* bm = s_max + c * 64 + x;
-            const float mn = fmaxf(m[c], fmaxf(fmaxf(bm[0], bm[16]), fmaxf(bm[32], bm[48])));
+            const float mn = fmaxf(m[c], fmaxf(fmaxf(bm[c][0], bm[c][1]), fmaxf(bm[c][2], bm[c][3])));
             alpha[c] = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[c] - mn);
             rises |= mn > m[c];
             m[c] = mn;
@@ -373,7 +409,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
                 p[r] = __builtin_amdgcn_exp2f(s[c][r] - msafe);
                 lsum[c] += p[r];
             }
-            *reinterpret_cast<b4_t*>(s_p + ((size_t)(c * 2 + (wave >> 1)) * 64 + lane) * 8 + (wave & 1) * 4) = to_b4(p);
+            *reinterpret_cast<b4_t*>(s_p + ((size_t)((part * C + c) * 2 + (page >> 1)) * 64 + lane) * 8 + (page & 1) * 4) = to_b4(p);
         }
         if (__any(rises)) {
 #pragma unroll
@@ -385,26 +421,33 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
         }
         latent_barrier();
         // ---- values: keys of pages (0, 1), then (2, 3)
+        b8_t pf[C];
+        auto load_weights = [&](int h) {
 #pragma unroll
-        for (int h = 0; h < 2; h++) {
-            b8_t pf[C];
+            for (int c = 0; c < C; c++) pf[c] = *reinterpret_cast<const b8_t*>(s_p + ((size_t)((part * C + c) * 2 + h) * 64 + lane) * 8);
+        };
+        load_weights(0);
+        auto value_frag = [&](int i) {   // fragment i of 2 * NT: half i / NT of the block, value tile page + 4 * (i % NT)
+            const int h = i / NT, n = EXACT ? page + 4 * (i % NT) : min(page + 4 * (i % NT), n_tiles - 1);
+            const __half* v = blk + (size_t)(2 * h) * nc * TILE_HALVES + (n >> 1) * TILE_HALVES + (tr_key + 16 * (2 * (n & 1) + tr_sub)) * 8 + tr_off;
+            const s4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)v);
+            const s4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(v + (size_t)nc * TILE_HALVES));
+            const s8_t both = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+            return __builtin_bit_cast(b8_t, both);
+        };
+        constexpr int VA = C == 2 || NT == 1 ? 2 : 4;
+        b8_t vf[VA];
 #pragma unroll
-            for (int c = 0; c < C; c++) pf[c] = *reinterpret_cast<const b8_t*>(s_p + ((size_t)(c * 2 + h) * 64 + lane) * 8);
-            const __half* v0 = blk + (size_t)(2 * h) * nc * TILE_HALVES + tr_off;
-            const __half* v1 = v0 + (size_t)nc * TILE_HALVES;
+        for (int i = 0; i < VA; i++) vf[i] = value_frag(i);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-            for (int i = 0; i < NT; i++) {
-                const int n = wave + 4 * i;
-                if (EXACT || n < n_tiles) {
-                    const int off = (n >> 1) * TILE_HALVES + (tr_key + 16 * (2 * (n & 1) + tr_sub)) * 8;
-                    const s4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(v0 + off));
-                    const s4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(v1 + off));
-                    const s8_t both = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-                    const b8_t vf = __builtin_bit_cast(b8_t, both);
+        for (int i = 0; i < 2 * NT; i++) {
+            // (a value tile past the end multiplies the last one again; its sums are never stored)
 #pragma unroll
-                    for (int c = 0; c < C; c++) acc[i][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[c], acc[i][c], 0, 0, 0);
-                }
-            }
+            for (int c = 0; c < C; c++) acc[i % NT][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i % VA], pf[c], acc[i % NT][c], 0, 0, 0);
+            if (i == NT - 1) load_weights(1);
+            if (i + VA < 2 * NT) vf[i % VA] = value_frag(i + VA);
+            __builtin_amdgcn_sched_barrier(0);
         }
     }
     // ---- the waves' partial sums meet; the sink; the result
@@ -412,32 +455,34 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentKArgs a) {
     for (int c = 0; c < C; c++) {
         lsum[c] += __shfl_xor(lsum[c], 16, 64);
         lsum[c] += __shfl_xor(lsum[c], 32, 64);
-        if (g == 0) s_sum[(c * 4 + wave) * 16 + x] = lsum[c];
+        if (g == 0) s_sum[((part * C + c) * 4 + page) * 16 + x] = lsum[c];
     }
     latent_barrier();
 #pragma unroll
     for (int c = 0; c < C; c++) {
-        const float* bs = s_sum + c * 64 + x;
+        const float* bs = s_sum + (part * C + c) * 64 + x;
         const float L = (bs[0] + bs[16]) + (bs[32] + bs[48]);
-        if (!valid[c]) continue;
+        int tok, h;
+        column(c, tok, h);
+        if (h < 0) continue;
         float f = 1.f;
-        const size_t th = (size_t)colt[c] * a.H + colh[c];
+        const size_t th = (size_t)(t0 + tok) * a.H + h;
         if (a.nsplit == 1) {
-            const float sk = a.sink[colh[c]] * 1.44269504088896340736f, top = fmaxf(m[c], sk);
+            const float sk = a.sink[h] * 1.44269504088896340736f, top = fmaxf(m[c], sk);
             const float w = __builtin_amdgcn_exp2f(m[c] - top);
             f = w / fmaf(L, w, __builtin_amdgcn_exp2f(sk - top));
-        } else if (wave == 0 && g == 0) {
+        } else if (page == 0 && g == 0) {
             a.part_ml[(th * a.nsplit + split) * 2] = m[c];
             a.part_ml[(th * a.nsplit + split) * 2 + 1] = L;
         }
 #pragma unroll
         for (int i = 0; i < NT; i++) {
-            const int n = wave + 4 * i;
+            const int n = page + 4 * i;
             if (!(EXACT || n < n_tiles)) continue;
             const int d = 16 * n + 4 * g;
             if (a.nsplit == 1) {
                 const float o[4] = {acc[i][c][0] * f, acc[i][c][1] * f, acc[i][c][2] * f, acc[i][c][3] * f};
-                store_b16_4(a.out, a.Kb_out, colt[c], colh[c] * a.rank_ld + d, o);
+                store_b16_4(a.out, a.Kb_out, t0 + tok, h * a.rank_ld + d, o);
             } else {
                 *reinterpret_cast<f4_t*>(a.part_acc + (th * a.nsplit + split) * a.rank_ld + d) = acc[i][c];
             }
@@ -470,26 +515,27 @@ __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict_
     }
 }
 
-template <int RC, int NT, int C>
+template <int RC, int NT, int C, int WC>
 static void launch_latent_c(const LatentKArgs& k, long units) {
-    const size_t lds = latent_attn_lds(k.chunks, C);
+    const size_t lds = latent_attn_lds(k.chunks, C * WC);
     const bool exact = k.chunks == RC && k.n_tiles == 4 * NT;
     static bool ready = false;
     if (!ready) {
-        const int most = (int)latent_attn_lds(RC, C);
+        const int most = (int)latent_attn_lds(RC, C * WC);
         if (most > 64 * 1024) {
-            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, true>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
-            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, false>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
+            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, WC, true>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
+            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, WC, false>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
         }
         ready = true;
     }
-    if (exact) NVLLM_LAUNCH((k_latent_attn<RC, NT, C, true>), dim3((unsigned)units), dim3(256), lds, k);
-    else NVLLM_LAUNCH((k_latent_attn<RC, NT, C, false>), dim3((unsigned)units), dim3(256), lds, k);
+    if (exact) NVLLM_LAUNCH((k_latent_attn<RC, NT, C, WC, true>), dim3((unsigned)units), dim3(256 * WC), lds, k);
+    else NVLLM_LAUNCH((k_latent_attn<RC, NT, C, WC, false>), dim3((unsigned)units), dim3(256 * WC), lds, k);
 }
 template <int RC, int NT>
-static void launch_latent_rc(const LatentKArgs& k, long units, int C) {
-    if (C == 1) launch_latent_c<RC, NT, 1>(k, units);
-    else launch_latent_c<RC, NT, 2>(k, units);
+static void launch_latent_rc(const LatentKArgs& k, long units, int columns) {
+    if (columns == 16) launch_latent_c<RC, NT, 1, 1>(k, units);
+    else if (columns == 32) launch_latent_c<RC, NT, 1, 2>(k, units);
+    else launch_latent_c<RC, NT, 2, 2>(k, units);
 }
 
 void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
@@ -515,8 +561,8 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
                          P.block_size, a.H, P.rank, P.rank_ld, row, a.out_f32, a.out_b16, 0);
         return;
     }
-    // columns per item: 32, or 16 when no item would fill more
-    const int C = (a.H <= 16 && a.H * st.max_run <= 16) ? 1 : 2, W = 16 * C;
+    // columns per item: 64, or 32 or 16 when no item would fill more
+    const int W = a.H * st.max_run <= 16 ? 16 : a.H * st.max_run <= 32 ? 32 : 64;
     LatentKArgs k{};
     k.base = (const __half*)P.base;
     k.q = (const __half*)a.q;
@@ -537,7 +583,7 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     k.Kb_out = a.H * P.rank_ld / 32;
     // slices of pages until the chip is full: as many workgroups as fit by LDS (at most two per CU), two blocks per slice at least
     const long items = (long)st.n_runs * k.n_sub * k.NG;
-    const int per_cu = latent_attn_lds(chunks, C) * 2 <= 160 * 1024 ? 2 : 1;
+    const int per_cu = latent_attn_lds(chunks, W / 16) * 2 <= 160 * 1024 ? 2 : 1;
     const int nblocks = cdiv(st.max_pos / LATENT_PAGE + 1, LATENT_BLOCK_PAGES);
     int nsplit = (int)(((long)per_cu * rt().num_cus + items / 2) / items);
     if (nsplit > cdiv(nblocks, 2)) nsplit = cdiv(nblocks, 2);
@@ -553,10 +599,10 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     {
         ProfScope ps(PC_LATENT_ATTN, bytes, flops);
         const long units = items * nsplit;
-        if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, C);
-        else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, C);
-        else if (chunks <= 10 && vt <= 4) launch_latent_rc<10, 4>(k, units, C);
-        else launch_latent_rc<18, 8>(k, units, C);
+        if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, W);
+        else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, W);
+        else if (chunks <= 10 && vt <= 4) launch_latent_rc<10, 4>(k, units, W);
+        else launch_latent_rc<18, 8>(k, units, W);
     }
     if (nsplit > 1) {
         ProfScope ps(PC_LATENT_COMBINE, (double)st.T * a.H * ((double)nsplit * (P.rank_ld + 2) * 4.0 + P.rank_ld * 2.0), 0);
