@@ -4,6 +4,7 @@
 // (one head per group of row blocks) is the same kernel with tiles that stay inside a group.
 #include "gemm_prefill_tile.h"
 #include "gemm_tile.h"
+#include "latent_kv.h"
 
 namespace nvllm {
 
@@ -14,8 +15,14 @@ constexpr int NW = 8, RW = 4, RA = 2;
 template <int NBW, int TB, int WAVES, int EPI, bool GRP>
 __global__ __launch_bounds__(WAVES * 64) void k_gemm_b16(GemmArgs p) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds_dyn[];
+    if constexpr (EPI == GemmEpilogue::LATENT_Q) {
+        if ((int)blockIdx.x >= p.ride_from) {
+            if (blockIdx.y == 0 && blockIdx.z == 0) latent_kv_ride(p.ride, ((int)blockIdx.x - p.ride_from) * WAVES + (int)(threadIdx.x >> 6), threadIdx.x & 63);
+            return;
+        }
+    }
     h8_t w[RW][NBW];
-    const TileIdx ix{(int)blockIdx.x, (int)blockIdx.y, (int)blockIdx.z, (int)gridDim.x};
+    const TileIdx ix{(int)blockIdx.x, (int)blockIdx.y, (int)blockIdx.z, EPI == GemmEpilogue::LATENT_Q ? p.ride_from : (int)gridDim.x};
     gemm_tile<NBW, TB, WAVES, RW, RA, EPI, float, false, 0, OpBf16, GRP>(p, ix, lds_dyn, w, [](int) {}, (int)threadIdx.x);
 }
 
@@ -34,7 +41,7 @@ void launch_stream(const GemmArgs& a, dim3 grid) {
 
 template <int EPI, bool GRP>
 void launch_stream_plan(const GemmArgs& a, const GemmPlan& pl) {
-    const dim3 grid(pl.tiles_n, pl.ks, pl.tiles_t);
+    const dim3 grid(pl.tiles_n + (EPI == GemmEpilogue::LATENT_Q && a.ride.base ? cdiv(a.ride.T, NW) : 0), pl.ks, pl.tiles_t);
     if constexpr (EPI == GemmEpilogue::SWIGLU_A16) {
         if (pl.nbw == 6) {
             launch_stream<6, 2, NW, EPI, GRP>(a, grid);
@@ -65,7 +72,7 @@ void launch_dense_tw(const GemmArgs& a, int tiles_n, int tiles_t, int nbuf) {
                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem));
         allowed = shmem;
     }
-    NVLLM_LAUNCH((k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP>), dim3(tiles_n * tiles_t), dim3(256), shmem, a, tiles_n, tiles_t, nbuf,
+    NVLLM_LAUNCH((k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP>), dim3(tiles_n * tiles_t + (EPI == GemmEpilogue::LATENT_Q && a.ride.base ? cdiv(a.ride.T, 4) : 0)), dim3(256), shmem, a, tiles_n, tiles_t, nbuf,
                  tiles_n * tiles_t);
 }
 
@@ -83,6 +90,7 @@ void launch_dense(GemmArgs a) {
     const int nbuf = per_cu >= 3 ? 3 : (per_cu == 2 ? 4 : 5);   // 16 KiB per stage (12 for the lower tiles)
     a.ksplit = 1;
     a.kb_per_split = a.Kb;
+    a.ride_from = total;
     if (low) launch_dense_tw<EPI, GRP, 2>(a, tiles_n, tiles_t, nbuf);
     else launch_dense_tw<EPI, GRP, 4>(a, tiles_n, tiles_t, nbuf);
 }
@@ -107,6 +115,7 @@ void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
         pl.tiles_n = a.group_tiles * groups;
         pl.nw = NW;
     }
+    a.ride_from = pl.tiles_n;
     a.ksplit = pl.ks;
     a.kb_per_split = pl.kb_per_split;
     const long wgs = (long)pl.tiles_n * pl.ks * pl.tiles_t;
@@ -124,7 +133,7 @@ void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
 
 }  // namespace
 
-void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls) {
+void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls, const LatentKvRider* ride) {
     if (T <= 0) return;
     ensure_init();
     if (w.K % 32) NVLLM_FATAL("bf16 projection: the input width %d is not padded to 32", w.K);
@@ -145,6 +154,10 @@ void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpi
     }
     a.counters = gemm_tile_counters();
     a.e = epi;
+    if (ride) {
+        if (epi.kind != GemmEpilogue::LATENT_Q) NVLLM_FATAL("cache rows ride on the query projection only");
+        a.ride = *ride;
+    }
     auto need32 = [&](int n, const char* what) {
         if (n % 32) NVLLM_FATAL("bf16 projection: %s of %d is not padded to 32", what, n);
     };

@@ -30,6 +30,20 @@ constexpr bool epi_is_point(int kind) { return kind >= GemmEpilogue::TILE_B16; }
 // epilogues that also leave sums of squares per 32 features
 constexpr bool epi_has_ss(int kind) { return kind == GemmEpilogue::RESID_A16 || kind == GemmEpilogue::LATENT_IN; }
 
+// What a launch may carry besides its tiles: the norm, rotation and cache write of the batch's latent rows (latent_kv.h)
+// in extra workgroups, a wave per token.  Their input comes from the launch before and their output is for the launch
+// after, so they cost no time of their own.
+struct LatentKvRider {
+    void* base = nullptr;   // null: nobody rides
+    const float* raw;
+    const float* gain;
+    const float2* rope;
+    const int* pos;
+    const int* kv_row;
+    float eps;
+    int raw_ld, rot_at, T, rank, rot, rank_ld, rot_ld;
+};
+
 struct GemmArgs {
     const __half* W;
     long nb_stride;   // halves between 16-row blocks
@@ -48,6 +62,8 @@ struct GemmArgs {
     int close_sc1;    // K split: the closing workgroup loads the partials past the vector cache instead of invalidating it
                       // (launches of at most one workgroup per CU over a hipMalloc slab)
     GemmEpilogue e;
+    LatentKvRider ride;
+    int ride_from;    // first workgroup (grid x) of the riders
 #ifdef NVLLM_STAMPS
     unsigned long long* stamps;   // diagnostic builds only: [workgroup][8] constant-rate clock readings
 #endif
@@ -138,28 +154,37 @@ __device__ __forceinline__ void store_b16_4(__half* act, int Kb_out, int t, int 
 // Hyper-connection update of one token's features n .. n+3 and the next sublayer's input from it:
 //   x_to <- sum_from mix[from][to] x_from + out[to] * (y + bias) * scale;   u = sum_s in[s] x_s;
 //   act = tanh(alpha u) w + b
+// in two halves: what does not depend on y is loaded early, so that it travels while the sums are completed.
 template <int SMAX>
-__device__ __forceinline__ void hyper_update_4(const GemmEpilogue& ep, int N, int t, int n, const float* y_in) {
+struct HyperIn {
+    f4_t xs[SMAX], scale, bias, w, b;
+};
+template <int SMAX>
+__device__ __forceinline__ void hyper_load_4(HyperIn<SMAX>& in, const GemmEpilogue& ep, int N, int t, int n) {
+    const float* xr = ep.x + (size_t)t * ep.streams * N + n;
+#pragma unroll
+    for (int s = 0; s < SMAX; s++) in.xs[s] = *reinterpret_cast<const f4_t*>(xr + (size_t)min(s, ep.streams - 1) * N);
+    in.scale = *reinterpret_cast<const f4_t*>(ep.hyper_scale + n);
+    in.bias = ep.bias ? *reinterpret_cast<const f4_t*>(ep.bias + n) : f4_t{0.f, 0.f, 0.f, 0.f};
+    in.w = *reinterpret_cast<const f4_t*>(ep.norm_w + n);
+    in.b = *reinterpret_cast<const f4_t*>(ep.norm_b + n);
+}
+template <int SMAX>
+__device__ __forceinline__ void hyper_update_4(const HyperIn<SMAX>& in, const GemmEpilogue& ep, int N, int t, int n, const float* y_in) {
     const int S = ep.streams;
     float y[4];
-    const f4_t ls = *reinterpret_cast<const f4_t*>(ep.hyper_scale + n);
-    const f4_t bias = ep.bias ? *reinterpret_cast<const f4_t*>(ep.bias + n) : f4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int r = 0; r < 4; r++) y[r] = (y_in[r] + bias[r]) * ls[r];
-    f4_t xs[SMAX];
+    for (int r = 0; r < 4; r++) y[r] = (y_in[r] + in.bias[r]) * in.scale[r];
     float* xr = ep.x + (size_t)t * S * N + n;
-#pragma unroll
-    for (int s = 0; s < SMAX; s++)
-        if (s < S) xs[s] = *reinterpret_cast<const f4_t*>(xr + (size_t)s * N);
     const float* mix = ep.hyper;
     const float* out = mix + S * S;
-    const float* in = out + S;
-    const float alpha = in[S];
+    const float* weight = out + S;
+    const float alpha = weight[S];
     f4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int to = 0; to < SMAX; to++)
         if (to < S) {
-            const float o = out[to], ii = in[to];
+            const float o = out[to], ii = weight[to];
             f4_t v;
 #pragma unroll
             for (int r = 0; r < 4; r++) v[r] = o * y[r];
@@ -168,20 +193,20 @@ __device__ __forceinline__ void hyper_update_4(const GemmEpilogue& ep, int N, in
                 if (s < S) {
                     const float m = mix[s * S + to];
 #pragma unroll
-                    for (int r = 0; r < 4; r++) v[r] = fmaf(m, xs[s][r], v[r]);
+                    for (int r = 0; r < 4; r++) v[r] = fmaf(m, in.xs[s][r], v[r]);
                 }
             *reinterpret_cast<f4_t*>(xr + (size_t)to * N) = v;
 #pragma unroll
             for (int r = 0; r < 4; r++) u[r] = fmaf(ii, v[r], u[r]);
         }
-    const f4_t w = *reinterpret_cast<const f4_t*>(ep.norm_w + n), b = *reinterpret_cast<const f4_t*>(ep.norm_b + n);
     float z[4];
 #pragma unroll
-    for (int r = 0; r < 4; r++) z[r] = fmaf(tanhf(alpha * u[r]), w[r], b[r]);
+    for (int r = 0; r < 4; r++) z[r] = fmaf(tanhf(alpha * u[r]), in.w[r], in.b[r]);
     store_b16_4(ep.a16_out, ep.Kb_out, t, n, z);
 }
+constexpr int hyper_streams(int kind) { return kind == GemmEpilogue::HYPER_2 ? 2 : kind == GemmEpilogue::HYPER_4 ? 4 : 0; }   // 0: another epilogue
 
-// One token's features n .. n+3 through a point epilogue; returns their share of the sum of squares.
+// One token's features n .. n+3 through a point epilogue other than HYPER_*; returns their share of the sum of squares.
 template <int EPI>
 __device__ __forceinline__ float epi_point(const GemmEpilogue& ep, int N, int t, int n, const float* y) {
     if constexpr (EPI == GemmEpilogue::TILE_B16) {
@@ -213,10 +238,6 @@ __device__ __forceinline__ float epi_point(const GemmEpilogue& ep, int N, int t,
                 }
             *reinterpret_cast<b4_t*>(ep.q_rows + ((size_t)t * ep.q_heads + h) * ep.q_row + ep.head_ld + d) = to_b4(z);
         }
-    } else if constexpr (EPI == GemmEpilogue::HYPER_2) {
-        hyper_update_4<2>(ep, N, t, n, y);
-    } else {
-        hyper_update_4<4>(ep, N, t, n, y);
     }
     return 0.f;
 }

@@ -42,6 +42,7 @@
 #pragma once
 
 #include "gemm_common.h"
+#include "latent_kv.h"
 #include <type_traits>
 #include <algorithm>
 
@@ -128,6 +129,12 @@ __device__ __forceinline__ void pf_epilogue(const GemmArgs& p, const f4_t (&v)[N
             pos = ep.pos[t];
             kv_row = ep.kv_row[t];
         }
+        constexpr int HS = hyper_streams(EPI);
+        HyperIn<HS ? HS : 1> hyper[HS ? NI : 1];   // the residual operands of all NI tiles of this token block travel together
+        if constexpr (HS > 0) {
+#pragma unroll
+            for (int i = 0; i < NI; i++) hyper_load_4<HS>(hyper[i], ep, p.N, min(t, p.T - 1), min((nb_first + i) * 16 + 4 * (lane >> 4), p.N - 4));
+        }
         float ssq[NI / 2];
 #pragma unroll
         for (int h = 0; h < NI / 2; h++) ssq[h] = 0.f;
@@ -137,7 +144,9 @@ __device__ __forceinline__ void pf_epilogue(const GemmArgs& p, const f4_t (&v)[N
             const int n = nb * 16 + 4 * (lane >> 4);
             const bool live = tok_live && nb < nb_lim;
             float y[4] = {v[i][j][0] * rinv, v[i][j][1] * rinv, v[i][j][2] * rinv, v[i][j][3] * rinv};
-            if constexpr (epi_is_point(EPI)) {
+            if constexpr (HS > 0) {
+                if (live) hyper_update_4<HS>(hyper[i], ep, p.N, t, n, y);
+            } else if constexpr (epi_is_point(EPI)) {
                 if (live) ssq[i >> 1] += epi_point<EPI>(ep, p.N, t, n, y);
             } else if (EPI == GemmEpilogue::F32) {
                 if constexpr (OP::PLANES == 1) {
@@ -292,6 +301,12 @@ __global__ __launch_bounds__(128 * WR * KG, WR == 4 ? 4 : 2) void k_gemm_prefill
     const int ablate = nbuf >> 8;   // diagnostic build: 1 no in-loop copies, 2 no multiplies, 4 no LDS reads, 8 no barrier, 16 no epilogue
     nbuf &= 255;
 #endif
+    if constexpr (EPI == GemmEpilogue::LATENT_Q) {
+        if ((int)blockIdx.x >= p.ride_from) {
+            latent_kv_ride(p.ride, ((int)blockIdx.x - p.ride_from) * (2 * WR * KG) + (int)(threadIdx.x >> 6), threadIdx.x & 63);
+            return;
+        }
+    }
     // all LDS is one object: 128 floats of 1/rms, then the ring [nbuf][STAGE_TILES][512 halves]
     extern __shared__ __attribute__((aligned(16))) __half lds_all[];
     float* s_rinv = reinterpret_cast<float*>(lds_all);

@@ -311,6 +311,17 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
             pf_g[s] = *reinterpret_cast<const float4*>(ep.gain_next + n);
         }
     }
+    constexpr int HS = hyper_streams(EPI);
+    HyperIn<HS ? HS : 1> pf_hyper[HS ? FPT : 1];
+    if constexpr (HS > 0) {
+#pragma unroll
+        for (int s = 0; s < FPT; s++) {
+            const int w_ = min(tid + s * NW * 64, WITEMS - 1);
+            const int h = w_ >> ITEMS_SHIFT, e = w_ & (ITEMS - 1);
+            const int l = e & 63, j = (e >> 6) % TB, i = (e >> 6) / TB;
+            hyper_load_4<HS>(pf_hyper[s], ep, p.N, min(tb0 * 16 + j * 16 + (l & 15), p.T - 1), min((nb0 + 2 * h + i) * 16 + 4 * (l >> 4), p.N - 4));
+        }
+    }
     if (EPI == GemmEpilogue::ROPE_KV) {   // all items of a thread belong to one token (NW*64 is a multiple of TB*64)
         const int e = min(tid, WITEMS - 1) & (ITEMS - 1);
         const int t = min(tb0 * 16 + ((e >> 6) % TB) * 16 + (e & 15), p.T - 1);
@@ -438,7 +449,9 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
             const bool live = t < p.T && tb0 + j < p.Tb && nb < nb_lim;
             const float rinv = ep.ss_in ? s_rinv[tl] : 1.0f;
             float y[4] = {v[s][0] * rinv, v[s][1] * rinv, v[s][2] * rinv, v[s][3] * rinv};
-            if constexpr (epi_is_point(EPI)) {
+            if constexpr (HS > 0) {
+                if (live) hyper_update_4<HS>(pf_hyper[s], ep, p.N, t, n, y);
+            } else if constexpr (epi_is_point(EPI)) {
                 if (live) ssq[s] += epi_point<EPI>(ep, p.N, t, n, y);
             } else if (EPI == GemmEpilogue::F32) {
                 if constexpr (OP::PLANES == 1) {

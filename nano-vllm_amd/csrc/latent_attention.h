@@ -32,6 +32,11 @@ static inline size_t latent_pool_bytes(const LatentPool& p, int num_blocks) { re
 void launch_latent_kv(const LatentPool& pool, const float* raw, int raw_ld, int rot_at, const float* gain, float eps, const float2* rope,
                       const StepArrays& st);
 
+// the same as a rider of the query projection (launch_gemm_b16)
+struct LatentKvRider;
+LatentKvRider latent_kv_rider(const LatentPool& pool, const float* raw, int raw_ld, int rot_at, const float* gain, float eps, const float2* rope,
+                              const StepArrays& st);
+
 struct LatentAttn {
     LatentPool pool;
     const void* q;         // [T][H][pool.row()], element type as the pool's
@@ -41,7 +46,7 @@ struct LatentAttn {
     float* out_f32;        // fp32 pool: [T][H][rank]
     __half* out_b16;       // bf16 pool: activation tiles of [T, H * rank_ld]
 };
-constexpr int LATENT_RUN = 32;   // stage_step(attn_ct): tokens per run at most
+constexpr int LATENT_RUN = 32;   // stage_step(attn_ct, multi_first): tokens per run at most
 void launch_latent_attention(const LatentAttn& a, const StepArrays& st);
 
 // fp32 models: q [T][H * (dim + rot)] -> rows [T][H][rank + rot] (W_uk [H * dim, rank] absorbed, rotated part turned)

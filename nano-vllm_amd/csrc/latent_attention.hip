@@ -21,6 +21,7 @@
 
 #include "attn_tile.h"
 #include "gemm_common.h"
+#include "latent_kv.h"
 
 namespace nvllm {
 
@@ -34,94 +35,36 @@ LatentPool latent_pool(void* base, int elem_bytes, int block_size, int rank, int
     return p;
 }
 
-// half index of element d of the row at pool row r (block * block_size + slot)
-__device__ __forceinline__ size_t latent_off(long r, int d, int row) {
-    return (size_t)(r >> 4) * 16 * row + (size_t)(d >> 5) * 512 + (size_t)(((int)r & 15) + 16 * ((d >> 3) & 3)) * 8 + (d & 7);
-}
 __device__ __forceinline__ float bf16_to_f32(unsigned short v) { return __builtin_bit_cast(float, (unsigned)v << 16); }
 
 // ------------------------------------------------------------------ cache write
 template <bool B16>
-__global__ __launch_bounds__(256) void k_latent_kv(void* base, const float* __restrict__ raw, int raw_ld, int rot_at, const float* __restrict__ gain,
-                                                   float eps, const float2* __restrict__ rope, const int* __restrict__ pos,
-                                                   const int* __restrict__ kv_row, int T, int rank, int rot, int rank_ld, int rot_ld) {
-    const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t >= T) return;
-    const long row = kv_row[t];
-    if (row < 0) return;
-    const float* src = raw + (size_t)t * raw_ld;
-    const int width = rank_ld + rot_ld;
-    float ss = 0.f;
-    for (int d = lane; d < rank; d += 64) ss = fmaf(src[d], src[d], ss);
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
-    const float rms = sqrtf(ss / (float)rank + eps);
-    const float2* tab = rope + (size_t)pos[t] * (rot >> 1);
-    for (int d = 2 * lane; d < width; d += 128) {   // a pair of elements per lane (rank_ld is even in the padded layout)
-        float v[2] = {0.f, 0.f};
-        if (d >= rank_ld) {
-            const int r = d - rank_ld;
-            if (r < rot) {
-                const float2 cs = tab[r >> 1];
-                const float u = src[rot_at + r], w = src[rot_at + r + 1];
-                v[0] = u * cs.x - w * cs.y;
-                v[1] = w * cs.x + u * cs.y;
-            }
-        } else {
-#pragma unroll
-            for (int e = 0; e < 2; e++)
-                if (d + e < rank) v[e] = src[d + e] / rms * gain[d + e];
-        }
-        if (B16) {
-            typedef __bf16 b2_t __attribute__((ext_vector_type(2)));
-            typedef float f2_t __attribute__((ext_vector_type(2)));
-            const f2_t f = {v[0], v[1]};
-            *reinterpret_cast<b2_t*>(reinterpret_cast<__half*>(base) + latent_off(row, d, width)) = __builtin_convertvector(f, b2_t);
-        } else {
-            float* dst = reinterpret_cast<float*>(base) + (size_t)row * width + d;
-            dst[0] = v[0];
-            dst[1] = v[1];
-        }
+__global__ __launch_bounds__(256) void k_latent_kv(LatentKvRider a) {
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (B16) {
+        latent_kv_ride(a, t, lane);
+        return;
     }
+    if (t >= a.T || a.kv_row[t] < 0) return;
+    float* dst = reinterpret_cast<float*>(a.base) + (size_t)a.kv_row[t] * (a.rank_ld + a.rot_ld);
+    latent_kv_token(a, t, lane, [&](int d, float v) { dst[d] = v; });
 }
-// fp32 rows whose latent size is odd: pairs would straddle the two parts, so one element per lane
-__global__ __launch_bounds__(256) void k_latent_kv_odd(float* base, const float* __restrict__ raw, int raw_ld, int rot_at, const float* __restrict__ gain,
-                                                       float eps, const float2* __restrict__ rope, const int* __restrict__ pos,
-                                                       const int* __restrict__ kv_row, int T, int rank, int rot) {
-    const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t >= T) return;
-    const long row = kv_row[t];
-    if (row < 0) return;
-    const float* src = raw + (size_t)t * raw_ld;
-    float ss = 0.f;
-    for (int d = lane; d < rank; d += 64) ss = fmaf(src[d], src[d], ss);
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
-    const float rms = sqrtf(ss / (float)rank + eps);
-    float* dst = base + (size_t)row * (rank + rot);
-    for (int d = lane; d < rank; d += 64) dst[d] = src[d] / rms * gain[d];
-    for (int i = lane; i < rot / 2; i += 64) {
-        const float2 cs = rope[(size_t)pos[t] * (rot >> 1) + i];
-        const float u = src[rot_at + 2 * i], w = src[rot_at + 2 * i + 1];
-        dst[rank + 2 * i] = u * cs.x - w * cs.y;
-        dst[rank + 2 * i + 1] = w * cs.x + u * cs.y;
-    }
+
+LatentKvRider latent_kv_rider(const LatentPool& pool, const float* raw, int raw_ld, int rot_at, const float* gain, float eps, const float2* rope,
+                              const StepArrays& st) {
+    LatentKvRider r;
+    r.base = pool.base; r.raw = raw; r.gain = gain; r.rope = rope; r.pos = st.d_pos; r.kv_row = st.d_kv_row; r.eps = eps;
+    r.raw_ld = raw_ld; r.rot_at = rot_at; r.T = st.T; r.rank = pool.rank; r.rot = pool.rot; r.rank_ld = pool.rank_ld; r.rot_ld = pool.rot_ld;
+    return r;
 }
 
 void launch_latent_kv(const LatentPool& pool, const float* raw, int raw_ld, int rot_at, const float* gain, float eps, const float2* rope,
                       const StepArrays& st) {
     if (st.T <= 0) return;
     ProfScope ps(PC_LATENT_KV, (double)st.T * ((double)raw_ld * 4.0 + (double)pool.row() * pool.elem_bytes), 0);
-    const dim3 grid(cdiv(st.T, 4));
-    if (pool.elem_bytes == 2)
-        NVLLM_LAUNCH((k_latent_kv<true>), grid, dim3(256), 0, pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
-                     pool.rot, pool.rank_ld, pool.rot_ld);
-    else if (pool.rank % 2)
-        NVLLM_LAUNCH(k_latent_kv_odd, grid, dim3(256), 0, (float*)pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
-                     pool.rot);
-    else
-        NVLLM_LAUNCH((k_latent_kv<false>), grid, dim3(256), 0, pool.base, raw, raw_ld, rot_at, gain, eps, rope, st.d_pos, st.d_kv_row, st.T, pool.rank,
-                     pool.rot, pool.rank_ld, pool.rot_ld);
+    const LatentKvRider r = latent_kv_rider(pool, raw, raw_ld, rot_at, gain, eps, rope, st);
+    if (pool.elem_bytes == 2) NVLLM_LAUNCH((k_latent_kv<true>), dim3(cdiv(st.T, 4)), dim3(256), 0, r);
+    else NVLLM_LAUNCH((k_latent_kv<false>), dim3(cdiv(st.T, 4)), dim3(256), 0, r);
 }
 
 // ------------------------------------------------------------------ attention, any size
@@ -216,6 +159,7 @@ struct LatentKArgs {
     const int* tables;
     const int4* runs;     // (first token, count, last position, table offset)
     int n_sub;            // items of CT tokens per run
+    int run_ld;           // tokens of the longest run: partial results are indexed [run][token of the run]
     int CT, HG, NG;       // tokens and heads per item; head groups
     int H, nsplit;
     int chunks;           // row / 32
@@ -224,8 +168,8 @@ struct LatentKArgs {
     int page_shift;       // log2(pages per block)
     __half* out;
     int Kb_out;
-    float* part_acc;      // [token][head][slice][rank_ld]
-    float* part_ml;       // [token][head][slice][2], log2 domain
+    float* part_acc;      // [run][token of the run][head][slice][rank_ld]
+    float* part_ml;       // [run][token of the run][head][slice][2], log2 domain
 };
 
 constexpr int LATENT_BLOCK_PAGES = 4;
@@ -269,25 +213,29 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
     const int hg = (int)(idx % (unsigned)a.NG);
     idx /= (unsigned)a.NG;
     const int sub = (int)(idx % (unsigned)a.n_sub);
-    const int4 run = a.runs[idx / (unsigned)a.n_sub];
+    const int run_id = (int)(idx / (unsigned)a.n_sub);
+    const int4 run = a.runs[run_id];
     const int first = sub * a.CT;
     if (first >= run.y) return;
     const int ntok = min(a.CT, run.y - first), t0 = run.x + first;
     const int plast = run.z - (run.y - first - ntok);
     const int h0 = hg * a.HG;
     const const_int_p table = (const_int_p)(uintptr_t)(a.tables + __builtin_amdgcn_readfirstlane(run.w));
-    const int npages = __builtin_amdgcn_readfirstlane((plast >> 4) + 1), nblocks = (npages + LATENT_BLOCK_PAGES - 1) / LATENT_BLOCK_PAGES;
-    const int per = (nblocks + a.nsplit - 1) / a.nsplit;
-    const int b0 = split * per, b1 = min(nblocks, b0 + per);
+    // this slice's pages [p0, p1), in blocks of four
+    const int npages = __builtin_amdgcn_readfirstlane((plast >> 4) + 1);
+    const int per = (npages + a.nsplit - 1) / a.nsplit;
+    const int p0 = split * per, p1 = min(npages, p0 + per);
+    const int nblocks = p0 < p1 ? (p1 - p0 + LATENT_BLOCK_PAGES - 1) / LATENT_BLOCK_PAGES : 0;
     const int row = nc * 32;
 
     // this lane's columns: (token of the item, head); -1 where the item has none.  (Formed again where needed: the page loop
     // keeps only the last position each column sees.)
     auto column = [&](int c, int& tok, int& h) {
-        const int j = 16 * (part * C + c) + (int)(threadIdx.x & 15);
-        tok = j / a.HG;
-        h = h0 + j - tok * a.HG;
-        const bool valid = tok < ntok && h < a.H;
+        // (tokens fastest: the 16 columns of a group are neighbouring rows of the output tiles)
+        const int j = 16 * (part * C + c) + (int)(threadIdx.x & 15), hl = j / a.CT;
+        tok = j - hl * a.CT;
+        h = h0 + hl;
+        const bool valid = tok < ntok && hl < a.HG && h < a.H;
         tok = valid ? tok : 0;
         h = valid ? h : -1;
     };
@@ -296,16 +244,19 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
     for (int c = 0; c < C; c++) {
         int tok, h;
         column(c, tok, h);
-        plim[c] = h >= 0 ? plast - (ntok - 1 - tok) : -1;
+        plim[c] = h >= 0 ? min(plast - (ntok - 1 - tok), p1 * LATENT_PAGE - 1) : -1;
     }
 
-    // the page id of a block's page `page` (past the end: the last page again, its keys are masked)
+    // the page id of a block's page `page`; past the slice's end its keys are masked, and the copy is the slice's last page
+    // again, or nothing once the buffer holds an earlier block's (finite) rows
     auto page_of = [&](int b) {
-        const int pg = min(b * LATENT_BLOCK_PAGES + page, npages - 1);
+        const int pg = min(p0 + b * LATENT_BLOCK_PAGES + page, npages - 1);
         return (table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1));
     };
     const unsigned lds0 = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(page * nc + part) * 1024u;
-    auto issue = [&](int page_id, int buf) {   // tiles part, part + WC, ... of the page
+    auto issue = [&](int page_id, int b) {   // tiles part, part + WC, ... of the page
+        if (b >= 2 && p0 + b * LATENT_BLOCK_PAGES + page >= p1) return;
+        const int buf = b & 1;
         const __half* src = a.base + (size_t)page_id * (LATENT_PAGE * row) + (size_t)part * TILE_HALVES + lane * 8;
         const unsigned dst = lds0 + (unsigned)(buf * LATENT_BLOCK_PAGES * nc) * 1024u;
 #pragma unroll
@@ -323,9 +274,8 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int n = 0; n < NT; n++) acc[n][c] = f4_t{0.f, 0.f, 0.f, 0.f};
     }
-    int next_page = page_of(min(b0, nblocks - 1));
-    if (b0 < b1) issue(next_page, 0);
-    next_page = page_of(min(b0 + 1, nblocks - 1));
+    if (nblocks > 0) issue(page_of(0), 0);
+    int next_page = page_of(1);
     // queries as the B operand: column x, dims 32k + 8g .. +7 (columns nobody owns read a real row; their scores are masked)
     b8_t qf[C][RC];
 #pragma unroll
@@ -346,19 +296,24 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
     // transpose read: 16 lanes bring 4 keys x 16 dims, lane i gets dim i of the 4 keys
     const int tr_key = 4 * g + (x >> 2), tr_sub = (x & 3) >> 1, tr_off = 4 * (x & 1);
 
-    for (int b = b0; b < b1; b++) {
-        const int buf = (b - b0) & 1;
+    // (no peeled iterations: their copies of the loop body would hold registers this one needs)
+#pragma clang loop unroll(disable)
+    for (int b = 0; b < nblocks; b++) {
+        const int buf = b & 1;
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // this wave's tiles of block b are in LDS
         latent_barrier();                                   // ... and everybody's; block b - 1 has been consumed
-        if (b + 1 < b1) {
-            issue(next_page, buf ^ 1);
-            next_page = page_of(min(b + 2, nblocks - 1));
+        if (b + 1 < nblocks) {
+            issue(next_page, b + 1);
+            next_page = page_of(b + 2);
         }
         const __half* blk = pages + (size_t)buf * LATENT_BLOCK_PAGES * nc * TILE_HALVES;
         // ---- scores of this wave's page; key fragments a few chunks ahead of the multiplies
-        f4_t s[C];
+        constexpr int CH = C == 1 ? 2 : 1;   // independent accumulator chains per column group
+        f4_t s[C], s2[CH][C];
 #pragma unroll
-        for (int c = 0; c < C; c++) s[c] = f4_t{0.f, 0.f, 0.f, 0.f};
+        for (int c = 0; c < C; c++)
+#pragma unroll
+            for (int h = 0; h < CH; h++) s2[h][c] = f4_t{0.f, 0.f, 0.f, 0.f};
         const b8_t* kp = reinterpret_cast<const b8_t*>(blk + (size_t)page * nc * TILE_HALVES) + lane;
         constexpr int KA = C == 2 ? 3 : RC < 6 ? RC : 6;
         b8_t kf[KA];
@@ -369,12 +324,14 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
         for (int k = 0; k < RC; k++) {
             if (EXACT || k < nc) {
 #pragma unroll
-                for (int c = 0; c < C; c++) s[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k % KA], qf[c][k], s[c], 0, 0, 0);
+                for (int c = 0; c < C; c++) s2[k % CH][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k % KA], qf[c][k], s2[k % CH][c], 0, 0, 0);
                 if (k + KA < RC && (EXACT || k + KA < nc)) kf[k % KA] = kp[(k + KA) * 64];
             }
             __builtin_amdgcn_sched_barrier(0);
         }
-        const int kfirst = (b * LATENT_BLOCK_PAGES + page) * LATENT_PAGE + 4 * g;
+#pragma unroll
+        for (int c = 0; c < C; c++) s[c] = CH == 2 ? s2[0][c] + s2[CH - 1][c] : s2[0][c];
+        const int kfirst = (p0 + b * LATENT_BLOCK_PAGES + page) * LATENT_PAGE + 4 * g;
 #pragma unroll
         for (int c = 0; c < C; c++) {
             float mx = -INFINITY;
@@ -466,7 +423,7 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
         column(c, tok, h);
         if (h < 0) continue;
         float f = 1.f;
-        const size_t th = (size_t)(t0 + tok) * a.H + h;
+        const size_t th = ((size_t)run_id * a.run_ld + first + tok) * a.H + h;   // place among the partial results
         if (a.nsplit == 1) {
             const float sk = a.sink[h] * 1.44269504088896340736f, top = fmaxf(m[c], sk);
             const float w = __builtin_amdgcn_exp2f(m[c] - top);
@@ -492,9 +449,13 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 
 // slices of one (token, head) -> the attended latent, the sink in the denominator
 __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
-                                                        const float* __restrict__ sink, int H, int nsplit, int rank_ld, __half* out, int Kb_out) {
-    const int t = blockIdx.x / H, h = blockIdx.x % H;
+                                                        const float* __restrict__ sink, const int4* __restrict__ runs, int run_ld, int H, int nsplit,
+                                                        int rank_ld, __half* out, int Kb_out) {
     const size_t th = blockIdx.x;
+    const int h = blockIdx.x % H, slot = blockIdx.x / H;
+    const int4 run = runs[slot / run_ld];
+    if (slot % run_ld >= run.y) return;
+    const int t = run.x + slot % run_ld;
     const float* ml = part_ml + th * nsplit * 2;
     const float sk = sink[h] * 1.44269504088896340736f;
     float top = sk;
@@ -515,7 +476,7 @@ __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict_
     }
 }
 
-template <int RC, int NT, int C, int WC>
+template <int RC, int NT, int C, int WC, bool EXACT_ONLY = false>
 static void launch_latent_c(const LatentKArgs& k, long units) {
     const size_t lds = latent_attn_lds(k.chunks, C * WC);
     const bool exact = k.chunks == RC && k.n_tiles == 4 * NT;
@@ -524,26 +485,27 @@ static void launch_latent_c(const LatentKArgs& k, long units) {
         const int most = (int)latent_attn_lds(RC, C * WC);
         if (most > 64 * 1024) {
             HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, WC, true>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
-            HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, WC, false>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
+            if constexpr (!EXACT_ONLY)
+                HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RC, NT, C, WC, false>), hipFuncAttributeMaxDynamicSharedMemorySize, most));
         }
         ready = true;
     }
     if (exact) NVLLM_LAUNCH((k_latent_attn<RC, NT, C, WC, true>), dim3((unsigned)units), dim3(256 * WC), lds, k);
-    else NVLLM_LAUNCH((k_latent_attn<RC, NT, C, WC, false>), dim3((unsigned)units), dim3(256 * WC), lds, k);
+    else if constexpr (!EXACT_ONLY) NVLLM_LAUNCH((k_latent_attn<RC, NT, C, WC, false>), dim3((unsigned)units), dim3(256 * WC), lds, k);
 }
 template <int RC, int NT>
 static void launch_latent_rc(const LatentKArgs& k, long units, int columns) {
     if (columns == 16) launch_latent_c<RC, NT, 1, 1>(k, units);
     else if (columns == 32) launch_latent_c<RC, NT, 1, 2>(k, units);
-    else launch_latent_c<RC, NT, 2, 2>(k, units);
+    else launch_latent_c<RC, NT, 2, 2, (RC > 10)>(k, units);
 }
 
 void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     if (st.T <= 0) return;
     const LatentPool& P = a.pool;
     const int row = P.row(), chunks = row / 32, vt = cdiv(P.rank_ld, 64);   // value tiles per wave
-    // algorithmic work: every run's rows read once; per (token, key, head) the two products
-    const double bytes = (double)st.kv_positions * row * P.elem_bytes + (double)st.T * a.H * (row + P.rank_ld) * P.elem_bytes;
+    // algorithmic work: every sequence's rows read once; per (token, key, head) the two products
+    const double bytes = (double)st.kv_rows * row * P.elem_bytes + (double)st.T * a.H * (row + P.rank_ld) * P.elem_bytes;
     const double flops = 2.0 * (double)st.qk_pairs * a.H * (row + P.rank_ld);
     const bool tiled = P.elem_bytes == 2 && ((chunks <= 4 && vt <= 1) || (chunks <= 6 && vt <= 2) || (chunks <= 10 && vt <= 4) || (chunks <= 18 && vt <= 8));
     int pages_per_block = P.block_size / LATENT_PAGE, page_shift = 0;
@@ -561,19 +523,12 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
                          P.block_size, a.H, P.rank, P.rank_ld, row, a.out_f32, a.out_b16, 0);
         return;
     }
-    // columns per item: 64, or 32 or 16 when no item would fill more
-    const int W = a.H * st.max_run <= 16 ? 16 : a.H * st.max_run <= 32 ? 32 : 64;
     LatentKArgs k{};
     k.base = (const __half*)P.base;
     k.q = (const __half*)a.q;
     k.sink = a.sink;
     k.scale = a.scale;
     k.tables = st.d_tables;
-    k.runs = (const int4*)st.d_runs;
-    k.HG = a.H < W ? a.H : W;
-    k.NG = cdiv(a.H, k.HG);
-    k.CT = W / k.HG;
-    k.n_sub = cdiv(st.max_run < LATENT_RUN ? st.max_run : LATENT_RUN, k.CT);
     k.H = a.H;
     k.chunks = chunks;
     k.n_tiles = P.rank_ld / 16;
@@ -581,33 +536,56 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     k.page_shift = page_shift;
     k.out = a.out_b16;
     k.Kb_out = a.H * P.rank_ld / 32;
-    // slices of pages until the chip is full: as many workgroups as fit by LDS (at most two per CU), two blocks per slice at least
-    const long items = (long)st.n_runs * k.n_sub * k.NG;
-    const int per_cu = latent_attn_lds(chunks, W / 16) * 2 <= 160 * 1024 ? 2 : 1;
-    const int nblocks = cdiv(st.max_pos / LATENT_PAGE + 1, LATENT_BLOCK_PAGES);
-    int nsplit = (int)(((long)per_cu * rt().num_cus + items / 2) / items);
-    if (nsplit > cdiv(nblocks, 2)) nsplit = cdiv(nblocks, 2);
-    if (nsplit > 64) nsplit = 64;
-    if (nsplit < 1) nsplit = 1;
-    k.nsplit = nsplit;
-    if (nsplit > 1) {
-        const size_t rows = (size_t)st.T * a.H * nsplit;
-        float* part = (float*)ws_get(WS_ATT_PART, rows * (P.rank_ld + 2) * sizeof(float));
-        k.part_acc = part;
-        k.part_ml = part + rows * P.rank_ld;
-    }
-    {
-        ProfScope ps(PC_LATENT_ATTN, bytes, flops);
-        const long units = items * nsplit;
-        if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, W);
-        else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, W);
-        else if (chunks <= 10 && vt <= 4) launch_latent_rc<10, 4>(k, units, W);
-        else launch_latent_rc<18, 8>(k, units, W);
-    }
-    if (nsplit > 1) {
-        ProfScope ps(PC_LATENT_COMBINE, (double)st.T * a.H * ((double)nsplit * (P.rank_ld + 2) * 4.0 + P.rank_ld * 2.0), 0);
-        NVLLM_LAUNCH(k_latent_combine, dim3((unsigned)st.T * a.H), dim3(128), 0, k.part_acc, k.part_ml, a.sink, a.H, nsplit, P.rank_ld, a.out_b16, k.Kb_out);
-    }
+    // prompt portions and single tokens want differently shaped items: a launch each when the batch has both
+    const int n_single = st.n_runs - st.n_multi;
+    const double share = st.kv_rows > 0 ? (double)st.kv_rows_single / (double)st.kv_rows : 0.0;
+    auto launch = [&](const int* runs, int n_runs, int max_run, double bytes, double flops) {
+        if (n_runs <= 0) return;
+        // columns per item: 64, or 32 or 16 when no item would fill more
+        // (64 columns of the widest class fit the register file only when the row is exactly that class's)
+        const bool wide = chunks > 10 || vt > 4, exact = chunks == 18 && vt * 64 == P.rank_ld;
+        const int W = a.H * max_run <= 16 ? 16 : a.H * max_run <= 32 || (wide && !exact) ? 32 : 64;
+        // up to 16 tokens per item (so that a column group is one head's neighbouring tokens), more only when there are few heads
+        int ct = 1;
+        while (ct < 16 && ct < max_run) ct *= 2;
+        k.runs = (const int4*)runs;
+        k.run_ld = max_run;
+        k.HG = a.H < W / ct ? a.H : W / ct;
+        k.NG = cdiv(a.H, k.HG);
+        k.CT = W / k.HG;
+        k.n_sub = cdiv(max_run, k.CT);
+        // slices of pages until the chip is full: as many workgroups as fit by LDS (at most two per CU), eight pages per slice at least
+        const long items = (long)n_runs * k.n_sub * k.NG;
+        const int per_cu = latent_attn_lds(chunks, W / 16) * 2 <= 160 * 1024 ? 2 : 1;
+        const int npages = st.max_pos / LATENT_PAGE + 1;
+        int nsplit = (int)(((long)per_cu * rt().num_cus + items / 2) / items);
+        if (nsplit > cdiv(npages, 8)) nsplit = cdiv(npages, 8);
+        if (nsplit > 64) nsplit = 64;
+        if (nsplit < 1) nsplit = 1;
+        k.nsplit = nsplit;
+        const size_t rows = (size_t)n_runs * max_run * a.H * nsplit;
+        if (nsplit > 1) {
+            float* part = (float*)ws_get(WS_ATT_PART, rows * (P.rank_ld + 2) * sizeof(float));
+            k.part_acc = part;
+            k.part_ml = part + rows * P.rank_ld;
+        }
+        {
+            ProfScope ps(PC_LATENT_ATTN, bytes, flops);
+            const long units = items * nsplit;
+            if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, W);
+            else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, W);
+            else if (chunks <= 10 && vt <= 4) launch_latent_rc<10, 4>(k, units, W);
+            else launch_latent_rc<18, 8>(k, units, W);
+        }
+        if (nsplit > 1) {
+            ProfScope ps(PC_LATENT_COMBINE, (double)rows * (P.rank_ld + 2) * 4.0, 0);
+            NVLLM_LAUNCH(k_latent_combine, dim3((unsigned)n_runs * max_run * a.H), dim3(128), 0, k.part_acc, k.part_ml, a.sink, k.runs, max_run, a.H, nsplit,
+                         P.rank_ld, a.out_b16, k.Kb_out);
+        }
+    };
+    const double single_flops = 2.0 * (double)st.kv_rows_single * a.H * (row + P.rank_ld);
+    launch(st.d_runs, st.n_multi, st.max_run, bytes * (1.0 - share), flops - single_flops);
+    launch(st.d_runs + 4 * st.n_multi, n_single, 1, bytes * share, single_flops);
 }
 
 // ------------------------------------------------------------------ fp32 head products

@@ -5,12 +5,12 @@
 // embeddings and soft-capped logits.
 //
 // Two forms of the forward pass:
-//   bf16  eight launches per layer run.  The Dynamic Tanh norm needs no statistics, so the residual projections'
+//   bf16  eight launches per layer run (nine when attention is cut into slices).  The Dynamic Tanh norm needs no statistics, so the residual projections'
 //         epilogues do the whole step between two sublayers: bias, layer scale, stream mixing, the next
 //         sublayer's input and its norm, stored as activation tiles.
 //           latent_in   [W_dq ; W_dkv]       query latent (x gain) -> tiles + sums of squares; rest -> fp32 rows
-//           latent_q    W_uq (rows reordered: unrotated parts of all heads, then rotated parts)  1/rms, rotation
-//           latent_kv   norm + rotation of the new cache rows
+//           latent_q    W_uq (rows reordered: unrotated parts of all heads, then rotated parts)  1/rms, rotation;
+//                       extra workgroups norm, rotate and write the new cache rows
 //           absorb      W_uk^T head by head  -> query rows over the latent
 //           attention   (+ merge of slices)
 //           value       W_uv head by head
@@ -20,6 +20,7 @@
 #include <algorithm>
 #include <memory>
 
+#include "gemm_common.h"
 #include "latent_attention.h"
 #include "model_dir.h"
 
@@ -187,7 +188,7 @@ void LatentHyperModel::load_layer(const ModelDir& dir, int i, const Json& cfg) {
     }
     const int Qp = pad32(m.q_rank), Cp = pad32(m.rank), Rp = pad32(m.rot), dimp = pad32(m.dim), vp = pad32(m.vdim);
     w.gain_q = vec(dir, M + "dq.norm", m.q_rank, Qp);
-    w.gain_kv = vec(dir, M + "dkv.norm", m.rank, m.rank);
+    w.gain_kv = vec(dir, M + "dkv.norm", m.rank, Cp);
     std::vector<uint16_t> src, dst;
     auto read = [&](const std::string& name, int rows, int cols) {
         src.resize((size_t)rows * cols);
@@ -366,7 +367,7 @@ void LatentHyperModel::init_kv(KVCacheManager* mgr, int block_size, int num_bloc
 }
 
 void LatentHyperModel::forward(const PassArgs& a) {
-    const StepArrays st = stage_step(a.tokens, a.pos, a.seq_ids, a.T, a.output_indices, a.B, a.tables, nullptr, 0, a.mgr->block_size, LATENT_RUN, a.token_src);
+    const StepArrays st = stage_step(a.tokens, a.pos, a.seq_ids, a.T, a.output_indices, a.B, a.tables, nullptr, 0, a.mgr->block_size, LATENT_RUN, a.token_src, true);
     if (st.table_short) NVLLM_FATAL("transformer_batch: a position lies beyond its sequence's block table (allocate the block first)");
     if (f32_) forward_f32(a, st);
     else forward_b16(a, st);
@@ -444,13 +445,13 @@ void LatentHyperModel::forward_b16(const PassArgs& a, const StepArrays& st) {
         e1.out = raw; e1.ldo = Cp + Rp;
         launch_gemm_b16(w.in, act, T, e1, PC_GEMM_LATENT_IN);
         const LatentPool pl = pool(a.mgr, s.run);
-        launch_latent_kv(pl, raw, Cp + Rp, Cp, w.gain_kv, eps_, rope, st);
+        const LatentKvRider ride = latent_kv_rider(pl, raw, Cp + Rp, Cp, w.gain_kv, eps_, rope, st);
         GemmEpilogue e2;
         e2.kind = GemmEpilogue::LATENT_Q;
         e2.ss_in = ss; e2.ss_tiles = Qp / 32; e2.d_in = m.q_rank; e2.eps = eps_;
         e2.q_plain = m.heads * dimp; e2.rot_ld = Rp; e2.rot_dim = m.rot; e2.rope = rope; e2.pos = st.d_pos;
         e2.a16_out = hid; e2.q_rows = q; e2.q_heads = m.heads; e2.q_row = Cp + Rp; e2.head_ld = Cp;
-        launch_gemm_b16(w.uq, qt, T, e2, PC_GEMM_LATENT_Q);
+        launch_gemm_b16(w.uq, qt, T, e2, PC_GEMM_LATENT_Q, &ride);
         GemmEpilogue e3;
         e3.kind = GemmEpilogue::ROWS_B16;
         e3.q_rows = q; e3.q_heads = m.heads; e3.q_row = Cp + Rp; e3.head_ld = Cp;

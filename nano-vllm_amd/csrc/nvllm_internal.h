@@ -349,7 +349,8 @@ struct B16Weight {
     int groups = 1;
 };
 static inline size_t b16_halves(int tokens, int K) { return (size_t)cdiv(tokens, 16) * cdiv(K, 32) * TILE_HALVES; }
-void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls);
+struct LatentKvRider;   // gemm_common.h: cache rows written by extra workgroups of a LATENT_Q launch
+void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls, const LatentKvRider* ride = nullptr);
 
 void launch_pack_a16(__half* a16, const float* in, int T, int K);
 void launch_matmul_f32w(float* out, const float* in, const float* w, int T, int K, int N);

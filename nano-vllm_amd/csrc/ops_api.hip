@@ -1,6 +1,7 @@
 // ops_api.hip -- the operator entry points of include/ops.h on top of the kernel
 // launchers: argument checking, host->HBM staging of the integer arrays and block
 // tables, and the host-side KV block allocator.
+#include <algorithm>
 #include <cstring>
 #include <unordered_map>
 #include <vector>
@@ -39,7 +40,7 @@ KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim) {
 // pinned region and upload it with a single copy.
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
-                      int pos0, int block_size, int attn_ct, const int* token_src) {
+                      int pos0, int block_size, int attn_ct, const int* token_src, bool multi_first) {
     StepArrays s{};
     s.T = T;
     s.B = B;
@@ -98,6 +99,30 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
                 if (tb < 4) s.runs_in_tb[tb]++;
             t += n;
         }
+        if (multi_first) {
+            std::vector<int> singles;
+            size_t keep = 0;
+            for (size_t i = 0; i < runs.size(); i += 4) {
+                if (runs[i + 1] == 1) {
+                    singles.insert(singles.end(), runs.begin() + (long)i, runs.begin() + (long)i + 4);
+                    s.kv_rows_single += runs[i + 2] + 1;
+                } else {
+                    std::copy(runs.begin() + (long)i, runs.begin() + (long)i + 4, runs.begin() + (long)keep);
+                    keep += 4;
+                }
+            }
+            std::copy(singles.begin(), singles.end(), runs.begin() + (long)keep);
+            s.n_multi = (int)(keep / 4);
+        }
+    }
+    if (attn_ct > 0) {
+        std::vector<int> seen_to(n_seqs, 0);
+        for (int t = 0; t < T; t++) {
+            int& last = seen_to[seq_ids ? seq_ids[t] : 0];
+            const int p = (pos_arr ? pos_arr[t] : pos0 + t) + 1;
+            if (p > last) last = p;
+        }
+        for (int v : seen_to) s.kv_rows += v;
     }
     {   // does any sequence occur twice?
         std::vector<char> seen(n_seqs, 0);
@@ -473,7 +498,8 @@ void nvllm_latent_attention(float* out, const float* q, KVCacheManager* mgr, Blo
                             const float* sink, float scale, int n_heads, int rank, int rot, int elem_bytes, int num_tokens) {
     ensure_init();
     if (num_tokens <= 0) return;
-    StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size, LATENT_RUN);
+    StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size, LATENT_RUN,
+                              nullptr, true);
     if (s.table_short) NVLLM_FATAL("latent attention: a position lies beyond its sequence's block table");
     LatentAttn a{};
     a.pool = latent_pool(mgr->pool_k, elem_bytes, mgr->block_size, rank, rot);

@@ -21,8 +21,11 @@ struct StepArrays {
     int* d_runs;      // [n_runs][4] (first token, count, last position, table offset): attention work items
     int n_runs;
     long kv_positions;
+    long kv_rows;            // sum over the batch's sequences of the positions their last token sees
     long qk_pairs;           // sum over tokens of the positions they see
     int max_run;             // tokens of the longest run
+    int n_multi;             // with `multi_first`: the first n_multi runs have several tokens, the others one each
+    long kv_rows_single;     // ... positions those others see
     int runs_in_tb[4];       // runs that touch each of the first four 16-token blocks
     bool one_token_per_seq;  // no sequence contributes more than one token (a pure decode step)
 };
@@ -32,10 +35,10 @@ struct StepArrays {
 // `tables` (indexed by seq id) or `single` (one table, positions pos0 + t) may be
 // null for operators that do not touch the pool.  attn_ct > 0 also cuts the batch into
 // attention work items: runs of at most attn_ct tokens of one sequence at
-// consecutive positions.
+// consecutive positions.  multi_first: runs of several tokens come before those of one.
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
-                      int pos0, int block_size, int attn_ct = 0, const int* token_src = nullptr);
+                      int pos0, int block_size, int attn_ct = 0, const int* token_src = nullptr, bool multi_first = false);
 
 KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim);
 
