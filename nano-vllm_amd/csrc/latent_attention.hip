@@ -274,7 +274,7 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int n = 0; n < NT; n++) acc[n][c] = f4_t{0.f, 0.f, 0.f, 0.f};
     }
-    if (nblocks > 0) issue(page_of(0), 0);
+    const int first_page = page_of(0);
     int next_page = page_of(1);
     // queries as the B operand: column x, dims 32k + 8g .. +7 (columns nobody owns read a real row; their scores are masked)
     b8_t qf[C][RC];
@@ -286,6 +286,7 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int k = 0; k < RC; k++) qf[c][k] = *reinterpret_cast<const b8_t*>(qr + 32 * (EXACT ? k : min(k, nc - 1)));
     }
+    if (nblocks > 0) issue(first_page, 0);
     // the queries have arrived before the loop: inside it the compiler then has no load of its own to wait for, and
     // the only waits on memory are the ones below
 #pragma unroll
@@ -554,11 +555,10 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
         k.NG = cdiv(a.H, k.HG);
         k.CT = W / k.HG;
         k.n_sub = cdiv(max_run, k.CT);
-        // slices of pages until the chip is full: as many workgroups as fit by LDS (at most two per CU), eight pages per slice at least
+        // slices of pages until every CU has a workgroup, eight pages per slice at least
         const long items = (long)n_runs * k.n_sub * k.NG;
-        const int per_cu = latent_attn_lds(chunks, W / 16) * 2 <= 160 * 1024 ? 2 : 1;
         const int npages = st.max_pos / LATENT_PAGE + 1;
-        int nsplit = (int)(((long)per_cu * rt().num_cus + items / 2) / items);
+        int nsplit = (int)((rt().num_cus + items / 2) / items);
         if (nsplit > cdiv(npages, 8)) nsplit = cdiv(npages, 8);
         if (nsplit > 64) nsplit = 64;
         if (nsplit < 1) nsplit = 1;

@@ -102,6 +102,7 @@ private:
     // row-major bf16 [N][K] on the host -> tiles in HBM
     B16Weight tile(const std::vector<uint16_t>& rm, int N, int K, int groups = 1);
     LatentPool pool(const KVCacheManager* mgr, int run) const;
+    size_t pool_bytes(int block_size, int num_blocks, int runs) const;   // of the first `runs` cache slices
     void load_layer(const ModelDir& dir, int i, const Json& cfg);
     void forward_b16(const PassArgs& a, const StepArrays& st);
     void forward_f32(const PassArgs& a, const StepArrays& st);
@@ -350,23 +351,29 @@ LatentHyperModel::LatentHyperModel(const ModelDir& dir, Config* p) {
     p->rope_theta = (float)m0.base;
 }
 
-LatentPool LatentHyperModel::pool(const KVCacheManager* mgr, int run) const {
-    size_t off = 0;
-    for (int r = 0; r < run; r++) {
+size_t LatentHyperModel::pool_bytes(int block_size, int num_blocks, int runs) const {
+    size_t bytes = 0;
+    for (int r = 0; r < runs; r++) {
         const Mixer& m = layers_[runs_[r]].m;
-        off += latent_pool_bytes(latent_pool(nullptr, f32_ ? 4 : 2, mgr->block_size, m.rank, m.rot), mgr->num_blocks);
+        bytes += latent_pool_bytes(latent_pool(nullptr, f32_ ? 4 : 2, block_size, m.rank, m.rot), num_blocks);
     }
+    return bytes;
+}
+
+LatentPool LatentHyperModel::pool(const KVCacheManager* mgr, int run) const {
     const Mixer& m = layers_[runs_[run]].m;
-    return latent_pool((char*)mgr->pool_k + off, f32_ ? 4 : 2, mgr->block_size, m.rank, m.rot);
+    return latent_pool((char*)mgr->pool_k + pool_bytes(mgr->block_size, mgr->num_blocks, run), f32_ ? 4 : 2, mgr->block_size, m.rank, m.rot);
 }
 
 void LatentHyperModel::init_kv(KVCacheManager* mgr, int block_size, int num_blocks) {
-    size_t bytes = 0;
-    for (int l : runs_) bytes += latent_pool_bytes(latent_pool(nullptr, f32_ ? 4 : 2, block_size, layers_[l].m.rank, layers_[l].m.rot), num_blocks);
-    init_block_pool(mgr, block_size, num_blocks, bytes);
+    init_block_pool(mgr, block_size, num_blocks, pool_bytes(block_size, num_blocks, (int)runs_.size()));
 }
 
 void LatentHyperModel::forward(const PassArgs& a) {
+    if (block_pool_bytes(a.mgr) != pool_bytes(a.mgr->block_size, a.mgr->num_blocks, (int)runs_.size()))
+        NVLLM_FATAL("transformer_batch: the block pool was not made for this model (nvllm_init_model_kv)");
+    for (int t = 0; t < a.T; t++)
+        if (a.pos[t] < 0 || a.tokens[t] < 0 || a.tokens[t] >= V_) NVLLM_FATAL("transformer_batch: token %d (id %d, position %d) is out of range", t, a.tokens[t], a.pos[t]);
     const StepArrays st = stage_step(a.tokens, a.pos, a.seq_ids, a.T, a.output_indices, a.B, a.tables, nullptr, 0, a.mgr->block_size, LATENT_RUN, a.token_src, true);
     if (st.table_short) NVLLM_FATAL("transformer_batch: a position lies beyond its sequence's block table (allocate the block first)");
     if (f32_) forward_f32(a, st);

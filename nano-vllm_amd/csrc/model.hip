@@ -144,6 +144,12 @@ static DirModelLoader find_architecture(const char* name) {
     return nullptr;
 }
 
+static const ModelPriv* g_dir_model = nullptr;   // the folder model loaded last
+DirModel* current_dir_model(int n_layers, int n_kv_heads, int head_dim) {
+    const ModelPriv* m = g_dir_model;
+    return m && m->cfg.n_layers == n_layers && m->cfg.n_kv_heads == n_kv_heads && m->cfg.head_dim == head_dim ? m->dir.get() : nullptr;
+}
+
 static void load_model_dir(Weights* w, Config* p, const char* path) {
     if (tp().active) {
         fprintf(stderr, "model folders are not split over tensor-parallel ranks\n");
@@ -163,6 +169,7 @@ static void load_model_dir(Weights* w, Config* p, const char* path) {
     std::unique_ptr<ModelPriv> m(new ModelPriv());
     m->dir.reset(load(dir, p));
     m->cfg = *p;
+    g_dir_model = m.get();
     w->_data_buffer = m.release();
     printf("Model loaded: %s, width %d, %d layer runs, vocabulary %d, %s\n", arch.c_str(), p->dim, p->n_layers, p->vocab_size,
            rt().compute_dtype == NVLLM_COMPUTE_F32 ? "fp32" : "bf16");
@@ -631,6 +638,7 @@ void nvllm_free_model(Weights* w) {
     if (m->arena) device_free(m->arena);
     if (m->chain_layers) device_free(m->chain_layers);
     for (void* q : m->f32_bufs) device_free(q);
+    if (g_dir_model == m) g_dir_model = nullptr;
     delete m;
     free(w->layers);
     memset(w, 0, sizeof *w);

@@ -75,6 +75,9 @@ DirModel* load_latent_hyper_model(const ModelDir& dir, Config* p);   // latent_m
 
 // ops_api.hip: host bookkeeping of a block pool whose storage is ONE HBM buffer of `bytes` bytes (pool_v stays null)
 void init_block_pool(KVCacheManager* mgr, int block_size, int num_blocks, size_t bytes);
+size_t block_pool_bytes(const KVCacheManager* mgr);   // of such a pool; 0 for any other
+// model.hip: the folder model loaded last, if its Config says these numbers
+DirModel* current_dir_model(int n_layers, int n_kv_heads, int head_dim);
 
 // model.hip: the previous pass's result rows have left the workspaces the classifier writes
 void wait_for_row_copies();

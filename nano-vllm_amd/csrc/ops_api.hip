@@ -19,6 +19,16 @@ struct PoolInfo {
     int elem_bytes;
     int n_layers, n_kv_heads, head_dim;
 };
+// Block pools of models that lay them out themselves: bytes behind pool_k.
+static std::unordered_map<const void*, size_t>& block_pools() {
+    static std::unordered_map<const void*, size_t> m;
+    return m;
+}
+size_t block_pool_bytes(const KVCacheManager* mgr) {
+    auto it = block_pools().find(mgr->pool_k);
+    return it == block_pools().end() ? 0 : it->second;
+}
+
 static std::unordered_map<const void*, PoolInfo>& pools() {
     static std::unordered_map<const void*, PoolInfo> m;
     return m;
@@ -267,6 +277,11 @@ static void init_free_stack(KVCacheManager* mgr, int block_size, int num_blocks)
 void init_kv_cache_manager(KVCacheManager* mgr, int block_size, int num_blocks, int n_layers,
                            int n_kv_heads, int head_dim) {
     ensure_init();
+    // a driver that knows only this entry point, with a folder model loaded: the pool is that model's own
+    if (DirModel* m = current_dir_model(n_layers, n_kv_heads, head_dim)) {
+        m->init_kv(mgr, block_size, num_blocks);
+        return;
+    }
     // tensor parallelism: the caller passes the model's head count (it sizes the pool from Config);
     // this process stores and reads the K/V of its own heads only
     if (tp().active && tp().world > 1) {
@@ -299,6 +314,7 @@ void nvllm::init_block_pool(KVCacheManager* mgr, int block_size, int num_blocks,
     HIP_CHECK(hipMemsetAsync(pool, 0, bytes, rt().stream));   // rows nobody has written are finite
     mgr->pool_k = (float*)pool;
     mgr->pool_v = nullptr;
+    block_pools()[pool] = bytes;
 }
 extern "C" {
 
@@ -307,6 +323,7 @@ void free_kv_cache_manager(KVCacheManager* mgr) {
     mgr->free_block_indices = nullptr;
     if (mgr->pool_k) {
         pools().erase(mgr->pool_k);
+        block_pools().erase(mgr->pool_k);
         device_free(mgr->pool_k);
     }
     if (mgr->pool_v) device_free(mgr->pool_v);
@@ -484,12 +501,18 @@ void nvllm_latent_pool_init(KVCacheManager* mgr, int block_size, int num_blocks,
     init_block_pool(mgr, block_size, num_blocks, latent_pool_bytes(latent_pool(nullptr, elem_bytes, block_size, rank, rot), num_blocks));
 }
 
+static void check_latent_pool(const KVCacheManager* mgr, int rank, int rot, int elem_bytes) {
+    if (block_pool_bytes(mgr) != latent_pool_bytes(latent_pool(nullptr, elem_bytes, mgr->block_size, rank, rot), mgr->num_blocks))
+        NVLLM_FATAL("this block pool does not hold rows of %d + %d values of %d bytes", rank, rot, elem_bytes);
+}
+
 void nvllm_latent_cache_write(KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr, const float* kv, const float* gain,
                               float eps, double base, int rank, int rot, int elem_bytes, int num_tokens) {
     ensure_init();
     if (num_tokens <= 0) return;
     StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size);
     if (s.table_short) NVLLM_FATAL("latent cache write: a position lies beyond its sequence's block table");
+    check_latent_pool(mgr, rank, rot, elem_bytes);
     launch_latent_kv(latent_pool(mgr->pool_k, elem_bytes, mgr->block_size, rank, rot), kv, rank + rot, rank, gain, eps,
                      rotation_table(base, rot, s.max_pos + 1), s);
 }
@@ -501,6 +524,7 @@ void nvllm_latent_attention(float* out, const float* q, KVCacheManager* mgr, Blo
     StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, block_tables, nullptr, 0, mgr->block_size, LATENT_RUN,
                               nullptr, true);
     if (s.table_short) NVLLM_FATAL("latent attention: a position lies beyond its sequence's block table");
+    check_latent_pool(mgr, rank, rot, elem_bytes);
     LatentAttn a{};
     a.pool = latent_pool(mgr->pool_k, elem_bytes, mgr->block_size, rank, rot);
     a.sink = sink;

@@ -231,3 +231,42 @@ def test_replaying_a_trace(tmp_path, dtype):
     assert U.error(np.fromfile(out / "0.f32", "<f4").reshape(-1, V), za[[19, 3]]) < lim
     assert not (out / "1.f32").exists()
     assert U.error(np.fromfile(out / "2.f32", "<f4").reshape(-1, V), np.stack([za[29], zb[8]])) < lim
+
+
+def test_generating_from_the_command_line(tmp_path, tmp_models):
+    """The same command generates from a folder and from a model file."""
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    path, cfg, w = U.model(tmp_path, "mixed", seed=4)
+
+    def run(model, vocab, *more):
+        prompts = [U.tokens(n, vocab, n).tolist() for n in (3, 11)]
+        r = subprocess.run([os.path.join(root, "bin", "generate"), "--model", model, "-n", "6"] + [f"--prompt={','.join(map(str, p))}" for p in prompts] +
+                           list(more), capture_output=True, text=True, timeout=100)
+        assert r.returncode == 0, r.stderr[-2000:]
+        lines = [[[int(t) for t in part.split(",")] for part in line.split("|")] for line in r.stdout.strip().split("\n")]
+        assert [l[0] for l in lines] == prompts and all(len(l[1]) == 6 for l in lines)
+        return lines
+    for prompt, new in run(path, cfg["vocab"], "--dtype", "float32"):
+        want, margins = greedy(cfg, w, prompt, 6)
+        assert new == want[len(prompt):] or min(margins) < 1e-4
+    file_path, shape = tmp_models("tiny")
+    run(file_path, shape.vocab_size, "--chunk-size", "4")
+
+
+def test_a_pool_of_another_model_is_refused(hip, tmp_path):
+    """init_kv_cache_manager, all an older driver knows, makes the loaded folder model's pool; nothing else fits it."""
+    import ctypes as C
+    path, cfg, w = U.model(tmp_path, "mixed", seed=4)
+    hip.nvllm_set_compute_dtype(capi.COMPUTE_BF16)
+    weights, config = capi.Weights(), capi.Config()
+    hip.load_model(C.byref(weights), C.byref(config), path.encode())
+    sizes = []
+    for make in (lambda m: hip.init_kv_cache_manager(C.byref(m), 16, 8, config.n_layers, config.n_kv_heads, config.head_dim),
+                 lambda m: hip.nvllm_init_model_kv(C.byref(m), 16, 8, C.byref(config), C.byref(weights)),
+                 lambda m: hip.init_kv_cache_manager(C.byref(m), 16, 8, 1, 2, 16)):
+        mgr = capi.KVCacheManager()
+        make(mgr)
+        sizes.append((bool(mgr.pool_k), bool(mgr.pool_v), mgr.free_blocks_count))
+        hip.free_kv_cache_manager(C.byref(mgr))
+    assert sizes == [(True, False, 8), (True, False, 8), (True, True, 8)]
+    hip.nvllm_free_model(C.byref(weights))

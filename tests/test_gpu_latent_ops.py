@@ -201,7 +201,7 @@ def filled_pool(hip, rank, rot, elem, bs, lengths, seed):
 
 # rank, rot, heads, block size: every register class of the tiled kernel, exact and not, one and several head groups,
 # rows too wide for it, a block of three pages
-SHAPES = [(64, 32, 4, 16), (16, 2, 1, 16), (40, 12, 5, 32), (96, 64, 16, 16), (128, 64, 12, 64), (200, 48, 3, 16), (256, 64, 20, 16), (320, 64, 2, 16),
+SHAPES = [(64, 32, 6, 16), (16, 2, 1, 16), (40, 12, 5, 32), (96, 64, 16, 16), (128, 64, 12, 64), (200, 48, 3, 16), (256, 64, 20, 16), (320, 64, 2, 16),
           (512, 64, 32, 16), (512, 64, 33, 32), (576, 64, 2, 16), (64, 128, 3, 16), (48, 16, 7, 48)]
 
 
@@ -234,7 +234,7 @@ def test_latent_attention_of_a_ragged_batch(hip, rank, rot, heads, bs, elem):
 def test_one_far_key_and_nothing_beyond_the_token(hip, elem, decode):
     """One key stands out by far: wherever it lies -- first token, either side of a page's, a 64-key block's or a slice's
     border, the token itself -- it is found; one place beyond the token it is not seen at all."""
-    rank, rot, heads, n = 64, 32, 4, 900
+    rank, rot, heads, n = 64, 32, 6, 900
     pool, rows_of = filled_pool(hip, rank, rot, elem, 16, [n], 3)
     rows = rows_of[0]
     places = [0, 1, 15, 16, 17, 31, 32, 63, 64, 65, 127, 128, 255, 256, 257, 447, 448, 639, 640, 700]
@@ -275,7 +275,7 @@ def test_sink_takes_its_share(hip, elem):
 
 def test_slices_of_pages_and_one_slice_agree(hip):
     """A lone long sequence is cut into slices whose partial results are merged; many of them are not: same rows, same result."""
-    rank, rot, heads, n = 64, 32, 4, 1500
+    rank, rot, heads, n = 64, 32, 5, 1500
     pool, _ = filled_pool(hip, rank, rot, 2, 16, [n], 9)
     q = rounded(rng(2).standard_normal((1, heads, rank + rot)), 2)
     sink = np.zeros(heads)
