@@ -537,9 +537,9 @@ void launch_paged_attention(const AttnArgs& a) {
         k.part_ml = part + rows * a.hd;
     }
     {
-        // algorithmic bytes: each (sequence run, kv head) reads its keys and values once
-        const double kvb = (double)a.kv_positions * 2.0 * a.KVH * a.hd * a.pool.elem_bytes;
-        ProfScope ps(PC_ATTN, kvb + (double)a.T * a.H * a.hd * 8.0, 4.0 * (double)a.kv_positions * CT * a.H * a.hd);
+        // algorithmic work: keys and values of every sequence read once per kv head; two products per (token, position) pair
+        const double kvb = (double)(a.kv_rows ? a.kv_rows : a.kv_positions) * 2.0 * a.KVH * a.hd * a.pool.elem_bytes;
+        ProfScope ps(PC_ATTN, kvb + (double)a.T * a.H * a.hd * 8.0, 4.0 * (a.qk_pairs ? (double)a.qk_pairs : (double)a.kv_positions * CT) * a.H * a.hd);
         switch (a.hd) {
             case 16: launch_hd<16>(k, waves, a.pool.elem_bytes, solo, once, merge_waves); break;
             case 32: launch_hd<32>(k, waves, a.pool.elem_bytes, solo, once, merge_waves); break;

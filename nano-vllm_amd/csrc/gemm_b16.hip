@@ -111,6 +111,13 @@ void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
     const int groups = GRP ? a.NB / a.group_nb : 1;
     GemmPlan pl = gemm_plan(GRP ? a.group_nb * 16 * groups : a.N, a.Kb * 32, a.T, EPI, GRP || EPI == GemmEpilogue::F32 ? 1 : 0, 1 << 16, 0);
     if (GRP) {
+        // a short K and no split: when 64-feature tiles leave half the CUs idle, 32-feature tiles x 32 or 16 tokens
+        const int cus = rt().num_cus;
+        if (cdiv(a.group_nb, pl.nbw) * groups * pl.tiles_t * 2 <= cus) {
+            pl.nbw = 2;
+            if (pl.TB > 1) pl.TB = cdiv(a.group_nb, 2) * groups * a.Tb > cus ? 2 : 1;
+            pl.tiles_t = cdiv(a.Tb, pl.TB);
+        }
         a.group_tiles = cdiv(a.group_nb, pl.nbw);
         pl.tiles_n = a.group_tiles * groups;
         pl.nw = NW;

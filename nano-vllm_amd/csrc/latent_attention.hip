@@ -230,15 +230,16 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 
     // this lane's columns: (token of the item, head); -1 where the item has none.  (Formed again where needed: the page loop
     // keeps only the last position each column sees.)
-    auto column = [&](int c, int& tok, int& h) {
+    auto column_of = [&](int j, int& tok, int& h) {
         // (tokens fastest: the 16 columns of a group are neighbouring rows of the output tiles)
-        const int j = 16 * (part * C + c) + (int)(threadIdx.x & 15), hl = j / a.CT;
+        const int hl = j / a.CT;
         tok = j - hl * a.CT;
         h = h0 + hl;
         const bool valid = tok < ntok && hl < a.HG && h < a.H;
         tok = valid ? tok : 0;
         h = valid ? h : -1;
     };
+    auto column = [&](int c, int& tok, int& h) { column_of(16 * (part * C + c) + (int)(threadIdx.x & 15), tok, h); };
     int plim[C];
 #pragma unroll
     for (int c = 0; c < C; c++) {
@@ -274,21 +275,28 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int n = 0; n < NT; n++) acc[n][c] = f4_t{0.f, 0.f, 0.f, 0.f};
     }
-    const int first_page = page_of(0);
+    // Queries as the B operand: column x, dims 32k + 8g .. +7.  Every fragment is one direct-to-LDS copy whose lanes gather the
+    // 16 columns' pieces, made once for the waves that share it, into the second page buffer (free until block 1 is
+    // requested); from there it goes to registers.  (Columns nobody owns read a real row; their scores are masked.)
+    const unsigned lds_q = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(LATENT_BLOCK_PAGES * nc) * 1024u;
+    for (int f = wave; f < C * WC * nc; f += 4 * WC) {
+        const int group = f / nc, k = f - group * nc;
+        int tok, h;
+        column_of(16 * group + x, tok, h);
+        latent_copy_tile(a.q + ((size_t)(t0 + tok) * a.H + max(h, 0)) * row + 32 * k + 8 * g, __builtin_amdgcn_readfirstlane(lds_q + (unsigned)f * 1024u));
+    }
     int next_page = page_of(1);
-    // queries as the B operand: column x, dims 32k + 8g .. +7 (columns nobody owns read a real row; their scores are masked)
+    if (nblocks > 0) issue(page_of(0), 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    latent_barrier();
     b8_t qf[C][RC];
 #pragma unroll
     for (int c = 0; c < C; c++) {
-        int tok, h;
-        column(c, tok, h);
-        const __half* qr = a.q + ((size_t)(t0 + tok) * a.H + max(h, 0)) * row + 8 * g;
+        const b8_t* qs = reinterpret_cast<const b8_t*>(pages + (size_t)(LATENT_BLOCK_PAGES + part * C + c) * nc * TILE_HALVES) + lane;
 #pragma unroll
-        for (int k = 0; k < RC; k++) qf[c][k] = *reinterpret_cast<const b8_t*>(qr + 32 * (EXACT ? k : min(k, nc - 1)));
+        for (int k = 0; k < RC; k++) qf[c][k] = qs[(EXACT ? k : min(k, nc - 1)) * 64];
     }
-    if (nblocks > 0) issue(first_page, 0);
-    // the queries have arrived before the loop: inside it the compiler then has no load of its own to wait for, and
-    // the only waits on memory are the ones below
+    // (the fragments are in registers before the loop: inside it the compiler has no load of its own to wait for)
 #pragma unroll
     for (int c = 0; c < C; c++)
 #pragma unroll
@@ -506,7 +514,8 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     const LatentPool& P = a.pool;
     const int row = P.row(), chunks = row / 32, vt = cdiv(P.rank_ld, 64);   // value tiles per wave
     // algorithmic work: every sequence's rows read once; per (token, key, head) the two products
-    const double bytes = (double)st.kv_rows * row * P.elem_bytes + (double)st.T * a.H * (row + P.rank_ld) * P.elem_bytes;
+    auto bytes_of = [&](double rows, double tokens) { return rows * row * P.elem_bytes + tokens * a.H * (row + P.rank_ld) * P.elem_bytes; };
+    const double bytes = bytes_of((double)st.kv_rows, st.T);
     const double flops = 2.0 * (double)st.qk_pairs * a.H * (row + P.rank_ld);
     const bool tiled = P.elem_bytes == 2 && ((chunks <= 4 && vt <= 1) || (chunks <= 6 && vt <= 2) || (chunks <= 10 && vt <= 4) || (chunks <= 18 && vt <= 8));
     int pages_per_block = P.block_size / LATENT_PAGE, page_shift = 0;
@@ -539,7 +548,6 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
     k.Kb_out = a.H * P.rank_ld / 32;
     // prompt portions and single tokens want differently shaped items: a launch each when the batch has both
     const int n_single = st.n_runs - st.n_multi;
-    const double share = st.kv_rows > 0 ? (double)st.kv_rows_single / (double)st.kv_rows : 0.0;
     auto launch = [&](const int* runs, int n_runs, int max_run, double bytes, double flops) {
         if (n_runs <= 0) return;
         // columns per item: 64, or 32 or 16 when no item would fill more
@@ -570,7 +578,7 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
             k.part_ml = part + rows * P.rank_ld;
         }
         {
-            ProfScope ps(PC_LATENT_ATTN, bytes, flops);
+            ProfScope ps(max_run == 1 ? PC_LATENT_ATTN_TOK : PC_LATENT_ATTN, bytes, flops);
             const long units = items * nsplit;
             if (chunks <= 4 && vt <= 1) launch_latent_rc<4, 1>(k, units, W);
             else if (chunks <= 6 && vt <= 2) launch_latent_rc<6, 2>(k, units, W);
@@ -583,9 +591,10 @@ void launch_latent_attention(const LatentAttn& a, const StepArrays& st) {
                          P.rank_ld, a.out_b16, k.Kb_out);
         }
     };
+    const double single_bytes = bytes_of((double)st.kv_rows_single, n_single);
     const double single_flops = 2.0 * (double)st.kv_rows_single * a.H * (row + P.rank_ld);
-    launch(st.d_runs, st.n_multi, st.max_run, bytes * (1.0 - share), flops - single_flops);
-    launch(st.d_runs + 4 * st.n_multi, n_single, 1, bytes * share, single_flops);
+    launch(st.d_runs, st.n_multi, st.max_run, bytes - single_bytes, flops - single_flops);
+    launch(st.d_runs + 4 * st.n_multi, n_single, 1, single_bytes, single_flops);
 }
 
 // ------------------------------------------------------------------ fp32 head products

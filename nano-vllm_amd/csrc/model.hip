@@ -348,6 +348,8 @@ static void forward_f32(const StepArrays& st, int T, int B, Config* p, RunState*
         at.runs = st.d_runs;
         at.n_runs = st.n_runs;
         at.kv_positions = st.kv_positions;
+        at.kv_rows = st.kv_rows;
+        at.qk_pairs = st.qk_pairs;
         launch_paged_attention(at);
         launch_matmul_f32w(s->xb, s->xb2, lw.wo, T, QD, D);
         launch_accum(s->x, s->xb, (long)T * D);
@@ -812,6 +814,8 @@ static long enqueue_pass(int* tokens, int num_tokens, int* pos_arr, int* seq_ids
         at.runs = st.d_runs;
         at.n_runs = st.n_runs;
         at.kv_positions = st.kv_positions;
+        at.kv_rows = st.kv_rows;
+        at.qk_pairs = st.qk_pairs;
         launch_paged_attention(at);
         // x += att . wo^T; a16_x = x * rms_ffn; ss_b                              (model.c:385-388)
         WeightEntry wwo{lp.wo, D, QD, QD / 32, (long)(QD / 32) * TILE_HALVES, nullptr};

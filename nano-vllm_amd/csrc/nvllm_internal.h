@@ -175,7 +175,8 @@ enum ProfClass {
     PC_GEMM_ABSORB,      // ... queries times the key up-projection, head by head
     PC_GEMM_VALUE,       // ... attended latents times the value up-projection, head by head
     PC_LATENT_KV,        // ... norm, rotation and cache write of a token's latent row
-    PC_LATENT_ATTN,
+    PC_LATENT_ATTN,      // attention over latents: prompt portions ...
+    PC_LATENT_ATTN_TOK,  // ... and single tokens
     PC_LATENT_COMBINE,
     PC_HYPER,            // hyper-connection update and norm as a launch of its own
     PC_COUNT
@@ -406,6 +407,8 @@ struct AttnArgs {
     const int* runs;       // device int4 (first token, count, last position, table offset): runs of consecutive
     int n_runs;            //   positions of one sequence, at most attn_tokens_per_item() tokens each
     long kv_positions;     // sum over runs of (last position + 1): rows of K/V each kv head reads
+    long kv_rows;          // kernel timing: rows of K/V of the batch's sequences, each counted once (0: kv_positions) ...
+    long qk_pairs;         // ... and (token, position) pairs
 };
 void launch_paged_attention(const AttnArgs& a);
 int attn_tokens_per_item(int H, int KVH);

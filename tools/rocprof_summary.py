@@ -15,7 +15,7 @@ from collections import defaultdict
 
 
 def short(name):
-    m = re.match(r"(?:void )?(?:nvllm::)?([A-Za-z0-9_]+)(<[^>]*>)?", name)
+    m = re.match(r"(?:void )?(?:nvllm::)?(?:\(anonymous namespace\)::)?([A-Za-z0-9_]+)(<[^>]*>)?", name)
     return (m.group(1) + (m.group(2) or "")) if m else name[:40]
 
 
