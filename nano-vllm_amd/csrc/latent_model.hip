@@ -28,6 +28,11 @@ namespace nvllm {
 
 namespace {
 
+[[noreturn]] void bad_config(const char* what) {
+    fprintf(stderr, "nvllm: config.json: %s\n", what);
+    exit(1);
+}
+
 inline int pad32(int n) { return (n + 31) & ~31; }
 
 struct Mixer {
@@ -157,7 +162,7 @@ void LatentHyperModel::load_layer(const ModelDir& dir, int i, const Json& cfg) {
             exit(1);
         }
         w.ff = json_int(*mlp, "ff", af.c_str());
-        if (w.ff < 1) NVLLM_FATAL("config.json: %s.ff is not positive", af.c_str());
+        if (w.ff < 1) bad_config((af + ".ff is not positive").c_str());
     }
     const int H = m.heads, QD = m.dim + m.rot;
     w.sink = vec(dir, M + "sink", H, H);
@@ -269,18 +274,18 @@ LatentHyperModel::LatentHyperModel(const ModelDir& dir, Config* p) {
     S_ = json_int(c, "streams", "config");
     eps_ = (float)json_num(json_get(c, "norm", Json::OBJECT, "config"), "eps", "config.norm");
     softcap_ = (float)json_num(c, "logit_softcap", "config");
-    if (D_ < 1 || V_ < 1 || S_ < 1 || S_ > 64 || !(softcap_ > 0.f)) NVLLM_FATAL("config.json: width, vocab, streams or logit_softcap is out of range");
+    if (D_ < 1 || V_ < 1 || S_ < 1 || S_ > 64 || !(softcap_ > 0.f)) bad_config("width, vocab, streams or logit_softcap is out of range");
     Dp_ = f32_ ? D_ : pad32(D_);
     const Json& list = json_get(c, "layers", Json::ARRAY, "config");
     const int n_layers = (int)list.items.size();
-    if (n_layers < 1) NVLLM_FATAL("config.json lists no layers");
+    if (n_layers < 1) bad_config("it lists no layers");
     int start = 0, stop = 0, times = 1;
     const Json* loop = c.find("loop");
     if (loop && !loop->is_null()) {
         start = json_int(*loop, "start", "config.loop");
         stop = json_int(*loop, "stop", "config.loop");
         times = json_int(*loop, "times", "config.loop");
-        if (start < 0 || stop < start || stop > n_layers || times < 0) NVLLM_FATAL("config.json: the loop does not fit %d layers", n_layers);
+        if (start < 0 || stop < start || stop > n_layers || times < 0) bad_config("the loop does not fit the layers");
     }
     for (int i = 0; i < start; i++) runs_.push_back(i);
     for (int r = 0; r < times; r++)
@@ -336,7 +341,7 @@ LatentHyperModel::LatentHyperModel(const ModelDir& dir, Config* p) {
         s.next_w = last ? final_w : layers_[subs_[i + 1].layer].norm_w[subs_[i + 1].part];
         s.next_b = last ? final_b : layers_[subs_[i + 1].layer].norm_b[subs_[i + 1].part];
     }
-    if (subs_.empty()) NVLLM_FATAL("config.json: no layer runs");
+    if (subs_.empty()) bad_config("no layer runs");
 
     const Mixer& m0 = layers_[0].m;
     p->dim = D_;

@@ -270,3 +270,24 @@ def test_a_pool_of_another_model_is_refused(hip, tmp_path):
         hip.free_kv_cache_manager(C.byref(mgr))
     assert sizes == [(True, False, 8), (True, False, 8), (True, True, 8)]
     hip.nvllm_free_model(C.byref(weights))
+
+
+@pytest.mark.parametrize("what", ["mixer", "architecture", "shape", "loop"])
+def test_a_folder_that_does_not_fit_is_refused(tmp_path, what):
+    """Configurations the library does not know, or that the tensors contradict, end with a message and an error status."""
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    path, cfg, _ = U.model(tmp_path, "mixed", seed=4)
+    cfg = json.loads(json.dumps(cfg))
+    if what == "mixer":
+        cfg["layers"][1]["type"] = "something_else"
+    elif what == "architecture":
+        cfg["architecture"] = "Unheardof"
+    elif what == "shape":
+        cfg["layers"][0]["mixer"]["kv_rank"] += 16
+    else:
+        cfg["loop"] = dict(start=1, stop=9, times=2)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    r = subprocess.run([os.path.join(root, "bin", "generate"), "--model", path, "-n", "1"], capture_output=True, text=True, timeout=100)
+    assert r.returncode != 0 and r.stdout == ""
+    assert {"mixer": "something_else", "architecture": "Unheardof", "shape": "asks for", "loop": "loop"}[what] in r.stderr
