@@ -242,6 +242,20 @@ __device__ __forceinline__ float epi_point(const GemmEpilogue& ep, int N, int t,
     return 0.f;
 }
 
+typedef __attribute__((address_space(3))) void lds_void;
+// One wave copies one 1-KiB tile global -> LDS without passing through registers: lane l's
+// 16 bytes land at lds_byte_address + 16*l.  Written as an asm statement on purpose: the
+// compiler then keeps no account of the copy, and the waits below are the only ones (with
+// the builtin it drains every copy in flight before the next read of the LDS array).
+// M0 carries the LDS address and is restored inside the statement.
+__device__ __forceinline__ void copy_tile_to_lds(const __half* lane_src, unsigned lds_byte_address) {
+    unsigned keep;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+                 : "=&s"(keep)
+                 : "v"(lane_src), "s"(lds_byte_address)
+                 : "memory");
+}
+
 // gemm_prefill.hip: 128 x 128 output tiles through LDS, for batches of hundreds of tokens
 void launch_gemm_prefill(GemmArgs a);
 

@@ -50,8 +50,6 @@ namespace nvllm {
 
 namespace {
 
-typedef __attribute__((address_space(3))) void lds_void;
-
 // FW = 16-row weight blocks per wave (4 or 8), KG = wave groups that split the K-steps, WR = rows of
 // the wave grid (WR x 2 waves per group: 2 -> 128-feature tiles; 4 -> 256-feature tiles compiles but measured
 // slower on this model's shapes and is not instantiated), TW = 16-token
@@ -69,19 +67,6 @@ struct PfGeom {
     static_assert(TW == 4 || KG == 1, "the two-group form exchanges halves of four token blocks");
     static constexpr int RINV_HALVES = 256;            // 128 floats in front of the ring (1/rms of up to 128 tokens)
 };
-
-// One wave copies one 1-KiB tile global -> LDS without passing through registers: lane l's
-// 16 bytes land at lds_byte_address + 16*l.  Written as an asm statement on purpose: the
-// compiler then keeps no account of the copy, and the waits below are the only ones (with
-// the builtin it drains every copy in flight before the next read of the LDS array).
-// M0 carries the LDS address and is restored inside the statement.
-__device__ __forceinline__ void copy_tile_to_lds(const __half* lane_src, unsigned lds_byte_address) {
-    unsigned keep;
-    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
-                 : "=&s"(keep)
-                 : "v"(lane_src), "s"(lds_byte_address)
-                 : "memory");
-}
 
 // The same copy for the steady state of the K loop: M0 is written and left (nothing else in
 // this kernel reads it: the compiler sets M0 itself right before any use of its own), the LDS address is a wave-uniform

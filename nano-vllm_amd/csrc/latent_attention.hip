@@ -149,7 +149,6 @@ __global__ __launch_bounds__(256) void k_latent_attn_any(const void* base, const
 typedef short s4_t __attribute__((ext_vector_type(4)));
 typedef short s8_t __attribute__((ext_vector_type(8)));
 typedef __attribute__((address_space(3))) s4_t lds_s4;
-typedef __attribute__((address_space(3))) void lds_void_t;
 
 struct LatentKArgs {
     const __half* base;
@@ -175,13 +174,6 @@ struct LatentKArgs {
 constexpr int LATENT_BLOCK_PAGES = 4;
 static size_t latent_attn_lds(int chunks, int C) { return (size_t)2 * LATENT_BLOCK_PAGES * chunks * 1024 + (size_t)C * 2048 + (size_t)C * 2 * 4 * 16 * 4; }
 
-__device__ __forceinline__ void latent_copy_tile(const __half* lane_src, unsigned lds_byte_address) {
-    unsigned keep;
-    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
-                 : "=&s"(keep)
-                 : "v"(lane_src), "s"(lds_byte_address)
-                 : "memory");
-}
 // LDS stores of this wave are done, then everybody meets (copies to LDS in flight stay in flight)
 __device__ __forceinline__ void latent_barrier() {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -254,7 +246,7 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
         const int pg = min(p0 + b * LATENT_BLOCK_PAGES + page, npages - 1);
         return (table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1));
     };
-    const unsigned lds0 = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(page * nc + part) * 1024u;
+    const unsigned lds0 = (unsigned)(size_t)(lds_void*)pages + (unsigned)(page * nc + part) * 1024u;
     auto issue = [&](int page_id, int b) {   // tiles part, part + WC, ... of the page
         if (b >= 2 && p0 + b * LATENT_BLOCK_PAGES + page >= p1) return;
         const int buf = b & 1;
@@ -263,7 +255,7 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
 #pragma unroll
         for (int c = 0; c < RC; c += WC)
             if (EXACT ? c + WC <= RC || c + part < RC : c + part < nc)
-                latent_copy_tile(src + (size_t)c * TILE_HALVES, __builtin_amdgcn_readfirstlane(dst + (unsigned)c * 1024u));
+                copy_tile_to_lds(src + (size_t)c * TILE_HALVES, __builtin_amdgcn_readfirstlane(dst + (unsigned)c * 1024u));
     };
 
     float m[C], lsum[C];
@@ -278,12 +270,12 @@ __global__ __launch_bounds__(256 * WC, WC) void k_latent_attn(LatentKArgs a) {
     // Queries as the B operand: column x, dims 32k + 8g .. +7.  Every fragment is one direct-to-LDS copy whose lanes gather the
     // 16 columns' pieces, made once for the waves that share it, into the second page buffer (free until block 1 is
     // requested); from there it goes to registers.  (Columns nobody owns read a real row; their scores are masked.)
-    const unsigned lds_q = (unsigned)(size_t)(lds_void_t*)pages + (unsigned)(LATENT_BLOCK_PAGES * nc) * 1024u;
+    const unsigned lds_q = (unsigned)(size_t)(lds_void*)pages + (unsigned)(LATENT_BLOCK_PAGES * nc) * 1024u;
     for (int f = wave; f < C * WC * nc; f += 4 * WC) {
         const int group = f / nc, k = f - group * nc;
         int tok, h;
         column_of(16 * group + x, tok, h);
-        latent_copy_tile(a.q + ((size_t)(t0 + tok) * a.H + max(h, 0)) * row + 32 * k + 8 * g, __builtin_amdgcn_readfirstlane(lds_q + (unsigned)f * 1024u));
+        copy_tile_to_lds(a.q + ((size_t)(t0 + tok) * a.H + max(h, 0)) * row + 32 * k + 8 * g, __builtin_amdgcn_readfirstlane(lds_q + (unsigned)f * 1024u));
     }
     int next_page = page_of(1);
     if (nblocks > 0) issue(page_of(0), 0);

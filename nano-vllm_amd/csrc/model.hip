@@ -711,7 +711,7 @@ static long enqueue_pass(int* tokens, int num_tokens, int* pos_arr, int* seq_ids
     if (m->dir) {
         if (tp().active) NVLLM_FATAL("model folders are not split over tensor-parallel ranks");
         const bool to_host = rt().logits_mode == NVLLM_LOGITS_ARGMAX && B > 0;
-        PassArgs a{tokens, pos_arr, seq_ids, output_indices, token_src, T, B, p->max_seq_len, block_tables, &g_kv_manager,
+        PassArgs a{tokens, pos_arr, seq_ids, output_indices, token_src, T, B, block_tables, &g_kv_manager,
                    (float*)ws_get(WS_LOGITS, (size_t)B * p->vocab_size * sizeof(float)),
                    (int*)ws_get(WS_ARGMAX, (size_t)(p->max_seq_len + 64) * sizeof(int)), to_host ? next_slot(B).host : nullptr};
         m->dir->forward(a);

@@ -54,7 +54,6 @@ struct PassArgs {
     const int* output_indices;
     const int* token_src;         // optional: >= 0 names the output row of the previous pass that the token continues
     int T, B;
-    int max_tokens;               // T never exceeds this
     BlockTable** tables;
     KVCacheManager* mgr;
     float* d_logits;              // [B, vocab] in HBM: to be filled
