@@ -242,6 +242,11 @@ long nvllm_forward_enqueue(int* tokens, int num_tokens, int* pos_arr, int* seq_i
  * num_outputs. */
 int nvllm_forward_collect(long ticket, int* argmax_out, int cap);
 
+/* Models whose layers carry a state from token to token: room for `n_slots` sequences (a sequence's slot is its id in
+ * seq_ids; a pass that brings a larger id makes room by itself).  A sequence that starts again at position 0 starts from
+ * an empty state.  No effect on other models. */
+void nvllm_init_model_states(const Weights* w, int n_slots);
+
 /* ------------------------------------------------------ N-sequence driver */
 /* The reference's scheduler with the sequence count as a parameter: arrival
  * gating, is_prefill = pos < n_prompt-1, chunked prefill, batch-capacity check,

@@ -166,6 +166,7 @@ _HIP_ONLY = {
     "nvllm_get_compute_dtype": (_I, []),
     "nvllm_has_architecture": (_I, [C.c_char_p]),
     "nvllm_init_model_kv": (_V, [C.POINTER(KVCacheManager), _I, _I, C.POINTER(Config), C.POINTER(Weights)]),
+    "nvllm_init_model_states": (_V, [C.POINTER(Weights), _I]),
     "nvllm_hyper_step": (_V, [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I]),
     "nvllm_swiglu_bias": (_V, [_P, _P, _P, _P, _P, _I, _I]),
     "nvllm_softcap": (_V, [_P, _F, _L]),

@@ -12,7 +12,7 @@ namespace {
 
 constexpr int NW = 8, RW = 4, RA = 2;
 
-template <int NBW, int TB, int WAVES, int EPI, bool GRP>
+template <int NBW, int TB, int WAVES, int EPI, bool GRP, bool EXP = false>
 __global__ __launch_bounds__(WAVES * 64) void k_gemm_b16(GemmArgs p) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds_dyn[];
     if constexpr (EPI == GemmEpilogue::LATENT_Q) {
@@ -23,20 +23,20 @@ __global__ __launch_bounds__(WAVES * 64) void k_gemm_b16(GemmArgs p) {
     }
     h8_t w[RW][NBW];
     const TileIdx ix{(int)blockIdx.x, (int)blockIdx.y, (int)blockIdx.z, EPI == GemmEpilogue::LATENT_Q ? p.ride_from : (int)gridDim.x};
-    gemm_tile<NBW, TB, WAVES, RW, RA, EPI, float, false, 0, OpBf16, GRP>(p, ix, lds_dyn, w, [](int) {}, (int)threadIdx.x);
+    gemm_tile<NBW, TB, WAVES, RW, RA, EPI, float, false, 0, OpBf16, GRP, EXP>(p, ix, lds_dyn, w, [](int) {}, (int)threadIdx.x);
 }
 
-template <int NBW, int TB, int WAVES, int EPI, bool GRP>
+template <int NBW, int TB, int WAVES, int EPI, bool GRP, bool EXP = false>
 void launch_stream(const GemmArgs& a, dim3 grid) {
     constexpr int shmem = gemm_tile_lds<NBW, TB, WAVES>();
     static_assert(shmem <= 160 * 1024, "partial tiles must fit the CU's LDS");
     static bool enabled = false;
     if (shmem > 64 * 1024 && !enabled) {
-        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemm_b16<NBW, TB, WAVES, EPI, GRP>),
+        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemm_b16<NBW, TB, WAVES, EPI, GRP, EXP>),
                                       hipFuncAttributeMaxDynamicSharedMemorySize, shmem));
         enabled = true;
     }
-    NVLLM_LAUNCH((k_gemm_b16<NBW, TB, WAVES, EPI, GRP>), grid, dim3(WAVES * 64), shmem, a);
+    NVLLM_LAUNCH((k_gemm_b16<NBW, TB, WAVES, EPI, GRP, EXP>), grid, dim3(WAVES * 64), shmem, a);
 }
 
 template <int EPI, bool GRP>
@@ -62,17 +62,17 @@ void launch_stream_plan(const GemmArgs& a, const GemmPlan& pl) {
     else launch_stream<4, 4, NW, EPI, GRP>(a, grid);
 }
 
-template <int EPI, bool GRP, int TW>
+template <int EPI, bool GRP, int TW, bool EXP = false>
 void launch_dense_tw(const GemmArgs& a, int tiles_n, int tiles_t, int nbuf) {
     using G = PfGeom<4, 1, 2, TW, 1>;
     const size_t shmem = (size_t)(G::RINV_HALVES + nbuf * G::STAGE_HALVES) * sizeof(__half);
     static size_t allowed = 0;
     if (shmem > allowed) {
-        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP>),
+        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP, EXP>),
                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem));
         allowed = shmem;
     }
-    NVLLM_LAUNCH((k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP>), dim3(tiles_n * tiles_t + (EPI == GemmEpilogue::LATENT_Q && a.ride.base ? cdiv(a.ride.T, 4) : 0)), dim3(256), shmem, a, tiles_n, tiles_t, nbuf,
+    NVLLM_LAUNCH((k_gemm_prefill<4, 1, EPI, float, 2, TW, OpBf16, GRP, EXP>), dim3(tiles_n * tiles_t + (EPI == GemmEpilogue::LATENT_Q && a.ride.base ? cdiv(a.ride.T, 4) : 0)), dim3(256), shmem, a, tiles_n, tiles_t, nbuf,
                  tiles_n * tiles_t);
 }
 
@@ -138,7 +138,69 @@ void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
     }
 }
 
+template <int EPI>
+void launch_experts_kind(GemmArgs a, int pad, bool dense, double bytes, double flops, int prof_cls) {
+    const int cus = rt().num_cus;
+    a.ksplit = 1;
+    a.kb_per_split = a.Kb;
+    ProfScope ps(prof_cls, bytes, flops);
+    if (dense) {
+        const int tiles_n = cdiv(a.NB, 8), tiles_t = a.Tb * 16 / pad, per_cu = cdiv(tiles_n * tiles_t, cus);
+        const int nbuf = per_cu >= 3 ? 3 : (per_cu == 2 ? 4 : 5);
+        a.ride_from = tiles_n * tiles_t;
+        if (pad == 64) launch_dense_tw<EPI, false, 2, true>(a, tiles_n, tiles_t, nbuf);
+        else launch_dense_tw<EPI, false, 4, true>(a, tiles_n, tiles_t, nbuf);
+        return;
+    }
+    const int TB = pad / 16, tiles_t = a.Tb / TB;
+    const bool narrow = cdiv(a.NB, 4) * tiles_t <= cus;   // (some of the row groups are empty)
+    const dim3 grid(cdiv(a.NB, narrow ? 2 : 4), 1, tiles_t);
+    a.ride_from = (int)grid.x;
+    if (narrow) {
+        if (TB == 1) launch_stream<2, 1, NW, EPI, false, true>(a, grid);
+        else launch_stream<2, 2, NW, EPI, false, true>(a, grid);
+    } else {
+        if (TB == 1) launch_stream<4, 1, NW, EPI, false, true>(a, grid);
+        else launch_stream<4, 2, NW, EPI, false, true>(a, grid);
+    }
+}
+
 }  // namespace
+
+void launch_gemm_experts(const B16Weight& w, int experts, const __half* act, const ExpertRows& rows, const GemmEpilogue& epi, int prof_cls) {
+    if (rows.capacity <= 0) return;
+    ensure_init();
+    const bool dense = rows.pad >= 64;
+    if (w.K % 32 || w.N % 32 || experts < 1 || rows.capacity % rows.pad || !(rows.pad == 16 || rows.pad == 32 || rows.pad == 64 || rows.pad == 128))
+        NVLLM_FATAL("expert projection: [%d, %d] on %d rows in groups of %d is not supported", w.N, w.K, rows.capacity, rows.pad);
+    GemmArgs a{};
+    a.W = w.tiles;
+    a.Kb = w.K / 32;
+    a.nb_stride = (long)a.Kb * TILE_HALVES;
+    a.NB = w.N / 16;
+    a.expert_stride = a.NB * a.nb_stride;
+    a.A = act;
+    a.Tb = rows.capacity / 16;
+    a.N = w.N;
+    a.T = rows.capacity;
+    a.act_Kb = a.Kb;
+    a.block_expert = rows.block_expert;
+    a.source = rows.source;
+    a.counters = gemm_tile_counters();
+    a.e = epi;
+    const double touched = std::min(experts, rows.live);   // matrices read
+    const double bytes = touched * w.N * w.K * 2.0 + (double)rows.live * w.K * 2.0 + (double)rows.live * w.N * (epi.kind == GemmEpilogue::F32 ? 4.0 : 1.0);
+    const double flops = 2.0 * rows.live * (double)w.N * w.K;
+    if (epi.kind == GemmEpilogue::SWIGLU_A16) {
+        if (w.N % 64) NVLLM_FATAL("expert projection: a hidden width of %d is not padded to 32", w.N / 2);
+        a.e.Kb_out = w.N / 64;
+        launch_experts_kind<GemmEpilogue::SWIGLU_A16>(a, rows.pad, dense, bytes, flops, prof_cls);
+    } else if (epi.kind == GemmEpilogue::F32) {
+        launch_experts_kind<GemmEpilogue::F32>(a, rows.pad, dense, bytes, flops, prof_cls);
+    } else {
+        NVLLM_FATAL("this epilogue has no form for experts");
+    }
+}
 
 void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls, const LatentKvRider* ride) {
     if (T <= 0) return;
@@ -177,6 +239,11 @@ void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpi
             out_bytes = (double)T * w.N;
             break;
         case GemmEpilogue::TILE_B16: need32(w.N, "an output width"); a.e.Kb_out = w.N / 32; break;
+        case GemmEpilogue::RESID_B16:
+            need32(w.N, "a residual width");
+            a.e.Kb_out = w.N / 32;
+            out_bytes = (double)T * w.N * 10.0;
+            break;
         case GemmEpilogue::LATENT_IN: need32(epi.latent_q, "a query latent"); a.e.Kb_out = epi.latent_q / 32; break;
         case GemmEpilogue::LATENT_Q: need32(epi.q_plain, "a query width"); a.e.Kb_out = epi.q_plain / 32; break;
         case GemmEpilogue::HYPER_2:
@@ -202,6 +269,7 @@ void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpi
             break;
         case GemmEpilogue::LATENT_IN: launch_kind<GemmEpilogue::LATENT_IN, false>(a, prof_cls, bytes, flops); break;
         case GemmEpilogue::LATENT_Q: launch_kind<GemmEpilogue::LATENT_Q, false>(a, prof_cls, bytes, flops); break;
+        case GemmEpilogue::RESID_B16: launch_kind<GemmEpilogue::RESID_B16, false>(a, prof_cls, bytes, flops); break;
         case GemmEpilogue::HYPER_2: launch_kind<GemmEpilogue::HYPER_2, false>(a, prof_cls, bytes, flops); break;
         case GemmEpilogue::HYPER_4: launch_kind<GemmEpilogue::HYPER_4, false>(a, prof_cls, bytes, flops); break;
         default: NVLLM_FATAL("this epilogue belongs to fp16 models");

@@ -26,9 +26,9 @@ struct OpBf16 {    // bf16 weights, bf16 activations
     }
 };
 // epilogues that act on four consecutive features of one token at a time (epi_point below)
-constexpr bool epi_is_point(int kind) { return kind >= GemmEpilogue::TILE_B16; }
+constexpr bool epi_is_point(int kind) { return kind >= GemmEpilogue::TILE_B16 && kind != GemmEpilogue::RESID_B16; }
 // epilogues that also leave sums of squares per 32 features
-constexpr bool epi_has_ss(int kind) { return kind == GemmEpilogue::RESID_A16 || kind == GemmEpilogue::LATENT_IN; }
+constexpr bool epi_has_ss(int kind) { return kind == GemmEpilogue::RESID_A16 || kind == GemmEpilogue::LATENT_IN || kind == GemmEpilogue::RESID_B16; }
 
 // What a launch may carry besides its tiles: the norm, rotation and cache write of the batch's latent rows (latent_kv.h)
 // in extra workgroups, a wave per token.  Their input comes from the launch before and their output is for the launch
@@ -55,6 +55,9 @@ struct GemmArgs {
     int act_Kb;       // k tiles per token block of A (Kb, or Kb * groups of a block-diagonal product)
     int group_nb;     // block-diagonal product: 16-row blocks per group, 0 = one group ...
     int group_tiles;  // ... and feature tiles per group (streaming kernel: grid columns)
+    const int* block_expert;   // rows sorted by expert (ExpertRows): expert of a row block ...
+    const int* source;         // ... row of A that a row reads (null: its own) ...
+    long expert_stride;        // ... and halves between the experts' matrices
     int kb_per_split;
     int ksplit;
     float* slab;      // [tile][slice][round][item] float4
@@ -206,14 +209,34 @@ __device__ __forceinline__ void hyper_update_4(const HyperIn<SMAX>& in, const Ge
 }
 constexpr int hyper_streams(int kind) { return kind == GemmEpilogue::HYPER_2 ? 2 : kind == GemmEpilogue::HYPER_4 ? 4 : 0; }   // 0: another epilogue
 
+// Residual add of one token's features n .. n+3: xr <- xo + y, x * gain -> tiles; returns their sum of squares.
+__device__ __forceinline__ float resid_b16_4(const GemmEpilogue& ep, int N, int t, int n, const float4 xo, const float4 g, const float* y) {
+    const float xn[4] = {xo.x + y[0], xo.y + y[1], xo.z + y[2], xo.w + y[3]};
+    *reinterpret_cast<float4*>(ep.x + (size_t)t * N + n) = make_float4(xn[0], xn[1], xn[2], xn[3]);
+    const float z[4] = {xn[0] * g.x, xn[1] * g.y, xn[2] * g.z, xn[3] * g.w};
+    store_b16_4(ep.a16_out, ep.Kb_out, t, n, z);
+    return xn[0] * xn[0] + xn[1] * xn[1] + xn[2] * xn[2] + xn[3] * xn[3];
+}
+
 // One token's features n .. n+3 through a point epilogue other than HYPER_*; returns their share of the sum of squares.
 template <int EPI>
 __device__ __forceinline__ float epi_point(const GemmEpilogue& ep, int N, int t, int n, const float* y) {
     if constexpr (EPI == GemmEpilogue::TILE_B16) {
+        if (ep.relu2) {
+            float z[4];
+#pragma unroll
+            for (int r = 0; r < 4; r++) z[r] = fmaxf(y[r], 0.f) * fmaxf(y[r], 0.f);
+            store_b16_4(ep.a16_out, ep.Kb_out, t, n, z);
+            return 0.f;
+        }
         store_b16_4(ep.a16_out, ep.Kb_out, t, n, y);
     } else if constexpr (EPI == GemmEpilogue::ROWS_B16) {
         const int h = n / ep.head_ld, d = n - h * ep.head_ld;
-        *reinterpret_cast<b4_t*>(ep.q_rows + ((size_t)t * ep.q_heads + h) * ep.q_row + d) = to_b4(y);
+        float z[4] = {y[0], y[1], y[2], y[3]};
+        if (n < ep.silu_to)
+#pragma unroll
+            for (int r = 0; r < 4; r++) z[r] = silu_mul(y[r], 1.f);
+        *reinterpret_cast<b4_t*>(ep.q_rows + ((size_t)t * ep.q_heads + h) * ep.q_row + d) = to_b4(z);
     } else if constexpr (EPI == GemmEpilogue::LATENT_IN) {
         if (n < ep.latent_q) {
             const f4_t g = *reinterpret_cast<const f4_t*>(ep.gain_next + n);

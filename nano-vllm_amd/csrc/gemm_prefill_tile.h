@@ -161,6 +161,10 @@ __device__ __forceinline__ void pf_epilogue(const GemmArgs& p, const f4_t (&v)[N
                                 gate += ep.bias[n + r];
                                 up += ep.bias[n + 16 + r];
                             }
+                            if (ep.row_weight) {
+                                gate *= ep.row_weight[t];
+                                up *= ep.row_weight[t];
+                            }
                         }
                         z[r] = silu_mul(gate, up);
                     }
@@ -168,6 +172,10 @@ __device__ __forceinline__ void pf_epilogue(const GemmArgs& p, const f4_t (&v)[N
                     if constexpr (OP::PLANES == 1) store_b16_4(ep.a16_out, ep.Kb_out, t, hid, z);
                     else store_a16_4(ep.a16_out, ep.Kb_out, t, hid, z);
                 }
+            } else if (EPI == GemmEpilogue::RESID_B16) {
+                if (live)
+                    ssq[i >> 1] += resid_b16_4(ep, p.N, t, n, *reinterpret_cast<const float4*>(ep.x + (size_t)t * p.N + n),
+                                               *reinterpret_cast<const float4*>(ep.gain_next + n), y);
             } else if (EPI == GemmEpilogue::RESID_A16) {
                 if (live) {
                     float* xr = ep.x + (size_t)t * p.N + n;
@@ -278,7 +286,7 @@ __device__ __forceinline__ bool pf_close_split(const GemmArgs& p, f4_t (&v)[NI][
     return true;
 }
 
-template <int FW, int KG, int EPI, typename KVT, int WR = 2, int TW = 4, typename OP = OpF16x2, bool GRP = false>
+template <int FW, int KG, int EPI, typename KVT, int WR = 2, int TW = 4, typename OP = OpF16x2, bool GRP = false, bool EXP = false>
 __global__ __launch_bounds__(128 * WR * KG, WR == 4 ? 4 : 2) void k_gemm_prefill(GemmArgs p, int tiles_n, int tiles_t, int nbuf, int split_from) {
     constexpr int PL = OP::PLANES;
     using G = PfGeom<FW, KG, WR, TW, PL>;
@@ -330,6 +338,12 @@ __global__ __launch_bounds__(128 * WR * KG, WR == 4 ? 4 : 2) void k_gemm_prefill
     const int nb0 = GRP ? grp * p.group_nb + (col - grp * p.group_tiles) * G::FB : col * G::FB;
     const int nb_lim = GRP ? min(p.NB, (grp + 1) * p.group_nb) : p.NB;   // row blocks this tile may touch
     const int tb0 = (id % tiles_t) * G::TB;
+    const __half* W = p.W;
+    if constexpr (EXP) {
+        const int e = __builtin_amdgcn_readfirstlane(p.block_expert[tb0]);
+        if (e < 0) return;   // fewer rows than the launch has room for
+        W += (size_t)e * p.expert_stride;
+    }
     // K-steps [kb_lo, kb_hi) of this workgroup
     const int kb_lo = split ? slice * p.kb_per_split : 0;
     const int kb_hi = split ? min(p.Kb, kb_lo + p.kb_per_split) : p.Kb;
@@ -346,11 +360,17 @@ __global__ __launch_bounds__(128 * WR * KG, WR == 4 ? 4 : 2) void k_gemm_prefill
         const int r = q % G::TPK;
         kofs[u] = q / G::TPK;
         if (r < G::FB) {
-            src[u] = p.W + (size_t)min(nb0 + r, nb_lim - 1) * p.nb_stride + lane * 8;
+            src[u] = W + (size_t)min(nb0 + r, nb_lim - 1) * p.nb_stride + lane * 8;
             step[u] = TILE_HALVES;
         } else {
             const int tb = min(tb0 + (r - G::FB) / PL, p.Tb - 1);
             src[u] = p.A + (((size_t)tb * (GRP ? p.act_Kb : p.Kb) + (GRP ? grp * p.Kb : 0)) * PL + (r - G::FB) % PL) * TILE_HALVES + lane * 8;
+            if constexpr (EXP) {
+                if (p.source) {   // every lane gathers its own row
+                    const int s = p.source[tb * 16 + (lane & 15)];
+                    src[u] = p.A + (size_t)(s >> 4) * p.Kb * TILE_HALVES + ((s & 15) + 16 * (lane >> 4)) * 8;
+                }
+            }
             step[u] = PL * TILE_HALVES;
         }
     }

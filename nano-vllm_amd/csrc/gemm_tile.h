@@ -136,8 +136,8 @@ __device__ __forceinline__ void gemm_tile_prefetch(const GemmArgs& p, const Tile
 // spread over its last RW steps: the place to start loads for later work, a few at a time.
 // PRE: 0 = the tile requests its first RW K-steps of weights itself; 1 = the caller has (gemm_tile_prefetch);
 // 2 = the caller says at run time (`prefetched`, uniform over the workgroup).
-// OP: operand format (gemm_common.h); GRP: a block-diagonal product, whose tiles never cross a group.
-template <int NBW, int TB, int NW, int RW, int RA, int EPI, typename KVT, bool COH, int PRE, typename OP = OpF16x2, bool GRP = false, typename Hook>
+// OP: operand format (gemm_common.h); GRP: a block-diagonal product, whose tiles never cross a group; EXP: rows sorted by expert.
+template <int NBW, int TB, int NW, int RW, int RA, int EPI, typename KVT, bool COH, int PRE, typename OP = OpF16x2, bool GRP = false, bool EXP = false, typename Hook>
 __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, unsigned char* lds_dyn, h8_t (&w)[RW][NBW],
                                           Hook&& slot_free, const int tid, const bool prefetched = true) {
     static_assert(NBW % 2 == 0, "row blocks are reduced in pairs");
@@ -173,12 +173,22 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
     const int kb_begin = ix.y * p.kb_per_split;
     const int kb_end = min(p.Kb, kb_begin + p.kb_per_split);
     const int tb0 = ix.z * TB;
+    const __half* W = p.W;
+    if constexpr (EXP) {
+        const int e = __builtin_amdgcn_readfirstlane(p.block_expert[tb0]);
+        if (e < 0) {   // fewer rows than the launch has room for
+#pragma unroll
+            for (int r = 0; r < RW; r++) slot_free(r);
+            return false;
+        }
+        W += (size_t)e * p.expert_stride;
+    }
     const int first = kb_begin + wave;
     const int nsteps = first < kb_end ? (kb_end - first + NW - 1) / NW : 0;
     const h8_t* wp[NBW];
 #pragma unroll
     for (int i = 0; i < NBW; i++)
-        wp[i] = reinterpret_cast<const h8_t*>(p.W + (size_t)min(nb0 + i, nb_lim - 1) * p.nb_stride) + lane;
+        wp[i] = reinterpret_cast<const h8_t*>(W + (size_t)min(nb0 + i, nb_lim - 1) * p.nb_stride) + lane;
     // activations: pointers (plain loads), or byte offsets into a buffer descriptor (sc1 loads)
     const h8_t* ap[TB];
     int aoff[TB];
@@ -186,6 +196,12 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
 #pragma unroll
     for (int j = 0; j < TB; j++) {
         ap[j] = reinterpret_cast<const h8_t*>(p.A + ((size_t)min(tb0 + j, p.Tb - 1) * (GRP ? p.act_Kb : p.Kb) + (GRP ? grp * p.Kb : 0)) * OP::PLANES * TILE_HALVES) + lane;
+        if constexpr (EXP) {
+            if (p.source) {   // every lane gathers its own row
+                const int r = p.source[(tb0 + j) * 16 + (lane & 15)];
+                ap[j] = reinterpret_cast<const h8_t*>(p.A + (size_t)(r >> 4) * p.Kb * TILE_HALVES) + (r & 15) + 16 * (lane >> 4);
+            }
+        }
         aoff[j] = min(tb0 + j, p.Tb - 1) * p.Kb * 2048 + lane * 16;
     }
     static_assert(!COH || (OP::PLANES == 2 && !GRP), "the one-launch step runs fp16 models");
@@ -296,7 +312,7 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
     __amdgpu_buffer_rsrc_t rs_x = gemm_rsrc(ep.x, (unsigned)p.T * (unsigned)p.N * 4u);
     __amdgpu_buffer_rsrc_t rs_o = gemm_rsrc(ep.a16_out, (unsigned)p.Tb * (unsigned)ep.Kb_out * 2048u);
     __amdgpu_buffer_rsrc_t rs_q = gemm_rsrc(ep.q_out, (unsigned)p.T * (unsigned)ep.QD * 4u);
-    if (EPI == GemmEpilogue::RESID_A16) {
+    if (EPI == GemmEpilogue::RESID_A16 || EPI == GemmEpilogue::RESID_B16) {
 #pragma unroll
         for (int s = 0; s < FPT; s++) {
             const int w_ = min(tid + s * NW * 64, WITEMS - 1);
@@ -502,6 +518,10 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
                                 gate += ep.bias[n + r];
                                 up += ep.bias[n + 16 + r];
                             }
+                            if (ep.row_weight) {
+                                gate *= ep.row_weight[t];
+                                up *= ep.row_weight[t];
+                            }
                         }
                         z[r] = silu_mul(gate, up);
                     }
@@ -510,6 +530,8 @@ __device__ __forceinline__ bool gemm_tile(const GemmArgs& p, const TileIdx ix, u
                     else if constexpr (COH) store_a16_4_sc1(rs_o, ep.Kb_out, t, hid, z, l);
                     else store_a16_4(ep.a16_out, ep.Kb_out, t, hid, z);
                 }
+            } else if (EPI == GemmEpilogue::RESID_B16) {
+                if (live) ssq[s] += resid_b16_4(ep, p.N, t, n, pf_x[s], pf_g[s], y);
             } else if (EPI == GemmEpilogue::RESID_A16) {
                 if (live) {
                     float* xr = ep.x + (size_t)t * p.N + n;

@@ -64,6 +64,36 @@ void launch_embed_streams(float* x, const void* table, bool bf16, const int* tok
     else NVLLM_LAUNCH((k_embed_streams<false>), dim3(T), dim3(256), 0, x, table, tokens, streams, ld, tok_src, prev);
 }
 
+// a thread per four features: eight neighbouring threads cover the 32 of a sum of squares
+__global__ __launch_bounds__(256) void k_embed_norm_b16(float* __restrict__ x, __half* __restrict__ act, float* __restrict__ ss, const __bf16* __restrict__ table,
+                                                        const int* __restrict__ tokens, const float* __restrict__ gain, int ld, const int* __restrict__ tok_src,
+                                                        const int* __restrict__ prev) {
+    const int t = blockIdx.x, Kb = ld >> 5;
+    const int tok = (tok_src && tok_src[t] >= 0) ? prev[tok_src[t]] : tokens[t];
+    for (int n = threadIdx.x * 4; n < ((ld + 255) & ~255); n += 1024) {
+        float sq = 0.f;
+        if (n < ld) {
+            const b4_t r = *reinterpret_cast<const b4_t*>(table + (size_t)tok * ld + n);
+            const f4_t g = *reinterpret_cast<const f4_t*>(gain + n);
+            const float v[4] = {(float)r[0], (float)r[1], (float)r[2], (float)r[3]};
+            const float z[4] = {v[0] * g[0], v[1] * g[1], v[2] * g[2], v[3] * g[3]};
+            *reinterpret_cast<float4*>(x + (size_t)t * ld + n) = make_float4(v[0], v[1], v[2], v[3]);
+            store_b16_4(act, Kb, t, n, z);
+            sq = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        }
+        sq += __shfl_xor(sq, 1, 64);
+        sq += __shfl_xor(sq, 2, 64);
+        sq += __shfl_xor(sq, 4, 64);
+        if ((threadIdx.x & 7) == 0 && n < ld) ss[(size_t)t * Kb + (n >> 5)] = sq;
+    }
+}
+void launch_embed_norm_b16(float* x, __half* act, float* ss, const void* table, const int* tokens, const float* gain, int T, int ld, const int* tok_src, const int* prev) {
+    if (T <= 0) return;
+    if (ld % 32) NVLLM_FATAL("embedding: a row of %d is not padded to 32", ld);
+    ProfScope ps(PC_EMBED, (double)T * ld * 8.0, 0);
+    NVLLM_LAUNCH(k_embed_norm_b16, dim3(T), dim3(256), 0, x, act, ss, (const __bf16*)table, tokens, gain, ld, tok_src, prev);
+}
+
 __global__ __launch_bounds__(256) void k_gather_b16(__half* __restrict__ dst, const __half* __restrict__ src, const int* __restrict__ idx, int Kb) {
     const int r = blockIdx.x, t = idx[r];
     for (int c = threadIdx.x; c < Kb * 4; c += 256) {   // 8-element chunks of the row

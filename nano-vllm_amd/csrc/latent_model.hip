@@ -28,13 +28,6 @@ namespace nvllm {
 
 namespace {
 
-[[noreturn]] void bad_config(const char* what) {
-    fprintf(stderr, "nvllm: config.json: %s\n", what);
-    exit(1);
-}
-
-inline int pad32(int n) { return (n + 31) & ~31; }
-
 struct Mixer {
     int heads, dim, rot, vdim, rank, q_rank;
     double base;
@@ -62,12 +55,9 @@ struct Sublayer {
     const float *next_w, *next_b;   // norm of the next sublayer, or the final norm
 };
 
-class LatentHyperModel : public DirModel {
+class LatentHyperModel : public HbmModel {
 public:
     LatentHyperModel(const ModelDir& dir, Config* p);
-    ~LatentHyperModel() override {
-        for (void* b : bufs_) device_free(b);
-    }
     void init_kv(KVCacheManager* mgr, int block_size, int num_blocks) override;
     void forward(const PassArgs& a) override;
 
@@ -81,53 +71,13 @@ private:
     const float* first_record_ = nullptr;   // input weights and alpha of the first sublayer
     const void* embed_ = nullptr;
     B16Weight head_;
-    std::vector<void*> bufs_;
 
-    void* alloc(size_t bytes, const char* what) {
-        void* d = nullptr;
-        if (device_malloc(&d, bytes) != 0) NVLLM_FATAL("cannot allocate %zu bytes of HBM for %s", bytes, what);
-        bufs_.push_back(d);
-        return d;
-    }
-    float* upload(const std::vector<float>& v) {
-        float* d = (float*)alloc(v.size() * sizeof(float), "a vector");
-        device_memcpy(d, v.data(), v.size() * sizeof(float), HOST_TO_DEVICE);
-        return d;
-    }
-    float* vec(const ModelDir& dir, const std::string& name, int n, int n_pad) {
-        std::vector<float> v((size_t)n_pad, 0.f);
-        dir.read_f32(name, {n}, v.data());
-        return upload(v);
-    }
-    float* matrix_f32(const ModelDir& dir, const std::string& name, int rows, int cols) {
-        std::vector<float> v((size_t)rows * cols);
-        dir.read_f32(name, {rows, cols}, v.data());
-        return upload(v);
-    }
-    // row-major bf16 [N][K] on the host -> tiles in HBM
-    B16Weight tile(const std::vector<uint16_t>& rm, int N, int K, int groups = 1);
     LatentPool pool(const KVCacheManager* mgr, int run) const;
     size_t pool_bytes(int block_size, int num_blocks, int runs) const;   // of the first `runs` cache slices
     void load_layer(const ModelDir& dir, int i, const Json& cfg);
     void forward_b16(const PassArgs& a, const StepArrays& st);
     void forward_f32(const PassArgs& a, const StepArrays& st);
 };
-
-B16Weight LatentHyperModel::tile(const std::vector<uint16_t>& rm, int N, int K, int groups) {
-    const int Kp = pad32(K), Nb = cdiv(N, 16);
-    B16Weight w;
-    w.N = N;
-    w.K = Kp;
-    w.groups = groups;
-    __half* tiles = (__half*)alloc((size_t)Nb * (Kp / 32) * TILE_HALVES * 2, "a projection");
-    void* stage = nullptr;
-    if (device_malloc(&stage, rm.size() * 2) != 0) NVLLM_FATAL("no memory for a load buffer of %zu bytes", rm.size() * 2);
-    device_memcpy(stage, rm.data(), rm.size() * 2, HOST_TO_DEVICE);
-    launch_tile_weights(tiles, (const __half*)stage, N, K, (long)(Kp / 32) * TILE_HALVES);   // moves 16-bit patterns
-    device_free(stage);
-    w.tiles = tiles;
-    return w;
-}
 
 void LatentHyperModel::load_layer(const ModelDir& dir, int i, const Json& cfg) {
     const std::string at = "layers[" + std::to_string(i) + "]", L = "l" + std::to_string(i) + ".", M = L + "mix.", P = L + "mlp.";

@@ -136,6 +136,7 @@ static const struct {
     const char* name;
     DirModelLoader load;
 } kArchitectures[] = {
+    {"Simivik", load_hybrid_model},
     {"Suselorn", load_latent_hyper_model},
 };
 static DirModelLoader find_architecture(const char* name) {
@@ -631,6 +632,12 @@ void nvllm_init_model_kv(KVCacheManager* mgr, int block_size, int num_blocks, co
     ModelPriv* m = (ModelPriv*)w->_data_buffer;
     if (m && m->dir) m->dir->init_kv(mgr, block_size, num_blocks);
     else init_kv_cache_manager(mgr, block_size, num_blocks, p->n_layers, p->n_kv_heads, p->head_dim);
+}
+
+void nvllm_init_model_states(const Weights* w, int n_slots) {
+    ensure_init();
+    ModelPriv* m = (ModelPriv*)w->_data_buffer;
+    if (m && m->dir) m->dir->init_states(n_slots);
 }
 
 void nvllm_free_model(Weights* w) {

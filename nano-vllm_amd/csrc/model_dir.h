@@ -67,10 +67,34 @@ class DirModel {
 public:
     virtual ~DirModel() {}
     virtual void init_kv(KVCacheManager* mgr, int block_size, int num_blocks) = 0;
+    // room for the state that `slots` sequences carry from token to token (a sequence's slot is its id)
+    virtual void init_states(int slots) { (void)slots; }
     virtual void forward(const PassArgs& a) = 0;
 };
+
+// What designs share: tensors on their way from the file to HBM.
+class HbmModel : public DirModel {
+public:
+    ~HbmModel() override {
+        for (void* b : bufs_) device_free(b);
+    }
+
+protected:
+    void* alloc(size_t bytes, const char* what);
+    float* upload(const std::vector<float>& v);
+    float* vec(const ModelDir& dir, const std::string& name, int n, int n_pad);   // padded with zeros
+    float* matrix_f32(const ModelDir& dir, const std::string& name, int rows, int cols);
+    // row-major bf16 [N][K] on the host -> tiles in HBM, K padded to 32
+    B16Weight tile(const std::vector<uint16_t>& rm, int N, int K, int groups = 1);
+
+private:
+    std::vector<void*> bufs_;
+};
+[[noreturn]] void bad_config(const char* what);   // ends the process with a message about config.json
+inline int pad32(int n) { return (n + 31) & ~31; }
 typedef DirModel* (*DirModelLoader)(const ModelDir& dir, Config* p);
 DirModel* load_latent_hyper_model(const ModelDir& dir, Config* p);   // latent_model.hip
+DirModel* load_hybrid_model(const ModelDir& dir, Config* p);         // hybrid_model.hip
 
 // ops_api.hip: host bookkeeping of a block pool whose storage is ONE HBM buffer of `bytes` bytes (pool_v stays null)
 void init_block_pool(KVCacheManager* mgr, int block_size, int num_blocks, size_t bytes);

@@ -1,4 +1,4 @@
-// model_dir.hip -- reading a model folder (model_dir.h).  Host code only.
+// model_dir.hip -- reading a model folder, and its tensors' way to HBM (model_dir.h).
 #include "model_dir.h"
 
 #include <cstring>
@@ -104,6 +104,48 @@ void ModelDir::read_bf16(const std::string& name, const std::vector<long>& shape
     } else {
         die("tensor '" + name + "' has type " + t.dtype + ", a bf16 or fp32 tensor was expected");
     }
+}
+
+void bad_config(const char* what) {
+    fprintf(stderr, "nvllm: config.json: %s\n", what);
+    exit(1);
+}
+
+void* HbmModel::alloc(size_t bytes, const char* what) {
+    void* d = nullptr;
+    if (device_malloc(&d, bytes) != 0) NVLLM_FATAL("cannot allocate %zu bytes of HBM for %s", bytes, what);
+    bufs_.push_back(d);
+    return d;
+}
+float* HbmModel::upload(const std::vector<float>& v) {
+    float* d = (float*)alloc(v.size() * sizeof(float), "a vector");
+    device_memcpy(d, v.data(), v.size() * sizeof(float), HOST_TO_DEVICE);
+    return d;
+}
+float* HbmModel::vec(const ModelDir& dir, const std::string& name, int n, int n_pad) {
+    std::vector<float> v((size_t)n_pad, 0.f);
+    dir.read_f32(name, {n}, v.data());
+    return upload(v);
+}
+float* HbmModel::matrix_f32(const ModelDir& dir, const std::string& name, int rows, int cols) {
+    std::vector<float> v((size_t)rows * cols);
+    dir.read_f32(name, {rows, cols}, v.data());
+    return upload(v);
+}
+B16Weight HbmModel::tile(const std::vector<uint16_t>& rm, int N, int K, int groups) {
+    const int Kp = pad32(K), Nb = cdiv(N, 16);
+    B16Weight w;
+    w.N = N;
+    w.K = Kp;
+    w.groups = groups;
+    __half* tiles = (__half*)alloc((size_t)Nb * (Kp / 32) * TILE_HALVES * 2, "a projection");
+    void* stage = nullptr;
+    if (device_malloc(&stage, rm.size() * 2) != 0) NVLLM_FATAL("no memory for a load buffer of %zu bytes", rm.size() * 2);
+    device_memcpy(stage, rm.data(), rm.size() * 2, HOST_TO_DEVICE);
+    launch_tile_weights(tiles, (const __half*)stage, N, K, (long)(Kp / 32) * TILE_HALVES);   // moves 16-bit patterns
+    device_free(stage);
+    w.tiles = tiles;
+    return w;
 }
 
 }  // namespace nvllm

@@ -179,6 +179,18 @@ enum ProfClass {
     PC_LATENT_ATTN_TOK,  // ... and single tokens
     PC_LATENT_COMBINE,
     PC_HYPER,            // hyper-connection update and norm as a launch of its own
+    PC_CONV_ROPE,        // short convolution over time, rotation, cache write
+    PC_WINDOW_ATTN,      // windowed attention: prompt portions ...
+    PC_WINDOW_ATTN_TOK,  // ... and single tokens
+    PC_LIGHTNING,        // linear attention with decay: prompt portions ...
+    PC_LIGHTNING_TOK,    // ... and single tokens
+    PC_GEMM_ROUTER,      // mixture of experts: router logits ...
+    PC_ROUTE,            // ... choice and sorting ...
+    PC_GEMM_EXPERT_UP,   // ... the chosen experts' two products ...
+    PC_GEMM_EXPERT_DOWN,
+    PC_GEMM_SHARED_UP,   // ... the shared expert's ...
+    PC_GEMM_SHARED_DOWN,
+    PC_MOE_COMBINE,      // ... and the sum of their results
     PC_COUNT
 };
 hipEvent_t prof_start_event();   // events of the enclosing ProfScope, or null when timing is off
@@ -216,7 +228,8 @@ struct GemmEpilogue {
         LATENT_IN = 6,   // query latent * gain -> tiles + sums of squares; key/value latent and rotated key part -> fp32 rows
         LATENT_Q = 7,    // unrotated query parts -> tiles; rotated parts -> query rows
         HYPER_2 = 8,     // hyper-connection update of up to 2 (4) residual streams, and the next sublayer's
-        HYPER_4 = 9      //   input (their weighted sum through the Dynamic Tanh norm) -> tiles
+        HYPER_4 = 9,     //   input (their weighted sum through the Dynamic Tanh norm) -> tiles
+        RESID_B16 = 10   // x += result; x * gain -> tiles; sums of squares: RESID_A16 with one bf16 plane
     } kind = F32;
     // Input normalisation.  When ss_in is set the activations fed to the projection are
     // x * gain (not yet divided by the RMS) and the result is scaled per token by
@@ -258,6 +271,11 @@ struct GemmEpilogue {
     // ---- bf16 models
     const float* bias = nullptr;   // SWIGLU_A16, HYPER_*: one fp32 per output feature, added before anything else
     float softcap = 0.f;           // F32: out = softcap * tanh(out / softcap) when positive
+    // ROWS_B16: features [0, silu_to) go through z * sigmoid(z);  TILE_B16: max(z, 0)^2 when relu2
+    int silu_to = 0;
+    bool relu2 = false;
+    // SWIGLU_A16: both halves of token t's input are scaled by row_weight[t] (the product is linear up to here)
+    const float* row_weight = nullptr;
     // LATENT_IN: features [0, latent_q) are the query latent (gain_next, a16_out, ss_out), the rest goes to out[t, ldo]
     int latent_q = 0;
     // LATENT_Q: features [0, q_plain) are the unrotated parts (a16_out); then per head rot_ld features, rotated by
@@ -352,6 +370,16 @@ struct B16Weight {
 static inline size_t b16_halves(int tokens, int K) { return (size_t)cdiv(tokens, 16) * cdiv(K, 32) * TILE_HALVES; }
 struct LatentKvRider;   // gemm_common.h: cache rows written by extra workgroups of a LATENT_Q launch
 void launch_gemm_b16(const B16Weight& w, const __half* act, int T, const GemmEpilogue& epi, int prof_cls, const LatentKvRider* ride = nullptr);
+// Rows sorted by expert (moe.h): every group of `pad` rows meets the matrix of ONE expert.
+struct ExpertRows {
+    const int* block_expert;   // [capacity / 16] expert of each 16-row block, -1: no rows (the same within a group)
+    const int* source;         // row -> row of the activations, null: rows are the activations' own
+    int capacity;              // rows, a multiple of pad: an upper bound known to the host
+    int pad;                   // 16, 32, 64 or 128
+    int live;                  // expected number of rows (bytes and flops of the kernel timing)
+};
+// w: [experts][N][K] stacked, N a multiple of 32.  Kinds SWIGLU_A16 and F32.
+void launch_gemm_experts(const B16Weight& w, int experts, const __half* act, const ExpertRows& rows, const GemmEpilogue& epi, int prof_cls);
 
 void launch_pack_a16(__half* a16, const float* in, int T, int K);
 void launch_matmul_f32w(float* out, const float* in, const float* w, int T, int K, int N);
@@ -434,6 +462,8 @@ struct HyperStep {
 void launch_hyper_step(const HyperStep& h, int T);
 // every stream of token t = its embedding row (fp32 or bf16 table rows of ld values); tok_src / prev as in launch_embed_prescale
 void launch_embed_streams(float* x, const void* table, bool bf16, const int* tokens, int T, int streams, int ld, const int* tok_src, const int* prev);
+// x[t,:] = table row (bf16, ld values); act = x * gain tiles; ss per 32 features; tok_src / prev as in launch_embed_prescale
+void launch_embed_norm_b16(float* x, __half* act, float* ss, const void* table, const int* tokens, const float* gain, int T, int ld, const int* tok_src, const int* prev);
 void launch_gather_b16(__half* dst, const __half* src, const int* idx, int B, int K);   // rows of activation tiles
 void launch_swiglu_bias(float* out, const float* g, const float* u, const float* bg, const float* bu, int T, int F);
 void launch_softcap(float* x, float cap, long n);

@@ -50,7 +50,7 @@ KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim) {
 // pinned region and upload it with a single copy.
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
-                      int pos0, int block_size, int attn_ct, const int* token_src, bool multi_first) {
+                      int pos0, int block_size, int attn_ct, const int* token_src, bool multi_first, bool spans) {
     StepArrays s{};
     s.T = T;
     s.B = B;
@@ -144,6 +144,29 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
         }
     }
     s.n_runs = (int)runs.size() / 4;
+    std::vector<int> span, span_of;
+    if (spans) {
+        auto pos_of = [&](int t) { return pos_arr ? pos_arr[t] : pos0 + t; };
+        auto seq_of = [&](int t) { return seq_ids ? seq_ids[t] : 0; };
+        std::vector<char> seen(n_seqs, 0);
+        span_of.resize(T);
+        for (int pass = 0; pass < 2; pass++)   // portions of several tokens, then single tokens
+            for (int t = 0; t < T;) {
+                int n = 1;
+                while (t + n < T && seq_of(t + n) == seq_of(t) && pos_of(t + n) == pos_of(t + n - 1) + 1) n++;
+                if ((n > 1) == (pass == 0)) {
+                    if (seen[seq_of(t)]) s.seq_split = true;
+                    seen[seq_of(t)] = 1;
+                    for (int i = 0; i < n; i++) span_of[t + i] = (int)span.size() / 4;
+                    span.insert(span.end(), {t, n, pos_of(t), seq_of(t)});
+                    if (n > s.max_span) s.max_span = n;
+                }
+                t += n;
+                if (pass == 0) s.n_spans_multi = (int)span.size() / 4;
+            }
+        s.n_spans = (int)span.size() / 4;
+        s.host_spans = span;
+    }
     // where each token's K/V row goes: resolves position -> (block table entry, slot) on
     // the host so the kernels that store K/V need one load instead of a chain of three
     std::vector<int> kv_row;
@@ -156,7 +179,7 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
         }
     }
     const size_t n_ints = (size_t)(tokens ? T : 0) + (token_src ? T : 0) + (pos_arr ? T : 0) + (seq_ids ? T : 0) + kv_row.size() +
-                          (output_indices ? B : 0) + n_seqs + total_tbl + runs.size() + 64;
+                          (output_indices ? B : 0) + n_seqs + total_tbl + runs.size() + span.size() + span_of.size() + 64;
     int* host = pinned_ints(n_ints);
     int* dev = (int*)ws_get(WS_STEP, n_ints * sizeof(int));
     size_t o = 0;
@@ -193,6 +216,8 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
     }
     o = (o + 3) & ~(size_t)3;  // int4 alignment
     s.d_runs = runs.empty() ? nullptr : put(runs.data(), runs.size());
+    s.d_spans = span.empty() ? nullptr : put(span.data(), span.size());
+    s.d_span_of = span_of.empty() ? nullptr : put(span_of.data(), span_of.size());
     if (o > 0) {
         static const int by_kernel = getenv("NVLLM_STAGE_COPY") ? atoi(getenv("NVLLM_STAGE_COPY")) == 0 : 1;
         if (by_kernel && o <= (1u << 16)) launch_copy_ints(dev, host, o);   // small: a kernel reads the pinned region itself

@@ -1,5 +1,8 @@
 // step_arrays.h -- device copies of the host-side description of one ragged batch.
 #pragma once
+#include <algorithm>
+#include <vector>
+
 #include "nvllm_internal.h"
 
 namespace nvllm {
@@ -28,6 +31,29 @@ struct StepArrays {
     long kv_rows_single;     // ... positions those others see
     int runs_in_tb[4];       // runs that touch each of the first four 16-token blocks
     bool one_token_per_seq;  // no sequence contributes more than one token (a pure decode step)
+    // with `spans`: every sequence's portion of the batch as a whole (models whose layers carry a state from token to token)
+    int* d_spans;            // [n_spans][4] (first token, count, first position, sequence); portions of several tokens come first
+    int* d_span_of;          // [T] the span of each token
+    int n_spans, n_spans_multi;
+    int max_span;            // tokens of the longest
+    bool seq_split;          // some sequence's tokens do not lie side by side at consecutive positions
+    std::vector<int> host_spans;
+    // Kernel timing, when a token sees at most `limit` positions: rows of K/V that the portions of several tokens (of one
+    // token) see, each counted once, and (token, position) pairs of the former.
+    long multi_rows(long limit) const { return count(0, n_spans_multi, limit, false); }
+    long multi_pairs(long limit) const { return count(0, n_spans_multi, limit, true); }
+    long single_rows(long limit) const { return count(n_spans_multi, n_spans, limit, false); }
+
+private:
+    long count(int from, int to, long limit, bool pairs) const {
+        long n = 0;
+        for (int i = from; i < to; i++) {
+            const long toks = host_spans[4 * i + 1], p0 = host_spans[4 * i + 2], last = p0 + toks;   // sees p0 + 1 .. last positions
+            const long rising = std::max(0L, std::min(last, limit) - p0);                          // tokens below the limit
+            n += pairs ? rising * p0 + rising * (rising + 1) / 2 + (toks - rising) * limit : std::min(last, limit + toks - 1);
+        }
+        return n;
+    }
 };
 
 // Copies the arrays into the pinned ring, lays the block tables of the sequences
@@ -38,7 +64,8 @@ struct StepArrays {
 // consecutive positions.  multi_first: runs of several tokens come before those of one.
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
-                      int pos0, int block_size, int attn_ct = 0, const int* token_src = nullptr, bool multi_first = false);
+                      int pos0, int block_size, int attn_ct = 0, const int* token_src = nullptr, bool multi_first = false,
+                      bool spans = false);
 
 KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim);
 

@@ -50,6 +50,9 @@ extern int nvllm_get_logits_mode(void) __attribute__((weak));
 extern void nvllm_init_model_kv(KVCacheManager* mgr, int block_size, int num_blocks, const Config* p, const Weights* w)
     __attribute__((weak));
 
+/* Optional: a backend whose models carry a state per sequence. */
+extern void nvllm_init_model_states(const Weights* w, int n_slots) __attribute__((weak));
+
 struct NvllmEngine {
     NvllmEngineOptions opt;
     Config config;
@@ -136,6 +139,7 @@ NvllmEngine* nvllm_engine_create(const char* model_path, int n_seqs, const Nvllm
     if (pool_blocks <= 0) pool_blocks = n_seqs * e->max_blocks_per_seq; /* main.c:189-193 */
     if (nvllm_init_model_kv) nvllm_init_model_kv(&g_kv_manager, bs, pool_blocks, &e->config, &e->weights);
     else init_kv_cache_manager(&g_kv_manager, bs, pool_blocks, e->config.n_layers, e->config.n_kv_heads, e->config.head_dim);
+    if (nvllm_init_model_states) nvllm_init_model_states(&e->weights, n_seqs);
     for (int i = 0; i < n_seqs; i++) {
         Sequence* s = &e->seqs[i];
         s->id = i;
