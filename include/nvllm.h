@@ -109,6 +109,33 @@ void nvllm_latent_cache_write(KVCacheManager* mgr, BlockTable** block_tables, in
 void nvllm_latent_attention(float* out, const float* q, KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr,
                             const float* sink, float scale, int n_heads, int rank, int rot, int elem_bytes, int num_tokens);
 
+/* Windowed attention (one layer): a pool of kv_heads key heads (dim values) and value heads (vdim) per position, fp32
+ * rows (elem_bytes 4) or bf16 pages of 16 positions (elem_bytes 2). */
+void nvllm_window_pool_init(KVCacheManager* mgr, int block_size, int num_blocks, int kv_heads, int dim, int vdim, int elem_bytes);
+/* raw [num_tokens][channels], channels = n_heads*dim query, kv_heads*dim key, kv_heads*vdim value:
+ *   y_t = sum_j taps[j][channel] u_(t - n_taps + 1 + j) per sequence, zeros before its start (taps null: y = u), the last
+ *   n_taps - 1 inputs kept in state [slot = sequence id][n_taps - 1][channels] (elem_bytes each);
+ *   dimension i < rot/2 of query and key heads turns with i + rot/2 by pos * base^(-2i/rot);
+ *   queries -> q [num_tokens][n_heads][dim], keys and values -> the pool.  A sequence's tokens lie side by side. */
+void nvllm_conv_rope(float* q, const float* raw, const float* taps, int n_taps, void* state, KVCacheManager* mgr, BlockTable** block_tables,
+                     int* seq_ids, int* pos_arr, double base, int rot, int n_heads, int kv_heads, int dim, int vdim, int elem_bytes, int num_tokens);
+/* out [num_tokens][n_heads][vdim]: softmax of cap * tanh(scale q.k / cap) (cap 0: of scale q.k) over the positions j <= i
+ * with i - j < size or j < keep_first. */
+void nvllm_window_attention(float* out, const float* q, KVCacheManager* mgr, BlockTable** block_tables, int* seq_ids, int* pos_arr, float scale,
+                            float cap, int size, int keep_first, int n_heads, int kv_heads, int dim, int vdim, int elem_bytes, int num_tokens);
+
+/* Linear attention with decay: per head S <- decay S + k v^T, o = S^T q, state [slot = sequence id][heads][dim][vdim], empty
+ * at position 0.  decay: host, one per head.  elem_bytes 4: out = o [num_tokens][heads][vdim].  elem_bytes 2 (q, k, v and
+ * gate rounded to bf16): out = o * gain * sigmoid(gate), ss[t] = sum over heads of o^2 (null: not wanted). */
+void nvllm_lightning(float* out, float* ss, const float* q, const float* k, const float* v, const float* gate, const float* gain,
+                     const float* decay, float* state, int* seq_ids, int* pos_arr, int heads, int dim, int vdim, int elem_bytes, int num_tokens);
+
+/* Mixture of experts on in [num_tokens][dim] with router logits z [num_tokens][experts]: the `top` largest are chosen, s =
+ * sigmoid of their logits; out = sum over them of down(silu(gate(s in)) * up(s in)).  gate, up [experts][ff][dim], down
+ * [experts][dim][ff].  choice, score [num_tokens][top]: wanted when not null; out null: only these. */
+void nvllm_expert_ff(float* out, int* choice, float* score, const float* in, const float* z, const float* gate, const float* up, const float* down,
+                     int dim, int ff, int experts, int top, int elem_bytes, int num_tokens);
+
 /* -------------------------------------------------- one launch per decode step */
 /* No counterpart in the reference, whose layer loop (src/model.c:358-394) calls one operator
  * after the other.  With the switch on (off by default; environment NVLLM_DECODE_CHAIN=1 turns it

@@ -175,6 +175,13 @@ _HIP_ONLY = {
                                       _F, C.c_double, _I, _I, _I, _I]),
     "nvllm_latent_attention": (_V, [_P, _P, C.POINTER(KVCacheManager), C.POINTER(C.POINTER(BlockTable)), c_int_p, c_int_p,
                                     _P, _F, _I, _I, _I, _I, _I]),
+    "nvllm_window_pool_init": (_V, [C.POINTER(KVCacheManager), _I, _I, _I, _I, _I, _I]),
+    "nvllm_conv_rope": (_V, [_P, _P, _P, _I, _P, C.POINTER(KVCacheManager), C.POINTER(C.POINTER(BlockTable)), c_int_p, c_int_p, C.c_double,
+                             _I, _I, _I, _I, _I, _I, _I]),
+    "nvllm_window_attention": (_V, [_P, _P, C.POINTER(KVCacheManager), C.POINTER(C.POINTER(BlockTable)), c_int_p, c_int_p, _F, _F,
+                                    _I, _I, _I, _I, _I, _I, _I, _I]),
+    "nvllm_lightning": (_V, [_P, _P, _P, _P, _P, _P, _P, C.POINTER(C.c_float), _P, c_int_p, c_int_p, _I, _I, _I, _I, _I]),
+    "nvllm_expert_ff": (_V, [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I]),
     "nvllm_prof_enable": (_V, [_I]),
     "nvllm_prof_reset": (_V, []),
     "nvllm_prof_num_classes": (_I, []),

@@ -11,7 +11,7 @@ struct RoutePlan {
     int T, E, top, pad;
     int capacity;          // rows, a multiple of pad: no batch of T tokens needs more
     int* block_expert;     // [capacity / 16]
-    int* source;           // [capacity] row -> token (padding: token 0)
+    int* source;           // [capacity] row -> token (padding and unused rows: token 0)
     float* weight;         // [capacity] row -> its expert's score (padding: 0)
     int* row_of;           // [T][top] row of a token's j-th choice
     int* choice;           // [T][top] expert

@@ -109,8 +109,11 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
     }
     __syncthreads();
     const int used = start[r.E];
-    for (int b = tid; b < r.capacity / 16; b += 1024)
-        if (b * 16 >= used) r.block_expert[b] = -1;
+    for (int b = used / 16 + tid; b < r.capacity / 16; b += 1024) r.block_expert[b] = -1;
+    for (int i = used + tid; i < r.capacity; i += 1024) {   // (a tile may look up rows behind its own: they name a token too)
+        r.source[i] = 0;
+        r.weight[i] = 0.f;
+    }
     for (int e = tid >> 4; e < r.E; e += 64) {   // 16 threads per expert: its blocks, and the padding of its segment
         const int lo = start[e], hi = start[e + 1], n = cursor[e];
         for (int b = lo / 16 + (tid & 15); b < hi / 16; b += 16) r.block_expert[b] = e;

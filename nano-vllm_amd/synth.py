@@ -173,9 +173,9 @@ def make_requests(n: int, prompt_lo: int, prompt_hi: int, vocab_size: int, seed:
 
 
 # ------------------------------------------------------------------ model folders
-# config.json + model.safetensors (random bf16 weights) of the "Suselorn" design.  Test-sized models come with
-# weights that make every mechanism matter (attention scores of several units, sinks of their size, streams that
-# mix); `plain=True` writes the same tensors from one repeated random block, for benchmark-sized files.
+# config.json + model.safetensors (random bf16 weights) of the "Suselorn" and "Simivik" designs.  Test-sized models
+# come with weights that make every mechanism matter (attention scores of several units, sinks of their size, streams
+# that mix, routers without close calls); `plain=True` writes the same tensors from one repeated random block, for benchmark-sized files.
 
 def latent_mixer(heads, dim, rot_dim, vdim, kv_rank, q_rank, scale=None, base=10000.0) -> dict:
     return dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank,
@@ -226,6 +226,81 @@ def latent_tensors(cfg: dict) -> dict:
     return out
 
 
+def lightning_mixer(heads, dim, vdim, decay=None) -> dict:
+    """decay: one number per head; default: half-lives from about a token to hundreds."""
+    if decay is None:
+        decay = [float(np.exp(-0.7 * 0.35 ** i)) for i in range(heads)]
+    return dict(heads=heads, dim=dim, vdim=vdim, decay=[float(d) for d in decay])
+
+
+def window_mixer(heads, kv_heads, dim, vdim, size, keep_first, taps=4, rot=None, base=10000.0, scale=None, softcap=30.0) -> dict:
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=taps, mask=dict(size=size, keep_first=keep_first), softcap=softcap,
+                rot=dict(base=float(base), dims=dim if rot is None else rot), scale=float(dim ** -0.5 if scale is None else scale))
+
+
+def expert_mlp(ff, experts, top, shared_ff=None) -> dict:
+    return dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top), shared=None if shared_ff is None else dict(ff=shared_ff))
+
+
+def hybrid_config(width, vocab, layers, eps=1e-5) -> dict:
+    """layers: (mixer dict, feed-forward) per layer -- the feed-forward a width (dense), an expert_mlp() or None -- or the
+    index of the layer whose tensors it shares."""
+    out = []
+    for layer in layers:
+        if isinstance(layer, int):
+            out.append(dict(out[layer], weights_of=layer))
+            continue
+        mixer, mlp = layer
+        out.append(dict(type="lightning" if "decay" in mixer else "attention", mixer=mixer, mlp=dict(kind="dense", ff=mlp) if isinstance(mlp, int) else mlp))
+    return dict(architecture="Simivik", width=width, vocab=vocab, norm=dict(eps=eps), layers=out)
+
+
+def hybrid_tensors(cfg: dict) -> dict:
+    D = cfg["width"]
+    out = {"embed": ((cfg["vocab"], D), "routed_embed")}
+    for i, layer in enumerate(cfg["layers"]):
+        if "weights_of" in layer:
+            continue
+        p, m, mlp = f"l{i}.", layer["mixer"], layer["mlp"]
+        out[p + "norm1"] = ((D,), "routed_zero_gain")
+        if mlp:
+            out[p + "norm2"] = ((D,), "routed_zero_gain")
+        x, H = p + "mix.", m["heads"]
+        G = m.get("kv_heads", H)
+        sizes = dict(q=H * m["dim"], k=G * m["dim"], v=G * m["vdim"])
+        for n, rows in sizes.items():
+            out[x + n] = ((rows, D), "matrix" if n == "v" else "sharp")
+        if layer["type"] == "lightning":
+            out[x + "g"] = ((H * m["vdim"], D), "matrix")
+            out[x + "norm"] = ((H * m["vdim"],), "gain")
+        elif m["conv"]:
+            for n, rows in sizes.items():
+                out[f"{x}{n}.conv"] = ((rows, m["conv"]), "taps")
+        out[x + "o"] = ((D, H * m["vdim"]), "routed_out")
+        x = p + "mlp."
+        if mlp and mlp["kind"] == "dense":
+            out[x + "up"], out[x + "down"] = ((mlp["ff"], D), "matrix"), ((D, mlp["ff"]), "routed_out")
+        elif mlp:
+            parts = [(f"{x}e{e}.", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])]
+            if mlp.get("shared"):
+                parts.append((x + "shared.", mlp["shared"]["ff"]))
+                out[x + "shared.sg"] = ((1, D), "matrix")
+            for n, ff in parts:
+                out[n + "gate"], out[n + "up"], out[n + "down"] = ((ff, D), "matrix"), ((ff, D), "matrix"), ((D, ff), "routed_out")
+            out[x + "router"] = ((mlp["router"]["experts"], D), "router")
+    out["final.norm"] = ((D,), "zero_gain")
+    return out
+
+
+def _routed_dims(cfg) -> int:
+    """The first dims of the residual belong to the routers of test-sized models: a token's embedding holds its experts' order
+    there, well apart, and no layer writes to them -- so that the choice never hangs on rounding."""
+    return max([l["mlp"]["router"]["experts"] for l in cfg.get("layers", []) if l.get("mlp") and l["mlp"]["kind"] == "moe"], default=0)
+
+
+DESIGN_TENSORS = {"Suselorn": latent_tensors, "Simivik": hybrid_tensors}
+
+
 def to_bf16(a: np.ndarray) -> np.ndarray:
     """fp32 -> bf16 bit patterns, to nearest even."""
     u = np.ascontiguousarray(a, np.float32).view(np.uint32)
@@ -236,13 +311,21 @@ def from_bf16(u: np.ndarray) -> np.ndarray:
     return (u.astype(np.uint32) << 16).view(np.float32)
 
 
-def _latent_values(shape, kind, rng) -> np.ndarray:
+def _tensor_values(shape, kind, rng, routed=0) -> np.ndarray:
+    if kind.startswith("routed_"):
+        v = _tensor_values(shape, kind[7:], rng)
+        if kind == "routed_embed" and routed:   # every row a permutation of evenly spaced numbers
+            v[:, :routed] = (rng.permuted(np.tile(np.arange(routed), (shape[0], 1)), axis=1) - (routed - 1) / 2)
+        else:
+            v[:routed] = 0.0
+        return v
     n = rng.standard_normal(shape)
     fan = shape[-1] if shape else 1
     return {"embed": lambda: n, "matrix": lambda: n * fan ** -0.5, "sharp": lambda: n * 1.7 * fan ** -0.5,
             "gain": lambda: 1.0 + 0.2 * n, "bias": lambda: 0.2 * n, "alpha": lambda: 0.6 + 0.2 * rng.random(shape),
             "sink": lambda: 1.5 + 2.0 * n, "weight": lambda: 0.4 + 0.8 * rng.random(shape),
-            "mix": lambda: 0.9 * np.eye(fan) + 0.2 * n}[kind]()
+            "mix": lambda: 0.9 * np.eye(fan) + 0.2 * n, "zero_gain": lambda: 0.2 * n, "out": lambda: n * fan ** -0.5,
+            "taps": lambda: 0.4 * n + np.eye(fan)[-1], "router": lambda: np.eye(*shape) * 1.5 + 0.005 * n}[kind]()
 
 
 def write_model_dir(path: str, cfg: dict, seed: int = 0, plain: bool = False, edit=None) -> dict:
@@ -251,7 +334,7 @@ def write_model_dir(path: str, cfg: dict, seed: int = 0, plain: bool = False, ed
     import json
     os.makedirs(path, exist_ok=True)
     rng = np.random.Generator(np.random.PCG64(seed))
-    tensors = latent_tensors(cfg)
+    tensors, routed = DESIGN_TENSORS[cfg["architecture"]](cfg), _routed_dims(cfg)
     header, at = {}, 0
     for name, (shape, _) in tensors.items():
         size = 2 * int(np.prod(shape, dtype=np.int64))
@@ -266,14 +349,14 @@ def write_model_dir(path: str, cfg: dict, seed: int = 0, plain: bool = False, ed
         f.write(struct.pack("<Q", len(text)))
         f.write(text)
         for name, (shape, kind) in tensors.items():
-            if plain and kind in ("embed", "matrix", "sharp"):
-                scale = {"embed": 1.0, "matrix": shape[-1] ** -0.5, "sharp": shape[-1] ** -0.5}[kind]
+            if plain and kind in ("embed", "routed_embed", "matrix", "sharp", "routed_out", "router"):
+                scale = 1.0 if kind.endswith("embed") else shape[-1] ** -0.5
                 chunk, left = to_bf16(block * np.float32(scale)), int(np.prod(shape, dtype=np.int64))
                 while left > 0:
                     chunk[:min(left, len(chunk))].tofile(f)
                     left -= len(chunk)
                 continue
-            v = np.asarray(_latent_values(shape, kind, rng), np.float32)
+            v = np.asarray(_tensor_values(shape, kind, rng, 0 if plain else routed), np.float32)
             if edit is not None:
                 new = edit(name, v)
                 v = v if new is None else np.asarray(new, np.float32)

@@ -98,7 +98,7 @@ def lightning_mixer(h, W, name, c, eps):
 def attention_mixer(h, W, name, c):
     n = len(h)
     u = {x: h @ W[name + x].T for x in "qkv"}
-    for x in u:
+    for x in u if c["conv"] else ():
         u[x] = causal_conv(u[x], W[name + x + ".conv"])
     q, k, v = u["q"].reshape(n, c["heads"], -1), u["k"].reshape(n, c["kv_heads"], -1), u["v"].reshape(n, c["kv_heads"], -1)
     q, k = (rotate_half(x, np.arange(n), c["rot"]["base"], c["rot"]["dims"]) for x in (q, k))
