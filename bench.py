@@ -313,7 +313,15 @@ def write_design_model(which, z, args):
         if not (os.path.exists(path) and os.path.getsize(path) == 28 + 2 * shape.n_params()):
             synth.write_model(path, shape, seed=0)
         return path
-    path = os.path.join(args.model_dir, f"nvllm_suselorn_{tag}")
+    path = os.path.join(args.model_dir, f"nvllm_{which}_{tag}")
+    if which == "simivik" and not os.path.exists(os.path.join(path, "config.json")):
+        # of four layers: linear attention with a dense feed-forward, then windowed attention with experts, dense, experts.  A token
+        # meets as many feed-forward weights in a layer of experts (two of 16, and the shared one) as in a dense one.
+        window = synth.window_mixer(z["heads"], z["kv_heads"], z["dim"], z["vdim"], size=512, keep_first=16)
+        lightning, experts = synth.lightning_mixer(z["heads"], z["dim"], z["vdim"]), synth.expert_mlp(z["ff"] // 4, 16, 2, z["ff"] // 2)
+        period = [(lightning, z["ff"]), (window, experts), (window, z["ff"]), (window, experts)]
+        synth.write_model_dir(path, synth.hybrid_config(z["width"], z["vocab"], [period[i % 4] for i in range(z["layers"])]), plain=True)
+        return path
     if not os.path.exists(os.path.join(path, "config.json")):
         m = synth.latent_mixer(z["heads"], z["dim"], z["rot"], z["vdim"], z["kv_rank"], z["q_rank"])
         synth.write_model_dir(path, synth.latent_config(z["width"], z["vocab"], [(m, z["ff"])] * z["layers"], streams=2), plain=True)
@@ -382,7 +390,7 @@ def run_design(lib, path, z, args, profile):
 
 
 def bench_designs(args):
-    """--design suselorn: the design beside the closest model at equal sizes, one JSON line per size."""
+    """--design NAME: the design beside the closest model at equal sizes, one JSON line per size."""
     from nvllm_amd import capi
     lib = capi.load_hip()
     lib.nvllm_set_kv_elem_bytes(2)
@@ -394,7 +402,7 @@ def bench_designs(args):
     for size in args.sizes.split(","):
         z = dict(DESIGN_SIZES[size])
         line = dict(metric="prefill and decode tokens/s, designs at equal size", size=size, shape=z, prompt_len=args.prompt_len, chunk=args.chunk,
-                    steps=args.steps, data="synthetic", dtype={"suselorn": "bf16", "llama": "f32 (fp16 hi/lo)"}, models={})
+                    steps=args.steps, data="synthetic", dtype={args.design: "bf16", "llama": "f32 (fp16 hi/lo)"}, models={})
         for which in args.design.split(",") + ([] if args.alone else ["llama"]):
             t0 = time.time()
             path = write_design_model(which, z, args)
@@ -478,7 +486,7 @@ def main():
                     help="skip the `variants` block (N = 1 only: the same workload with the fp32 row pool and with logits rows to the host)")
     ap.add_argument("--cpu-steps", type=int, default=8, help="decode steps of the CPU baseline leg (about 1.7 s each on 16 cores); 0 disables it")
     ap.add_argument("--model-dir", default=os.environ.get("NVLLM_MODEL_DIR", "/tmp"))
-    ap.add_argument("--design", default=None, choices=("suselorn",),
+    ap.add_argument("--design", default=None, choices=("simivik", "suselorn"),
                     help="another benchmark: prefill and decode throughput of this design beside the closest model at equal sizes (bf16, random weights)")
     ap.add_argument("--sizes", default=",".join(DESIGN_SIZES), help="with --design: which of " + ", ".join(DESIGN_SIZES))
     ap.add_argument("--alone", action="store_true", help="with --design: without the closest model")

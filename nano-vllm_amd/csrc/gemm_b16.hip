@@ -98,7 +98,9 @@ void launch_dense(GemmArgs a) {
 template <int EPI, bool GRP>
 void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
     static const int pf_min_t = getenv("NVLLM_GEMM_PREFILL_T") ? atoi(getenv("NVLLM_GEMM_PREFILL_T")) : 256;
-    if (a.T >= pf_min_t) {
+    // few features: the chip fills with token groups of 16 or 32, not with dense tiles
+    const bool narrow = !GRP && EPI == GemmEpilogue::F32 && !a.e.amax_out && a.NB <= 8 && a.Tb <= 4 * rt().num_cus;
+    if (a.T >= pf_min_t && !narrow) {
         {
             ProfScope ps(prof_cls, bytes, flops);
             a.e.amax_pairs = nullptr;   // the dense-tile kernel does not emit pairs: the rows are scanned afterwards
@@ -109,7 +111,14 @@ void launch_kind(GemmArgs a, int prof_cls, double bytes, double flops) {
     }
     // a block-diagonal product has a short K and no K split; its plan is that of one group times the groups
     const int groups = GRP ? a.NB / a.group_nb : 1;
-    GemmPlan pl = gemm_plan(GRP ? a.group_nb * 16 * groups : a.N, a.Kb * 32, a.T, EPI, GRP || EPI == GemmEpilogue::F32 ? 1 : 0, 1 << 16, 0);
+    GemmPlan pl = gemm_plan(GRP ? a.group_nb * 16 * groups : a.N, a.Kb * 32, a.T, EPI, GRP || narrow || (EPI == GemmEpilogue::F32 && a.e.amax_out) ? 1 : 0, 1 << 16, 0);
+    if (narrow) {
+        pl.nw = NW;
+        pl.nbw = 2;
+        pl.TB = a.Tb * cdiv(a.NB, 2) <= rt().num_cus ? 1 : 2;
+        pl.tiles_n = cdiv(a.NB, 2);
+        pl.tiles_t = cdiv(a.Tb, pl.TB);
+    }
     if (GRP) {
         // a short K and no split: when 64-feature tiles leave half the CUs idle, 32-feature tiles x 32 or 16 tokens
         const int cus = rt().num_cus;

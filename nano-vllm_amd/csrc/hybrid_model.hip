@@ -487,7 +487,7 @@ void HybridModel::forward(const PassArgs& a) {
 void HybridModel::forward_b16(const PassArgs& a, const StepArrays& st) {
     const int T = a.T, B = a.B, x_tiles = Dp_ / 32;
     // workspaces of the widest layer
-    size_t rows = 0, raw = 0, hid = 0, heads_ss = 0, shared_hid = 0, y_rows = 0, z_ld = 0, ints = 0;
+    size_t sorted = 0, rows = 0, raw = 0, hid = 0, heads_ss = 0, shared_hid = 0, y_rows = 0, z_ld = 0, ints = 0;
     for (const auto& l : layers_) {
         const MixerSizes& m = l.m;
         const FfSizes& f = l.f;
@@ -503,6 +503,7 @@ void HybridModel::forward_b16(const PassArgs& a, const StepArrays& st) {
             const int cap = route_plan(nullptr, T, f.experts, f.top, pad).capacity;
             hid = std::max(hid, b16_halves(cap, pad32(f.expert_ff)));
             y_rows = std::max(y_rows, (size_t)cap);
+            if (pad >= 64) sorted = std::max(sorted, b16_halves(cap, Dp_));
             shared_hid = std::max(shared_hid, b16_halves(T, pad32(f.shared_ff)));
             z_ld = std::max(z_ld, (size_t)pad32(f.experts + 1));
             ints = std::max(ints, w);
@@ -520,6 +521,7 @@ void HybridModel::forward_b16(const PassArgs& a, const StepArrays& st) {
     float* y_shared = (float*)ws_get(WS_F32_B, (shared_hid ? (size_t)T * Dp_ : 0) * sizeof(float));
     float* z = (float*)ws_get(WS_F32_C, (size_t)T * z_ld * sizeof(float));
     int* route_mem = (int*)ws_get(WS_LATENT, ints * sizeof(int));
+    __half* act_sorted = (__half*)ws_get(WS_A16_SORTED, sorted * sizeof(__half));
 
     launch_embed_norm_b16(x, act, ss, embed_, st.d_tokens, layers_[source_[0]].norm[0], T, Dp_, st.d_tok_src, a.d_argmax);
     auto normed = [&](GemmEpilogue::Kind kind) {   // a projection of the normed residual
@@ -578,7 +580,11 @@ void HybridModel::forward_b16(const PassArgs& a, const StepArrays& st) {
             ExpertRows er{plan.block_expert, plan.source, plan.capacity, plan.pad, T * f.top};
             GemmEpilogue eu = normed(GemmEpilogue::SWIGLU_A16);
             eu.ss_gather = plan.source; eu.row_weight = plan.weight; eu.a16_out = wide;
-            launch_gemm_experts(w.experts_up, f.experts, act, er, eu, PC_GEMM_EXPERT_UP);
+            if (plan.pad >= 64) {   // many rows per expert: sorted once (a gathering tile copy touches a cache line per 16 bytes)
+                launch_expert_rows(act_sorted, x, w.norm[1], plan, Dp_);
+                er.source = nullptr;
+            }
+            launch_gemm_experts(w.experts_up, f.experts, er.source ? act : act_sorted, er, eu, PC_GEMM_EXPERT_UP);
             er.source = nullptr;
             GemmEpilogue ed;
             ed.kind = GemmEpilogue::F32;

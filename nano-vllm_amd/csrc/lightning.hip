@@ -86,6 +86,7 @@ __global__ __launch_bounds__(256, 2) void k_lightning_chunk(Lightning a, const i
     // ---- the chunk's rows, a chunk ahead in registers: 16-byte pieces, a row's pieces by neighbouring threads
     const int qk_pieces = a.dim_ld / 8;
     u4_t rq[DC], rk[DC], rv[2];
+    u2_t rg[4];   // this lane's gates: columns my_v + 4 g .. + 3 of tokens 16 i + x
     auto fetch = [&](int c0) {
 #pragma unroll
         for (int u = 0; u < DC; u++) {
@@ -101,6 +102,11 @@ __global__ __launch_bounds__(256, 2) void k_lightning_chunk(Lightning a, const i
             const bool live = c0 + row < n_tok && v0 + piece * 8 < a.vdim_ld;
             const __half* src = a.rows + (size_t)(span.x + c0 + row) * a.ld + 2 * a.H * a.dim_ld + h * a.vdim_ld + v0 + piece * 8;
             rv[u] = live ? *reinterpret_cast<const u4_t*>(src) : u4_t{0, 0, 0, 0};
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int tok = min(c0 + 16 * i + x, n_tok - 1);
+            rg[i] = has_v ? *reinterpret_cast<const u2_t*>(a.rows + (size_t)(span.x + tok) * a.ld + 2 * a.H * a.dim_ld + (a.H + h) * a.vdim_ld + my_v + 4 * g) : u2_t{0, 0};
         }
     };
     fetch(0);
@@ -120,6 +126,9 @@ __global__ __launch_bounds__(256, 2) void k_lightning_chunk(Lightning a, const i
             const int i = tid + 256 * u, row = i >> 3, piece = i & 7;
             *reinterpret_cast<u4_t*>(s_v + row * VROW + piece * 8) = rv[u];
         }
+        u2_t gates[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) gates[i] = rg[i];
         __syncthreads();
         if (c0 + CH < n_tok) fetch(c0 + CH);
         // operands over dims in the order of the state's registers: {32 c + 4 g .., 32 c + 16 + 4 g ..} of row 16 i + x
@@ -204,10 +213,9 @@ __global__ __launch_bounds__(256, 2) void k_lightning_chunk(Lightning a, const i
                 sq += __shfl_xor(sq, 32, 64);
                 if (tl < n) {
                     const int col = h * a.vdim_ld + my_v;
-                    const u2_t gate = *reinterpret_cast<const u2_t*>(a.rows + (size_t)t * a.ld + 2 * a.H * a.dim_ld + a.H * a.vdim_ld + col + 4 * g);
                     float y[4];
 #pragma unroll
-                    for (int r = 0; r < 4; r++) y[r] = o[r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gate[r >> 1] >> (16 * (r & 1)))));
+                    for (int r = 0; r < 4; r++) y[r] = o[r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gates[i][r >> 1] >> (16 * (r & 1)))));
                     store_b16_4(a.out_b16, Kb_out, t, col + 4 * g, y);
                     if (g == 0) a.ss_out[(size_t)t * ss_ld + (col >> 4)] = sq;
                 }

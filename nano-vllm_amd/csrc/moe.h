@@ -23,6 +23,9 @@ RoutePlan route_plan(int* mem, int T, int E, int top, int pad);
 // z: [T][ldz] router logits in columns 0 .. E-1; the `top` largest (the first of equals) are chosen
 void launch_route(const RoutePlan& r, const float* z, int ldz);
 
+// the rows x * gain of a batch in the plan's order, as activation tiles (x [T][ld])
+void launch_expert_rows(__half* dst, const float* x, const float* gain, const RoutePlan& r, int ld);
+
 // x += sum of the chosen experts' rows + sigmoid(z_shared) * shared;  then what the next sublayer needs of x
 struct MoeCombine {
     float* x;                  // [T][ld]

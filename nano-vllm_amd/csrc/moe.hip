@@ -80,17 +80,58 @@ __global__ __launch_bounds__(256) void k_route(RoutePlan r, const float* __restr
 // result does not depend on its place).
 template <bool CHOOSE>
 __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* __restrict__ z, int ldz) {
-    extern __shared__ int lds_r[];   // count / cursor [E], segment start [E + 1]
+    extern __shared__ int lds_r[];   // count / cursor [E], segment start [E + 1], CHOOSE: choices and scores [T * top]
     int* cursor = lds_r;
     int* start = lds_r + r.E;
-    const int tid = threadIdx.x, pairs = r.T * r.top;
-    if (CHOOSE) {
-        for (int t = tid >> 6; t < r.T; t += 16) route_token(r, z + (size_t)t * ldz, t, tid & 63);
-        __threadfence_block();
-    }
+    const int tid = threadIdx.x, lane = tid & 63, pairs = r.T * r.top;
+    int *choice = CHOOSE ? start + r.E + 1 : r.choice, *out_choice = r.choice;
+    float* out_score = r.score;
+    float* score = CHOOSE ? reinterpret_cast<float*>(choice + pairs) : r.score;
     for (int e = tid; e < r.E; e += 1024) cursor[e] = 0;
+    if (CHOOSE) {
+        r.choice = choice;   // (route_token fills the LDS copies)
+        r.score = score;
+        if (r.E <= 64) {   // a logit per lane, four tokens at a time
+            for (int t0 = tid >> 6; t0 < r.T; t0 += 64) {
+                float v[4];
+#pragma unroll
+                for (int u = 0; u < 4; u++) v[u] = lane < r.E ? z[(size_t)min(t0 + 16 * u, r.T - 1) * ldz + lane] : -INFINITY;
+                for (int j = 0; j < r.top; j++) {
+                    float best[4];
+                    int best_e[4];
+#pragma unroll
+                    for (int u = 0; u < 4; u++) {
+                        best[u] = v[u];
+                        best_e[u] = v[u] > -INFINITY ? lane : 64;
+                    }
+#pragma unroll
+                    for (int o = 32; o > 0; o >>= 1)
+#pragma unroll
+                        for (int u = 0; u < 4; u++) {
+                            const float w = __shfl_xor(best[u], o, 64);
+                            const int e = __shfl_xor(best_e[u], o, 64);
+                            if (w > best[u] || (w == best[u] && e < best_e[u])) {
+                                best[u] = w;
+                                best_e[u] = e;
+                            }
+                        }
+#pragma unroll
+                    for (int u = 0; u < 4; u++) {
+                        const int t = t0 + 16 * u, e = best_e[u] < r.E ? best_e[u] : 0;   // (no number compares: NaN logits)
+                        if (lane == e) v[u] = -INFINITY;
+                        if (lane == 0 && t < r.T) {
+                            choice[t * r.top + j] = e;
+                            score[t * r.top + j] = 1.f / (1.f + expf(-best[u]));
+                        }
+                    }
+                }
+            }
+        } else {
+            for (int t = tid >> 6; t < r.T; t += 16) route_token(r, z + (size_t)t * ldz, t, lane);
+        }
+    }
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) atomicAdd(cursor + r.choice[i], 1);
+    for (int i = tid; i < pairs; i += 1024) atomicAdd(cursor + choice[i], 1);
     __syncthreads();
     if (tid < 64) {   // the first wave sums the padded counts
         int base = 0;
@@ -126,10 +167,14 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
     for (int e = tid; e < r.E; e += 1024) cursor[e] = start[e];
     __syncthreads();
     for (int i = tid; i < pairs; i += 1024) {
-        const int row = atomicAdd(cursor + r.choice[i], 1);
+        const int row = atomicAdd(cursor + choice[i], 1);
         r.source[row] = i / r.top;
-        r.weight[row] = r.score[i];
+        r.weight[row] = score[i];
         r.row_of[i] = row;
+        if (CHOOSE) {
+            out_choice[i] = choice[i];
+            out_score[i] = score[i];
+        }
     }
 }
 
@@ -138,9 +183,10 @@ void launch_route(const RoutePlan& r, const float* z, int ldz) {
     if (r.E < 1 || r.E > MAX_EXPERTS || r.top < 1 || r.top > r.E) NVLLM_FATAL("routing: %d of %d experts per token", r.top, r.E);
     const size_t lds = ((size_t)2 * r.E + 1) * sizeof(int);
     const double bytes = (double)r.T * (r.E * 4.0 + r.top * 20.0);
-    if (r.T <= ROUTE_ONE) {
+    const size_t lds_one = lds + (size_t)r.T * r.top * 8;
+    if (r.T <= ROUTE_ONE && lds_one <= 64 * 1024) {
         ProfScope ps(PC_ROUTE, bytes, 0);
-        NVLLM_LAUNCH((k_route_sort<true>), dim3(1), dim3(1024), lds, r, z, ldz);
+        NVLLM_LAUNCH((k_route_sort<true>), dim3(1), dim3(1024), lds_one, r, z, ldz);
         return;
     }
     {
@@ -149,6 +195,30 @@ void launch_route(const RoutePlan& r, const float* z, int ldz) {
     }
     ProfScope ps(PC_ROUTE, (double)r.T * r.top * 28.0, 0);
     NVLLM_LAUNCH((k_route_sort<false>), dim3(1), dim3(1024), lds, r, z, ldz);
+}
+
+// A workgroup per 16 rows, a wave per tile: lane (row, k group) reads 32 bytes of its row and writes its piece of the tile.
+__global__ __launch_bounds__(256) void k_expert_rows(__half* __restrict__ dst, const float* __restrict__ x, const float* __restrict__ gain, RoutePlan r, int ld) {
+    const int blk = blockIdx.x, lane = threadIdx.x & 63, Kb = ld >> 5;
+    if (r.block_expert[blk] < 0) return;
+    const float* row = x + (size_t)r.source[blk * 16 + (lane & 15)] * ld + 8 * (lane >> 4);
+    for (int kb = threadIdx.x >> 6; kb < Kb; kb += 4) {
+        const f4_t a = *reinterpret_cast<const f4_t*>(row + kb * 32), b = *reinterpret_cast<const f4_t*>(row + kb * 32 + 4);
+        const f4_t ga = *reinterpret_cast<const f4_t*>(gain + kb * 32 + 8 * (lane >> 4)), gb = *reinterpret_cast<const f4_t*>(gain + kb * 32 + 8 * (lane >> 4) + 4);
+        b8_t v;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            v[e] = (__bf16)(a[e] * ga[e]);
+            v[4 + e] = (__bf16)(b[e] * gb[e]);
+        }
+        *reinterpret_cast<b8_t*>(dst + ((size_t)blk * Kb + kb) * TILE_HALVES + lane * 8) = v;
+    }
+}
+void launch_expert_rows(__half* dst, const float* x, const float* gain, const RoutePlan& r, int ld) {
+    if (r.T <= 0) return;
+    if (ld % 32) NVLLM_FATAL("expert rows: a row of %d is not padded to 32", ld);
+    ProfScope ps(PC_EXPERT_ROWS, (double)r.T * r.top * ld * 2.0 + (double)r.T * ld * 4.0, 0);
+    NVLLM_LAUNCH(k_expert_rows, dim3(r.capacity / 16), dim3(256), 0, dst, x, gain, r, ld);
 }
 
 // One workgroup per token.  VEC 4: eight neighbouring threads cover 32 features.

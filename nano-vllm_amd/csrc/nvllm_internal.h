@@ -135,6 +135,7 @@ enum WsSlot {
     WS_KV_RAW,      // latent attention: a batch's latents and rotated key parts before norm and rotation
     WS_Q_ROWS,      // ... its absorbed queries
     WS_LATENT,      // ... its attended latents
+    WS_A16_SORTED,  // mixture of experts: a batch's rows sorted by expert
     WS_F32_A,       // fp32 models: activations between operators
     WS_F32_B,
     WS_F32_C,
@@ -186,6 +187,7 @@ enum ProfClass {
     PC_LIGHTNING_TOK,    // ... and single tokens
     PC_GEMM_ROUTER,      // mixture of experts: router logits ...
     PC_ROUTE,            // ... choice and sorting ...
+    PC_EXPERT_ROWS,      // ... a batch's rows in that order ...
     PC_GEMM_EXPERT_UP,   // ... the chosen experts' two products ...
     PC_GEMM_EXPERT_DOWN,
     PC_GEMM_SHARED_UP,   // ... the shared expert's ...

@@ -191,7 +191,7 @@ static const char* kProfNames[PC_COUNT] = {
     "embed",      "rmsnorm",  "gemm_qkv", "gemm_wo",      "gemm_gateup", "gemm_down", "gemm_head",
     "gemm_other", "rope_kv",  "attn",     "attn_combine", "elementwise", "argmax",    "pack",
     "decode_chain", "gemm_latent_in", "gemm_latent_q", "gemm_absorb", "gemm_value", "latent_kv", "latent_attn", "latent_attn_tok", "latent_combine", "hyper",
-    "conv_rope", "window_attn", "window_attn_tok", "lightning", "lightning_tok", "gemm_router", "route", "gemm_expert_up", "gemm_expert_down",
+    "conv_rope", "window_attn", "window_attn_tok", "lightning", "lightning_tok", "gemm_router", "route", "expert_rows", "gemm_expert_up", "gemm_expert_down",
     "gemm_shared_up", "gemm_shared_down", "moe_combine"};
 
 // --------------------------------------------------------------------- init

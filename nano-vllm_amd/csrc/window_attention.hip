@@ -191,6 +191,142 @@ __global__ __launch_bounds__(256) void k_conv_rope(ConvKArgs a) {
     }
 }
 
+// The same for bf16 rows of 16-byte pieces and KEEP + 1 taps: a thread walks TOK neighbouring tokens with the taps and the
+// last KEEP inputs in registers, and on to the end of those that see the state of a portion that starts among them.
+struct alignas(16) Piece {
+    __bf16 v[8];
+};
+template <int KEEP>
+__global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int TOK) {
+    const int item = blockIdx.y * 256 + threadIdx.x, t0 = blockIdx.x * TOK;
+    if (item >= a.items) return;
+    int part, head, at, i = item;
+    if (i < a.c.H * a.items_q) {
+        part = 0;
+        head = i / a.items_q;
+        at = i - head * a.items_q;
+    } else if ((i -= a.c.H * a.items_q) < a.pool.G * a.items_k) {
+        part = 1;
+        head = i / a.items_k;
+        at = i - head * a.items_k;
+    } else {
+        i -= a.pool.G * a.items_k;
+        part = 2;
+        head = i / a.items_v;
+        at = i - head * a.items_v;
+    }
+    const int half = part == 2 ? 0 : a.c.rot >> 1, turning = half / 8;
+    const bool turns = at < turning;
+    const int d0 = turns ? at * 8 : 2 * half + (at - turning) * 8;
+    const int dim = part == 2 ? a.pool.vdim : a.pool.dim;
+    const bool live = d0 < dim;   // (past it: the padding of a query row)
+    const int ch = (part == 0 ? 0 : part == 1 ? a.QD : a.QD + a.KD) + head * dim + (live ? d0 : 0), partner = turns ? half : 0;
+    const __bf16* raw = reinterpret_cast<const __bf16*>(a.c.raw) + ch;
+    float w[KEEP + 1][8], wz[KEEP + 1][8];
+#pragma unroll
+    for (int j = 0; j <= KEEP; j++)
+#pragma unroll
+        for (int e = 0; e < 8; e += 4) {
+            const f4_t one = {1.f, 1.f, 1.f, 1.f};
+            const f4_t u = a.c.taps ? *reinterpret_cast<const f4_t*>(a.c.taps + (size_t)j * a.channels + ch + e) : one;
+            const f4_t v = a.c.taps ? *reinterpret_cast<const f4_t*>(a.c.taps + (size_t)j * a.channels + ch + partner + e) : one;
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                w[j][e + r] = u[r];
+                wz[j][e + r] = v[r];
+            }
+        }
+    Piece win[KEEP + 1], winz[KEEP + 1];   // inputs of tokens t - KEEP .. t
+    int have = -1;                         // the token they are complete for, but for its own input
+    for (int t = t0; t < T; t++) {
+        const int4 span = a.spans[a.span_of[t]];   // (first token, count, first position, sequence)
+        const int off = t - span.x;
+        const bool old_state = off > 0 && off < KEEP;
+        if (t < t0 + TOK ? old_state && span.x < t0 : !(old_state && span.x >= t0)) {
+            if (t < t0 + TOK) continue;   // belongs to the thread of the portion's first token
+            break;
+        }
+        __bf16* state = reinterpret_cast<__bf16*>(a.c.state) + (size_t)span.w * KEEP * a.channels + ch;
+        if (have != t || off == 0) {
+#pragma unroll
+            for (int j = 0; j < KEEP; j++) {
+                const int o = off - KEEP + j;
+                const Piece zero = {};
+                win[j] = winz[j] = zero;
+                if (span.z + o >= 0) {
+                    const __bf16* src = o >= 0 ? raw + (size_t)(span.x + o) * a.c.raw_ld : state + (size_t)(KEEP + o) * a.channels;
+                    win[j] = *reinterpret_cast<const Piece*>(src);
+                    winz[j] = *reinterpret_cast<const Piece*>(src + partner);
+                }
+            }
+        }
+        win[KEEP] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld);
+        winz[KEEP] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner);
+        float y[8], z[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) y[e] = z[e] = 0.f;
+#pragma unroll
+        for (int j = 0; j <= KEEP; j++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                y[e] = fmaf(w[j][e], (float)win[j].v[e], y[e]);
+                z[e] = fmaf(wz[j][e], (float)winz[j].v[e], z[e]);
+            }
+        if (turns) {
+            const float4* cs = reinterpret_cast<const float4*>(a.c.rope + (size_t)(span.z + off) * half + d0);   // {cos, sin} x 2
+#pragma unroll
+            for (int e = 0; e < 8; e += 2) {
+                const float4 r = cs[e >> 1];
+                const float u0 = y[e], v0 = z[e], u1 = y[e + 1], v1 = z[e + 1];
+                y[e] = u0 * r.x - v0 * r.y;
+                z[e] = v0 * r.x + u0 * r.y;
+                y[e + 1] = u1 * r.z - v1 * r.w;
+                z[e + 1] = v1 * r.z + u1 * r.w;
+            }
+        }
+        Piece py, pz;
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            py.v[e] = (__bf16)(live ? y[e] : 0.f);
+            pz.v[e] = (__bf16)z[e];
+        }
+        if (part == 0) {
+            __bf16* q = reinterpret_cast<__bf16*>(a.c.q_out) + ((size_t)t * a.c.H + head) * a.pool.dim_ld + d0;
+            *reinterpret_cast<Piece*>(q) = py;
+            if (turns) *reinterpret_cast<Piece*>(q + half) = pz;
+        } else if (const int row = a.kv_row[t]; row >= 0) {
+            if (part == 1) {
+                __bf16* k = reinterpret_cast<__bf16*>(a.pool.keys);
+                *reinterpret_cast<Piece*>(k + key_off(row, head, a.pool.G, d0, a.pool.dim_ld)) = py;
+                if (turns) *reinterpret_cast<Piece*>(k + key_off(row, head, a.pool.G, d0 + half, a.pool.dim_ld)) = pz;
+            } else {
+                __bf16* v = reinterpret_cast<__bf16*>(a.pool.values) + value_off(row, head, a.pool.G, d0, a.pool.vdim_ld);
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[4 * e] = py.v[e];   // (d0 is a multiple of 8: the dims stay in one tile)
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            win[j] = win[j + 1];
+            winz[j] = winz[j + 1];
+        }
+        have = t + 1;
+        if (KEEP > 0 && live && off == min(span.y, KEEP) - 1) {   // nobody needs the old state any more
+#pragma unroll
+            for (int j = 0; j < KEEP; j++) {
+                Piece u = win[j], v = winz[j];
+                if (span.y > KEEP) {
+                    const __bf16* src = raw + (size_t)(span.x + span.y - KEEP + j) * a.c.raw_ld;
+                    u = *reinterpret_cast<const Piece*>(src);
+                    v = *reinterpret_cast<const Piece*>(src + partner);
+                }
+                *reinterpret_cast<Piece*>(state + (size_t)j * a.channels) = u;
+                if (turns) *reinterpret_cast<Piece*>(state + (size_t)j * a.channels + half) = v;
+            }
+        }
+    }
+}
+
 void launch_conv_rope(const ConvRope& c, const KvPages& pool, const StepArrays& st) {
     if (st.T <= 0) return;
     if (!st.d_spans || !st.d_kv_row) NVLLM_FATAL("convolution over time: the batch was staged without its portions");
@@ -214,6 +350,18 @@ void launch_conv_rope(const ConvRope& c, const KvPages& pool, const StepArrays& 
     const double elems = (double)st.T * a.channels * 2.0;
     ProfScope ps(PC_CONV_ROPE, elems * pool.elem_bytes + (double)a.channels * c.n_taps * 4.0, elems * c.n_taps);
     const dim3 grid(st.T, cdiv(a.items, 256));
+    if (wide && c.n_taps <= 5 && (c.taps || c.n_taps == 1)) {
+        const int TOK = st.T >= 1024 ? 4 : st.T >= 256 ? 2 : 1, threads = std::min(256, (a.items + 63) & ~63);
+        const dim3 walk(cdiv(st.T, TOK), cdiv(a.items, 256));
+        switch (c.n_taps) {
+            case 1: NVLLM_LAUNCH((k_conv_rope_walk<0>), walk, dim3(threads), 0, a, st.T, TOK); break;
+            case 2: NVLLM_LAUNCH((k_conv_rope_walk<1>), walk, dim3(threads), 0, a, st.T, TOK); break;
+            case 3: NVLLM_LAUNCH((k_conv_rope_walk<2>), walk, dim3(threads), 0, a, st.T, TOK); break;
+            case 4: NVLLM_LAUNCH((k_conv_rope_walk<3>), walk, dim3(threads), 0, a, st.T, TOK); break;
+            default: NVLLM_LAUNCH((k_conv_rope_walk<4>), walk, dim3(threads), 0, a, st.T, TOK); break;
+        }
+        return;
+    }
     if (pool.elem_bytes == 4) NVLLM_LAUNCH((k_conv_rope<float, 1>), grid, dim3(256), 0, a);
     else if (wide) NVLLM_LAUNCH((k_conv_rope<__bf16, 8>), grid, dim3(256), 0, a);
     else NVLLM_LAUNCH((k_conv_rope<__bf16, 1>), grid, dim3(256), 0, a);
@@ -635,15 +783,24 @@ void launch_window_attention(const WindowAttn& w, const StepArrays& st) {
     if (st.n_multi > 0) {
         a.runs = (const int4*)st.d_runs;
         a.n_runs = st.n_multi;
-        const int C = cls == 0 ? 4 : cls == 1 ? 2 : 1;
-        a.HW = rep >= C ? C : rep >= 2 && C >= 2 ? 2 : 1;
-        a.NHG = cdiv(rep, a.HW);
-        a.n_sub = cdiv(std::min(st.max_run, WINDOW_RUN), 16 * C / a.HW);
-        const int grid = cdiv(a.G * a.n_runs * a.n_sub * a.NHG, 4);
+        // wide items share more of a page's load, narrow ones are more waves: the widest that still gives every SIMD two
+        static const int force = getenv("NVLLM_WINDOW_C") ? atoi(getenv("NVLLM_WINDOW_C")) : 0;
+        int C = cls == 0 ? 4 : cls == 1 ? 2 : 1, waves = 0;
+        for (;; C /= 2) {
+            a.HW = rep >= C ? C : rep >= 2 && C >= 2 ? 2 : 1;
+            a.NHG = cdiv(rep, a.HW);
+            a.n_sub = cdiv(std::min(st.max_run, WINDOW_RUN), 16 * C / a.HW);
+            waves = a.G * a.n_runs * a.n_sub * a.NHG;
+            if (C == 1 || (force ? C <= force : waves >= 8 * rt().num_cus)) break;
+        }
+        const int grid = cdiv(waves, 4);
         const double rows = (double)st.multi_rows(seen_cap), pairs = (double)st.multi_pairs(seen_cap);
         ProfScope ps(PC_WINDOW_ATTN, rows * kv_bytes + (double)(st.T - (st.n_runs - st.n_multi)) * io_bytes, pairs * pair_flops);
-        if (cls == 0) launch_win_cap<2, 4, 4, false>(a, grid);
-        else if (cls == 1) launch_win_cap<4, 8, 2, false>(a, grid);
+        if (cls == 0 && C == 4) launch_win_cap<2, 4, 4, false>(a, grid);
+        else if (cls == 0 && C == 2) launch_win_cap<2, 4, 2, false>(a, grid);
+        else if (cls == 0) launch_win_cap<2, 4, 1, false>(a, grid);
+        else if (cls == 1 && C == 2) launch_win_cap<4, 8, 2, false>(a, grid);
+        else if (cls == 1) launch_win_cap<4, 8, 1, false>(a, grid);
         else launch_win_cap<8, 16, 1, false>(a, grid);
     }
     const int n_single = st.n_runs - st.n_multi;
