@@ -1,13 +1,13 @@
 // lightning.hip -- linear attention with decay (lightning.h).
 //
-// k_lightning_chunk (bf16, portions of several tokens): a workgroup takes a portion's head x 64 value columns and walks
-// the portion in chunks of 64 tokens, its four waves owning 16 columns of the state each, in registers:
-//   P[s, t]  = decay^(t-s) (k_s . q_t), s <= t        one wave per 16 tokens t, to LDS as the operand of the next product
-//   o_t      = decay^(t+1) S^T q_t + sum_s P[s, t] v_s
-//   S        = decay^n S + sum_s k_s (decay^(n-1-s) v_s)^T
-// q, k and v are bf16 values.  The 32-bit factors -- S, P and the decayed v -- enter the matrix cores as three bf16
-// parts (truncations: 8 + 8 + 8 bits, together the exact value), so every product is that of the 32-bit numbers.
-// The state's result registers are already in the k order of S^T q, P's in that of P v.
+// Portions of several tokens (bf16) are cut into chunks of 64 tokens, all at once, in three launches:
+//   k_lightning_add    U_c = sum_s k_s (decay^(n-1-s) v_s)^T of every chunk
+//   k_lightning_scan   S_c = decay^n S_(c-1) + U_c over a portion's chunks, element by element; U_c gives way to S_(c-1)
+//   k_lightning_out    o_t = decay^(t+1) S_(c-1)^T q_t + sum_{s <= t} decay^(t-s) (k_s . q_t) v_s
+// A workgroup takes a chunk's head x 64 value columns, a wave 16 of them.  q, k and v are bf16 values.  The 32-bit factors
+// -- S, the decayed products P[s, t] of queries and keys, the decayed v -- enter the matrix cores as three bf16 parts
+// (truncations: 8 + 8 + 8 bits, together the exact value), so every product is that of the 32-bit numbers.  The state's
+// result registers are already in the k order of S^T q, P's in that of P v.
 //
 // k_lightning_step (single tokens, and everything in fp32): a workgroup per (portion, head), the state streamed once per
 // token as float4 columns.
@@ -21,7 +21,7 @@ typedef short s4_t __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) s4_t lds_s4;
 typedef unsigned int u2_t __attribute__((ext_vector_type(2)));
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(z * -1.44269504088896340736f)); }
 __device__ __forceinline__ float b16_f(unsigned short v) { return __builtin_bit_cast(float, (unsigned)v << 16); }
 
 // x = a + b + c exactly, each with at most 8 significant bits (their upper halves are bf16 values)
@@ -50,212 +50,270 @@ __device__ __forceinline__ void split3_frag(const float (&v)[8], b8_t (&out)[3])
 
 constexpr int CH = LIGHTNING_CHUNK;
 constexpr int VROW = 64 + 8;   // LDS row of a chunk's values, halves (rows 16-byte aligned, banks shifted)
-constexpr int lightning_lds(int DC) { return 2 * CH * (DC * 32 + 8) * 2 + CH * VROW * 2 + 4 * 2 * 3 * 1024 + (CH + 1) * 4; }
+constexpr int qk_row(int DC) { return DC * 32 + 8; }
+constexpr int add_lds(int DC) { return CH * qk_row(DC) * 2 + CH * VROW * 2 + (CH + 1) * 4; }
+constexpr int out_lds(int DC) { return 2 * CH * qk_row(DC) * 2 + CH * VROW * 2 + 4 * 2 * 3 * 1024 + (CH + 1) * 4; }
 
-template <int DC>
-__global__ __launch_bounds__(256, 2) void k_lightning_chunk(Lightning a, const int4* __restrict__ spans, int vslices) {
-    constexpr int QROW = DC * 32 + 8;
-    extern __shared__ __attribute__((aligned(16))) unsigned char lds_l[];
-    __half* s_q = reinterpret_cast<__half*>(lds_l);   // [CH][QROW]
-    __half* s_k = s_q + CH * QROW;                    // [CH][QROW]
-    __half* s_v = s_k + CH * QROW;                    // [CH][VROW]
-    b8_t* s_p = reinterpret_cast<b8_t*>(s_v + CH * VROW);   // [t tile][s pair][part][64]
-    float* s_dec = reinterpret_cast<float*>(s_p + 4 * 2 * 3 * 64);   // [CH + 1]
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), x = lane & 15, g = lane >> 4;
+// What the chunk kernels share: a workgroup = chunk x head x 64 value columns, a wave = 16 of the columns.
+struct ChunkArgs {
+    Lightning a;
+    const int4* spans;     // (first token, count, first position, sequence)
+    const int2* chunks;    // (span, chunk of the span)
+    int n_spans, vslices;
+    float* mem;            // [chunk][H][value tile][dim tile][64][4]: a tile as the matrix cores leave it, lane (x, g) = S[16 i + 4 g + r][16 j + x]
+    int d_tiles, v_tiles;
+};
+struct ChunkId {
+    int slot, h, vs, first, n;   // first: token of the batch
+    int4 span;
+};
+__device__ __forceinline__ ChunkId chunk_id(const ChunkArgs& c) {
+    ChunkId id;
     int idx = blockIdx.x;
-    const int vs = idx % vslices;
-    idx /= vslices;
-    const int h = idx % a.H, span_id = idx / a.H;
-    const int4 span = spans[span_id];
-    const int n_tok = span.y;
-    const int v0 = vs * 64, my_v = v0 + wave * 16;         // this wave's value columns
-    const bool has_v = my_v < a.vdim_ld;
-    if (tid <= CH) s_dec[tid] = a.decay[h * (CH + 1) + tid];
+    id.vs = idx % c.vslices;
+    idx /= c.vslices;
+    id.h = idx % c.a.H;
+    id.slot = idx / c.a.H;
+    const int2 ch = c.chunks[id.slot];
+    id.span = c.spans[ch.x];
+    id.first = id.span.x + ch.y * CH;
+    id.n = min(CH, id.span.y - ch.y * CH);
+    return id;
+}
+__device__ __forceinline__ f4_t* chunk_tiles(const ChunkArgs& c, int slot, int h, int vtile) {   // dim tile 0, lane 0
+    return reinterpret_cast<f4_t*>(c.mem) + (((size_t)slot * c.a.H + h) * c.v_tiles + vtile) * c.d_tiles * 64;
+}
+// rows of the chunk, 16-byte pieces, zeros behind its end: `base` = first row's first element, `pieces` live pieces, to LDS rows of ROW halves
+template <int PER, int ROW, int U>
+__device__ __forceinline__ void chunk_rows(u4_t (&r)[U], const __half* base, int ld, int n, int pieces) {
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+        const int i = (int)threadIdx.x + 256 * u, row = i / PER, piece = i - row * PER;
+        r[u] = row < n && piece < pieces ? *reinterpret_cast<const u4_t*>(base + (size_t)row * ld + piece * 8) : u4_t{0, 0, 0, 0};
+    }
+}
+template <int PER, int ROW, int U>
+__device__ __forceinline__ void chunk_rows_to_lds(__half* dst, const u4_t (&r)[U]) {
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+        const int i = (int)threadIdx.x + 256 * u, row = i / PER, piece = i - row * PER;
+        *reinterpret_cast<u4_t*>(dst + row * ROW + piece * 8) = r[u];
+    }
+}
+// tokens as k of an operand: {32 pair + 4 g .., 32 pair + 16 + 4 g ..} of 16 columns, by the LDS transpose read (16 lanes bring
+// 4 rows x 16 columns, lane x receives column x of the four rows)
+__device__ __forceinline__ b8_t token_frag(const __half* lds, int row_halves, int col0, int pair) {
+    const int x = threadIdx.x & 15, g = (threadIdx.x >> 4) & 3;
+    const __half* p = lds + (size_t)(32 * pair + 4 * g + (x >> 2)) * row_halves + col0 + 4 * (x & 3);
+    const u2_t lo = __builtin_bit_cast(u2_t, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)p));
+    const u2_t hi = __builtin_bit_cast(u2_t, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(p + (size_t)16 * row_halves)));
+    return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
+}
 
-    // ---- the state's tiles: S[d = 16 i + 4 g + r][v = my_v + x]
-    float* st = a.state + ((size_t)span.w * a.H + h) * a.dim * a.vdim;
+// ---- 1. what a chunk adds to the state: sum_s k_s (decay^(n-1-s) v_s)^T
+template <int DC>
+__global__ __launch_bounds__(256, 2) void k_lightning_add(ChunkArgs c) {
+    constexpr int ROW = qk_row(DC);
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds_l[];
+    __half* s_k = reinterpret_cast<__half*>(lds_l);   // [CH][ROW]
+    __half* s_v = s_k + CH * ROW;                     // [CH][VROW]
+    float* s_dec = reinterpret_cast<float*>(s_v + CH * VROW);
+    const Lightning& a = c.a;
+    const ChunkId id = chunk_id(c);
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4;
+    const int n = id.n, v0 = id.vs * 64, my_v = v0 + wave * 16;
+    const __half* base = a.rows + (size_t)id.first * a.ld;
+    u4_t rk[DC], rv[2];
+    chunk_rows<4 * DC, ROW>(rk, base + (a.H + id.h) * a.dim_ld, a.ld, n, a.dim_ld / 8);
+    chunk_rows<8, VROW>(rv, base + 2 * a.H * a.dim_ld + id.h * a.vdim_ld + v0, a.ld, n, (a.vdim_ld - v0) / 8);
+    if (tid <= CH) s_dec[tid] = a.decay[id.h * (CH + 1) + tid];
+    chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
+    chunk_rows_to_lds<8, VROW>(s_v, rv);
+    __syncthreads();
+    if (my_v >= a.vdim_ld) return;
     f4_t S[2 * DC];
 #pragma unroll
-    for (int i = 0; i < 2 * DC; i++)
+    for (int i = 0; i < 2 * DC; i++) S[i] = f4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            const int d = 16 * i + 4 * g + r, v = my_v + x;
-            S[i][r] = span.z > 0 && d < a.dim && v < a.vdim ? st[(size_t)d * a.vdim + v] : 0.f;
+    for (int pair = 0; pair < 2; pair++) {
+        float e[8];
+        const b8_t vv = token_frag(s_v, VROW, wave * 16, pair);
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            const int s = 32 * pair + 16 * (i >> 2) + 4 * g + (i & 3);
+            e[i] = s < n ? (float)vv[i] * s_dec[max(n - 1 - s, 0)] : 0.f;
         }
-
-    // ---- the chunk's rows, a chunk ahead in registers: 16-byte pieces, a row's pieces by neighbouring threads
-    const int qk_pieces = a.dim_ld / 8;
-    u4_t rq[DC], rk[DC], rv[2];
-    u2_t rg[4];   // this lane's gates: columns my_v + 4 g .. + 3 of tokens 16 i + x
-    auto fetch = [&](int c0) {
+        b8_t parts[3];
+        split3_frag(e, parts);
 #pragma unroll
-        for (int u = 0; u < DC; u++) {
-            const int i = tid + 256 * u, row = i / (4 * DC), piece = i - row * (4 * DC);
-            const bool live = c0 + row < n_tok && piece < qk_pieces;
-            const __half* src = a.rows + (size_t)(span.x + c0 + row) * a.ld + h * a.dim_ld + piece * 8;
-            rq[u] = live ? *reinterpret_cast<const u4_t*>(src) : u4_t{0, 0, 0, 0};
-            rk[u] = live ? *reinterpret_cast<const u4_t*>(src + a.H * a.dim_ld) : u4_t{0, 0, 0, 0};
+        for (int i = 0; i < 2 * DC; i++) {
+            const b8_t kt = token_frag(s_k, ROW, 16 * i, pair);
+#pragma unroll
+            for (int k = 2; k >= 0; k--) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt, parts[k], S[i], 0, 0, 0);
         }
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const int i = tid + 256 * u, row = i >> 3, piece = i & 7;
-            const bool live = c0 + row < n_tok && v0 + piece * 8 < a.vdim_ld;
-            const __half* src = a.rows + (size_t)(span.x + c0 + row) * a.ld + 2 * a.H * a.dim_ld + h * a.vdim_ld + v0 + piece * 8;
-            rv[u] = live ? *reinterpret_cast<const u4_t*>(src) : u4_t{0, 0, 0, 0};
-        }
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int tok = min(c0 + 16 * i + x, n_tok - 1);
-            rg[i] = has_v ? *reinterpret_cast<const u2_t*>(a.rows + (size_t)(span.x + tok) * a.ld + 2 * a.H * a.dim_ld + (a.H + h) * a.vdim_ld + my_v + 4 * g) : u2_t{0, 0};
-        }
-    };
-    fetch(0);
-    const int ss_ld = a.H * a.vdim_ld / 16, Kb_out = a.H * a.vdim_ld / 32;
-    const f4_t gain = has_v ? *reinterpret_cast<const f4_t*>(a.gain + h * a.vdim_ld + my_v + 4 * g) : f4_t{0.f, 0.f, 0.f, 0.f};
-
-    for (int c0 = 0; c0 < n_tok; c0 += CH) {
-        const int n = min(CH, n_tok - c0);
-#pragma unroll
-        for (int u = 0; u < DC; u++) {
-            const int i = tid + 256 * u, row = i / (4 * DC), piece = i - row * (4 * DC);
-            *reinterpret_cast<u4_t*>(s_q + row * QROW + piece * 8) = rq[u];
-            *reinterpret_cast<u4_t*>(s_k + row * QROW + piece * 8) = rk[u];
-        }
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const int i = tid + 256 * u, row = i >> 3, piece = i & 7;
-            *reinterpret_cast<u4_t*>(s_v + row * VROW + piece * 8) = rv[u];
-        }
-        u2_t gates[4];
-#pragma unroll
-        for (int i = 0; i < 4; i++) gates[i] = rg[i];
-        __syncthreads();
-        if (c0 + CH < n_tok) fetch(c0 + CH);
-        // operands over dims in the order of the state's registers: {32 c + 4 g .., 32 c + 16 + 4 g ..} of row 16 i + x
-        auto frag = [&](const __half* base, int i, int c) {
-            const __half* p = base + (16 * i + x) * QROW + 32 * c + 4 * g;
-            const u2_t lo = *reinterpret_cast<const u2_t*>(p), hi = *reinterpret_cast<const u2_t*>(p + 16);
-            return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
-        };
-        // ---- P of token tile `wave`: rows s (tiles 0 .. wave), columns t
-        if (wave * 16 < n) {
-            b8_t qf[DC];
-#pragma unroll
-            for (int c = 0; c < DC; c++) qf[c] = frag(s_q, wave, c);
-            const int t = wave * 16 + x;
-#pragma unroll
-            for (int pair = 0; pair < 2; pair++) {
-                if (2 * pair > wave) break;
-                float e[8];
-#pragma unroll
-                for (int half = 0; half < 2; half++) {
-                    f4_t p = {0.f, 0.f, 0.f, 0.f};
-                    const int i = 2 * pair + half;
-                    if (i <= wave) {
-#pragma unroll
-                        for (int c = 0; c < DC; c++) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(s_k, i, c), qf[c], p, 0, 0, 0);
-                    }
-#pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        const int s = 16 * i + 4 * g + r;
-                        e[4 * half + r] = s <= t ? p[r] * s_dec[max(t - s, 0)] : 0.f;
-                    }
-                }
-                b8_t parts[3];
-                split3_frag(e, parts);
-#pragma unroll
-                for (int k = 0; k < 3; k++) s_p[((wave * 2 + pair) * 3 + k) * 64 + lane] = parts[k];
-            }
-        }
-        __syncthreads();
-        if (has_v) {
-            // values of this wave's columns with tokens as k: {pair * 32 + 4 g .., pair * 32 + 16 + 4 g ..}, by the LDS transpose read
-            // (16 lanes bring 4 rows x 16 columns, lane x receives column x of the four rows)
-            s4_t vt[2][2];
-#pragma unroll
-            for (int pair = 0; pair < 2; pair++)
-#pragma unroll
-                for (int half = 0; half < 2; half++)
-                    vt[pair][half] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                        (lds_s4*)(s_v + (32 * pair + 16 * half + 4 * g + (x >> 2)) * VROW + wave * 16 + 4 * (x & 3)));
-            auto vfrag = [&](int pair) {
-                const u2_t lo = __builtin_bit_cast(u2_t, vt[pair][0]), hi = __builtin_bit_cast(u2_t, vt[pair][1]);
-                return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
-            };
-            // the state as operand, three exact parts
-            b8_t sf[DC][3];
-#pragma unroll
-            for (int c = 0; c < DC; c++) {
-                const float e[8] = {S[2 * c][0], S[2 * c][1], S[2 * c][2], S[2 * c][3], S[2 * c + 1][0], S[2 * c + 1][1], S[2 * c + 1][2], S[2 * c + 1][3]};
-                split3_frag(e, sf[c]);
-            }
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                if (i * 16 >= n) break;
-                f4_t o = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int c = 0; c < DC; c++) {
-                    const b8_t qf = frag(s_q, i, c);
-#pragma unroll
-                    for (int k = 2; k >= 0; k--) o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf[c][k], qf, o, 0, 0, 0);
-                }
-                const int tl = i * 16 + x, t = span.x + c0 + tl;
-                o *= s_dec[tl + 1];
-#pragma unroll
-                for (int pair = 0; pair < 2; pair++) {
-                    if (2 * pair > i) break;
-#pragma unroll
-                    for (int k = 2; k >= 0; k--)
-                        o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vfrag(pair), s_p[((i * 2 + pair) * 3 + k) * 64 + lane], o, 0, 0, 0);
-                }
-                float sq = o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
-                sq += __shfl_xor(sq, 16, 64);
-                sq += __shfl_xor(sq, 32, 64);
-                if (tl < n) {
-                    const int col = h * a.vdim_ld + my_v;
-                    float y[4];
-#pragma unroll
-                    for (int r = 0; r < 4; r++) y[r] = o[r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gates[i][r >> 1] >> (16 * (r & 1)))));
-                    store_b16_4(a.out_b16, Kb_out, t, col + 4 * g, y);
-                    if (g == 0) a.ss_out[(size_t)t * ss_ld + (col >> 4)] = sq;
-                }
-            }
-            // ---- the state behind the chunk
-            const float fade = s_dec[n];
-#pragma unroll
-            for (int i = 0; i < 2 * DC; i++) S[i] *= fade;
-#pragma unroll
-            for (int pair = 0; pair < 2; pair++) {
-                float e[8];
-                const b8_t vv = vfrag(pair);
-#pragma unroll
-                for (int i = 0; i < 8; i++) {
-                    const int s = 32 * pair + 16 * (i >> 2) + 4 * g + (i & 3);
-                    e[i] = s < n ? (float)vv[i] * s_dec[max(n - 1 - s, 0)] : 0.f;
-                }
-                b8_t parts[3];
-                split3_frag(e, parts);
-#pragma unroll
-                for (int i = 0; i < 2 * DC; i++) {
-                    const s4_t k0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(s_k + (32 * pair + 4 * g + (x >> 2)) * QROW + 16 * i + 4 * (x & 3)));
-                    const s4_t k1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)(s_k + (32 * pair + 16 + 4 * g + (x >> 2)) * QROW + 16 * i + 4 * (x & 3)));
-                    const u2_t lo = __builtin_bit_cast(u2_t, k0), hi = __builtin_bit_cast(u2_t, k1);
-                    const b8_t kt = __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
-#pragma unroll
-                    for (int k = 2; k >= 0; k--) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt, parts[k], S[i], 0, 0, 0);
-                }
-            }
-        }
-        __syncthreads();   // the chunk's rows and P have been read
     }
-    if (has_v && my_v + x < a.vdim)
+    f4_t* out = chunk_tiles(c, id.slot, id.h, my_v >> 4) + lane;
 #pragma unroll
-        for (int i = 0; i < 2 * DC; i++)
+    for (int i = 0; i < 2 * DC; i++)
+        if (i < c.d_tiles) out[i * 64] = S[i];
+}
+
+// ---- 2. from what chunks add to the states they start from, and the sequence's state behind its portion.  A thread per four
+// elements of a state; chunk_of_span: the first chunk of every portion.
+__global__ __launch_bounds__(256) void k_lightning_scan(ChunkArgs c, const int* __restrict__ first_chunk) {
+    const Lightning& a = c.a;
+    const int tiles = c.v_tiles * c.d_tiles, item = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y;
+    if (item >= tiles * 64) return;
+    const int4 span = c.spans[blockIdx.z];
+    const int lane = item & 63, j = (item >> 6) / c.d_tiles, i = (item >> 6) - j * c.d_tiles;
+    const int v = 16 * j + (lane & 15), d0 = 16 * i + 4 * (lane >> 4);
+    float* st = a.state + ((size_t)span.w * a.H + h) * a.dim * a.vdim;
+    f4_t S;
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int d = 16 * i + 4 * g + r;
-                if (d < a.dim) st[(size_t)d * a.vdim + my_v + x] = S[i][r];
+    for (int r = 0; r < 4; r++) S[r] = span.z > 0 && d0 + r < a.dim && v < a.vdim ? st[(size_t)(d0 + r) * a.vdim + v] : 0.f;
+    const int n_chunks = (span.y + CH - 1) / CH;
+    const size_t stride = (size_t)a.H * tiles * 64;
+    f4_t* p = reinterpret_cast<f4_t*>(c.mem) + (size_t)first_chunk[blockIdx.z] * stride + (size_t)h * tiles * 64 + item;
+    const float* dec = a.decay + h * (CH + 1);
+    const float whole = dec[CH], tail = dec[span.y - (n_chunks - 1) * CH];
+    for (int k0 = 0; k0 < n_chunks; k0 += 8) {
+        f4_t u[8];
+#pragma unroll
+        for (int k = 0; k < 8; k++) u[k] = p[min(k0 + k, n_chunks - 1) * stride];
+#pragma unroll
+        for (int k = 0; k < 8; k++)
+            if (k0 + k < n_chunks) {
+                p[(k0 + k) * stride] = S;
+                S = S * (k0 + k == n_chunks - 1 ? tail : whole) + u[k];
             }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; r++)
+        if (d0 + r < a.dim && v < a.vdim) st[(size_t)(d0 + r) * a.vdim + v] = S[r];
+}
+
+// ---- 3. the chunk's results
+template <int DC>
+__global__ __launch_bounds__(256, 2) void k_lightning_out(ChunkArgs c) {
+    constexpr int ROW = qk_row(DC);
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds_l[];
+    __half* s_q = reinterpret_cast<__half*>(lds_l);   // [CH][ROW]
+    __half* s_k = s_q + CH * ROW;                     // [CH][ROW]
+    __half* s_v = s_k + CH * ROW;                     // [CH][VROW]
+    b8_t* s_p = reinterpret_cast<b8_t*>(s_v + CH * VROW);            // [t tile][s pair][part][64]
+    float* s_dec = reinterpret_cast<float*>(s_p + 4 * 2 * 3 * 64);   // [CH + 1]
+    const Lightning& a = c.a;
+    const ChunkId id = chunk_id(c);
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), x = lane & 15, g = lane >> 4;
+    const int n = id.n, h = id.h, v0 = id.vs * 64, my_v = v0 + wave * 16;
+    const bool has_v = my_v < a.vdim_ld;
+    const __half* base = a.rows + (size_t)id.first * a.ld;
+    u4_t rq[DC], rk[DC], rv[2];
+    chunk_rows<4 * DC, ROW>(rq, base + h * a.dim_ld, a.ld, n, a.dim_ld / 8);
+    chunk_rows<4 * DC, ROW>(rk, base + (a.H + h) * a.dim_ld, a.ld, n, a.dim_ld / 8);
+    chunk_rows<8, VROW>(rv, base + 2 * a.H * a.dim_ld + h * a.vdim_ld + v0, a.ld, n, (a.vdim_ld - v0) / 8);
+    // this wave's columns of the state, of the gates (tokens 16 i + x) and of the gain
+    f4_t S[2 * DC], gain = {0.f, 0.f, 0.f, 0.f};
+    u2_t gates[4];
+    if (has_v) {
+        const f4_t* in = chunk_tiles(c, id.slot, h, my_v >> 4) + lane;
+#pragma unroll
+        for (int i = 0; i < 2 * DC; i++) S[i] = i < c.d_tiles ? in[i * 64] : f4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            gates[i] = *reinterpret_cast<const u2_t*>(base + (size_t)min(16 * i + x, n - 1) * a.ld + 2 * a.H * a.dim_ld + (a.H + h) * a.vdim_ld + my_v + 4 * g);
+        gain = *reinterpret_cast<const f4_t*>(a.gain + h * a.vdim_ld + my_v + 4 * g);
+    }
+    if (tid <= CH) s_dec[tid] = a.decay[h * (CH + 1) + tid];
+    chunk_rows_to_lds<4 * DC, ROW>(s_q, rq);
+    chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
+    chunk_rows_to_lds<8, VROW>(s_v, rv);
+    __syncthreads();
+    // operands over dims in the order of the state's registers: {32 cc + 4 g .., 32 cc + 16 + 4 g ..} of row 16 i + x
+    auto frag = [&](const __half* lds, int i, int cc) {
+        const __half* p = lds + (16 * i + x) * ROW + 32 * cc + 4 * g;
+        const u2_t lo = *reinterpret_cast<const u2_t*>(p), hi = *reinterpret_cast<const u2_t*>(p + 16);
+        return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
+    };
+    // ---- P of token tile `wave`: rows s (tiles 0 .. wave), columns t
+    if (wave * 16 < n) {
+        b8_t qf[DC];
+#pragma unroll
+        for (int cc = 0; cc < DC; cc++) qf[cc] = frag(s_q, wave, cc);
+        const int t = wave * 16 + x;
+#pragma unroll
+        for (int pair = 0; pair < 2; pair++) {
+            if (2 * pair > wave) break;
+            float e[8];
+#pragma unroll
+            for (int half = 0; half < 2; half++) {
+                f4_t p = {0.f, 0.f, 0.f, 0.f};
+                const int i = 2 * pair + half;
+                if (i <= wave) {
+#pragma unroll
+                    for (int cc = 0; cc < DC; cc++) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(s_k, i, cc), qf[cc], p, 0, 0, 0);
+                }
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    const int s = 16 * i + 4 * g + r;
+                    e[4 * half + r] = s <= t ? p[r] * s_dec[max(t - s, 0)] : 0.f;
+                }
+            }
+            b8_t parts[3];
+            split3_frag(e, parts);
+#pragma unroll
+            for (int k = 0; k < 3; k++) s_p[((wave * 2 + pair) * 3 + k) * 64 + lane] = parts[k];
+        }
+    }
+    b8_t sf[DC][3];   // the state as operand, three exact parts
+#pragma unroll
+    for (int cc = 0; cc < DC; cc++) {
+        float e[8];
+#pragma unroll
+        for (int i = 0; i < 8; i++) e[i] = S[2 * cc + (i >> 2)][i & 3];
+        split3_frag(e, sf[cc]);
+    }
+    __syncthreads();
+    if (!has_v) return;
+    const b8_t vf[2] = {token_frag(s_v, VROW, wave * 16, 0), token_frag(s_v, VROW, wave * 16, 1)};
+    // (the four token tiles are independent chains of products)
+    f4_t o[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) o[i] = f4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int cc = 0; cc < DC; cc++) {
+        b8_t qf[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) qf[i] = frag(s_q, i, cc);
+#pragma unroll
+        for (int k = 2; k >= 0; k--)
+#pragma unroll
+            for (int i = 0; i < 4; i++) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf[cc][k], qf[i], o[i], 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) o[i] *= s_dec[i * 16 + x + 1];
+#pragma unroll
+    for (int pair = 0; pair < 2; pair++)
+#pragma unroll
+        for (int k = 2; k >= 0; k--)
+#pragma unroll
+            for (int i = 2 * pair; i < 4; i++)   // (P of tiles past the chunk's end is whatever LDS holds; their results are not stored)
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pair], s_p[((i * 2 + pair) * 3 + k) * 64 + lane], o[i], 0, 0, 0);
+    const int ss_ld = a.H * a.vdim_ld / 16, Kb_out = a.H * a.vdim_ld / 32, col = h * a.vdim_ld + my_v;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        float sq = o[i][0] * o[i][0] + o[i][1] * o[i][1] + o[i][2] * o[i][2] + o[i][3] * o[i][3];
+        sq += __shfl_xor(sq, 16, 64);
+        sq += __shfl_xor(sq, 32, 64);
+        const int tl = i * 16 + x, t = id.first + tl;
+        if (tl < n) {
+            float y[4];
+#pragma unroll
+            for (int r = 0; r < 4; r++) y[r] = o[i][r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gates[i][r >> 1] >> (16 * (r & 1)))));
+            store_b16_4(a.out_b16, Kb_out, t, col + 4 * g, y);
+            if (g == 0) a.ss_out[(size_t)t * ss_ld + (col >> 4)] = sq;
+        }
+    }
 }
 
 // A workgroup per (portion, head).  Thread = VEC neighbouring value columns x every ROWS-th dim.
@@ -357,15 +415,53 @@ __global__ __launch_bounds__(256) void k_lightning_step(Lightning a, const int4*
 }
 
 template <int DC>
-static void launch_chunk(const Lightning& a, const StepArrays& st) {
-    constexpr int shmem = lightning_lds(DC);
+static void launch_add(const ChunkArgs& c, int n_chunks) {
+    constexpr int shmem = add_lds(DC);
+    static_assert(shmem <= 64 * 1024, "no attribute needed");
+    NVLLM_LAUNCH((k_lightning_add<DC>), dim3(n_chunks * c.a.H * c.vslices), dim3(256), shmem, c);
+}
+template <int DC>
+static void launch_out(const ChunkArgs& c, int n_chunks) {
+    constexpr int shmem = out_lds(DC);
     static bool enabled = false;
     if (shmem > 64 * 1024 && !enabled) {
-        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_lightning_chunk<DC>), hipFuncAttributeMaxDynamicSharedMemorySize, shmem));
+        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_lightning_out<DC>), hipFuncAttributeMaxDynamicSharedMemorySize, shmem));
         enabled = true;
     }
-    const int vslices = cdiv(a.vdim_ld, 64);
-    NVLLM_LAUNCH((k_lightning_chunk<DC>), dim3(st.n_spans_multi * a.H * vslices), dim3(256), shmem, a, (const int4*)st.d_spans, vslices);
+    NVLLM_LAUNCH((k_lightning_out<DC>), dim3(n_chunks * c.a.H * c.vslices), dim3(256), shmem, c);
+}
+// Portions of several tokens: the chunks' additions, the scan over them, the chunks' results.
+static void launch_chunks(const Lightning& a, const StepArrays& st, double bytes, double flops) {
+    ChunkArgs c{};
+    c.a = a;
+    c.spans = (const int4*)st.d_spans;
+    c.chunks = (const int2*)st.d_chunks;
+    c.n_spans = st.n_spans_multi;
+    c.vslices = cdiv(a.vdim_ld, 64);
+    c.d_tiles = a.dim_ld / 16;
+    c.v_tiles = a.vdim_ld / 16;
+    const size_t tiles = (size_t)a.H * c.d_tiles * c.v_tiles;   // of a state
+    c.mem = (float*)ws_get(WS_STATES, st.n_chunks * tiles * 1024);
+    const int DC = a.dim_ld / 32, n = st.n_chunks;
+    // the algorithm's bytes and flops: those of the recurrence, split over the three launches
+    {
+        ProfScope ps(PC_LIGHTNING, bytes / 3, flops / 3);
+        if (DC == 1) launch_add<1>(c, n);
+        else if (DC == 2) launch_add<2>(c, n);
+        else if (DC == 3) launch_add<3>(c, n);
+        else if (DC == 4) launch_add<4>(c, n);
+        else launch_add<8>(c, n);
+    }
+    {
+        ProfScope ps(PC_LIGHTNING, bytes / 3, flops / 3);
+        NVLLM_LAUNCH(k_lightning_scan, dim3(cdiv(c.d_tiles * c.v_tiles * 64, 256), a.H, c.n_spans), dim3(256), 0, c, (const int*)st.d_first_chunk);
+    }
+    ProfScope ps(PC_LIGHTNING, bytes / 3, flops / 3);
+    if (DC == 1) launch_out<1>(c, n);
+    else if (DC == 2) launch_out<2>(c, n);
+    else if (DC == 3) launch_out<3>(c, n);
+    else if (DC == 4) launch_out<4>(c, n);
+    else launch_out<8>(c, n);
 }
 
 void launch_lightning(const Lightning& a, const StepArrays& st) {
@@ -379,15 +475,8 @@ void launch_lightning(const Lightning& a, const StepArrays& st) {
     const int DC = a.dim_ld / 32;
     const bool chunked = b16 && DC <= 8;
     if (chunked && st.n_spans_multi > 0) {
-        ProfScope ps(PC_LIGHTNING, st.n_spans_multi * state_bytes + multi_tokens * token_bytes,
-                     multi_tokens * (token_flops + pair * 0.5 * std::min(st.max_span, CH)));
-        switch (DC) {
-            case 1: launch_chunk<1>(a, st); break;
-            case 2: launch_chunk<2>(a, st); break;
-            case 3: launch_chunk<3>(a, st); break;
-            case 4: launch_chunk<4>(a, st); break;
-            default: launch_chunk<8>(a, st); break;
-        }
+        if (st.chunk_len != CH) NVLLM_FATAL("linear attention: the batch was staged in chunks of %d tokens", st.chunk_len);
+        launch_chunks(a, st, st.n_spans_multi * state_bytes + multi_tokens * token_bytes, multi_tokens * (token_flops + pair * 0.5 * std::min(st.max_span, CH)));
     }
     const int from = chunked ? st.n_spans_multi : 0, n = st.n_spans - from;
     if (n <= 0) return;

@@ -135,6 +135,7 @@ enum WsSlot {
     WS_KV_RAW,      // latent attention: a batch's latents and rotated key parts before norm and rotation
     WS_Q_ROWS,      // ... its absorbed queries
     WS_LATENT,      // ... its attended latents
+    WS_STATES,      // linear attention: the states a batch's chunks start from
     WS_A16_SORTED,  // mixture of experts: a batch's rows sorted by expert
     WS_F32_A,       // fp32 models: activations between operators
     WS_F32_B,

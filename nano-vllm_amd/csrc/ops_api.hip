@@ -50,7 +50,7 @@ KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim) {
 // pinned region and upload it with a single copy.
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
-                      int pos0, int block_size, int attn_ct, const int* token_src, bool multi_first, bool spans) {
+                      int pos0, int block_size, int attn_ct, const int* token_src, bool multi_first, bool spans, int chunk_len) {
     StepArrays s{};
     s.T = T;
     s.B = B;
@@ -167,6 +167,15 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
         s.n_spans = (int)span.size() / 4;
         s.host_spans = span;
     }
+    std::vector<int> chunks, first_chunk;
+    if (spans && chunk_len > 0) {
+        s.chunk_len = chunk_len;
+        for (int i = 0; i < s.n_spans_multi; i++) {
+            first_chunk.push_back((int)chunks.size() / 2);
+            for (int c = 0; c * chunk_len < span[4 * i + 1]; c++) chunks.insert(chunks.end(), {i, c});
+        }
+        s.n_chunks = (int)chunks.size() / 2;
+    }
     // where each token's K/V row goes: resolves position -> (block table entry, slot) on
     // the host so the kernels that store K/V need one load instead of a chain of three
     std::vector<int> kv_row;
@@ -179,7 +188,7 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
         }
     }
     const size_t n_ints = (size_t)(tokens ? T : 0) + (token_src ? T : 0) + (pos_arr ? T : 0) + (seq_ids ? T : 0) + kv_row.size() +
-                          (output_indices ? B : 0) + n_seqs + total_tbl + runs.size() + span.size() + span_of.size() + 64;
+                          (output_indices ? B : 0) + n_seqs + total_tbl + runs.size() + span.size() + span_of.size() + chunks.size() + first_chunk.size() + 64;
     int* host = pinned_ints(n_ints);
     int* dev = (int*)ws_get(WS_STEP, n_ints * sizeof(int));
     size_t o = 0;
@@ -217,6 +226,8 @@ StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids,
     o = (o + 3) & ~(size_t)3;  // int4 alignment
     s.d_runs = runs.empty() ? nullptr : put(runs.data(), runs.size());
     s.d_spans = span.empty() ? nullptr : put(span.data(), span.size());
+    s.d_chunks = chunks.empty() ? nullptr : put(chunks.data(), chunks.size());   // (pairs, behind quadruples)
+    s.d_first_chunk = first_chunk.empty() ? nullptr : put(first_chunk.data(), first_chunk.size());
     s.d_span_of = span_of.empty() ? nullptr : put(span_of.data(), span_of.size());
     if (o > 0) {
         static const int by_kernel = getenv("NVLLM_STAGE_COPY") ? atoi(getenv("NVLLM_STAGE_COPY")) == 0 : 1;

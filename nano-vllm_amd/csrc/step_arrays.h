@@ -37,6 +37,10 @@ struct StepArrays {
     int n_spans, n_spans_multi;
     int max_span;            // tokens of the longest
     bool seq_split;          // some sequence's tokens do not lie side by side at consecutive positions
+    // chunk_len > 0: the portions of several tokens cut into chunks of that many
+    int chunk_len, n_chunks;
+    int* d_chunks;           // [n_chunks][2] (span, its chunk)
+    int* d_first_chunk;      // [n_spans_multi]
     std::vector<int> host_spans;
     // Kernel timing, when a token sees at most `limit` positions: rows of K/V that the portions of several tokens (of one
     // token) see, each counted once, and (token, position) pairs of the former.
@@ -65,7 +69,7 @@ private:
 StepArrays stage_step(const int* tokens, const int* pos_arr, const int* seq_ids, int T,
                       const int* output_indices, int B, BlockTable** tables, const BlockTable* single,
                       int pos0, int block_size, int attn_ct = 0, const int* token_src = nullptr, bool multi_first = false,
-                      bool spans = false);
+                      bool spans = false, int chunk_len = 0);
 
 KvPoolView pool_view(const KVCacheManager* mgr, int n_kv_heads, int head_dim);
 

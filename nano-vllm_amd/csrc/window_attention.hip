@@ -3,8 +3,8 @@
 // k_window_attn (bf16 pages).  Pages are stored in the operand order of the matrix cores, so a wave reads a key page
 // (operand A of S^T = K Q^T) and a value page (operand A of O^T = V^T P^T) straight from memory into registers; a score
 // tile's result registers are already in the k order of the second product, and a column (one query) stays on its lane
-// through scores, weights, sums and results: no LDS and no barrier in the loop.  A step takes two pages (32 keys):
-// the keys of the next step are requested when the scores are done, its values when the products are.
+// through scores, weights, sums and results: no LDS and no barrier in the loop.  A step takes two pages (32 keys) while
+// the next step's travel.
 //   prompts        a wave owns C groups of 16 neighbouring tokens x up to four heads of a key/value group;
 //   single tokens  the columns are the heads of a group; the waves of a workgroup (and, when there are few items,
 //                  several workgroups) take every n-th pair of pages and their sums meet in LDS (and in a merge launch).
@@ -538,24 +538,33 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
     auto page_at = [&](int i) { return i < n_kept ? i : first_pg + i - n_kept; };   // position / 16
     auto page_id = [&](int pg) { return (table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1)); };
 
-    h8_t kf[2][KC];
-    u2_t vf[2][VT];
-    auto load_keys = [&](int it) {
+    // Pages in registers: of two steps (DEEP: a step's are requested before the step ahead of it is computed) or of one.
+    constexpr bool DEEP = 2 * (8 * KC + 4 * VT) + C * 4 * (KC + VT) <= 176;
+    constexpr int SETS = DEEP ? 2 : 1;
+    h8_t kf[SETS][2][KC];
+    u2_t vf[SETS][2][VT];
+    int ids[2] = {0, 0};   // pages of the step that is requested next
+    auto look_up = [&](int it) {
+        if (it < it1)
+#pragma unroll
+            for (int p = 0; p < 2; p++) ids[p] = page_id(page_at(min(2 * it + p, n_pages - 1)));
+    };
+    auto load_keys = [&](int set) {
 #pragma unroll
         for (int p = 0; p < 2; p++) {
-            const h8_t* src = reinterpret_cast<const h8_t*>(a.keys + ((size_t)page_id(page_at(min(2 * it + p, n_pages - 1))) * a.G + grp) * (KV_PAGE * 32 * kc)) + lane;
+            const h8_t* src = reinterpret_cast<const h8_t*>(a.keys + ((size_t)ids[p] * a.G + grp) * (KV_PAGE * 32 * kc)) + lane;
 #pragma unroll
             for (int k = 0; k < KC; k++)
-                if (EXACT || k < kc) kf[p][k] = src[k * 64];
+                if (EXACT || k < kc) kf[set][p][k] = src[k * 64];
         }
     };
-    auto load_values = [&](int it) {
+    auto load_values = [&](int set) {
 #pragma unroll
         for (int p = 0; p < 2; p++) {
-            const u2_t* src = reinterpret_cast<const u2_t*>(a.values + ((size_t)page_id(page_at(min(2 * it + p, n_pages - 1))) * a.G + grp) * (KV_PAGE * 16 * vt)) + lane;
+            const u2_t* src = reinterpret_cast<const u2_t*>(a.values + ((size_t)ids[p] * a.G + grp) * (KV_PAGE * 16 * vt)) + lane;
 #pragma unroll
             for (int v = 0; v < VT; v++)
-                if (EXACT || v < vt) vf[p][v] = src[v * 64];
+                if (EXACT || v < vt) vf[set][p][v] = src[v * 64];
         }
     };
 
@@ -572,12 +581,19 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
     const float grow = CAP ? 2.f * a.scale / a.cap * LOG2E : 0.f;                   // cap: tanh(s/cap) = 1 - 2 / (1 + 2^(grow s))
     const float top = a.cap * LOG2E;
 
+    look_up(it0);
     if (it0 < it1) {
-        load_keys(it0);
-        load_values(it0);
+        load_keys(0);
+        load_values(0);
     }
-#pragma clang loop unroll(disable)
-    for (int it = it0; it < it1; it += STRIDE) {
+    look_up(it0 + STRIDE);
+    auto step = [&](const int it, const int set) __attribute__((always_inline)) {   // set: where this step's pages are
+        const bool more = it + STRIDE < it1;
+        if (DEEP && more) {
+            load_keys(set ^ 1);
+            load_values(set ^ 1);
+            look_up(it + 2 * STRIDE);
+        }
         f4_t s[2][C];
 #pragma unroll
         for (int p = 0; p < 2; p++)
@@ -590,8 +606,8 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
                 for (int p = 0; p < 2; p++)
 #pragma unroll
                     for (int c = 0; c < C; c++)
-                        s[p][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, kf[p][k]), qf[c][k], s[p][c], 0, 0, 0);
-        if (it + STRIDE < it1) load_keys(it + STRIDE);
+                        s[p][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, kf[set][p][k]), qf[c][k], s[p][c], 0, 0, 0);
+        if (!DEEP && more) load_keys(0);
         // ---- weights
         const int pg0 = page_at(2 * it), pg1 = 2 * it + 1 < n_pages ? page_at(2 * it + 1) : 1 << 26;   // (a page that is not there lies past every query)
         auto open = [&](int pg) { return pg * 16 + 15 <= pos_lo && (pg * 16 > pos_hi - a.size || pg * 16 + 15 < a.keep); };
@@ -646,12 +662,25 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
 #pragma unroll
         for (int v = 0; v < VT; v++)
             if (EXACT || v < vt) {
-                const u4_t both = {vf[0][v][0], vf[0][v][1], vf[1][v][0], vf[1][v][1]};
+                const u4_t both = {vf[set][0][v][0], vf[set][0][v][1], vf[set][1][v][0], vf[set][1][v][1]};
 #pragma unroll
                 for (int c = 0; c < C; c++)
                     acc[v][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, both), pw[c], acc[v][c], 0, 0, 0);
             }
-        if (it + STRIDE < it1) load_values(it + STRIDE);
+        if (!DEEP && more) {
+            load_values(0);
+            look_up(it + 2 * STRIDE);
+        }
+    };
+    if constexpr (DEEP) {
+#pragma clang loop unroll(disable)
+        for (int it = it0; it < it1; it += 2 * STRIDE) {
+            step(it, 0);
+            if (it + STRIDE < it1) step(it + STRIDE, 1);
+        }
+    } else {
+#pragma clang loop unroll(disable)
+        for (int it = it0; it < it1; it += STRIDE) step(it, 0);
     }
 #pragma unroll
     for (int c = 0; c < C; c++) {   // the four lane rows of a column hold different keys
