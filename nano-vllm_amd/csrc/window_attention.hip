@@ -192,12 +192,13 @@ __global__ __launch_bounds__(256) void k_conv_rope(ConvKArgs a) {
 }
 
 // The same for bf16 rows of 16-byte pieces and KEEP + 1 taps: a thread walks TOK neighbouring tokens with the taps and the
-// last KEEP inputs in registers, and on to the end of those that see the state of a portion that starts among them.
+// last KEEP inputs in registers (what the tokens need is requested up front), and on to the end of those that see the state
+// of a portion that starts among them.
 struct alignas(16) Piece {
     __bf16 v[8];
 };
-template <int KEEP>
-__global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int TOK) {
+template <int KEEP, int TOK>
+__global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T) {
     const int item = blockIdx.y * 256 + threadIdx.x, t0 = blockIdx.x * TOK;
     if (item >= a.items) return;
     int part, head, at, i = item;
@@ -222,6 +223,17 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int 
     const bool live = d0 < dim;   // (past it: the padding of a query row)
     const int ch = (part == 0 ? 0 : part == 1 ? a.QD : a.QD + a.KD) + head * dim + (live ? d0 : 0), partner = turns ? half : 0;
     const __bf16* raw = reinterpret_cast<const __bf16*>(a.c.raw) + ch;
+    int4 spans[TOK];   // (first token, count, first position, sequence)
+    int rows[TOK];
+    Piece in[TOK], inz[TOK];
+#pragma unroll
+    for (int u = 0; u < TOK; u++) {
+        const int t = min(t0 + u, T - 1);
+        spans[u] = a.spans[a.span_of[t]];
+        rows[u] = a.kv_row[t];
+        in[u] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld);
+        inz[u] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner);
+    }
     float w[KEEP + 1][8], wz[KEEP + 1][8];
 #pragma unroll
     for (int j = 0; j <= KEEP; j++)
@@ -238,14 +250,8 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int 
         }
     Piece win[KEEP + 1], winz[KEEP + 1];   // inputs of tokens t - KEEP .. t
     int have = -1;                         // the token they are complete for, but for its own input
-    for (int t = t0; t < T; t++) {
-        const int4 span = a.spans[a.span_of[t]];   // (first token, count, first position, sequence)
+    auto token = [&](const int t, const int4 span, const int row, const Piece own, const Piece ownz) __attribute__((always_inline)) {
         const int off = t - span.x;
-        const bool old_state = off > 0 && off < KEEP;
-        if (t < t0 + TOK ? old_state && span.x < t0 : !(old_state && span.x >= t0)) {
-            if (t < t0 + TOK) continue;   // belongs to the thread of the portion's first token
-            break;
-        }
         __bf16* state = reinterpret_cast<__bf16*>(a.c.state) + (size_t)span.w * KEEP * a.channels + ch;
         if (have != t || off == 0) {
 #pragma unroll
@@ -260,8 +266,8 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int 
                 }
             }
         }
-        win[KEEP] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld);
-        winz[KEEP] = *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner);
+        win[KEEP] = own;
+        winz[KEEP] = ownz;
         float y[8], z[8];
 #pragma unroll
         for (int e = 0; e < 8; e++) y[e] = z[e] = 0.f;
@@ -294,7 +300,7 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int 
             __bf16* q = reinterpret_cast<__bf16*>(a.c.q_out) + ((size_t)t * a.c.H + head) * a.pool.dim_ld + d0;
             *reinterpret_cast<Piece*>(q) = py;
             if (turns) *reinterpret_cast<Piece*>(q + half) = pz;
-        } else if (const int row = a.kv_row[t]; row >= 0) {
+        } else if (row >= 0) {
             if (part == 1) {
                 __bf16* k = reinterpret_cast<__bf16*>(a.pool.keys);
                 *reinterpret_cast<Piece*>(k + key_off(row, head, a.pool.G, d0, a.pool.dim_ld)) = py;
@@ -324,7 +330,25 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T, int 
                 if (turns) *reinterpret_cast<Piece*>(state + (size_t)j * a.channels + half) = v;
             }
         }
+    };
+#pragma unroll
+    for (int u = 0; u < TOK; u++) {
+        const int t = t0 + u, off = t - spans[u].x;
+        // (a token that sees the state of a portion that starts in front of these belongs to the thread of its first token)
+        if (t < T && !(off > 0 && off < KEEP && spans[u].x < t0)) token(t, spans[u], rows[u], in[u], inz[u]);
     }
+    const int4 last = spans[TOK - 1];   // the portion the next tokens may belong to
+    for (int t = t0 + TOK; t < last.x + min(last.y, KEEP) && last.x >= t0; t++)
+        token(t, last, a.kv_row[t], *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld), *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner));
+}
+
+template <int KEEP>
+static void launch_walk(const ConvKArgs& a, int T) {
+    const dim3 threads(std::min(256, (a.items + 63) & ~63));
+    const int y = cdiv(a.items, 256);
+    if (T >= 1024) NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 4>), dim3(cdiv(T, 4), y), threads, 0, a, T);
+    else if (T >= 256) NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 2>), dim3(cdiv(T, 2), y), threads, 0, a, T);
+    else NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 1>), dim3(T, y), threads, 0, a, T);
 }
 
 void launch_conv_rope(const ConvRope& c, const KvPages& pool, const StepArrays& st) {
@@ -351,14 +375,12 @@ void launch_conv_rope(const ConvRope& c, const KvPages& pool, const StepArrays& 
     ProfScope ps(PC_CONV_ROPE, elems * pool.elem_bytes + (double)a.channels * c.n_taps * 4.0, elems * c.n_taps);
     const dim3 grid(st.T, cdiv(a.items, 256));
     if (wide && c.n_taps <= 5 && (c.taps || c.n_taps == 1)) {
-        const int TOK = st.T >= 1024 ? 4 : st.T >= 256 ? 2 : 1, threads = std::min(256, (a.items + 63) & ~63);
-        const dim3 walk(cdiv(st.T, TOK), cdiv(a.items, 256));
         switch (c.n_taps) {
-            case 1: NVLLM_LAUNCH((k_conv_rope_walk<0>), walk, dim3(threads), 0, a, st.T, TOK); break;
-            case 2: NVLLM_LAUNCH((k_conv_rope_walk<1>), walk, dim3(threads), 0, a, st.T, TOK); break;
-            case 3: NVLLM_LAUNCH((k_conv_rope_walk<2>), walk, dim3(threads), 0, a, st.T, TOK); break;
-            case 4: NVLLM_LAUNCH((k_conv_rope_walk<3>), walk, dim3(threads), 0, a, st.T, TOK); break;
-            default: NVLLM_LAUNCH((k_conv_rope_walk<4>), walk, dim3(threads), 0, a, st.T, TOK); break;
+            case 1: launch_walk<0>(a, st.T); break;
+            case 2: launch_walk<1>(a, st.T); break;
+            case 3: launch_walk<2>(a, st.T); break;
+            case 4: launch_walk<3>(a, st.T); break;
+            default: launch_walk<4>(a, st.T); break;
         }
         return;
     }
