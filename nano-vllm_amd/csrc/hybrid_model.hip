@@ -477,8 +477,11 @@ void HybridModel::forward(const PassArgs& a) {
         slots = std::max(slots, a.seq_ids[t] + 1);
     }
     init_states(slots);
+    int group = LIGHTNING_CHUNK;
+    for (const auto& l : layers_)
+        if (l.m.lightning) group = std::max(group, lightning_group(a.T, l.m.heads, l.m.vdim));
     const StepArrays st = stage_step(a.tokens, a.pos, a.seq_ids, a.T, a.output_indices, a.B, a.tables, nullptr, 0, a.mgr->block_size, WINDOW_RUN, a.token_src, true, true,
-                                     LIGHTNING_CHUNK);
+                                     group);
     if (st.table_short) NVLLM_FATAL("transformer_batch: a position lies beyond its sequence's block table (allocate the block first)");
     if (st.seq_split) NVLLM_FATAL("transformer_batch: the tokens of a sequence must lie side by side in the batch");
     if (f32_) forward_f32(a, st);

@@ -123,7 +123,7 @@ void nvllm_lightning(float* out, float* ss, const float* q, const float* k, cons
                      int* seq_ids, int* pos_arr, int heads, int dim, int vdim, int elem_bytes, int num_tokens) {
     ensure_init();
     if (num_tokens <= 0) return;
-    const StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, nullptr, nullptr, 0, 1, 0, nullptr, false, true, LIGHTNING_CHUNK);
+    const StepArrays s = stage_step(nullptr, pos_arr, seq_ids, num_tokens, nullptr, 0, nullptr, nullptr, 0, 1, 0, nullptr, false, true, lightning_group(num_tokens, heads, vdim));
     if (s.seq_split) NVLLM_FATAL("linear attention: a sequence's tokens must lie side by side in the batch");
     std::vector<float> powers((size_t)heads * (LIGHTNING_CHUNK + 1));
     for (int h = 0; h < heads; h++)

@@ -7,7 +7,9 @@
 
 namespace nvllm {
 
-constexpr int LIGHTNING_CHUNK = 64;   // tokens per step of the chunked kernel
+constexpr int LIGHTNING_CHUNK = 64;   // tokens per step of the chunked kernels
+// stage_step(chunk_len) for a batch of T tokens: tokens a workgroup of the chunked kernels walks
+int lightning_group(int T, int H, int vdim);
 
 // One layer run over a batch.  Every sequence's portion starts from its slot's state (from zero at position 0) and
 // leaves the state behind its last token there.

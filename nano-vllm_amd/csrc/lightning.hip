@@ -1,13 +1,14 @@
 // lightning.hip -- linear attention with decay (lightning.h).
 //
-// Portions of several tokens (bf16) are cut into chunks of 64 tokens, all at once, in three launches:
-//   k_lightning_add    U_c = sum_s k_s (decay^(n-1-s) v_s)^T of every chunk
-//   k_lightning_scan   S_c = decay^n S_(c-1) + U_c over a portion's chunks, element by element; U_c gives way to S_(c-1)
-//   k_lightning_out    o_t = decay^(t+1) S_(c-1)^T q_t + sum_{s <= t} decay^(t-s) (k_s . q_t) v_s
-// A workgroup takes a chunk's head x 64 value columns, a wave 16 of them.  q, k and v are bf16 values.  The 32-bit factors
-// -- S, the decayed products P[s, t] of queries and keys, the decayed v -- enter the matrix cores as three bf16 parts
-// (truncations: 8 + 8 + 8 bits, together the exact value), so every product is that of the 32-bit numbers.  The state's
-// result registers are already in the k order of S^T q, P's in that of P v.
+// Portions of several tokens (bf16) go in chunks of 64 tokens, a few neighbouring chunks (a group) to a workgroup, as many as
+// still leave the chip full; three launches:
+//   k_lightning_add    what a group adds to the state, chunk by chunk: U = decay^n U + sum_s k_s (decay^(n-1-s) v_s)^T
+//   k_lightning_scan   the states groups start from, over a portion's groups, element by element; U gives way to S
+//   k_lightning_out    o_t = decay^(t+1) S^T q_t + sum_{s <= t} decay^(t-s) (k_s . q_t) v_s chunk by chunk, S carried along
+// A workgroup takes a group's head x 64 value columns, a wave 16 of them, the state in its registers.  q, k and v are bf16
+// values.  The 32-bit factors -- S, the decayed products P[s, t] of queries and keys, the decayed v -- enter the matrix
+// cores as three bf16 parts (truncations: 8 + 8 + 8 bits, together the exact value), so every product is that of the 32-bit
+// numbers.  The state's result registers are already in the k order of S^T q, P's in that of P v.
 //
 // k_lightning_step (single tokens, and everything in fp32): a workgroup per (portion, head), the state streamed once per
 // token as float4 columns.
@@ -54,18 +55,17 @@ constexpr int qk_row(int DC) { return DC * 32 + 8; }
 constexpr int add_lds(int DC) { return CH * qk_row(DC) * 2 + CH * VROW * 2 + (CH + 1) * 4; }
 constexpr int out_lds(int DC) { return 2 * CH * qk_row(DC) * 2 + CH * VROW * 2 + 4 * 2 * 3 * 1024 + (CH + 1) * 4; }
 
-// What the chunk kernels share: a workgroup = chunk x head x 64 value columns, a wave = 16 of the columns.
+// What the chunk kernels share: a workgroup = group of chunks x head x 64 value columns, a wave = 16 of the columns.
 struct ChunkArgs {
     Lightning a;
     const int4* spans;     // (first token, count, first position, sequence)
-    const int2* chunks;    // (span, chunk of the span)
-    int n_spans, vslices;
-    float* mem;            // [chunk][H][value tile][dim tile][64][4]: a tile as the matrix cores leave it, lane (x, g) = S[16 i + 4 g + r][16 j + x]
+    const int2* groups;    // (span, group of the span): `per_group` neighbouring chunks
+    int n_spans, vslices, per_group;
+    float* mem;            // [group][H][value tile][dim tile][64][4]: a tile as the matrix cores leave it, lane (x, g) = S[16 i + 4 g + r][16 j + x]
     int d_tiles, v_tiles;
 };
 struct ChunkId {
-    int slot, h, vs, first, n;   // first: token of the batch
-    int4 span;
+    int slot, h, vs, first, n;   // the group, its first token of the batch and its number of tokens
 };
 __device__ __forceinline__ ChunkId chunk_id(const ChunkArgs& c) {
     ChunkId id;
@@ -74,17 +74,17 @@ __device__ __forceinline__ ChunkId chunk_id(const ChunkArgs& c) {
     idx /= c.vslices;
     id.h = idx % c.a.H;
     id.slot = idx / c.a.H;
-    const int2 ch = c.chunks[id.slot];
-    id.span = c.spans[ch.x];
-    id.first = id.span.x + ch.y * CH;
-    id.n = min(CH, id.span.y - ch.y * CH);
+    const int2 gr = c.groups[id.slot];
+    const int4 span = c.spans[gr.x];
+    id.first = span.x + gr.y * c.per_group * CH;
+    id.n = min(c.per_group * CH, span.y - gr.y * c.per_group * CH);
     return id;
 }
 __device__ __forceinline__ f4_t* chunk_tiles(const ChunkArgs& c, int slot, int h, int vtile) {   // dim tile 0, lane 0
     return reinterpret_cast<f4_t*>(c.mem) + (((size_t)slot * c.a.H + h) * c.v_tiles + vtile) * c.d_tiles * 64;
 }
-// rows of the chunk, 16-byte pieces, zeros behind its end: `base` = first row's first element, `pieces` live pieces, to LDS rows of ROW halves
-template <int PER, int ROW, int U>
+// rows of a chunk, PER 16-byte pieces each by neighbouring threads, zeros behind the n-th row and the last of `pieces`
+template <int PER, int U>
 __device__ __forceinline__ void chunk_rows(u4_t (&r)[U], const __half* base, int ld, int n, int pieces) {
 #pragma unroll
     for (int u = 0; u < U; u++) {
@@ -110,7 +110,33 @@ __device__ __forceinline__ b8_t token_frag(const __half* lds, int row_halves, in
     return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
 }
 
-// ---- 1. what a chunk adds to the state: sum_s k_s (decay^(n-1-s) v_s)^T
+// S <- decay^n S + sum_s k_s (decay^(n-1-s) v_s)^T over a chunk of n tokens
+template <int DC>
+__device__ __forceinline__ void chunk_update(f4_t (&S)[2 * DC], const __half* s_k, const b8_t (&vf)[2], const float* s_dec, int n) {
+    const int g = (threadIdx.x >> 4) & 3;
+    const float fade = s_dec[n];
+#pragma unroll
+    for (int i = 0; i < 2 * DC; i++) S[i] *= fade;
+#pragma unroll
+    for (int pair = 0; pair < 2; pair++) {
+        float e[8];
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            const int s = 32 * pair + 16 * (i >> 2) + 4 * g + (i & 3);
+            e[i] = s < n ? (float)vf[pair][i] * s_dec[max(n - 1 - s, 0)] : 0.f;
+        }
+        b8_t parts[3];
+        split3_frag(e, parts);
+#pragma unroll
+        for (int i = 0; i < 2 * DC; i++) {
+            const b8_t kt = token_frag(s_k, qk_row(DC), 16 * i, pair);
+#pragma unroll
+            for (int k = 2; k >= 0; k--) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt, parts[k], S[i], 0, 0, 0);
+        }
+    }
+}
+
+// ---- 1. what a group of chunks adds to the state
 template <int DC>
 __global__ __launch_bounds__(256, 2) void k_lightning_add(ChunkArgs c) {
     constexpr int ROW = qk_row(DC);
@@ -120,47 +146,41 @@ __global__ __launch_bounds__(256, 2) void k_lightning_add(ChunkArgs c) {
     float* s_dec = reinterpret_cast<float*>(s_v + CH * VROW);
     const Lightning& a = c.a;
     const ChunkId id = chunk_id(c);
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4;
-    const int n = id.n, v0 = id.vs * 64, my_v = v0 + wave * 16;
-    const __half* base = a.rows + (size_t)id.first * a.ld;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int v0 = id.vs * 64, my_v = v0 + wave * 16;
+    const bool has_v = my_v < a.vdim_ld;
     u4_t rk[DC], rv[2];
-    chunk_rows<4 * DC, ROW>(rk, base + (a.H + id.h) * a.dim_ld, a.ld, n, a.dim_ld / 8);
-    chunk_rows<8, VROW>(rv, base + 2 * a.H * a.dim_ld + id.h * a.vdim_ld + v0, a.ld, n, (a.vdim_ld - v0) / 8);
+    auto fetch = [&](int c0) {
+        const __half* base = a.rows + (size_t)(id.first + c0) * a.ld;
+        chunk_rows<4 * DC>(rk, base + (a.H + id.h) * a.dim_ld, a.ld, id.n - c0, a.dim_ld / 8);
+        chunk_rows<8>(rv, base + 2 * a.H * a.dim_ld + id.h * a.vdim_ld + v0, a.ld, id.n - c0, (a.vdim_ld - v0) / 8);
+    };
+    fetch(0);
     if (tid <= CH) s_dec[tid] = a.decay[id.h * (CH + 1) + tid];
-    chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
-    chunk_rows_to_lds<8, VROW>(s_v, rv);
-    __syncthreads();
-    if (my_v >= a.vdim_ld) return;
     f4_t S[2 * DC];
 #pragma unroll
     for (int i = 0; i < 2 * DC; i++) S[i] = f4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int pair = 0; pair < 2; pair++) {
-        float e[8];
-        const b8_t vv = token_frag(s_v, VROW, wave * 16, pair);
-#pragma unroll
-        for (int i = 0; i < 8; i++) {
-            const int s = 32 * pair + 16 * (i >> 2) + 4 * g + (i & 3);
-            e[i] = s < n ? (float)vv[i] * s_dec[max(n - 1 - s, 0)] : 0.f;
+    for (int c0 = 0; c0 < id.n; c0 += CH) {
+        chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
+        chunk_rows_to_lds<8, VROW>(s_v, rv);
+        __syncthreads();
+        if (c0 + CH < id.n) fetch(c0 + CH);
+        if (has_v) {
+            const b8_t vf[2] = {token_frag(s_v, VROW, wave * 16, 0), token_frag(s_v, VROW, wave * 16, 1)};
+            chunk_update<DC>(S, s_k, vf, s_dec, min(CH, id.n - c0));
         }
-        b8_t parts[3];
-        split3_frag(e, parts);
-#pragma unroll
-        for (int i = 0; i < 2 * DC; i++) {
-            const b8_t kt = token_frag(s_k, ROW, 16 * i, pair);
-#pragma unroll
-            for (int k = 2; k >= 0; k--) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt, parts[k], S[i], 0, 0, 0);
-        }
+        __syncthreads();   // the chunk's rows have been read
     }
+    if (!has_v) return;
     f4_t* out = chunk_tiles(c, id.slot, id.h, my_v >> 4) + lane;
 #pragma unroll
     for (int i = 0; i < 2 * DC; i++)
         if (i < c.d_tiles) out[i * 64] = S[i];
 }
 
-// ---- 2. from what chunks add to the states they start from, and the sequence's state behind its portion.  A thread per four
-// elements of a state; chunk_of_span: the first chunk of every portion.
-__global__ __launch_bounds__(256) void k_lightning_scan(ChunkArgs c, const int* __restrict__ first_chunk) {
+// ---- 2. from what groups add to the states they start from, and the sequence's state behind its portion.  A thread per four
+// elements of a state; first_group: of every portion.
+__global__ __launch_bounds__(256) void k_lightning_scan(ChunkArgs c, const int* __restrict__ first_group) {
     const Lightning& a = c.a;
     const int tiles = c.v_tiles * c.d_tiles, item = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y;
     if (item >= tiles * 64) return;
@@ -171,20 +191,25 @@ __global__ __launch_bounds__(256) void k_lightning_scan(ChunkArgs c, const int* 
     f4_t S;
 #pragma unroll
     for (int r = 0; r < 4; r++) S[r] = span.z > 0 && d0 + r < a.dim && v < a.vdim ? st[(size_t)(d0 + r) * a.vdim + v] : 0.f;
-    const int n_chunks = (span.y + CH - 1) / CH;
+    const int len = c.per_group * CH, n_groups = (span.y + len - 1) / len;
     const size_t stride = (size_t)a.H * tiles * 64;
-    f4_t* p = reinterpret_cast<f4_t*>(c.mem) + (size_t)first_chunk[blockIdx.z] * stride + (size_t)h * tiles * 64 + item;
+    f4_t* p = reinterpret_cast<f4_t*>(c.mem) + (size_t)first_group[blockIdx.z] * stride + (size_t)h * tiles * 64 + item;
     const float* dec = a.decay + h * (CH + 1);
-    const float whole = dec[CH], tail = dec[span.y - (n_chunks - 1) * CH];
-    for (int k0 = 0; k0 < n_chunks; k0 += 8) {
+    auto faded = [&](int tokens) {   // decay^tokens
+        float f = 1.f;
+        for (; tokens > CH; tokens -= CH) f *= dec[CH];
+        return f * dec[tokens];
+    };
+    const float whole = faded(len), tail = faded(span.y - (n_groups - 1) * len);
+    for (int k0 = 0; k0 < n_groups; k0 += 8) {
         f4_t u[8];
 #pragma unroll
-        for (int k = 0; k < 8; k++) u[k] = p[min(k0 + k, n_chunks - 1) * stride];
+        for (int k = 0; k < 8; k++) u[k] = p[min(k0 + k, n_groups - 1) * stride];
 #pragma unroll
         for (int k = 0; k < 8; k++)
-            if (k0 + k < n_chunks) {
+            if (k0 + k < n_groups) {
                 p[(k0 + k) * stride] = S;
-                S = S * (k0 + k == n_chunks - 1 ? tail : whole) + u[k];
+                S = S * (k0 + k == n_groups - 1 ? tail : whole) + u[k];
             }
     }
 #pragma unroll
@@ -192,7 +217,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(ChunkArgs c, const int* 
         if (d0 + r < a.dim && v < a.vdim) st[(size_t)(d0 + r) * a.vdim + v] = S[r];
 }
 
-// ---- 3. the chunk's results
+// ---- 3. the results, chunk by chunk from the state the group starts from
 template <int DC>
 __global__ __launch_bounds__(256, 2) void k_lightning_out(ChunkArgs c) {
     constexpr int ROW = qk_row(DC);
@@ -205,114 +230,131 @@ __global__ __launch_bounds__(256, 2) void k_lightning_out(ChunkArgs c) {
     const Lightning& a = c.a;
     const ChunkId id = chunk_id(c);
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), x = lane & 15, g = lane >> 4;
-    const int n = id.n, h = id.h, v0 = id.vs * 64, my_v = v0 + wave * 16;
+    const int h = id.h, v0 = id.vs * 64, my_v = v0 + wave * 16;
     const bool has_v = my_v < a.vdim_ld;
-    const __half* base = a.rows + (size_t)id.first * a.ld;
     u4_t rq[DC], rk[DC], rv[2];
-    chunk_rows<4 * DC, ROW>(rq, base + h * a.dim_ld, a.ld, n, a.dim_ld / 8);
-    chunk_rows<4 * DC, ROW>(rk, base + (a.H + h) * a.dim_ld, a.ld, n, a.dim_ld / 8);
-    chunk_rows<8, VROW>(rv, base + 2 * a.H * a.dim_ld + h * a.vdim_ld + v0, a.ld, n, (a.vdim_ld - v0) / 8);
-    // this wave's columns of the state, of the gates (tokens 16 i + x) and of the gain
+    u2_t rg[4];   // gates of this wave's columns my_v + 4 g .. + 3, tokens 16 i + x
+    auto fetch = [&](int c0) {
+        const __half* base = a.rows + (size_t)(id.first + c0) * a.ld;
+        const int left = id.n - c0;
+        chunk_rows<4 * DC>(rq, base + h * a.dim_ld, a.ld, left, a.dim_ld / 8);
+        chunk_rows<4 * DC>(rk, base + (a.H + h) * a.dim_ld, a.ld, left, a.dim_ld / 8);
+        chunk_rows<8>(rv, base + 2 * a.H * a.dim_ld + h * a.vdim_ld + v0, a.ld, left, (a.vdim_ld - v0) / 8);
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            rg[i] = has_v ? *reinterpret_cast<const u2_t*>(base + (size_t)min(16 * i + x, left - 1) * a.ld + 2 * a.H * a.dim_ld + (a.H + h) * a.vdim_ld + my_v + 4 * g) : u2_t{0, 0};
+    };
+    fetch(0);
     f4_t S[2 * DC], gain = {0.f, 0.f, 0.f, 0.f};
-    u2_t gates[4];
+#pragma unroll
+    for (int i = 0; i < 2 * DC; i++) S[i] = f4_t{0.f, 0.f, 0.f, 0.f};
     if (has_v) {
         const f4_t* in = chunk_tiles(c, id.slot, h, my_v >> 4) + lane;
 #pragma unroll
-        for (int i = 0; i < 2 * DC; i++) S[i] = i < c.d_tiles ? in[i * 64] : f4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int i = 0; i < 4; i++)
-            gates[i] = *reinterpret_cast<const u2_t*>(base + (size_t)min(16 * i + x, n - 1) * a.ld + 2 * a.H * a.dim_ld + (a.H + h) * a.vdim_ld + my_v + 4 * g);
+        for (int i = 0; i < 2 * DC; i++)
+            if (i < c.d_tiles) S[i] = in[i * 64];
         gain = *reinterpret_cast<const f4_t*>(a.gain + h * a.vdim_ld + my_v + 4 * g);
     }
     if (tid <= CH) s_dec[tid] = a.decay[h * (CH + 1) + tid];
-    chunk_rows_to_lds<4 * DC, ROW>(s_q, rq);
-    chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
-    chunk_rows_to_lds<8, VROW>(s_v, rv);
-    __syncthreads();
-    // operands over dims in the order of the state's registers: {32 cc + 4 g .., 32 cc + 16 + 4 g ..} of row 16 i + x
-    auto frag = [&](const __half* lds, int i, int cc) {
-        const __half* p = lds + (16 * i + x) * ROW + 32 * cc + 4 * g;
-        const u2_t lo = *reinterpret_cast<const u2_t*>(p), hi = *reinterpret_cast<const u2_t*>(p + 16);
-        return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
-    };
-    // ---- P of token tile `wave`: rows s (tiles 0 .. wave), columns t
-    if (wave * 16 < n) {
-        b8_t qf[DC];
+    const int ss_ld = a.H * a.vdim_ld / 16, Kb_out = a.H * a.vdim_ld / 32, col = h * a.vdim_ld + my_v;
+    for (int c0 = 0; c0 < id.n; c0 += CH) {
+        const int n = min(CH, id.n - c0);
+        chunk_rows_to_lds<4 * DC, ROW>(s_q, rq);
+        chunk_rows_to_lds<4 * DC, ROW>(s_k, rk);
+        chunk_rows_to_lds<8, VROW>(s_v, rv);
+        u2_t gates[4];
 #pragma unroll
-        for (int cc = 0; cc < DC; cc++) qf[cc] = frag(s_q, wave, cc);
-        const int t = wave * 16 + x;
+        for (int i = 0; i < 4; i++) gates[i] = rg[i];
+        __syncthreads();
+        const bool more = c0 + CH < id.n;
+        if (more) fetch(c0 + CH);
+        // operands over dims in the order of the state's registers: {32 cc + 4 g .., 32 cc + 16 + 4 g ..} of row 16 i + x
+        auto frag = [&](const __half* lds, int i, int cc) {
+            const __half* p = lds + (16 * i + x) * ROW + 32 * cc + 4 * g;
+            const u2_t lo = *reinterpret_cast<const u2_t*>(p), hi = *reinterpret_cast<const u2_t*>(p + 16);
+            return __builtin_bit_cast(b8_t, u4_t{lo[0], lo[1], hi[0], hi[1]});
+        };
+        // ---- P of token tile `wave`: rows s (tiles 0 .. wave), columns t
+        if (wave * 16 < n) {
+            b8_t qf[DC];
 #pragma unroll
-        for (int pair = 0; pair < 2; pair++) {
-            if (2 * pair > wave) break;
+            for (int cc = 0; cc < DC; cc++) qf[cc] = frag(s_q, wave, cc);
+            const int t = wave * 16 + x;
+#pragma unroll
+            for (int pair = 0; pair < 2; pair++) {
+                if (2 * pair > wave) break;
+                float e[8];
+#pragma unroll
+                for (int half = 0; half < 2; half++) {
+                    f4_t p = {0.f, 0.f, 0.f, 0.f};
+                    const int i = 2 * pair + half;
+                    if (i <= wave) {
+#pragma unroll
+                        for (int cc = 0; cc < DC; cc++) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(s_k, i, cc), qf[cc], p, 0, 0, 0);
+                    }
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int s = 16 * i + 4 * g + r;
+                        e[4 * half + r] = s <= t ? p[r] * s_dec[max(t - s, 0)] : 0.f;
+                    }
+                }
+                b8_t parts[3];
+                split3_frag(e, parts);
+#pragma unroll
+                for (int k = 0; k < 3; k++) s_p[((wave * 2 + pair) * 3 + k) * 64 + lane] = parts[k];
+            }
+        }
+        b8_t sf[DC][3];   // the state as operand, three exact parts
+#pragma unroll
+        for (int cc = 0; cc < DC; cc++) {
             float e[8];
 #pragma unroll
-            for (int half = 0; half < 2; half++) {
-                f4_t p = {0.f, 0.f, 0.f, 0.f};
-                const int i = 2 * pair + half;
-                if (i <= wave) {
+            for (int i = 0; i < 8; i++) e[i] = S[2 * cc + (i >> 2)][i & 3];
+            split3_frag(e, sf[cc]);
+        }
+        __syncthreads();
+        if (has_v) {
+            const b8_t vf[2] = {token_frag(s_v, VROW, wave * 16, 0), token_frag(s_v, VROW, wave * 16, 1)};
+            // (the four token tiles are independent chains of products)
+            f4_t o[4];
 #pragma unroll
-                    for (int cc = 0; cc < DC; cc++) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(s_k, i, cc), qf[cc], p, 0, 0, 0);
-                }
+            for (int i = 0; i < 4; i++) o[i] = f4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    const int s = 16 * i + 4 * g + r;
-                    e[4 * half + r] = s <= t ? p[r] * s_dec[max(t - s, 0)] : 0.f;
+            for (int cc = 0; cc < DC; cc++) {
+                b8_t qf[4];
+#pragma unroll
+                for (int i = 0; i < 4; i++) qf[i] = frag(s_q, i, cc);
+#pragma unroll
+                for (int k = 2; k >= 0; k--)
+#pragma unroll
+                    for (int i = 0; i < 4; i++) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf[cc][k], qf[i], o[i], 0, 0, 0);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++) o[i] *= s_dec[i * 16 + x + 1];
+#pragma unroll
+            for (int pair = 0; pair < 2; pair++)
+#pragma unroll
+                for (int k = 2; k >= 0; k--)
+#pragma unroll
+                    for (int i = 2 * pair; i < 4; i++)   // (P of tiles past the chunk's end is whatever LDS holds; their results are not stored)
+                        o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pair], s_p[((i * 2 + pair) * 3 + k) * 64 + lane], o[i], 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                float sq = o[i][0] * o[i][0] + o[i][1] * o[i][1] + o[i][2] * o[i][2] + o[i][3] * o[i][3];
+                sq += __shfl_xor(sq, 16, 64);
+                sq += __shfl_xor(sq, 32, 64);
+                const int tl = i * 16 + x, t = id.first + c0 + tl;
+                if (tl < n) {
+                    float y[4];
+#pragma unroll
+                    for (int r = 0; r < 4; r++) y[r] = o[i][r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gates[i][r >> 1] >> (16 * (r & 1)))));
+                    store_b16_4(a.out_b16, Kb_out, t, col + 4 * g, y);
+                    if (g == 0) a.ss_out[(size_t)t * ss_ld + (col >> 4)] = sq;
                 }
             }
-            b8_t parts[3];
-            split3_frag(e, parts);
-#pragma unroll
-            for (int k = 0; k < 3; k++) s_p[((wave * 2 + pair) * 3 + k) * 64 + lane] = parts[k];
+            if (more) chunk_update<DC>(S, s_k, vf, s_dec, n);
         }
-    }
-    b8_t sf[DC][3];   // the state as operand, three exact parts
-#pragma unroll
-    for (int cc = 0; cc < DC; cc++) {
-        float e[8];
-#pragma unroll
-        for (int i = 0; i < 8; i++) e[i] = S[2 * cc + (i >> 2)][i & 3];
-        split3_frag(e, sf[cc]);
-    }
-    __syncthreads();
-    if (!has_v) return;
-    const b8_t vf[2] = {token_frag(s_v, VROW, wave * 16, 0), token_frag(s_v, VROW, wave * 16, 1)};
-    // (the four token tiles are independent chains of products)
-    f4_t o[4];
-#pragma unroll
-    for (int i = 0; i < 4; i++) o[i] = f4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int cc = 0; cc < DC; cc++) {
-        b8_t qf[4];
-#pragma unroll
-        for (int i = 0; i < 4; i++) qf[i] = frag(s_q, i, cc);
-#pragma unroll
-        for (int k = 2; k >= 0; k--)
-#pragma unroll
-            for (int i = 0; i < 4; i++) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf[cc][k], qf[i], o[i], 0, 0, 0);
-    }
-#pragma unroll
-    for (int i = 0; i < 4; i++) o[i] *= s_dec[i * 16 + x + 1];
-#pragma unroll
-    for (int pair = 0; pair < 2; pair++)
-#pragma unroll
-        for (int k = 2; k >= 0; k--)
-#pragma unroll
-            for (int i = 2 * pair; i < 4; i++)   // (P of tiles past the chunk's end is whatever LDS holds; their results are not stored)
-                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pair], s_p[((i * 2 + pair) * 3 + k) * 64 + lane], o[i], 0, 0, 0);
-    const int ss_ld = a.H * a.vdim_ld / 16, Kb_out = a.H * a.vdim_ld / 32, col = h * a.vdim_ld + my_v;
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        float sq = o[i][0] * o[i][0] + o[i][1] * o[i][1] + o[i][2] * o[i][2] + o[i][3] * o[i][3];
-        sq += __shfl_xor(sq, 16, 64);
-        sq += __shfl_xor(sq, 32, 64);
-        const int tl = i * 16 + x, t = id.first + tl;
-        if (tl < n) {
-            float y[4];
-#pragma unroll
-            for (int r = 0; r < 4; r++) y[r] = o[i][r] * gain[r] * sigmoid_f(b16_f((unsigned short)(gates[i][r >> 1] >> (16 * (r & 1)))));
-            store_b16_4(a.out_b16, Kb_out, t, col + 4 * g, y);
-            if (g == 0) a.ss_out[(size_t)t * ss_ld + (col >> 4)] = sq;
-        }
+        __syncthreads();   // the chunk's rows and P have been read
     }
 }
 
@@ -415,27 +457,28 @@ __global__ __launch_bounds__(256) void k_lightning_step(Lightning a, const int4*
 }
 
 template <int DC>
-static void launch_add(const ChunkArgs& c, int n_chunks) {
+static void launch_add(const ChunkArgs& c, int n_groups) {
     constexpr int shmem = add_lds(DC);
     static_assert(shmem <= 64 * 1024, "no attribute needed");
-    NVLLM_LAUNCH((k_lightning_add<DC>), dim3(n_chunks * c.a.H * c.vslices), dim3(256), shmem, c);
+    NVLLM_LAUNCH((k_lightning_add<DC>), dim3(n_groups * c.a.H * c.vslices), dim3(256), shmem, c);
 }
 template <int DC>
-static void launch_out(const ChunkArgs& c, int n_chunks) {
+static void launch_out(const ChunkArgs& c, int n_groups) {
     constexpr int shmem = out_lds(DC);
     static bool enabled = false;
     if (shmem > 64 * 1024 && !enabled) {
         HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_lightning_out<DC>), hipFuncAttributeMaxDynamicSharedMemorySize, shmem));
         enabled = true;
     }
-    NVLLM_LAUNCH((k_lightning_out<DC>), dim3(n_chunks * c.a.H * c.vslices), dim3(256), shmem, c);
+    NVLLM_LAUNCH((k_lightning_out<DC>), dim3(n_groups * c.a.H * c.vslices), dim3(256), shmem, c);
 }
 // Portions of several tokens: the chunks' additions, the scan over them, the chunks' results.
 static void launch_chunks(const Lightning& a, const StepArrays& st, double bytes, double flops) {
     ChunkArgs c{};
     c.a = a;
     c.spans = (const int4*)st.d_spans;
-    c.chunks = (const int2*)st.d_chunks;
+    c.groups = (const int2*)st.d_chunks;
+    c.per_group = st.chunk_len / CH;
     c.n_spans = st.n_spans_multi;
     c.vslices = cdiv(a.vdim_ld, 64);
     c.d_tiles = a.dim_ld / 16;
@@ -464,6 +507,13 @@ static void launch_chunks(const Lightning& a, const StepArrays& st, double bytes
     else launch_out<8>(c, n);
 }
 
+int lightning_group(int T, int H, int vdim) {
+    const long wgs = (long)cdiv(T, CH) * H * cdiv(vdim, 64);   // with one chunk each
+    int per = 1;
+    while (per < 8 && wgs / (2 * per) >= 2 * rt().num_cus) per *= 2;
+    return per * CH;
+}
+
 void launch_lightning(const Lightning& a, const StepArrays& st) {
     if (st.T <= 0) return;
     if (!st.d_spans) NVLLM_FATAL("linear attention: the batch was staged without its portions");
@@ -475,7 +525,7 @@ void launch_lightning(const Lightning& a, const StepArrays& st) {
     const int DC = a.dim_ld / 32;
     const bool chunked = b16 && DC <= 8;
     if (chunked && st.n_spans_multi > 0) {
-        if (st.chunk_len != CH) NVLLM_FATAL("linear attention: the batch was staged in chunks of %d tokens", st.chunk_len);
+        if (st.chunk_len < CH || st.chunk_len % CH) NVLLM_FATAL("linear attention: the batch was staged in chunks of %d tokens", st.chunk_len);
         launch_chunks(a, st, st.n_spans_multi * state_bytes + multi_tokens * token_bytes, multi_tokens * (token_flops + pair * 0.5 * std::min(st.max_span, CH)));
     }
     const int from = chunked ? st.n_spans_multi : 0, n = st.n_spans - from;
