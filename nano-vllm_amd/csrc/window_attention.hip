@@ -558,23 +558,28 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
     const int it0 = split * per + (SINGLE ? wave : 0), it1 = min(n_pairs, split * per + per);
     constexpr int STRIDE = SINGLE ? WAVES : 1;
     auto page_at = [&](int i) { return i < n_kept ? i : first_pg + i - n_kept; };   // position / 16
-    auto page_id = [&](int pg) { return (table[pg >> a.page_shift] << a.page_shift) + (pg & ((1 << a.page_shift) - 1)); };
 
     // Pages in registers: of two steps (DEEP: a step's are requested before the step ahead of it is computed) or of one.
-    constexpr bool DEEP = 2 * (8 * KC + 4 * VT) + C * 4 * (KC + VT) <= 176;
+    constexpr bool DEEP = EXACT && 2 * (8 * KC + 4 * VT) + C * 4 * (KC + VT) <= 176;
     constexpr int SETS = DEEP ? 2 : 1;
     h8_t kf[SETS][2][KC];
     u2_t vf[SETS][2][VT];
-    int ids[2] = {0, 0};   // pages of the step that is requested next
+    // The step that is requested next: entries of the block table (looked up a step earlier; used as late as possible, so that
+    // nothing waits for the look-up) and the pages' places in their blocks.
+    int entry[2], inside[2];
     auto look_up = [&](int it) {
-        if (it < it1)
 #pragma unroll
-            for (int p = 0; p < 2; p++) ids[p] = page_id(page_at(min(2 * it + p, n_pages - 1)));
+        for (int p = 0; p < 2; p++) {
+            const int pg = page_at(min(2 * it + p, n_pages - 1));
+            entry[p] = table[pg >> a.page_shift];
+            inside[p] = pg & ((1 << a.page_shift) - 1);
+        }
     };
+    auto page_id = [&](int p) { return (entry[p] << a.page_shift) + inside[p]; };
     auto load_keys = [&](int set) {
 #pragma unroll
         for (int p = 0; p < 2; p++) {
-            const h8_t* src = reinterpret_cast<const h8_t*>(a.keys + ((size_t)ids[p] * a.G + grp) * (KV_PAGE * 32 * kc)) + lane;
+            const h8_t* src = reinterpret_cast<const h8_t*>(a.keys + ((size_t)page_id(p) * a.G + grp) * (KV_PAGE * 32 * kc)) + lane;
 #pragma unroll
             for (int k = 0; k < KC; k++)
                 if (EXACT || k < kc) kf[set][p][k] = src[k * 64];
@@ -583,7 +588,7 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
     auto load_values = [&](int set) {
 #pragma unroll
         for (int p = 0; p < 2; p++) {
-            const u2_t* src = reinterpret_cast<const u2_t*>(a.values + ((size_t)ids[p] * a.G + grp) * (KV_PAGE * 16 * vt)) + lane;
+            const u2_t* src = reinterpret_cast<const u2_t*>(a.values + ((size_t)page_id(p) * a.G + grp) * (KV_PAGE * 16 * vt)) + lane;
 #pragma unroll
             for (int v = 0; v < VT; v++)
                 if (EXACT || v < vt) vf[set][p][v] = src[v * 64];
@@ -603,15 +608,10 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
     const float grow = CAP ? 2.f * a.scale / a.cap * LOG2E : 0.f;                   // cap: tanh(s/cap) = 1 - 2 / (1 + 2^(grow s))
     const float top = a.cap * LOG2E;
 
-    look_up(it0);
-    if (it0 < it1) {
-        load_keys(0);
-        load_values(0);
-    }
-    look_up(it0 + STRIDE);
-    auto step = [&](const int it, const int set) __attribute__((always_inline)) {   // set: where this step's pages are
-        const bool more = it + STRIDE < it1;
-        if (DEEP && more) {
+    // set: where this step's pages are.  The next step's are requested whether or not there is one (the last pages again, then:
+    // no memory traffic): where paths with and without requests meet, the compiler waits for every request in flight.
+    auto step = [&](const int it, const int set) __attribute__((always_inline)) {
+        if (DEEP && (!SINGLE || it + STRIDE < it1)) {   // (single tokens: few steps, so that the last one's would weigh)
             load_keys(set ^ 1);
             load_values(set ^ 1);
             look_up(it + 2 * STRIDE);
@@ -629,7 +629,7 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
 #pragma unroll
                     for (int c = 0; c < C; c++)
                         s[p][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, kf[set][p][k]), qf[c][k], s[p][c], 0, 0, 0);
-        if (!DEEP && more) load_keys(0);
+        if (!DEEP) load_keys(0);
         // ---- weights
         const int pg0 = page_at(2 * it), pg1 = 2 * it + 1 < n_pages ? page_at(2 * it + 1) : 1 << 26;   // (a page that is not there lies past every query)
         auto open = [&](int pg) { return pg * 16 + 15 <= pos_lo && (pg * 16 > pos_hi - a.size || pg * 16 + 15 < a.keep); };
@@ -676,8 +676,9 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
             for (int i = 0; i < 8; i++) {
                 e[i] = __builtin_amdgcn_exp2f(e[i]);
                 part += e[i];
-                pw[c][i] = (__bf16)e[i];
             }
+            const f4_t lo = {e[0], e[1], e[2], e[3]}, hi = {e[4], e[5], e[6], e[7]};
+            pw[c] = __builtin_shufflevector(__builtin_convertvector(lo, b4_t), __builtin_convertvector(hi, b4_t), 0, 1, 2, 3, 4, 5, 6, 7);
             lsum[c] += part;
         }
         // ---- values
@@ -689,20 +690,26 @@ __global__ __launch_bounds__(64 * window_waves(VT, SINGLE), 2) void k_window_att
                 for (int c = 0; c < C; c++)
                     acc[v][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(b8_t, both), pw[c], acc[v][c], 0, 0, 0);
             }
-        if (!DEEP && more) {
+        if (!DEEP) {
             load_values(0);
             look_up(it + 2 * STRIDE);
         }
     };
-    if constexpr (DEEP) {
+    if (it0 < it1) {
+        look_up(it0);
+        load_keys(0);
+        load_values(0);
+        look_up(it0 + STRIDE);
+        if constexpr (DEEP) {
 #pragma clang loop unroll(disable)
-        for (int it = it0; it < it1; it += 2 * STRIDE) {
-            step(it, 0);
-            if (it + STRIDE < it1) step(it + STRIDE, 1);
+            for (int it = it0; it < it1; it += 2 * STRIDE) {
+                step(it, 0);
+                if (it + STRIDE < it1) step(it + STRIDE, 1);
+            }
+        } else {
+#pragma clang loop unroll(disable)
+            for (int it = it0; it < it1; it += STRIDE) step(it, 0);
         }
-    } else {
-#pragma clang loop unroll(disable)
-        for (int it = it0; it < it1; it += STRIDE) step(it, 0);
     }
 #pragma unroll
     for (int c = 0; c < C; c++) {   // the four lane rows of a column hold different keys
@@ -834,15 +841,14 @@ void launch_window_attention(const WindowAttn& w, const StepArrays& st) {
     if (st.n_multi > 0) {
         a.runs = (const int4*)st.d_runs;
         a.n_runs = st.n_multi;
-        // wide items share more of a page's load, narrow ones are more waves: the widest that still gives every SIMD two
-        static const int force = getenv("NVLLM_WINDOW_C") ? atoi(getenv("NVLLM_WINDOW_C")) : 0;
+        // wide items share more of a page's load, narrow ones are more waves: the widest that still gives every SIMD one
         int C = cls == 0 ? 4 : cls == 1 ? 2 : 1, waves = 0;
         for (;; C /= 2) {
             a.HW = rep >= C ? C : rep >= 2 && C >= 2 ? 2 : 1;
             a.NHG = cdiv(rep, a.HW);
             a.n_sub = cdiv(std::min(st.max_run, WINDOW_RUN), 16 * C / a.HW);
             waves = a.G * a.n_runs * a.n_sub * a.NHG;
-            if (C == 1 || (force ? C <= force : waves >= 8 * rt().num_cus)) break;
+            if (C == 1 || waves >= 4 * rt().num_cus) break;
         }
         const int grid = cdiv(waves, 4);
         const double rows = (double)st.multi_rows(seen_cap), pairs = (double)st.multi_pairs(seen_cap);

@@ -162,7 +162,7 @@ def reference(kv, q, pos, seq, scale, cap, size, keep):
 # heads, groups, dim, vdim, block size: every register class of the tiled kernel, exact and not; one and several heads per
 # group, more than 16, none that divides the item; sizes too wide for it, a block of three pages
 SHAPES = [(6, 2, 64, 64, 16), (4, 4, 16, 24, 32), (5, 1, 40, 80, 16), (8, 2, 128, 128, 64), (3, 1, 33, 112, 16), (3, 3, 192, 256, 16), (2, 1, 256, 64, 16),
-          (33, 1, 32, 32, 16), (16, 1, 64, 48, 16), (2, 1, 300, 40, 16), (6, 2, 24, 24, 48)]
+          (2, 2, 256, 256, 32), (4, 1, 128, 64, 16), (33, 1, 32, 32, 16), (16, 1, 64, 48, 16), (2, 1, 300, 40, 16), (6, 2, 24, 24, 48)]
 MASKS = [(72, 4, 30.0), (1, 0, 0.0), (33, 17, 60.0), (1 << 30, 0, 5.0), (16, 32, 0.0)]
 
 
@@ -185,6 +185,25 @@ def test_windowed_attention_of_a_ragged_batch(hip, H, G, dim, vdim, bs, elem):
         want = reference(kv, q, pos, seq, 2.5 * dim ** -0.5, cap, size, keep)
         worst = np.abs(got - want).max() / np.abs(want).max()
         assert worst < (2e-5 if elem == 4 else 8e-3) * 1.5, (size, keep, cap, worst)
+    pool.close()
+
+
+# batches large enough for items of two and four column groups: one head per group and several, exact sizes and not
+@pytest.mark.parametrize("H,G,dim,vdim,tokens", [(32, 32, 64, 64, 2048), (32, 8, 64, 64, 2048), (32, 8, 40, 48, 2048), (32, 32, 64, 64, 1024), (24, 8, 64, 64, 1536), (24, 8, 48, 40, 1536),
+                                                 (32, 32, 128, 128, 1024), (32, 16, 80, 112, 1024), (6, 2, 192, 160, 600)])
+def test_windowed_attention_of_large_batches(hip, H, G, dim, vdim, tokens):
+    n = tokens // 4
+    pool, kv = filled(hip, G, dim, vdim, 2, 16, [n + 30] * 4, tokens + dim)
+    r = rng(11)
+    seq = np.repeat(np.arange(4), n)
+    pos = np.concatenate([np.arange(n) + first for first in (0, 7, 16, 30)])
+    q = rounded(r.standard_normal((tokens, H, dim)), 2)
+    some = np.unique(np.concatenate([r.integers(0, tokens, 60), [0, n - 1, n, n + 1, tokens - 1]]))
+    for size, keep, cap in ((50, 5, 30.0), (77, 0, 0.0), (16, 40, 45.0)):
+        got = pool.attend(seq.tolist(), pos.tolist(), q, 2.5 * dim ** -0.5, cap, size, keep)
+        want = reference(kv, q[some], pos[some], seq[some], 2.5 * dim ** -0.5, cap, size, keep)
+        worst = np.abs(got[some] - want).max() / np.abs(want).max()
+        assert np.isfinite(got).all() and worst < 1.2e-2, (size, keep, cap, worst)
     pool.close()
 
 
