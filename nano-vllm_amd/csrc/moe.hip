@@ -3,6 +3,7 @@
 
 #include <algorithm>
 
+#include "attn_tile.h"
 #include "gemm_common.h"
 
 namespace nvllm {
@@ -37,6 +38,21 @@ RoutePlan route_plan(int* mem, int T, int E, int top, int pad) {
     return r;
 }
 
+// Maximum over a wave, in every lane, on the vector unit alone (many waves of one CU would queue for the LDS crossbar):
+// rotations within rows of 16 lanes, then the rows.
+template <int N>
+__device__ __forceinline__ float row_rotate(float x) {
+    const int v = __builtin_bit_cast(int, x);
+    return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(v, v, 0x120 + N, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float wave_max(float x) {
+    x = fmaxf(x, row_rotate<8>(x));
+    x = fmaxf(x, row_rotate<4>(x));
+    x = fmaxf(x, row_rotate<2>(x));
+    x = fmaxf(x, row_rotate<1>(x));
+    return rows_max(x);
+}
+
 // One wave chooses for one token: `top` times the best of what comes after the previous choice in the order
 // (score descending, index ascending).
 __device__ __forceinline__ void route_token(const RoutePlan& r, const float* __restrict__ z, int t, int lane) {
@@ -53,15 +69,12 @@ __device__ __forceinline__ void route_token(const RoutePlan& r, const float* __r
                 best_e = e;
             }
         }
+        const float top = wave_max(best);
+        int first = best == top ? best_e : 0x7fffffff;
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float v = __shfl_xor(best, o, 64);
-            const int e = __shfl_xor(best_e, o, 64);
-            if (v > best || (v == best && e < best_e)) {
-                best = v;
-                best_e = e;
-            }
-        }
+        for (int o = 32; o > 0; o >>= 1) first = min(first, __shfl_xor(first, o, 64));
+        best = top;
+        best_e = first;
         if (best_e >= r.E) best_e = 0;   // (no number compares: NaN logits)
         last = best;
         last_e = best_e;
@@ -80,14 +93,15 @@ __global__ __launch_bounds__(256) void k_route(RoutePlan r, const float* __restr
 // result does not depend on its place).
 template <bool CHOOSE>
 __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* __restrict__ z, int ldz) {
-    extern __shared__ int lds_r[];   // count / cursor [E], segment start [E + 1], CHOOSE: choices and scores [T * top]
-    int* cursor = lds_r;
-    int* start = lds_r + r.E;
+    extern __shared__ int lds_r[];   // counts [E], next free row [E], segment start [E + 1], CHOOSE: choices and scores [T * top]
+    int* count = lds_r;
+    int* cursor = count + r.E;
+    int* start = cursor + r.E;
     const int tid = threadIdx.x, lane = tid & 63, pairs = r.T * r.top;
     int *choice = CHOOSE ? start + r.E + 1 : r.choice, *out_choice = r.choice;
     float* out_score = r.score;
     float* score = CHOOSE ? reinterpret_cast<float*>(choice + pairs) : r.score;
-    for (int e = tid; e < r.E; e += 1024) cursor[e] = 0;
+    for (int e = tid; e < r.E; e += 1024) count[e] = 0;
     if (CHOOSE) {
         r.choice = choice;   // (route_token fills the LDS copies)
         r.score = score;
@@ -98,26 +112,13 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
                 for (int u = 0; u < 4; u++) v[u] = lane < r.E ? z[(size_t)min(t0 + 16 * u, r.T - 1) * ldz + lane] : -INFINITY;
                 for (int j = 0; j < r.top; j++) {
                     float best[4];
-                    int best_e[4];
+#pragma unroll
+                    for (int u = 0; u < 4; u++) best[u] = wave_max(v[u]);
 #pragma unroll
                     for (int u = 0; u < 4; u++) {
-                        best[u] = v[u];
-                        best_e[u] = v[u] > -INFINITY ? lane : 64;
-                    }
-#pragma unroll
-                    for (int o = 32; o > 0; o >>= 1)
-#pragma unroll
-                        for (int u = 0; u < 4; u++) {
-                            const float w = __shfl_xor(best[u], o, 64);
-                            const int e = __shfl_xor(best_e[u], o, 64);
-                            if (w > best[u] || (w == best[u] && e < best_e[u])) {
-                                best[u] = w;
-                                best_e[u] = e;
-                            }
-                        }
-#pragma unroll
-                    for (int u = 0; u < 4; u++) {
-                        const int t = t0 + 16 * u, e = best_e[u] < r.E ? best_e[u] : 0;   // (no number compares: NaN logits)
+                        const int t = t0 + 16 * u;
+                        const unsigned long long at = __ballot(v[u] == best[u] && lane < r.E);
+                        const int e = at ? __ffsll(at) - 1 : 0;   // (no number compares: NaN logits)
                         if (lane == e) v[u] = -INFINITY;
                         if (lane == 0 && t < r.T) {
                             choice[t * r.top + j] = e;
@@ -131,24 +132,24 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
         }
     }
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) atomicAdd(cursor + choice[i], 1);
+    for (int i = tid; i < pairs; i += 1024) atomicAdd(count + choice[i], 1);
     __syncthreads();
     if (tid < 64) {   // the first wave sums the padded counts
         int base = 0;
         for (int e0 = 0; e0 < r.E; e0 += 64) {
-            const int e = e0 + tid, n = e < r.E ? (cursor[e] + r.pad - 1) / r.pad * r.pad : 0;
+            const int e = e0 + tid, n = e < r.E ? (count[e] + r.pad - 1) / r.pad * r.pad : 0;
             int sum = n;
 #pragma unroll
             for (int o = 1; o < 64; o <<= 1) {
                 const int v = __shfl_up(sum, o, 64);
                 if (tid >= o) sum += v;
             }
-            if (e < r.E) start[e] = base + sum - n;
+            if (e < r.E) start[e] = cursor[e] = base + sum - n;
             base += __shfl(sum, 63, 64);
         }
         if (tid == 0) start[r.E] = base;
     }
-    __syncthreads();
+    __syncthreads();   // the last one: from here on everybody only writes results (a barrier would wait for the stores)
     const int used = start[r.E];
     for (int b = used / 16 + tid; b < r.capacity / 16; b += 1024) r.block_expert[b] = -1;
     for (int i = used + tid; i < r.capacity; i += 1024) {   // (a tile may look up rows behind its own: they name a token too)
@@ -156,16 +157,13 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
         r.weight[i] = 0.f;
     }
     for (int e = tid >> 4; e < r.E; e += 64) {   // 16 threads per expert: its blocks, and the padding of its segment
-        const int lo = start[e], hi = start[e + 1], n = cursor[e];
+        const int lo = start[e], hi = start[e + 1], n = count[e];
         for (int b = lo / 16 + (tid & 15); b < hi / 16; b += 16) r.block_expert[b] = e;
         for (int i = lo + n + (tid & 15); i < hi; i += 16) {
             r.source[i] = 0;
             r.weight[i] = 0.f;
         }
     }
-    __syncthreads();
-    for (int e = tid; e < r.E; e += 1024) cursor[e] = start[e];
-    __syncthreads();
     for (int i = tid; i < pairs; i += 1024) {
         const int row = atomicAdd(cursor + choice[i], 1);
         r.source[row] = i / r.top;
@@ -181,7 +179,7 @@ __global__ __launch_bounds__(1024) void k_route_sort(RoutePlan r, const float* _
 void launch_route(const RoutePlan& r, const float* z, int ldz) {
     if (r.T <= 0) return;
     if (r.E < 1 || r.E > MAX_EXPERTS || r.top < 1 || r.top > r.E) NVLLM_FATAL("routing: %d of %d experts per token", r.top, r.E);
-    const size_t lds = ((size_t)2 * r.E + 1) * sizeof(int);
+    const size_t lds = ((size_t)3 * r.E + 1) * sizeof(int);
     const double bytes = (double)r.T * (r.E * 4.0 + r.top * 20.0);
     const size_t lds_one = lds + (size_t)r.T * r.top * 8;
     if (r.T <= ROUTE_ONE && lds_one <= 64 * 1024) {
