@@ -250,7 +250,14 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T) {
         }
     Piece win[KEEP + 1], winz[KEEP + 1];   // inputs of tokens t - KEEP .. t
     int have = -1;                         // the token they are complete for, but for its own input
-    auto token = [&](const int t, const int4 span, const int row, const Piece own, const Piece ownz) __attribute__((always_inline)) {
+    // values of four tokens that are a quarter of a page: stored together, a dim's four keys lie side by side
+    bool quarter = false;
+    if (TOK % 4 == 0 && part == 2) {
+        const int off = t0 - spans[0].x;
+        quarter = t0 + TOK <= T && spans[TOK - 1].x == spans[0].x && (spans[0].z + off) % 4 == 0 && (off == 0 || off >= KEEP) && rows[0] >= 0 && rows[TOK - 1] >= 0;
+    }
+    Piece values[TOK];
+    auto token = [&](const int t, const int4 span, const int row, const Piece own, const Piece ownz, Piece& value) __attribute__((always_inline)) {
         const int off = t - span.x;
         __bf16* state = reinterpret_cast<__bf16*>(a.c.state) + (size_t)span.w * KEEP * a.channels + ch;
         if (have != t || off == 0) {
@@ -305,6 +312,8 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T) {
                 __bf16* k = reinterpret_cast<__bf16*>(a.pool.keys);
                 *reinterpret_cast<Piece*>(k + key_off(row, head, a.pool.G, d0, a.pool.dim_ld)) = py;
                 if (turns) *reinterpret_cast<Piece*>(k + key_off(row, head, a.pool.G, d0 + half, a.pool.dim_ld)) = pz;
+            } else if (quarter) {
+                value = py;
             } else {
                 __bf16* v = reinterpret_cast<__bf16*>(a.pool.values) + value_off(row, head, a.pool.G, d0, a.pool.vdim_ld);
 #pragma unroll
@@ -335,18 +344,29 @@ __global__ __launch_bounds__(256) void k_conv_rope_walk(ConvKArgs a, int T) {
     for (int u = 0; u < TOK; u++) {
         const int t = t0 + u, off = t - spans[u].x;
         // (a token that sees the state of a portion that starts in front of these belongs to the thread of its first token)
-        if (t < T && !(off > 0 && off < KEEP && spans[u].x < t0)) token(t, spans[u], rows[u], in[u], inz[u]);
+        if (t < T && !(off > 0 && off < KEEP && spans[u].x < t0)) token(t, spans[u], rows[u], in[u], inz[u], values[u]);
     }
+    if (quarter) {
+#pragma unroll
+        for (int u = 0; u + 3 < TOK; u += 4) {
+            b4_t* v = reinterpret_cast<b4_t*>(reinterpret_cast<__bf16*>(a.pool.values) + value_off(rows[u], head, a.pool.G, d0, a.pool.vdim_ld));
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = b4_t{values[u].v[e], values[u + 1].v[e], values[u + 2].v[e], values[u + 3].v[e]};
+        }
+    }
+    Piece unused;
+    quarter = false;
     const int4 last = spans[TOK - 1];   // the portion the next tokens may belong to
     for (int t = t0 + TOK; t < last.x + min(last.y, KEEP) && last.x >= t0; t++)
-        token(t, last, a.kv_row[t], *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld), *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner));
+        token(t, last, a.kv_row[t], *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld), *reinterpret_cast<const Piece*>(raw + (size_t)t * a.c.raw_ld + partner), unused);
 }
 
 template <int KEEP>
 static void launch_walk(const ConvKArgs& a, int T) {
     const dim3 threads(std::min(256, (a.items + 63) & ~63));
     const int y = cdiv(a.items, 256);
-    if (T >= 1024) NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 4>), dim3(cdiv(T, 4), y), threads, 0, a, T);
+    if ((long)T * a.items >= 4L * 64 * 16 * rt().num_cus)   // (enough waves even so; fewer loads of the taps)
+        NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 4>), dim3(cdiv(T, 4), y), threads, 0, a, T);
     else if (T >= 256) NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 2>), dim3(cdiv(T, 2), y), threads, 0, a, T);
     else NVLLM_LAUNCH((k_conv_rope_walk<KEEP, 1>), dim3(T, y), threads, 0, a, T);
 }

@@ -130,6 +130,39 @@ def test_convolution_rotation_and_cache(hip, H, G, dim, vdim, taps, rot, bs, ele
     pool.close()
 
 
+@pytest.mark.parametrize("H,G,dim,vdim,cuts", [(4, 2, 32, 32, [[257, 300], [1, 90], [40]]), (96, 96, 128, 128, [[301, 1], [402, 7], [200, 95]])])
+def test_convolution_of_large_batches(hip, H, G, dim, vdim, cuts):
+    """Batches large enough for threads that walk two and four tokens: portions that start anywhere among them."""
+    r = rng(H)
+    channels, taps, base = H * dim + G * (dim + vdim), 4, 500.0
+    w = np.asarray(r.standard_normal((channels, taps)), np.float32).astype(np.float64)
+    pool = WindowPool(hip, G, dim, vdim, 2, 16, 150)
+    seqs = [pool.sequence(list(range(50 * i, 50 * i + 50))) for i in range(3)]
+    u = [rounded(r.standard_normal((sum(c), channels)), 2) for c in cuts]
+    state = hip.to_device(np.zeros(3 * 3 * channels, np.uint16))
+    at, got = [0, 0, 0], [[], [], []]
+    for step in range(2):
+        ids, pos, raw = [], [], []
+        for s in (1, 0, 2):
+            k = cuts[s][step] if step < len(cuts[s]) else 0
+            ids += [s] * k
+            pos += list(range(at[s], at[s] + k))
+            raw.append(u[s][at[s]:at[s] + k])
+            at[s] += k
+        q = pool.conv(ids, pos, np.concatenate(raw), H, w, state, base, dim)
+        for s in seqs:
+            got[s].append(q[[i for i, x in enumerate(ids) if x == s]])
+    for s in seqs:
+        n = len(u[s])
+        q, k, v = np.split(O.causal_conv(u[s], w), [H * dim, (H + G) * dim], axis=1)
+        q, k = (O.rotate_half(z.reshape(n, -1, dim), np.arange(n), base, dim) for z in (q, k))
+        have_k, have_v = pool.rows(s, n)
+        for have, want in ((np.concatenate(got[s]), q), (have_k, k), (have_v, v.reshape(n, G, vdim))):
+            np.testing.assert_allclose(have, want, rtol=2.0 ** -7, atol=2e-3)
+    hip.free(state)
+    pool.close()
+
+
 # ------------------------------------------------------------------ attention
 def filled(hip, G, dim, vdim, elem, bs, lengths, seed, spread=1.0):
     r = rng(seed)
