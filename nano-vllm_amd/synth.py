@@ -233,7 +233,7 @@ def lightning_mixer(heads, dim, vdim, decay=None) -> dict:
     return dict(heads=heads, dim=dim, vdim=vdim, decay=[float(d) for d in decay])
 
 
-def window_mixer(heads, kv_heads, dim, vdim, size, keep_first, taps=4, rot=None, base=10000.0, scale=None, softcap=30.0) -> dict:
+def window_mixer(heads, kv_heads, dim, vdim, size, keep_first, taps=4, rot=None, base=10000.0, scale=None, softcap=25.0) -> dict:
     return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=taps, mask=dict(size=size, keep_first=keep_first), softcap=softcap,
                 rot=dict(base=float(base), dims=dim if rot is None else rot), scale=float(dim ** -0.5 if scale is None else scale))
 

@@ -196,7 +196,7 @@ def reference(kv, q, pos, seq, scale, cap, size, keep):
 # group, more than 16, none that divides the item; sizes too wide for it, a block of three pages
 SHAPES = [(6, 2, 64, 64, 16), (4, 4, 16, 24, 32), (5, 1, 40, 80, 16), (8, 2, 128, 128, 64), (3, 1, 33, 112, 16), (3, 3, 192, 256, 16), (2, 1, 256, 64, 16),
           (2, 2, 256, 256, 32), (4, 1, 128, 64, 16), (33, 1, 32, 32, 16), (16, 1, 64, 48, 16), (2, 1, 300, 40, 16), (6, 2, 24, 24, 48)]
-MASKS = [(72, 4, 30.0), (1, 0, 0.0), (33, 17, 60.0), (1 << 30, 0, 5.0), (16, 32, 0.0)]
+MASKS = [(70, 5, 28.0), (1, 0, 0.0), (33, 17, 60.0), (1 << 30, 0, 5.0), (16, 32, 0.0)]
 
 
 @BOTH
@@ -232,7 +232,7 @@ def test_windowed_attention_of_large_batches(hip, H, G, dim, vdim, tokens):
     pos = np.concatenate([np.arange(n) + first for first in (0, 7, 16, 30)])
     q = rounded(r.standard_normal((tokens, H, dim)), 2)
     some = np.unique(np.concatenate([r.integers(0, tokens, 60), [0, n - 1, n, n + 1, tokens - 1]]))
-    for size, keep, cap in ((50, 5, 30.0), (77, 0, 0.0), (16, 40, 45.0)):
+    for size, keep, cap in ((50, 5, 27.0), (77, 0, 0.0), (16, 40, 45.0)):
         got = pool.attend(seq.tolist(), pos.tolist(), q, 2.5 * dim ** -0.5, cap, size, keep)
         want = reference(kv, q[some], pos[some], seq[some], 2.5 * dim ** -0.5, cap, size, keep)
         worst = np.abs(got[some] - want).max() / np.abs(want).max()
@@ -269,7 +269,7 @@ def test_one_key_stands_out(hip, elem, decode, size, keep):
 @pytest.mark.parametrize("cap", [0.0, 20.0, 60.0])
 def test_slices_of_pages_and_one_slice_agree(hip, cap):
     """A lone long sequence is cut into slices whose partial results are merged; many of them are not: same rows, same result."""
-    H, G, dim, vdim, n = 6, 2, 64, 80, 3000
+    H, G, dim, vdim, n = 6, 2, 64, 88, 3000
     pool, kv = filled(hip, G, dim, vdim, 2, 16, [n], 9)
     q = rounded(rng(2).standard_normal((1, H, dim)), 2)
     one = pool.attend([0], [n - 1], q, 0.2, cap, 2900, 5)
